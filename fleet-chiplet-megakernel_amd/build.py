@@ -1,35 +1,38 @@
-"""Build libfleet_mk.so (HIP kernel + C-ABI host library) for gfx950 with hipcc.
+"""Build libfleet_mk.so (HIP kernels + C-ABI host library) for gfx950 with hipcc.
 
 Usage: python build.py            (from anywhere; output lands next to this file: the library, then the Cython binding
                                    mirage/_cython/core.*.so that links against it)
+
+Every kernel instantiation is a translation unit of its own; they compile side by side.  `build(kernels=...)` makes a
+library with only some of them (a graph that needs a missing one is refused by mk_compile); `ensure_library()` is what a
+program calls that wants to run one kind of graph from a fresh checkout.
 """
 import os
 import shutil
 import subprocess
 import sys
+import tempfile
+from concurrent.futures import ThreadPoolExecutor
 
 HERE = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(HERE, "csrc")
 LIB = os.path.join(HERE, "libfleet_mk.so")
+
+# kernel instantiations of mk_kernel.hip (-DMK_KERNEL_<name>)
+KERNELS = ("GENERAL", "M1", "FLEX", "FLEX_M1", "FLEX_F32")
 
 HIPCC_FLAGS = [
     "--offload-arch=gfx950",
     "-O3",
     "-std=c++17",
     "-fPIC",
-    "-shared",
     # packed fp32 VALU forms are disabled for all device code
     "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",
-    "-Wno-unused-command-line-argument",
+    "-Wno-unused-command-line-argument", "-Wno-pass-failed",
 ]
 
 
-def build(verbose: bool = True, defines=(), out: str = None) -> str:
-    hipcc = shutil.which("hipcc") or "/opt/rocm/bin/hipcc"
-    if not os.path.exists(hipcc):
-        raise RuntimeError("hipcc not found: the megakernel library cannot be built")
-    lib = out or LIB
-    cmd = [hipcc] + HIPCC_FLAGS + ["-D" + d for d in defines] + [os.path.join(CSRC, "fleet_mk.hip"), "-o", lib]
+def _run(cmd, verbose):
     if verbose:
         print(" ".join(cmd), flush=True)
     res = subprocess.run(cmd, cwd=CSRC, stdout=subprocess.PIPE, stderr=subprocess.STDOUT, text=True)
@@ -38,6 +41,37 @@ def build(verbose: bool = True, defines=(), out: str = None) -> str:
         raise RuntimeError("hipcc failed:\n" + out)
     if verbose and out.strip():
         print(out)
+
+
+def build(verbose: bool = True, defines=(), out: str = None, kernels=KERNELS) -> str:
+    hipcc = shutil.which("hipcc") or "/opt/rocm/bin/hipcc"
+    if not os.path.exists(hipcc):
+        raise RuntimeError("hipcc not found: the megakernel library cannot be built")
+    lib = out or LIB
+    extra = ["-D" + d for d in defines]
+    with tempfile.TemporaryDirectory(prefix="fleet_mk_build_") as tmp:
+        units = [(k.lower(), ["-DMK_KERNEL_" + k, "mk_kernel.hip"]) for k in kernels]
+        units.append(("pack", ["mk_pack.hip"]))
+        units.append(("host", ["-DMK_HAVE_KERNEL_" + k for k in kernels] + ["-x", "hip", "mk_host.cpp"]))
+        objs = [os.path.join(tmp, name + ".o") for name, _ in units]
+        workers = min(len(units), int(os.environ.get("MAX_JOBS", "8")))
+        with ThreadPoolExecutor(workers) as pool:
+            list(pool.map(lambda u: _run([hipcc] + HIPCC_FLAGS + extra + ["-c"] + u[0][1] + ["-o", u[1]], verbose), zip(units, objs)))
+        part = os.path.join(os.path.dirname(lib), f".{os.path.basename(lib)}.{os.getpid()}")
+        _run([hipcc, "--offload-arch=gfx950", "-shared", "-fPIC"] + objs + ["-o", part], verbose)
+        os.replace(part, lib)  # a program that finds the library finds all of it
+    return lib
+
+
+def ensure_library(kernels) -> str:
+    """Path of a built library that holds `kernels`: the full one when it is there, else one with exactly these, compiled
+    on first use."""
+    if os.path.exists(LIB):
+        return LIB
+    lib = os.path.join(HERE, "libfleet_mk_" + "_".join(k.lower() for k in kernels) + ".so")
+    if not os.path.exists(lib):
+        print("compiling " + ", ".join(kernels), file=sys.stderr, flush=True)
+        build(verbose=False, out=lib, kernels=kernels)
     return lib
 
 

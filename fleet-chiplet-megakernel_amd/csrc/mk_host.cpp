@@ -22,6 +22,26 @@
 #include "../../include/fleet_mk.h"
 #include "mk_types.h"
 
+typedef unsigned u32x4 __attribute__((ext_vector_type(4)));
+
+// the kernels, each from a translation unit of its own (build.py); a library may be built without some of them
+extern "C" __global__ void mk_pack_weights_kernel(const MkWeight w, int n, int k, int silu, int half, u32x4 *dst, long long total);
+#define MK_DECLARE_KERNEL(name) extern "C" __global__ void name(const MkRuntime rt, const MkRuntime *rtp, int max_iters, int run_scheduler)
+#ifdef MK_HAVE_KERNEL_GENERAL
+MK_DECLARE_KERNEL(mk_persistent_kernel);
+#endif
+#ifdef MK_HAVE_KERNEL_M1
+MK_DECLARE_KERNEL(mk_persistent_kernel_m1);
+#endif
+#ifdef MK_HAVE_KERNEL_FLEX
+MK_DECLARE_KERNEL(mk_persistent_kernel_flex);
+#endif
+#ifdef MK_HAVE_KERNEL_FLEX_M1
+MK_DECLARE_KERNEL(mk_persistent_kernel_flex_m1);
+#endif
+#ifdef MK_HAVE_KERNEL_FLEX_F32
+MK_DECLARE_KERNEL(mk_persistent_kernel_flex_f32);
+#endif
 
 namespace {
 
@@ -44,6 +64,7 @@ int fail(int code, const char *fmt, ...) {
   } while (0)
 
 enum TensorKind { T_ATTACHED, T_OWNED, T_SHUFFLED };
+enum FlexKind { FLEX_NONE, FLEX_BF16, FLEX_F32 };  // which stage set (and activation type) a graph runs on
 
 struct Tensor {
   std::string name;
@@ -126,6 +147,9 @@ struct mk_graph {
   void *profiler_ptr = nullptr;  // the caller's profiler tensor (mk_set_profiler)
   long long profiler_cap = 0;
   int64_t row_major_bytes = 0;
+  int flex = FLEX_NONE;
+  size_t flex_items = 0;     // most work items of a flex attention stage (row tiles x kv heads x value slices)
+  size_t flex_part = 0;      // floats of split-KV partials the flex attention stages need
 };
 
 namespace {
@@ -181,11 +205,11 @@ bool linear_kind(const std::string &n, bool *res, bool *silu, int *n_extra_input
   return false;
 }
 
-int resolve_weight(mk_graph *g, int id, int64_t k, MkWeight *w, int64_t *rows_out, int *group_half) {
+int resolve_weight(mk_graph *g, int id, int64_t k, MkWeight *w, int64_t *rows_out, int *group_half, int dtype = MK_DT_BF16) {
   const Tensor &t = g->tensors[id];
   memset(w, 0, sizeof(*w));
   if (t.ndims != 2) return fail(MK_EINVAL, "weight '%s' must be 2-D", t.name.c_str());
-  if (t.dtype != MK_DT_BF16) return fail(MK_EINVAL, "weight '%s' must be bf16", t.name.c_str());
+  if (t.dtype != dtype) return fail(MK_EINVAL, "weight '%s' must be %s", t.name.c_str(), dtype == MK_DT_F32 ? "fp32, like the activations" : "bf16");
   if (t.dims[1] != k) return fail(MK_EINVAL, "weight '%s' has k=%lld, expected %lld", t.name.c_str(), (long long)t.dims[1], (long long)k);
   *rows_out = t.dims[0];
   *group_half = 0;
@@ -230,7 +254,24 @@ int num_outputs(const Task &t) {
   if (t.name == "gang_attn_split_kv_mi300") return 3;
   if (t.name == "paged_attention_ck_fmha_split_kv_mi300" || t.name == "paged_attention_split_kv_mi300") return 2;
   if (t.name == "moe_topk_softmax_mi300") return 3;
+  if (t.name == "embedding_scaled" || t.name == "residual_rmsnorm") return 2;
   return 1;
+}
+
+// constants of the flex tasks travel as the bits of a float in an int parameter
+float bits_f32(int bits) {
+  float f;
+  memcpy(&f, &bits, sizeof(f));
+  return f;
+}
+
+// a graph holds flex stages of one activation type, and none of the fixed-shape stages next to them (checked after lowering)
+int set_flex(mk_graph *g, int dtype, const char *task) {
+  const int kind = dtype == MK_DT_F32 ? FLEX_F32 : FLEX_BF16;
+  if (dtype != MK_DT_F32 && dtype != MK_DT_BF16) return fail(MK_EINVAL, "task '%s': activations must be bf16 or fp32", task);
+  if (g->flex != FLEX_NONE && g->flex != kind) return fail(MK_EINVAL, "task '%s': the graph mixes bf16 and fp32 activations", task);
+  g->flex = kind;
+  return MK_OK;
 }
 
 // Lower one linear-type task (optionally preceded by a norm task whose output it consumes, optionally
@@ -264,16 +305,21 @@ int lower_linear(mk_graph *g, size_t &i) {
   const Tensor &tin = g->tensors[in_id];
   Tensor &tout = g->tensors[out_id];
   if (tin.ndims != 2 || tout.ndims != 2) return fail(MK_EINVAL, "task '%s': input/output must be 2-D", lt.name.c_str());
-  if (tin.dtype != MK_DT_BF16 || tout.dtype != MK_DT_BF16) return fail(MK_EINVAL, "task '%s': activations must be bf16", lt.name.c_str());
+  const bool f32 = tin.dtype == MK_DT_F32;  // 32-bit linear: plain or SwiGLU, part of a flex graph
+  if (tin.dtype != tout.dtype || (tin.dtype != MK_DT_BF16 && (!f32 || res || norm))) return fail(MK_EINVAL, "task '%s': activations must be bf16", lt.name.c_str());
+  if (f32) {
+    int rc = set_flex(g, MK_DT_F32, lt.name.c_str());
+    if (rc) return rc;
+  }
   MkStage st;
   memset(&st, 0, sizeof(st));
-  st.op = MK_OP_LINEAR;
+  st.op = f32 ? MK_OP_LINEAR_F32 : MK_OP_LINEAR;
   st.k = (int)tin.dims[1];
   if (st.k % 8) return fail(MK_EINVAL, "task '%s': reduction length %d must be a multiple of 8", lt.name.c_str(), st.k);
   if (g->cfg.max_num_batched_tokens > 1 && st.k % 32) return fail(MK_EINVAL, "task '%s': reduction length %d must be a multiple of 32 when more than one token is batched", lt.name.c_str(), st.k);
   int64_t rows;
   int half;
-  int rc = resolve_weight(g, w_id, st.k, &st.w, &rows, &half);
+  int rc = resolve_weight(g, w_id, st.k, &st.w, &rows, &half, tin.dtype);
   if (rc) return rc;
   st.n = (int)rows;
   st.eps = g->cfg.rms_eps;
@@ -299,6 +345,7 @@ int lower_linear(mk_graph *g, size_t &i) {
   }
   const Tensor &tfo = g->tensors[final_out];
   const int n_out = (st.flags & MK_F_SILU) ? st.n / 2 : st.n;
+  if (tfo.dtype != tin.dtype) return fail(MK_EINVAL, "task '%s': output '%s' has another type than the input", lt.name.c_str(), tfo.name.c_str());
   if (tfo.ndims != 2 || tfo.dims[1] < n_out) return fail(MK_EINVAL, "task '%s': output '%s' has %lld columns, need %d", lt.name.c_str(), tfo.name.c_str(), (long long)tfo.dims[1], n_out);
   if (tin.dims[0] < g->cfg.max_num_batched_tokens || tfo.dims[0] < g->cfg.max_num_batched_tokens)
     return fail(MK_EINVAL, "task '%s': activations need at least max_num_batched_tokens=%d rows", lt.name.c_str(), g->cfg.max_num_batched_tokens);
@@ -348,10 +395,10 @@ int lower_linear(mk_graph *g, size_t &i) {
     st.ld_norm = (int)no.strides[0];
   }
   g->stages.push_back(st);
-  g->stage_desc.push_back(fmt("LINEAR%s%s%s %s x %s -> %s n=%d k=%d segs=%d", (st.flags & MK_F_NORM) ? "+norm" : "", (st.flags & MK_F_RES) ? "+res" : "",
+  g->stage_desc.push_back(fmt("LINEAR%s%s%s%s %s x %s -> %s n=%d k=%d segs=%d", f32 ? "_F32" : "", (st.flags & MK_F_NORM) ? "+norm" : "", (st.flags & MK_F_RES) ? "+res" : "",
                               (st.flags & MK_F_SILU) ? "+silu" : "", tin.name.c_str(), g->tensors[w_id].name.c_str(), tfo.name.c_str(), st.n, st.k,
                               st.w.nseg));
-  g->weight_bytes += (int64_t)st.n * st.k * 2;
+  g->weight_bytes += (int64_t)st.n * st.k * (int64_t)dtype_size(tin.dtype);
   g->stage_weight.resize(g->stages.size(), -1);
   g->stage_weight.back() = w_id;
   g->last_linear_task = (int)i;
@@ -582,6 +629,195 @@ int lower_attention(mk_graph *g, size_t &i) {
 }
 
 
+// ---- flex tasks (mk_flex.hip): sizes and constants are data --------------------------------------------------------
+// embedding_scaled [ids, table, residual rows (fp32), rows] params [source, scale bits]
+int lower_embedding_scaled(mk_graph *g, size_t &i) {
+  const Task &t = g->ltasks[i];
+  if (t.ops.size() != 4 || t.params.size() != 2) return fail(MK_EINVAL, "embedding_scaled expects 4 operands / 2 params");
+  const Tensor &ids = g->tensors[t.ops[0]], &w = g->tensors[t.ops[1]], &r = g->tensors[t.ops[2]], &o = g->tensors[t.ops[3]];
+  const int B = g->cfg.max_num_batched_tokens;
+  if (ids.dtype != MK_DT_I64 || (int64_t)ids.elems() < B) return fail(MK_EINVAL, "embedding_scaled: ids must be int64, one per token row");
+  if (w.ndims != 2 || o.ndims != 2 || r.ndims != 2 || o.dims[1] < w.dims[1] || r.dims[1] < w.dims[1] || o.dims[0] < B || r.dims[0] < B || w.dtype != o.dtype || r.dtype != MK_DT_F32 ||
+      w.kind == T_SHUFFLED || (o.strides[0] & 3) || (r.strides[0] & 3))
+    return fail(MK_EINVAL, "embedding_scaled shapes mismatch");
+  int rc = set_flex(g, o.dtype, "embedding_scaled");
+  if (rc) return rc;
+  MkStage st;
+  memset(&st, 0, sizeof(st));
+  st.op = MK_OP_FX_EMBED;
+  st.k = (int)w.dims[1];
+  st.in = ids.ptr;
+  st.out = o.ptr;
+  st.ld_out = (int)o.strides[0];
+  st.out2 = r.ptr == o.ptr ? nullptr : r.ptr;
+  st.ld_out2 = (int)r.strides[0];
+  st.alpha = bits_f32(t.params[1]);
+  st.w.nseg = 1;
+  st.w.seg[0] = w.ptr;
+  if (t.params[0] == 0) st.flags |= MK_F_EMBED_FROM_TOKENS;
+  g->stages.push_back(st);
+  g->stage_desc.push_back(fmt("FX_EMBED %s[%s] * %g -> %s, %s k=%d", w.name.c_str(), ids.name.c_str(), st.alpha, r.name.c_str(), o.name.c_str(), st.k));
+  i++;
+  return MK_OK;
+}
+
+// residual_rmsnorm [y (optional), residual (fp32), weight (fp32), new residual (fp32), rows] params [width, alpha bits, eps
+// bits, weight offset bits]: v = alpha * residual + y, both outputs = v / rms(v) * (offset + weight).  A bf16 linear that
+// reads the rows next forms them itself when an iteration has one token; a linear that wrote y may leave its K-slice sum.
+int lower_residual_rmsnorm(mk_graph *g, size_t &i) {
+  const Task t = g->ltasks[i];
+  if (t.ops.size() != 5 || t.params.size() != 4) return fail(MK_EINVAL, "residual_rmsnorm expects 5 operands / 4 params");
+  const Tensor *y = t.ops[0] >= 0 ? &g->tensors[t.ops[0]] : nullptr;
+  const Tensor x = g->tensors[t.ops[1]], w = g->tensors[t.ops[2]], xo = g->tensors[t.ops[3]], o = g->tensors[t.ops[4]];
+  const int B = g->cfg.max_num_batched_tokens, width = t.params[0];
+  const int64_t n = o.dims[1];
+  int rc = set_flex(g, o.dtype, "residual_rmsnorm");
+  if (rc) return rc;
+  if (o.ndims != 2 || x.ndims != 2 || xo.ndims != 2 || n % 4 || width < 1 || width > n || x.dims[1] != n || xo.dims[1] != n || (int64_t)w.elems() != n ||
+      (y && (y->ndims != 2 || y->dims[1] != n || y->dtype != o.dtype || y->dims[0] < B)) || o.dims[0] < B || x.dims[0] < B || xo.dims[0] < B)
+    return fail(MK_EINVAL, "residual_rmsnorm: every row tensor is [tokens, %lld] (a multiple of 4), the weight has as many entries, width=%d of them real", (long long)n, width);
+  if (x.dtype != MK_DT_F32 || xo.dtype != MK_DT_F32 || w.dtype != MK_DT_F32) return fail(MK_EINVAL, "residual_rmsnorm: residual rows and norm weight are fp32");
+  if (n > 12 * 4 * MK_THREADS) return fail(MK_EUNSUPPORTED, "residual_rmsnorm: rows of %lld values (most %d)", (long long)n, 12 * 4 * MK_THREADS);
+  if (x.ptr == xo.ptr && xo.ptr != o.ptr) return fail(MK_EINVAL, "residual_rmsnorm: the new residual rows must not overwrite the old ones (other workgroups may still read them)");
+  MkStage st;
+  memset(&st, 0, sizeof(st));
+  st.op = MK_OP_FX_ADDNORM;
+  st.n = (int)n;
+  st.k = width;
+  st.alpha = bits_f32(t.params[1]);
+  st.eps = bits_f32(t.params[2]);
+  st.w_offset = bits_f32(t.params[3]);
+  st.in = y ? y->ptr : nullptr;
+  st.ld_in = y ? (int)y->strides[0] : 0;
+  st.res = x.ptr;
+  st.ld_res = (int)x.strides[0];
+  st.norm_w = w.ptr;
+  st.out = o.ptr;
+  st.ld_out = (int)o.strides[0];
+  st.out2 = xo.ptr == o.ptr ? nullptr : xo.ptr;
+  st.ld_out2 = (int)xo.strides[0];
+  if ((st.ld_in | st.ld_res | st.ld_out | st.ld_out2) & 3) return fail(MK_EINVAL, "residual_rmsnorm: row strides must be multiples of 4");
+  if (!g->stages.empty()) {
+    MkStage &pl = g->stages.back();
+    if (pl.op == MK_OP_LINEAR && !(pl.flags & (MK_F_SILU | MK_F_RES)) && y && pl.out == st.in && pl.ld_out == st.ld_in && pl.n == st.n && width == n)
+      pl.flags |= MK_F_DEFER_SUM;
+    if (pl.out != st.res && pl.out2 != st.res && pl.norm_out != st.res) st.flags |= MK_F_RES_EARLY;
+  }
+  bool res, silu;
+  int extra;
+  const bool fuse = g->flex == FLEX_BF16 && i + 1 < g->ltasks.size() && linear_kind(g->ltasks[i + 1].name, &res, &silu, &extra) && !res && g->ltasks[i + 1].ops[0] == t.ops[4];
+  if (fuse) st.flags |= MK_F_ONLY_MULTI;
+  g->stages.push_back(st);
+  g->stage_desc.push_back(fmt("FX_ADDNORM%s %g * %s + %s -> %s, %s k=%d", fuse ? "[multi-token only]" : "", st.alpha, x.name.c_str(), y ? y->name.c_str() : "0", xo.name.c_str(), o.name.c_str(), width));
+  i++;
+  if (!fuse) return MK_OK;
+  rc = lower_linear(g, i);
+  if (rc) return rc;
+  MkStage &l = g->stages.back();
+  l.flags |= MK_F_NORM | MK_F_ADDNORM | (st.flags & MK_F_RES_EARLY);
+  l.y_in = st.in;
+  l.ld_y = st.ld_in;
+  l.res = st.res;
+  l.ld_res = st.ld_res;
+  l.norm_w = st.norm_w;
+  l.norm_out = st.out;
+  l.ld_norm = st.ld_out;
+  l.out2 = st.out2;
+  l.ld_out2 = st.ld_out2;
+  l.alpha = st.alpha;
+  l.w_offset = st.w_offset;
+  l.norm_eps = st.eps;
+  l.k_real = width;
+  return MK_OK;
+}
+
+// flex_attention [qkv rows, k cache, v cache, cos (optional), sin (optional), sink (optional), q workspace, output]
+// params [q heads, kv heads, head dim, value dim, rotated dims, unit norm 0/1, eps bits, scale bits, softcap bits].  The
+// qkv rows are all query heads, then all key heads, then all value heads; caches are [pages, page_size, kv heads, padded
+// dim] with a layout of the library's own inside a page.
+int lower_flex_attention(mk_graph *g, size_t &i) {
+  const Task &t = g->ltasks[i];
+  if (t.ops.size() != 8 || t.params.size() != 9) return fail(MK_EINVAL, "flex_attention expects 8 operands / 9 params");
+  const Tensor &in = g->tensors[t.ops[0]], &kc = g->tensors[t.ops[1]], &vc = g->tensors[t.ops[2]], &qw = g->tensors[t.ops[6]], &o = g->tensors[t.ops[7]];
+  const int B = g->cfg.max_num_batched_tokens, ps = g->cfg.page_size;
+  const int H = t.params[0], G = t.params[1], D = t.params[2], DV = t.params[3], rot = t.params[4];
+  int rc = set_flex(g, in.dtype, "flex_attention");
+  if (rc) return rc;
+  const bool f32 = in.dtype == MK_DT_F32;
+  const int es = f32 ? 4 : 2, KW = f32 ? 16 : 32, TP = f32 ? 16 : 32;
+  if (H < 1 || G < 1 || H % G || D < 1 || DV < 1 || rot < 0 || rot > D || rot % 2) return fail(MK_EINVAL, "flex_attention: heads %d / %d, dims %d / %d, rotated %d", H, G, D, DV, rot);
+  if (D > MK_FX_MAX_HEAD_DIM) return fail(MK_EUNSUPPORTED, "flex_attention: head dim %d (most %d)", D, MK_FX_MAX_HEAD_DIM);
+  const int dk = (D + KW - 1) / KW * KW, dv = (DV + 15) / 16 * 16;
+  if (in.ndims != 2 || in.dims[0] < B || in.dims[1] < (int64_t)H * D + (int64_t)G * (D + DV)) return fail(MK_EINVAL, "flex_attention: input must be [tokens, >= (q + kv) * dim + kv * value dim]");
+  if (o.ndims != 2 || o.dims[0] < B || o.dims[1] < (int64_t)H * DV || o.dtype != in.dtype) return fail(MK_EINVAL, "flex_attention: output must be [tokens, >= q heads * value dim] of the input's type");
+  if (qw.ndims != 2 || qw.dims[0] < B || qw.dims[1] < (int64_t)H * dk || qw.dtype != in.dtype || (qw.strides[0] * es) % 16) return fail(MK_EINVAL, "flex_attention: q workspace must be [tokens, >= q heads * %d]", dk);
+  if (kc.ndims != 4 || vc.ndims != 4 || kc.dtype != in.dtype || vc.dtype != in.dtype || kc.dims[0] < g->cfg.max_num_pages || vc.dims[0] < g->cfg.max_num_pages || kc.dims[1] != ps ||
+      vc.dims[1] != ps || kc.dims[2] != G || vc.dims[2] != G || kc.dims[3] != dk || vc.dims[3] != dv)
+    return fail(MK_EINVAL, "flex_attention: caches must be [>= %d pages, %d, %d, %d] and [.., %d], of the input's type", g->cfg.max_num_pages, ps, G, dk, dv);
+  if (ps % TP) return fail(MK_EINVAL, "flex_attention: page_size %d must be a multiple of %d", ps, TP);
+  if ((int64_t)kc.elems() / 8 > 0x7fffffffll * 16) return fail(MK_EUNSUPPORTED, "flex_attention: cache too large");
+  MkStage st;
+  memset(&st, 0, sizeof(st));
+  st.op = MK_OP_FX_ATTN;
+  st.in = in.ptr;
+  st.ld_in = (int)in.strides[0];
+  st.out = o.ptr;
+  st.ld_out = (int)o.strides[0];
+  st.k_cache = kc.ptr;
+  st.v_cache = vc.ptr;
+  st.q_ws = qw.ptr;
+  st.ld_qws = (int)qw.strides[0];
+  st.num_q_heads = H;
+  st.num_kv_heads = G;
+  st.head_dim = D;
+  st.v_dim = DV;
+  st.rot_dims = rot;
+  st.eps = bits_f32(t.params[6]);
+  st.sm_scale = bits_f32(t.params[7]);
+  st.softcap = bits_f32(t.params[8]);
+  if (t.params[5]) st.flags |= MK_F_QK_NORM;
+  if (rot > 0) {
+    if (t.ops[3] < 0 || t.ops[4] < 0) return fail(MK_EINVAL, "flex_attention: rotated dims without cos / sin tables");
+    const Tensor &c = g->tensors[t.ops[3]], &s = g->tensors[t.ops[4]];
+    if (c.dtype != MK_DT_F32 || s.dtype != MK_DT_F32 || c.ndims != 2 || s.ndims != 2 || c.dims[1] != rot / 2 || s.dims[1] != rot / 2 || c.dims[0] < g->cfg.max_seq_length ||
+        s.dims[0] < g->cfg.max_seq_length || c.strides[0] != s.strides[0])
+      return fail(MK_EINVAL, "flex_attention: cos / sin tables must be fp32 [>= max_seq_length, rotated dims / 2]");
+    st.flags |= MK_F_ROPE;
+    st.cos_tab = c.ptr;
+    st.sin_tab = s.ptr;
+    st.ld_cos = (int)c.strides[0];
+  }
+  if (t.ops[5] >= 0) {
+    const Tensor &s = g->tensors[t.ops[5]];
+    if (s.dtype != MK_DT_F32 || (int64_t)s.elems() != H) return fail(MK_EINVAL, "flex_attention: the sink holds one fp32 value per query head");
+    st.sink = s.ptr;
+  }
+  // instantiation: 16-byte key operand rows and 16-wide value blocks a tile load holds (mk_flex.hip: stage_fx_attn)
+  st.k_tiles = f32 ? 8 : (dk <= 64 && dv <= 64 ? 2 : 4);
+  st.v_tiles = f32 ? 8 : (dv <= 64 ? 4 : 8);
+  const int nkc = dk / KW, nkg = (nkc + st.k_tiles - 1) / st.k_tiles, nvs = (dv / 16 + st.v_tiles - 1) / st.v_tiles;
+  const int64_t pages = ((int64_t)g->cfg.max_seq_length + ps - 1) / ps;
+  const int64_t lds = (int64_t)nkg * st.k_tiles * 1024 + (int64_t)(dk + dv) * es + 16 + 4 * 16 * (st.v_tiles * 16 + 4) * 4 + (128 + 96 + 2 * MK_ATTN_MAX_CHUNKS * 16 + 4) * 4 + pages * 4;
+  if (lds > MK_LDS_BYTES) return fail(MK_EUNSUPPORTED, "flex_attention: needs %lld bytes of LDS (head dim %d, %lld pages per request)", (long long)lds, D, (long long)pages);
+  const size_t items = (size_t)B * ((H / G + 15) / 16) * G * nvs;
+  g->flex_items = std::max(g->flex_items, items);
+  g->flex_part = std::max(g->flex_part, (size_t)g->G * 16 * (st.v_tiles * 16 + 32));
+  if (!g->stages.empty()) {
+    MkStage &pl = g->stages.back();  // the q/k/v linear may leave its K-slice sum to this stage's row fetch
+    if (pl.op == MK_OP_LINEAR && !(pl.flags & (MK_F_SILU | MK_F_RES)) && pl.out == st.in && pl.ld_out == st.ld_in && pl.n >= H * D + G * (D + DV)) pl.flags |= MK_F_DEFER_SUM;
+  }
+  if (B > 1) {
+    MkStage sp = st;
+    sp.op = MK_OP_FX_PREP;
+    g->stages.push_back(sp);
+    g->stage_desc.push_back(fmt("FX_PREP[portions] %s", in.name.c_str()));
+  }
+  g->stages.push_back(st);
+  g->stage_desc.push_back(fmt("FX_ATTN %s -> %s q=%d kv=%d d=%d dv=%d rot=%d norm=%d softcap=%g sink=%d", in.name.c_str(), o.name.c_str(), H, G, D, DV, rot, t.params[5], st.softcap, t.ops[5] >= 0));
+  i++;
+  return MK_OK;
+}
+
 bool is_moe_linear(const std::string &n) {
   return n == "moe_w13_linear_mi300" || n == "moe_w2_linear_mi300" || n == "gang_moe_w13_linear_mi300" || n == "gang_moe_w2_linear_mi300";
 }
@@ -759,6 +995,8 @@ int lower(mk_graph *g) {
   g->stage_weight.clear();
   g->weight_bytes = 0;
   g->last_linear_task = g->last_linear_stage = -1;
+  g->flex = FLEX_NONE;
+  g->flex_items = g->flex_part = 0;
   const int B = g->cfg.max_num_batched_tokens;
   // The list that is lowered: the recorded tasks, with the composite ones spelt out as the tasks they stand for (the
   // task graph handed back to the caller keeps them as recorded).
@@ -882,6 +1120,15 @@ int lower(mk_graph *g) {
                t.name == "paged_attention_split_kv_mi300" || t.name == "attention" || t.name == "single_batch_extend_attention") {
       int rc = lower_attention(g, i);
       if (rc) return rc;
+    } else if (t.name == "embedding_scaled") {
+      int rc = lower_embedding_scaled(g, i);
+      if (rc) return rc;
+    } else if (t.name == "residual_rmsnorm") {
+      int rc = lower_residual_rmsnorm(g, i);
+      if (rc) return rc;
+    } else if (t.name == "flex_attention") {
+      int rc = lower_flex_attention(g, i);
+      if (rc) return rc;
     } else if (t.name == "moe_topk_softmax_mi300") {
       bool inline_next = false;
       int rc = lower_moe_topk(g, i, &inline_next);
@@ -943,7 +1190,7 @@ int lower(mk_graph *g) {
       // partial + reduce pair, over library-owned partials
       if (t.ops.size() != 2) return fail(MK_EINVAL, "argmax expects 2 operands");
       const Tensor &x = g->tensors[t.ops[0]], &o = g->tensors[t.ops[1]];
-      if (x.ndims != 2 || x.dtype != MK_DT_BF16 || o.dtype != MK_DT_I64) return fail(MK_EINVAL, "argmax: logits must be 2-D bf16 and the output int64");
+      if (x.ndims != 2 || (x.dtype != MK_DT_BF16 && x.dtype != MK_DT_F32) || o.dtype != MK_DT_I64) return fail(MK_EINVAL, "argmax: logits must be 2-D bf16 or fp32 and the output int64");
       void *pv = nullptr, *pi = nullptr;
       int rc = dev_alloc(g, &pv, sizeof(float) * (size_t)B * g->G);
       if (rc) return rc;
@@ -951,7 +1198,7 @@ int lower(mk_graph *g) {
       if (rc) return rc;
       MkStage st;
       memset(&st, 0, sizeof(st));
-      st.op = MK_OP_ARGMAX_PARTIAL;
+      st.op = x.dtype == MK_DT_F32 ? MK_OP_FX_ARGMAX_F32 : MK_OP_ARGMAX_PARTIAL;
       st.n = (int)x.dims[1];
       st.in = x.ptr;
       st.ld_in = (int)x.strides[0];
@@ -973,7 +1220,7 @@ int lower(mk_graph *g) {
       if (i + 1 >= g->ltasks.size() || g->ltasks[i + 1].name != "argmax_reduce" || g->ltasks[i + 1].ops.size() != 3)
         return fail(MK_EUNSUPPORTED, "argmax_partial must be followed by argmax_reduce");
       const Tensor &x = g->tensors[t.ops[0]], &o = g->tensors[g->ltasks[i + 1].ops[2]];
-      if (x.ndims != 2 || x.dtype != MK_DT_BF16 || o.dtype != MK_DT_I64) return fail(MK_EINVAL, "argmax: logits must be 2-D bf16 and the output int64");
+      if (x.ndims != 2 || (x.dtype != MK_DT_BF16 && x.dtype != MK_DT_F32) || o.dtype != MK_DT_I64) return fail(MK_EINVAL, "argmax: logits must be 2-D bf16 or fp32 and the output int64");
       void *pv = nullptr, *pi = nullptr;
       int rc = dev_alloc(g, &pv, sizeof(float) * (size_t)B * g->G);
       if (rc) return rc;
@@ -981,7 +1228,7 @@ int lower(mk_graph *g) {
       if (rc) return rc;
       MkStage st;
       memset(&st, 0, sizeof(st));
-      st.op = MK_OP_ARGMAX_PARTIAL;
+      st.op = x.dtype == MK_DT_F32 ? MK_OP_FX_ARGMAX_F32 : MK_OP_ARGMAX_PARTIAL;
       st.n = (int)x.dims[1];
       st.in = x.ptr;
       st.ld_in = (int)x.strides[0];
@@ -1068,6 +1315,13 @@ int lower(mk_graph *g) {
     }
   }
   g->stage_weight.resize(g->stages.size(), -1);
+  for (size_t s = 0; s < g->stages.size(); s++) {
+    const int op = g->stages[s].op;
+    const bool f32_op = op == MK_OP_LINEAR_F32 || op == MK_OP_FX_ARGMAX_F32;
+    const bool fixed_op = op == MK_OP_EMBED || op == MK_OP_NORM || op == MK_OP_ATTN || op == MK_OP_SILU_MUL || op == MK_OP_MOE_TOPK || op == MK_OP_MOE_LINEAR || op == MK_OP_MOE_COMBINE;
+    const bool ok = g->flex == FLEX_NONE ? !f32_op : g->flex == FLEX_BF16 ? !f32_op && !fixed_op : !fixed_op && op != MK_OP_LINEAR && op != MK_OP_ARGMAX_PARTIAL;
+    if (!ok) return fail(MK_EUNSUPPORTED, "stage %zu (%s) cannot run in one graph with the others", s, g->stage_desc[s].c_str());
+  }
   for (auto &st : g->stages) {  // the task type a stage is shown as in a profiler trace (runtime_header.h:91-188)
     switch (st.op) {
       case MK_OP_EMBED: st.prof_event = 101; break;
@@ -1080,6 +1334,12 @@ int lower(mk_graph *g) {
       case MK_OP_MOE_TOPK: st.prof_event = 172; break;
       case MK_OP_MOE_LINEAR: st.prof_event = (st.flags & MK_F_MOE_COMBINE) || st.ld_in_slot ? 171 : 170; break;
       case MK_OP_MOE_COMBINE: st.prof_event = 173; break;
+      case MK_OP_FX_EMBED: st.prof_event = 101; break;
+      case MK_OP_FX_ADDNORM: st.prof_event = 119; break;
+      case MK_OP_FX_PREP:
+      case MK_OP_FX_ATTN: st.prof_event = 116; break;
+      case MK_OP_LINEAR_F32: st.prof_event = 120; break;
+      case MK_OP_FX_ARGMAX_F32: st.prof_event = 110; break;
       case MK_OP_NGRAM_PARTIAL: st.prof_event = 112; break;
       case MK_OP_NGRAM_GLOBAL: st.prof_event = 113; break;
       case MK_OP_VERIFY: st.prof_event = 114; break;
@@ -1133,7 +1393,8 @@ int task_type_id(const std::string &n) {
       {"paged_attention", 116}, {"paged_attention_split_kv_mi300", 130}, {"paged_attention_split_kv_merge_mi300", 131},
       {"paged_attention_ck_fmha_merge_mi300", 131}, {"gang_attn_merge_mi300", 139}, {"splitk_reduce_mi300", 132},
       {"silu_mul_linear_with_residual", 105}, {"rmsnorm_linear", 102}, {"identity", 121}, {"argmax", 109}, {"attention", 103},
-      {"find_ngram_partial", 112}, {"find_ngram_global", 113}, {"target_verify_greedy", 114}, {"single_batch_extend_attention", 115}};
+      {"find_ngram_partial", 112}, {"find_ngram_global", 113}, {"target_verify_greedy", 114}, {"single_batch_extend_attention", 115},
+      {"embedding_scaled", 101}, {"residual_rmsnorm", 119}, {"flex_attention", 116}};
   auto it = ids.find(n);
   return it == ids.end() ? 0 : it->second;
 }
@@ -1425,9 +1686,32 @@ int upload_runtime(mk_graph *g) {
 }
 
 // `rt` is the runtime block the kernel receives by value; `cleared_by_caller`: its barrier state has been zeroed already
-// graphs that never run more than one token per iteration use the kernel instantiated for exactly that
+// graphs with flex stages (mk_flex.hip) have kernels of their own; graphs that never run more than one token per iteration
+// use the instantiation for exactly that.  Null: not in this build of the library.
 static const void *kernel_of(const mk_graph *g) {
-  return g->cfg.max_num_batched_tokens == 1 ? (const void *)mk_persistent_kernel_m1 : (const void *)mk_persistent_kernel;
+  const bool m1 = g->cfg.max_num_batched_tokens == 1;
+  const void *k = nullptr;
+  if (g->flex == FLEX_NONE) {
+#ifdef MK_HAVE_KERNEL_GENERAL
+    if (!m1) k = (const void *)mk_persistent_kernel;
+#endif
+#ifdef MK_HAVE_KERNEL_M1
+    if (m1) k = (const void *)mk_persistent_kernel_m1;
+#endif
+  } else if (g->flex == FLEX_BF16) {
+#ifdef MK_HAVE_KERNEL_FLEX
+    if (!m1) k = (const void *)mk_persistent_kernel_flex;
+#endif
+#ifdef MK_HAVE_KERNEL_FLEX_M1
+    if (m1) k = (const void *)mk_persistent_kernel_flex_m1;
+#endif
+  } else {
+#ifdef MK_HAVE_KERNEL_FLEX_F32
+    k = (const void *)mk_persistent_kernel_flex_f32;
+#endif
+  }
+  (void)m1;
+  return k;
 }
 
 int do_launch(mk_graph *g, hipStream_t stream, int max_iters, int run_scheduler, const MkRuntime *rt = nullptr, bool cleared_by_caller = false) {
@@ -1716,8 +2000,10 @@ int mk_add_task(mk_graph *g, const char *task_name, const int grid_dim[3], const
   }
   for (int i = 0; i < n_operands; i++) {
     // id -1 = optional operand that is absent: only the q/k-norm weights and the cos/sin tables of the attention tasks
-    const bool optional = (t.name == "gang_attn_split_kv_mi300" || t.name == "kv_cache_update_mi300" || t.name == "paged_attention" ||
-                           t.name == "paged_attention_split_kv_mi300" || t.name == "attention" || t.name == "single_batch_extend_attention") && i >= 3 && i <= 6;
+    // (and the sink of flex_attention, the summand of residual_rmsnorm)
+    const bool optional = ((t.name == "gang_attn_split_kv_mi300" || t.name == "kv_cache_update_mi300" || t.name == "paged_attention" ||
+                           t.name == "paged_attention_split_kv_mi300" || t.name == "attention" || t.name == "single_batch_extend_attention") && i >= 3 && i <= 6) ||
+                          (t.name == "flex_attention" && i >= 3 && i <= 5) || (t.name == "residual_rmsnorm" && i == 0);
     if (tensor_ids[i] >= (int)g->tensors.size() || tensor_ids[i] < (optional ? -1 : 0))
       return fail(MK_EINVAL, "task '%s': bad tensor id %d for operand %d", task_name, tensor_ids[i], i);
     t.ops.push_back(tensor_ids[i]);
@@ -1735,7 +2021,8 @@ int mk_add_task(mk_graph *g, const char *task_name, const int grid_dim[3], const
                                 "moe_w2_linear_mi300", "gang_moe_w13_linear_mi300", "gang_moe_w2_linear_mi300", "moe_silu_mul", "moe_mul_sum_add_mi300",
                                 "paged_attention", "paged_attention_split_kv_mi300", "paged_attention_split_kv_merge_mi300",
                                 "paged_attention_ck_fmha_merge_mi300", "gang_attn_merge_mi300", "splitk_reduce_mi300", "silu_mul_linear_with_residual", "rmsnorm_linear", "identity", "argmax", "attention",
-                                "find_ngram_partial", "find_ngram_global", "target_verify_greedy", "single_batch_extend_attention"};
+                                "find_ngram_partial", "find_ngram_global", "target_verify_greedy", "single_batch_extend_attention",
+                                "embedding_scaled", "residual_rmsnorm", "flex_attention"};
   bool ok = linear_kind(t.name, &a, &b, &c);
   for (auto k : known) ok = ok || t.name == k;
   if (!ok) return fail(MK_EUNSUPPORTED, "Unsupported task name: %s", task_name);
@@ -1812,6 +2099,7 @@ int mk_compile(mk_graph *g) {
   if (rc) return rc;
   rc = build_task_graph_json(g);
   if (rc) return rc;
+  if (!kernel_of(g)) return fail(MK_EUNSUPPORTED, "this build of the library leaves out the kernel this graph runs on");
   // co-residency: every workgroup must be resident for the in-kernel barriers to make progress
   HIP_TRY(hipFuncSetAttribute(kernel_of(g), hipFuncAttributeMaxDynamicSharedMemorySize, MK_LDS_BYTES));
   int per_cu = 0;
@@ -1863,10 +2151,15 @@ int mk_compile(mk_graph *g) {
       g->max_qpk = std::max(g->max_qpk, s.num_q_heads / s.num_kv_heads);
     }
   g->max_kv_heads = max_kv;
-  g->attn_cnt_n = (size_t)rt.max_tokens * max_kv * 32 * 2;
+  g->attn_cnt_n = std::max((size_t)rt.max_tokens * max_kv * 2, g->flex_items) * 32;
   if ((rc = dev_alloc(g, &p, sizeof(unsigned) * g->attn_cnt_n))) return rc;
   rt.attn_cnt = (unsigned *)p;
   rt.attn_part = nullptr;
+  if (g->flex_part) {
+    // the flex attention stages share one buffer of chunk partials, handed over at device scope
+    if ((rc = dev_alloc(g, &p, g->flex_part * sizeof(float), false))) return rc;
+    rt.attn_part = (float *)p;
+  }
   for (auto &s : g->stages)
     if (s.op == MK_OP_ATTN) {
       // a work unit is (token, kv head, chunk) with chunks = clamp(G / (tokens * kv heads), 1, MK_ATTN_MAX_CHUNKS): never
@@ -2012,6 +2305,8 @@ int mk_enqueue_steps_static(mk_graph *g, void *stream, int max_iterations) {
   if (g->h_rt.max_tokens * g->max_kv_heads > MK_STATIC_MAX_ITEMS || g->max_qpk > MK_STATIC_MAX_QPK)
     return fail(MK_EINVAL, "the static launch scratch holds %d (token, kv head) pairs of up to %d q heads each; this graph needs %d x %d",
                 MK_STATIC_MAX_ITEMS, MK_STATIC_MAX_QPK, g->h_rt.max_tokens * g->max_kv_heads, g->max_qpk);
+  if (g->flex_items > (size_t)MK_STATIC_MAX_ITEMS || g->flex_part > MK_STATIC_ATTN_HEADS * MK_ATTN_PSTRIDE)
+    return fail(MK_EINVAL, "the static launch scratch is too small for this graph's attention stages (%zu work items)", g->flex_items);
   int rc = resolve_scratch(g->cfg.device);  // already resolved by mk_compile on this device; no allocation either way
   if (rc) return rc;
   if (g->launch_pending) return fail(MK_ESTATE, "a launch is still pending: call mk_wait first");

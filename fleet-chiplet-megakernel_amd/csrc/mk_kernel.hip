@@ -733,38 +733,6 @@ __device__ __forceinline__ const u32x4 *weight_row(CWeight &w, int r, int k8) {
   return (const u32x4 *)w.seg[s] + (size_t)(g * w.seg_rows[s] + o) * k8;
 }
 
-// Re-lays the weights of one linear stage in matrix-core tile order (MkStage::wpack); one thread per 16-byte operand.
-// Rows past the last output repeat it (their products are never stored).
-extern "C" __global__ __launch_bounds__(256) void mk_pack_weights_kernel(const MkWeight w, int n, int k, int silu, int half, u32x4 *dst, long long total) {
-  const int k8 = k / 8, nsteps = k >> 6;
-  const int n_out = silu ? n / 2 : n;
-  for (long long idx = (long long)blockIdx.x * 256 + threadIdx.x; idx < total; idx += (long long)gridDim.x * 256) {
-    const int lane = (int)(idx & 63);
-    long long r = idx >> 6;
-    const int h = (int)(r & 1);
-    r >>= 1;
-    const int step = (int)(r % nsteps), ti = (int)(r / nsteps);
-    const int lr = lane & 15, lg = lane >> 4;
-    int vr;
-    if (silu) {
-      const int o = min((ti >> 1) * 16 + lr, n_out - 1), gi = o / half;
-      vr = gi * 2 * half + (o - gi * half) + ((ti & 1) ? half : 0);
-    } else {
-      vr = min(ti * 16 + lr, n_out - 1);
-    }
-    const u32x4 *row;
-    if (w.nseg == 1) {
-      row = (const u32x4 *)w.seg[0] + (size_t)vr * k8;
-    } else {
-      const int g = vr / w.group_rows;
-      int o = vr - g * w.group_rows, sg = 0;
-      while (sg + 1 < w.nseg && o >= w.seg_rows[sg]) o -= w.seg_rows[sg++];
-      row = (const u32x4 *)w.seg[sg] + (size_t)(g * w.seg_rows[sg] + o) * k8;
-    }
-    dst[idx] = row[step * 8 + h * 4 + lg];
-  }
-}
-
 // ----------------------------------------------------------------------------- stages
 // Every stage function posts barrier_wait(c) itself, after any work that does not depend on the previous
 // stage (weight prefetch), and the main loop posts barrier_arrive(c) when the function returns.
@@ -919,10 +887,42 @@ __device__ __forceinline__ float silu_mul(float g, float u) { return g / (1.f + 
 
 // Stage the single input row of a one-token linear in LDS as packed bf16, applying the fused RMSNorm when the
 // stage asks for it (virtual workgroup 0 also stores the normalised row, which is the norm task's output tensor).
+// FX: the norm in front may be an FX_ADDNORM (see mk_flex.hip): alpha * residual + y, both rows in memory, then the norm.
+template <bool FX>
 __device__ __forceinline__ void stage_x_m1(CStage &st, const Ctx &c, uint32_t *xs, float *red) {
   const int tid = threadIdx.x, k4 = st.k / 4;
   const unsigned long long *xin = (const unsigned long long *)st.in;
   unsigned long long *xs2 = (unsigned long long *)xs;
+  if constexpr (FX) {
+    if (st.flags & MK_F_ADDNORM) {
+      f32x4 *vs = (f32x4 *)((char *)xs + MK_MOE_OFFSET);  // the sum, 32-bit
+      float ss = 0.f;
+      for (int i = tid; i < k4; i += MK_THREADS) {
+        const f32x4 x = __builtin_bit_cast(f32x4, ldc_16B((const u32x4 *)st.res + i));
+        const unsigned long long u = st.y_in ? ldc_u64((const unsigned long long *)st.y_in + i) : 0ull;
+        const uint32_t a = (uint32_t)u, b = (uint32_t)(u >> 32);
+        const f32x4 v = {fmaf(st.alpha, x[0], bf_lo(a)), fmaf(st.alpha, x[1], bf_hi(a)), fmaf(st.alpha, x[2], bf_lo(b)), fmaf(st.alpha, x[3], bf_hi(b))};
+        vs[i] = v;
+        ss += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+      }
+      ss = block_sum(ss, red);
+      const float r = 1.f / sqrtf(ss / (float)st.k_real + st.norm_eps);
+      for (int i = tid; i < k4; i += MK_THREADS) {
+        const f32x4 g = ((const f32x4 *)st.norm_w)[i], v = vs[i];
+        f32x4 o;
+#pragma unroll
+        for (int e = 0; e < 4; e++) o[e] = (v[e] * r) * (st.w_offset + g[e]);
+        const unsigned long long h = (unsigned long long)pack2(o[0], o[1]) | ((unsigned long long)pack2(o[2], o[3]) << 32);
+        xs2[i] = h;
+        if (c.vid == 0) {
+          if (st.out2) stc_16B((u32x4 *)st.out2 + i, __builtin_bit_cast(u32x4, o));
+          stc_u64((unsigned long long *)st.norm_out + i, h);
+        }
+      }
+      __syncthreads();
+      return;
+    }
+  }
   if (st.flags & MK_F_NORM) {
     float ss = 0.f;
     for (int i = tid; i < k4; i += MK_THREADS) {
@@ -984,6 +984,60 @@ __device__ __forceinline__ void stage_x_m1_wave(CStage &st, const Ctx &c, uint32
   }
 }
 
+// ... with an FX_ADDNORM in front: the norm weights and, where the previous stage does not write them, the residual values
+// were requested before the barrier was awaited.
+template <int KL>
+__device__ __forceinline__ void stage_x_m1_addnorm_wave(CStage &st, Ctx &c, uint32_t *xs, int lane) {
+  const f32x4 *w4 = (const f32x4 *)st.norm_w;
+  const u32x4 *x4 = (const u32x4 *)st.res;
+  f32x4 g[KL][2], x[KL][2];
+  auto load_x = [&]() {
+#pragma unroll
+    for (int kc = 0; kc < KL; kc++)
+#pragma unroll
+      for (int h = 0; h < 2; h++) x[kc][h] = __builtin_bit_cast(f32x4, ldc_16B(x4 + (kc * 64 + lane) * 2 + h));
+  };
+#pragma unroll
+  for (int kc = 0; kc < KL; kc++)
+#pragma unroll
+    for (int h = 0; h < 2; h++) g[kc][h] = w4[(kc * 64 + lane) * 2 + h];
+  const bool early = st.flags & MK_F_RES_EARLY;
+  if (early) load_x();
+  if (c.pending && lane == 0) barrier_poll(c);
+  if (!early) load_x();
+  u32x4 y[KL];
+#pragma unroll
+  for (int kc = 0; kc < KL; kc++) y[kc] = st.y_in ? ldc_16B((const u32x4 *)st.y_in + kc * 64 + lane) : (u32x4){0u, 0u, 0u, 0u};
+  float ss = 0.f;
+#pragma unroll
+  for (int kc = 0; kc < KL; kc++)
+#pragma unroll
+    for (int h = 0; h < 2; h++)
+#pragma unroll
+      for (int e = 0; e < 4; e++) {
+        const uint32_t u = y[kc][h * 2 + (e >> 1)];
+        x[kc][h][e] = fmaf(st.alpha, x[kc][h][e], (e & 1) ? bf_hi(u) : bf_lo(u));
+        ss += x[kc][h][e] * x[kc][h][e];
+      }
+  ss = wave_sum(ss);
+  const float r = 1.f / sqrtf(ss / (float)st.k_real + st.norm_eps);
+#pragma unroll
+  for (int kc = 0; kc < KL; kc++) {
+    u32x4 o16;
+#pragma unroll
+    for (int h = 0; h < 2; h++) {
+      f32x4 o;
+#pragma unroll
+      for (int e = 0; e < 4; e++) o[e] = (x[kc][h][e] * r) * (st.w_offset + g[kc][h][e]);
+      o16[h * 2] = pack2(o[0], o[1]);
+      o16[h * 2 + 1] = pack2(o[2], o[3]);
+      if (c.vid == 0 && st.out2) stc_16B((u32x4 *)st.out2 + (kc * 64 + lane) * 2 + h, __builtin_bit_cast(u32x4, o));
+    }
+    ((u32x4 *)xs)[kc * 64 + lane] = o16;
+    if (c.vid == 0) stc_16B((u32x4 *)st.norm_out + kc * 64 + lane, o16);
+  }
+}
+
 // Single-token linear: out[n] = bf16(sum_k W[n,k] * x[k] (+ res[n])), optionally with the RMSNorm of x
 // fused in front and with the SwiGLU epilogue fused behind.  The weight matrix is streamed from HBM
 // exactly once with 128-bit loads, one 1 KB row segment per wavefront instruction; x lives in LDS as
@@ -999,7 +1053,7 @@ __device__ __forceinline__ void stage_x_m1_wave(CStage &st, const Ctx &c, uint32
 // busy across the grid barrier, and a slot is refilled from the workgroup's ticket counter as soon as it is consumed.
 // Reference tasks: linear_kernel_ck (tasks/mi300/linear_ck_mi300.cuh:289-619), gang_linear_silu_kernel
 // (tasks/mi300/gang_linear_mi300.cuh:359-576).
-template <int KL, int R, bool SILU, bool W0OK>
+template <int KL, int R, bool SILU, bool W0OK, bool FX>
 __device__ __forceinline__ void stage_linear_m1_t(CStage &st, Ctx &c, char *smem) {
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   constexpr int K8 = KL * 64;
@@ -1070,6 +1124,8 @@ __device__ __forceinline__ void stage_linear_m1_t(CStage &st, Ctx &c, char *smem
         if (uo[j] >= 0) load_unit(uo[j], buf[j]);
       }
     }
+  } else if (FX && (st.flags & MK_F_ADDNORM)) {
+    if constexpr (FX && KL <= 8) stage_x_m1_addnorm_wave<KL>(st, c, xs, lane);  // (longer rows take the generic form)
   } else {
     u32x4 nwv[KL];
     if (st.flags & MK_F_NORM) {
@@ -1177,13 +1233,14 @@ __device__ __forceinline__ void stage_linear_m1_t(CStage &st, Ctx &c, char *smem
 
 // Generic single-token linear for reduction lengths that are not a multiple of 512 or have no tuned
 // instantiation: same arithmetic, no cross-barrier prefetch.
+template <bool FX>
 __device__ __forceinline__ void stage_linear_m1_generic(CStage &st, Ctx &c, char *smem) {
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int K = st.k, k8 = K / 8;
   uint32_t *xs = (uint32_t *)smem;
   float *red = (float *)(smem + MK_RED_OFFSET);
   barrier_wait(c);
-  stage_x_m1(st, c, xs, red);
+  stage_x_m1<FX>(st, c, xs, red);
   const bool silu = st.flags & MK_F_SILU;
   const int n_out = silu ? st.n / 2 : st.n;
   const int nwaves = c.G * MK_WAVES;
@@ -1220,25 +1277,25 @@ __device__ __forceinline__ void stage_linear_m1_generic(CStage &st, Ctx &c, char
   }
 }
 
-template <bool W0OK>
+template <bool W0OK, bool FX>
 __device__ __forceinline__ void stage_linear_m1(CStage &st, Ctx &c, char *smem) {
   const bool silu = st.flags & MK_F_SILU;
   // the tuned forms collect a workgroup's outputs in the LDS window [MK_OUT_OFFSET, MK_MOE_OFFSET)
   const bool fits = ((silu ? st.n / 2 : st.n) / c.G + 1) * 2 <= MK_MOE_OFFSET - MK_OUT_OFFSET;
-  if (!fits) {
-    stage_linear_m1_generic(st, c, smem);
+  if (!fits || (FX && (st.flags & MK_F_ADDNORM) && st.k > 4096)) {
+    stage_linear_m1_generic<FX>(st, c, smem);
   } else if (st.k == 4096) {
-    if (silu) stage_linear_m1_t<8, MK_TUNE_R8, true, W0OK>(st, c, smem);
-    else stage_linear_m1_t<8, MK_TUNE_R8N, false, W0OK>(st, c, smem);
+    if (silu) stage_linear_m1_t<8, MK_TUNE_R8, true, W0OK, FX>(st, c, smem);
+    else stage_linear_m1_t<8, MK_TUNE_R8N, false, W0OK, FX>(st, c, smem);
   } else if (st.k == 12288 && !silu) {
-    stage_linear_m1_t<24, MK_TUNE_R24, false, W0OK>(st, c, smem);
+    stage_linear_m1_t<24, MK_TUNE_R24, false, W0OK, FX>(st, c, smem);
   } else if (st.k == 2048) {
-    if (silu) stage_linear_m1_t<4, 4, true, W0OK>(st, c, smem);
-    else stage_linear_m1_t<4, MK_TUNE_R4, false, W0OK>(st, c, smem);
+    if (silu) stage_linear_m1_t<4, 4, true, W0OK, FX>(st, c, smem);
+    else stage_linear_m1_t<4, MK_TUNE_R4, false, W0OK, FX>(st, c, smem);
   } else if (st.k == 1024 && !silu) {
-    stage_linear_m1_t<2, 4, false, W0OK>(st, c, smem);
+    stage_linear_m1_t<2, 4, false, W0OK, FX>(st, c, smem);
   } else {
-    stage_linear_m1_generic(st, c, smem);
+    stage_linear_m1_generic<FX>(st, c, smem);
   }
 }
 
@@ -1444,7 +1501,7 @@ __device__ __forceinline__ void stage_linear_small(CStage &st, Ctx &c, int M, ch
 #define MK_TUNE_SMALL_MAX 2
 #endif
 __device__ __forceinline__ bool linear_small_ok(CStage &st, const Ctx &c, int M) {
-  if (M > MK_TUNE_SMALL_MAX || (st.k != 4096 && st.k != 2048)) return false;
+  if (M > MK_TUNE_SMALL_MAX || (st.k != 4096 && st.k != 2048) || (st.flags & MK_F_ADDNORM)) return false;
   const int n_out = (st.flags & MK_F_SILU) ? st.n / 2 : st.n;
   return (size_t)M * st.k * 2 <= (size_t)(MK_LDS_BYTES - MK_MOE_X_OFFSET) && (size_t)M * (n_out / c.G + 1) * 2 <= (size_t)MK_MOE_OFFSET;
 }
@@ -4024,15 +4081,31 @@ __device__ __attribute__((noinline)) void mk_verify_greedy(int stage, const MkRu
   }
 }
 
-template <int MAXM>
+#if defined(MK_KERNEL_FLEX) || defined(MK_KERNEL_FLEX_M1) || defined(MK_KERNEL_FLEX_F32)
+#include "mk_flex.hip"
+#define MK_HAVE_FLEX 1
+#else
+#define MK_HAVE_FLEX 0
+#endif
+
+// The stage set of an instantiation: the fixed-shape stages (E = void), or the flex stages for E-typed activations.
+template <int MAXM, typename E>
 __device__ __forceinline__ void run_stage_program(const MkRuntime &rt, const MkRuntime *rtp, Ctx &c, const int M, char *smem) {
+    constexpr bool FX = !std::is_void<E>::value;
+    constexpr bool F32 = std::is_same<E, float>::value;
+    bool single = M == 1;  // every request of the iteration brings one token
+    if constexpr (FX && MAXM > 1) {
+      const int lane = threadIdx.x & 63;
+      single = __all(lane >= M || c.sh_tok[2 * MK_MAX_TOKENS + lane] == lane);
+    }
     for (int s = 0; s < rt.num_stages && !c.dead; s++) {
       CStage &st = ((CStage *)(unsigned long long)rt.stages)[s];
       const int op = st.op, flags = st.flags;
       // (a handle that holds only the matrix-core copies of its weights runs every linear in a matrix-core form, which
       // reads normalised rows from the NORM stage's output: that stage then runs for one and two tokens as well)
       const bool packed_only = MAXM > 1 && rt.packed_only;
-      if ((flags & MK_F_ONLY_MULTI) && M == 1 && !(packed_only && op == MK_OP_NORM)) continue;
+      if ((flags & MK_F_ONLY_MULTI) && M == 1 && !(packed_only && (op == MK_OP_NORM || (FX && op == MK_OP_FX_ADDNORM)))) continue;
+      if (FX && op == MK_OP_FX_PREP && single) continue;
       if ((flags & MK_F_ONLY_MULTI) && op == MK_OP_NORM && s + 1 < rt.num_stages && !packed_only) {
         // the few-token linear normalises its rows itself
         CStage &nx = ((CStage *)(unsigned long long)rt.stages)[s + 1];
@@ -4040,11 +4113,26 @@ __device__ __forceinline__ void run_stage_program(const MkRuntime &rt, const MkR
       }
       const long long t_in = (long long)wall_clock64();
       switch (op) {
-        case MK_OP_EMBED: stage_embed(st, c, rt, M); break;
-        case MK_OP_NORM: stage_norm(st, c, M, smem); break;
+#if MK_HAVE_FLEX
+        case MK_OP_FX_EMBED: if constexpr (FX) stage_fx_embed<E>(st, c, rt, M); break;
+        case MK_OP_FX_ADDNORM: if constexpr (FX) stage_fx_addnorm<E>(st, c, M, smem); break;
+        case MK_OP_FX_PREP: if constexpr (FX) stage_fx_prep<E>(st, c, rt, M); break;
+        case MK_OP_FX_ATTN: if constexpr (FX) stage_fx_attn<E>(st, c, rt, M, MAXM == 1 || single, smem); break;
+        case MK_OP_LINEAR_F32:
+          if constexpr (F32) {
+            if (M <= 16) stage_fx_linear_f32<1>(st, c, M, smem);
+            else if (M <= 32) stage_fx_linear_f32<2>(st, c, M, smem);
+            else stage_fx_linear_f32<4>(st, c, M, smem);
+          }
+          break;
+        case MK_OP_FX_ARGMAX_F32: if constexpr (F32) stage_fx_argmax_f32(st, c, rt, M); break;
+#endif
+        case MK_OP_EMBED: if constexpr (!FX) stage_embed(st, c, rt, M); break;
+        case MK_OP_NORM: if constexpr (!FX) stage_norm(st, c, M, smem); break;
         case MK_OP_LINEAR:
-          if constexpr (MAXM == 1) stage_linear_m1<true>(st, c, smem);
-          else if (M == 1 && !(packed_only && st.wpack)) stage_linear_m1<false>(st, c, smem);
+          if constexpr (F32) barrier_wait(c);
+          else if constexpr (MAXM == 1) stage_linear_m1<true, FX>(st, c, smem);
+          else if (M == 1 && !(packed_only && st.wpack)) stage_linear_m1<false, FX>(st, c, smem);
           else if (linear_small_ok(st, c, M) && !(packed_only && st.wpack)) {
             if (M <= 2) stage_linear_small_dispatch<2>(st, c, M, smem);
             else if (M <= 4) stage_linear_small_dispatch<4>(st, c, M, smem);
@@ -4080,7 +4168,7 @@ __device__ __forceinline__ void run_stage_program(const MkRuntime &rt, const MkR
             }
           }
           break;
-        case MK_OP_SILU_MUL: stage_silu_mul(st, c, M); break;
+        case MK_OP_SILU_MUL: if constexpr (!FX) stage_silu_mul(st, c, M); break;
         case MK_OP_COPY: stage_copy(st, c, M); break;
         case MK_OP_NGRAM_PARTIAL:
         case MK_OP_NGRAM_GLOBAL:
@@ -4094,7 +4182,9 @@ __device__ __forceinline__ void run_stage_program(const MkRuntime &rt, const MkR
           }
           break;
         case MK_OP_ATTN:
-          if constexpr (MAXM == 1) {
+          if constexpr (FX) {
+            barrier_wait(c);
+          } else if constexpr (MAXM == 1) {
             if (st.num_q_heads == 4 * st.num_kv_heads) stage_attn<4, false>(st, c, rt, M, smem);
             else if (st.num_q_heads == 8 * st.num_kv_heads) stage_attn<8, false>(st, c, rt, M, smem);
             else barrier_wait(c);
@@ -4112,10 +4202,10 @@ __device__ __forceinline__ void run_stage_program(const MkRuntime &rt, const MkR
             }
           }
           break;
-        case MK_OP_MOE_TOPK: stage_moe_topk(st, c, M); break;
-        case MK_OP_MOE_LINEAR: stage_moe_linear(st, c, M, smem); break;
-        case MK_OP_MOE_COMBINE: stage_moe_combine(st, c, M); break;
-        case MK_OP_ARGMAX_PARTIAL: stage_argmax_partial(st, c, rt, M, smem); break;
+        case MK_OP_MOE_TOPK: if constexpr (!FX) stage_moe_topk(st, c, M); break;
+        case MK_OP_MOE_LINEAR: if constexpr (!FX) stage_moe_linear(st, c, M, smem); break;
+        case MK_OP_MOE_COMBINE: if constexpr (!FX) stage_moe_combine(st, c, M); break;
+        case MK_OP_ARGMAX_PARTIAL: if constexpr (!F32) stage_argmax_partial(st, c, rt, M, smem); break;
         case MK_OP_ARGMAX_REDUCE: stage_argmax_reduce(st, c, rt, M); break;
         default: barrier_wait(c); break;
       }
@@ -4150,7 +4240,7 @@ __device__ __forceinline__ void run_stage_program(const MkRuntime &rt, const MkR
 // The kernel body, instantiated twice: MAXM = 1 for graphs that never run more than one token per iteration (every
 // multi-token stage form is compiled out, so the single-token loops get the register file to themselves), and the
 // general one.
-template <int MAXM>
+template <int MAXM, typename E>
 __device__ __forceinline__ void mk_kernel_body(const MkRuntime &rt, const MkRuntime *rtp, int max_iters, int run_scheduler) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
   __shared__ int sh_bcast[4];
@@ -4271,20 +4361,38 @@ __device__ __forceinline__ void mk_kernel_body(const MkRuntime &rt, const MkRunt
       pr[2] = (long long)wall_clock64();
     }
     if (M == 0 || c.dead) break;
-    run_stage_program<MAXM>(rt, rtp, c, MAXM == 1 ? 1 : M, smem);
+    run_stage_program<MAXM, E>(rt, rtp, c, MAXM == 1 ? 1 : M, smem);
   }
   barrier_wait(c);  // drain: nobody leaves while another workgroup may still poll
   if (rt.profiler && threadIdx.x == 0) rt.profiler_count[c.vid] = c.prof_n;
   if (c.vid == 0 && threadIdx.x == 0 && rt.timing) rt.timing[0] = (long long)wall_clock64();
 }
 
-
-extern "C" __global__ __launch_bounds__(MK_THREADS, 1) void mk_persistent_kernel(const MkRuntime rt, const MkRuntime *rtp, int max_iters,
-                                                                                int run_scheduler) {
-  mk_kernel_body<MK_MAX_TOKENS>(rt, rtp, max_iters, run_scheduler);
+// Each instantiation is a translation unit of its own (build.py compiles this file once per -DMK_KERNEL_*), so they
+// compile side by side and a build may leave out the ones it does not need.
+#define MK_KERNEL_ARGS const MkRuntime rt, const MkRuntime *rtp, int max_iters, int run_scheduler
+#ifdef MK_KERNEL_GENERAL
+extern "C" __global__ __launch_bounds__(MK_THREADS, 1) void mk_persistent_kernel(MK_KERNEL_ARGS) {
+  mk_kernel_body<MK_MAX_TOKENS, void>(rt, rtp, max_iters, run_scheduler);
 }
-// the same for graphs with max_num_batched_tokens == 1
-extern "C" __global__ __launch_bounds__(MK_THREADS, 1) void mk_persistent_kernel_m1(const MkRuntime rt, const MkRuntime *rtp, int max_iters,
-                                                                                   int run_scheduler) {
-  mk_kernel_body<1>(rt, rtp, max_iters, run_scheduler);
+#endif
+#ifdef MK_KERNEL_M1  // graphs with max_num_batched_tokens == 1
+extern "C" __global__ __launch_bounds__(MK_THREADS, 1) void mk_persistent_kernel_m1(MK_KERNEL_ARGS) {
+  mk_kernel_body<1, void>(rt, rtp, max_iters, run_scheduler);
 }
+#endif
+#ifdef MK_KERNEL_FLEX  // graphs with flex stages (mk_flex.hip), 16-bit activations
+extern "C" __global__ __launch_bounds__(MK_THREADS, 1) void mk_persistent_kernel_flex(MK_KERNEL_ARGS) {
+  mk_kernel_body<MK_MAX_TOKENS, uint16_t>(rt, rtp, max_iters, run_scheduler);
+}
+#endif
+#ifdef MK_KERNEL_FLEX_M1
+extern "C" __global__ __launch_bounds__(MK_THREADS, 1) void mk_persistent_kernel_flex_m1(MK_KERNEL_ARGS) {
+  mk_kernel_body<1, uint16_t>(rt, rtp, max_iters, run_scheduler);
+}
+#endif
+#ifdef MK_KERNEL_FLEX_F32  // 32-bit activations, weights and caches
+extern "C" __global__ __launch_bounds__(MK_THREADS, 1) void mk_persistent_kernel_flex_f32(MK_KERNEL_ARGS) {
+  mk_kernel_body<MK_MAX_TOKENS, float>(rt, rtp, max_iters, run_scheduler);
+}
+#endif

@@ -51,6 +51,13 @@ enum MkOp {
   MK_OP_NGRAM_PARTIAL = 12,  // out[slot, task] = earliest position among the task's share where the request's last k tokens occurred before
   MK_OP_NGRAM_GLOBAL = 13,   // out[row] = this iteration's token ids: the scheduler's, and for a decoding request the tokens after that position
   MK_OP_VERIFY = 14,         // num_new_tokens[request] = 1 + leading candidates the sampled tokens agree with
+  // stages whose sizes and constants are data (mk_flex.hip); a graph that holds one runs on the flex kernels
+  MK_OP_FX_EMBED = 15,       // out2 = table[id] * alpha in 32 bits, out = the same rounded
+  MK_OP_FX_ADDNORM = 16,     // v = alpha * res + in; out2 = v / rms(v) * (w_offset + w) in 32 bits, out = the same rounded
+  MK_OP_FX_PREP = 17,        // rotate / normalise q and k rows, append K/V (iterations in which a request brings several tokens)
+  MK_OP_FX_ATTN = 18,        // paged attention with softcap and sink (single-token iterations: preparation and append included)
+  MK_OP_LINEAR_F32 = 19,     // LINEAR with 32-bit operands
+  MK_OP_FX_ARGMAX_F32 = 20,  // ARGMAX_PARTIAL over 32-bit logits
 };
 
 enum MkStageFlags {
@@ -64,7 +71,11 @@ enum MkStageFlags {
   MK_F_MOE_INLINE_TOPK = 128,   // MOE_LINEAR: a single-token iteration routes inside this stage (the MOE_TOPK stage before it is multi-token only)
   MK_F_MOE_COMBINE = 256,       // MOE_LINEAR: a single-token iteration also forms res + sum_k w_k * y_k (the MOE_COMBINE stage after it is multi-token only)
   MK_F_DEFER_SUM = 512,  // LINEAR: the next stage is a full-row NORM over this stage's output, which may be handed the K-slice partials to sum
+  MK_F_ADDNORM = 1024,   // LINEAR (set together with MK_F_NORM): the norm in front is an FX_ADDNORM; a single-token iteration forms it inside this stage
+  MK_F_RES_EARLY = 2048, // FX_ADDNORM / LINEAR+ADDNORM: the stage before this one does not write the residual rows, so they may be requested before its barrier
 };
+
+#define MK_FX_MAX_HEAD_DIM 512  // largest q/k head the flex attention keeps in a wavefront's registers
 
 #define MK_MOE_MAX_EXPERTS 256  // one thread per expert when the routing lists are built
 #define MK_MOE_MAX_TOPK 16
@@ -122,6 +133,17 @@ struct MkStage {
   int num_experts, topk, ld_logits, ld_topk_w;
   int ld_routing, ld_in_slot, ld_out_slot, ld_out2;
   int ld_out2_slot, pad4, pad5, pad6;
+  // flex stages.  FX_ADDNORM and LINEAR+ADDNORM: rows are `n_pad` long in memory with `k_real` of them real (a linear's
+  // k is n_pad then); y_in / ld_y: the rows added to alpha * res (null: none); out2 / ld_out2: the 32-bit result.
+  const void *y_in;
+  const void *sink;      // [num_q_heads] fp32, null: none
+  float alpha, w_offset; // residual (or embedding) factor; constant added to the norm weight
+  float sm_scale, softcap;  // FX_ATTN: score factor, tanh cap (0: none)
+  int k_real, ld_y;
+  int v_dim, rot_dims;   // FX_ATTN: value size per head, rotated dims (head_dim: query/key size)
+  int k_tiles, v_tiles;  // FX_ATTN: instantiation -- operand rows of a key / 16-wide value blocks held at a time
+  float norm_eps;        // LINEAR+ADDNORM: eps of the fused norm
+  int pad7;
 };
 
 // Hierarchical barrier state.  One 128-byte line per counter so that XCD-local

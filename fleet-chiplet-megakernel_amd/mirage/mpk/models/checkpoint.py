@@ -11,6 +11,7 @@ model.safetensors.index.json + shards), or the reference's per-rank file `model{
 Only safetensors files are read (nothing is unpickled).
 """
 import json
+import math
 import os
 
 import torch
@@ -36,8 +37,9 @@ def _weight_files(model_path: str, rank: int, world_size: int):
     raise FileNotFoundError(f"no safetensors weights under {model_path} (model.safetensors, model.safetensors.index.json or model{rank}-mp{world_size}.safetensors)")
 
 
-def load_checkpoint(model_path: str, device="cuda", rank: int = 0, world_size: int = 1, dtype=torch.bfloat16):
-    """Returns (config dict, state dict of contiguous `dtype` tensors on `device`)."""
+def load_checkpoint(model_path: str, device="cuda", rank: int = 0, world_size: int = 1, dtype=torch.bfloat16,
+                    required=("model.embed_tokens.weight", "model.norm.weight")):
+    """Returns (config dict, state dict of contiguous `dtype` tensors on `device`).  dtype None keeps the stored types."""
     from safetensors import safe_open
     cfg = load_config(model_path)
     state = {}
@@ -45,11 +47,10 @@ def load_checkpoint(model_path: str, device="cuda", rank: int = 0, world_size: i
         with safe_open(path, framework="pt", device="cpu") as f:
             for name in f.keys():
                 t = f.get_tensor(name)
-                if t.is_floating_point():
+                if dtype is not None and t.is_floating_point():
                     t = t.to(dtype)
                 state[name] = t.to(device).contiguous()
-    need = ["model.embed_tokens.weight", "model.norm.weight"]
-    missing = [n for n in need if n not in state]
+    missing = [n for n in required if n not in state]
     if missing:
         raise KeyError(f"checkpoint under {model_path} lacks {missing}")
     return cfg, state
@@ -74,3 +75,22 @@ def rotary_tables(head_dim: int, theta: float, n_pos: int, device="cuda"):
     freqs = torch.arange(n_pos, dtype=torch.float32, device=device)[:, None] * inv_freq[None, :]
     emb = torch.cat((freqs, freqs), dim=-1)
     return emb.cos().to(torch.bfloat16)[None].contiguous(), emb.sin().to(torch.bfloat16)[None].contiguous()
+
+
+def rotary_frequencies(dims: int, base: float, scaling: dict = None) -> torch.Tensor:
+    """float64 [dims / 2] angular frequencies base^(-2i/dims).  `scaling` {factor, low, high, original}: the scaling of
+    Llama 3.1 -- wavelengths beyond original / low are stretched by `factor`, those below original / high are kept, the
+    band in between is blended linearly in original / wavelength."""
+    f = torch.pow(torch.tensor(float(base), dtype=torch.float64), -torch.arange(0, dims, 2, dtype=torch.float64) / dims)
+    if scaling:
+        factor, low, high, original = (float(scaling[k]) for k in ("factor", "low", "high", "original"))
+        turns = original * f / (2.0 * math.pi)  # original / wavelength
+        blend = ((turns - low) / (high - low)).clamp(0.0, 1.0) if high != low else (turns >= low).to(torch.float64)
+        f = f * (blend + (1.0 - blend) / factor)
+    return f
+
+
+def rotary_tables_f32(dims: int, base: float, scaling: dict, n_pos: int, device="cuda"):
+    """(cos, sin), fp32 [n_pos, dims / 2]; the angles are formed in float64 so that far positions keep a 32-bit result."""
+    ang = torch.arange(n_pos, dtype=torch.float64)[:, None] * rotary_frequencies(dims, base, scaling)[None, :]
+    return ang.cos().to(torch.float32).to(device).contiguous(), ang.sin().to(torch.float32).to(device).contiguous()

@@ -24,6 +24,8 @@ class MirageModelConfig:
     # model weights under the checkpoint's names ("model.layers.0.self_attn.q_proj.weight", ...)
     state_dict: Optional[dict] = None
     with_lm_head: bool = True
+    # the whole parsed config.json, for architectures the fields above do not describe (layer lists and the like)
+    architecture: Optional[dict] = None
 
     def info_as_string(self):
         fields = [("Hidden size", self.hidden_size), ("Intermediate size", self.intermediate_size), ("Vocab size", self.vocab_size),
@@ -38,9 +40,24 @@ class MirageModelConfig:
 
 
 class GraphBuilder(abc.ABC):
+    owns_kv_cache = False        # True: the builder allocates the K/V caches when the caller brings none
+    default_eos_token_id = None  # used when neither the caller nor the checkpoint names one
+    dtypes = (torch.bfloat16,)   # activation / weight types the model can be built in
+
     def __init__(self, mpk, weights: Optional[Dict[str, Any]] = None):
         self.mpk = mpk
         self.weights = weights or {}
+        self.dtype = torch.bfloat16
+
+    def set_dtype(self, dtype: torch.dtype):
+        if dtype not in self.dtypes:
+            raise NotImplementedError(f"{type(self).__name__} runs in {', '.join(str(d) for d in self.dtypes)}, not {dtype}")
+        self.dtype = dtype
+
+    @classmethod
+    def kernels(cls, dtype: torch.dtype, max_num_batched_tokens: int):
+        """Kernel instantiations of the library (build.py: KERNELS) a graph of this builder runs on."""
+        return ("M1",) if max_num_batched_tokens == 1 else ("GENERAL",)
 
     @abc.abstractmethod
     def build_from_model(self, model_name: str = None, model_path: str = None):

@@ -26,8 +26,10 @@ from ..graph_builder import GraphBuilder, MirageModelConfig
 from ..utils import grid_for_rmsnorm_linear_layer
 
 
-@register_model_builder("Qwen3", "Qwen/Qwen3-8B", "Qwen/Qwen3-1.7B", "Qwen/Qwen3-14B", "Qwen/Qwen3-0.6B")
+@register_model_builder("Qwen3", "Qwen3ForCausalLM", "Qwen/Qwen3-8B", "Qwen/Qwen3-1.7B", "Qwen/Qwen3-14B", "Qwen/Qwen3-0.6B")
 class Qwen3Builder(GraphBuilder):
+    default_eos_token_id = 151645
+
     def __init__(self, mpk: PersistentKernel, weights: Optional[dict] = None):
         super().__init__(mpk, weights)
         self.max_num_pages = mpk.max_num_pages

@@ -17,7 +17,7 @@ from typing import Optional
 import torch
 
 from ..utils import get_configurations_from_gpu
-from .model_registry import get_builder
+from .model_registry import get_builder, model_name_of
 from .models.graph_builder import MirageModelConfig
 from .persistent_kernel import PersistentKernel
 from .speculative import spec_decode_class
@@ -71,14 +71,30 @@ class MPKMetadata:
     eos_token_id: Optional[int] = None
     max_tokens_per_request: Optional[int] = None
     single_weight_copy: Optional[bool] = None  # keep every linear weight once, in tile order (see PersistentKernel)
+    dtype: torch.dtype = torch.bfloat16  # activations, weights and caches; the builder refuses what its model cannot run in
 
     def check_valid(self):
         if self.weight_from_model:
             assert (self.model_name is not None) or (self.model_path is not None), "model_name or model_path is required when weight_from_model is True"
         else:
             assert self.model_config is not None and self.model_config.state_dict is not None, "state_dict is required when weight_from_model is False"
+            if get_builder(self.resolved_model_name()).owns_kv_cache:
+                return
             assert self.model_config.k_cache is not None, "k_cache is required when weight_from_model is False"
             assert self.model_config.v_cache is not None, "v_cache is required when weight_from_model is False"
+
+    def resolved_model_name(self):
+        """The caller's model name, else what the config (given, or the checkpoint's config.json) says, else Qwen3."""
+        if self.model_name is not None:
+            return self.model_name
+        if self.model_config is not None and self.model_config.architecture is not None:
+            return model_name_of(self.model_config.architecture)
+        if self.weight_from_model and self.model_path is not None:
+            from .models.checkpoint import load_config
+            cfg = load_config(self.model_path)
+            if cfg.get("architecture") or cfg.get("architectures"):
+                return model_name_of(cfg)
+        return "Qwen3"
 
     def info_as_string(self):
         shape = lambda t: None if t is None else tuple(t.shape)
@@ -112,7 +128,8 @@ class MPK:
         meta.check_valid()
         self.metadata = meta
         self.world_size, self.rank = 1, 0
-        self.model_name = meta.model_name or "Qwen3"
+        self.model_name = meta.resolved_model_name()
+        builder_cls = get_builder(self.model_name)
         self.device = meta.device
         self.weight_from_model = meta.weight_from_model
         self.max_seq_length = meta.max_seq_length
@@ -159,7 +176,7 @@ class MPK:
                 "paged_kv_indptr_buffer": self.paged_kv_indptr_buffer, "paged_kv_indices_buffer": self.paged_kv_indices_buffer,
                 "paged_kv_last_page_len_buffer": self.paged_kv_last_page_len_buffer},
             profiler_tensor=self.profiler_tensor, trace_name=meta.trace_name, spec_decode_config=meta.spec_decode_config,
-            use_cutlass_kernel=False, eos_token_id=meta.eos_token_id if meta.eos_token_id is not None else 151645,
+            use_cutlass_kernel=False, eos_token_id=next(e for e in (meta.eos_token_id, builder_cls.default_eos_token_id, -1) if e is not None),
             max_tokens_per_request=meta.max_tokens_per_request, single_weight_copy=meta.single_weight_copy)
         self.is_built = self.task_graph_generated = self.is_compiled = False
 
@@ -251,7 +268,8 @@ class MPK:
 
     def build(self):
         """Record the model graph through the builder registered for the model name (mpk.py:351-367)."""
-        self.model_builder = get_builder(self.model_name or "Qwen3")(self.persistent_kernel)
+        self.model_builder = get_builder(self.model_name)(self.persistent_kernel)
+        self.model_builder.set_dtype(self.metadata.dtype)
         if not self.weight_from_model:
             self.model_builder.build_from_config(self.model_config)
         else:

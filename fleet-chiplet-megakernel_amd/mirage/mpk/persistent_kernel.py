@@ -9,6 +9,7 @@ whole generation.  Nothing here computes: without libfleet_mk.so and a gfx950 de
 import ctypes
 import math
 import os
+import struct
 import sys
 
 import torch
@@ -23,6 +24,11 @@ _META_ORDER = ["step", "tokens", "input_tokens", "output_tokens", "num_new_token
                "qo_indptr_buffer", "paged_kv_indptr_buffer", "paged_kv_indices_buffer", "paged_kv_last_page_len_buffer"]
 
 _REPL = (-1, -1, -1)
+
+
+def _f32_bits(x: float) -> int:
+    """A task parameter is an int; constants of the flex tasks travel as the bits of a 32-bit float."""
+    return struct.unpack("<i", struct.pack("<f", float(x)))[0]
 
 
 class PersistentKernel:
@@ -622,6 +628,41 @@ class PersistentKernel:
                    [(input, (-1, 1, 0), 1), (weight, (0, 1, -1), 1), (residual, (1, -1, 0), 1), (workspace, (1, -1, 0), 1),
                     (done_counter, (0, -1, 1), 1), (output, (1, -1, 0), -1)], [k_splits])
 
+    # ------------------------------------------------------------------ layers whose sizes and constants are data (csrc/mk_flex.hip)
+    # No counterpart in the reference.  A graph uses them in one activation type, bf16 or fp32 (weights and caches of the same
+    # type); the residual stream, norms, angles, scores and softmax are 32-bit in both.
+    def embed_scaled_layer(self, input: DTensor, weight: DTensor, residual: DTensor, output: DTensor, scale: float = 1.0, input_source: int = 1):
+        """residual (fp32) = weight[id] * scale, output = the same rounded to the activation type (the two may be one
+        tensor in an fp32 graph).  input_source as in embed_layer."""
+        assert input.num_dims == 2 and weight.num_dims == 2 and residual.num_dims == 2 and output.num_dims == 2
+        self._task("embedding_scaled", (1, 1, 1), (256, 1, 1),
+                   [(input, _REPL, -1), (weight, _REPL, -1), (residual, _REPL, -1), (output, _REPL, -1)], [input_source, _f32_bits(scale)])
+
+    def residual_rmsnorm_layer(self, input: DTensor, residual: DTensor, weight: DTensor, new_residual: DTensor, output: DTensor, width: int = None,
+                               alpha: float = 1.0, eps: float = 1e-6, weight_offset: float = 0.0):
+        """v = alpha * residual + input (input None: no sum); new_residual (fp32) = v / sqrt(mean(v^2) + eps) *
+        (weight_offset + weight), output = the same rounded.  `width` of the row's entries are real, the rest is zero
+        padding.  A linear_layer over `output` right behind forms it itself when an iteration has one token."""
+        assert residual.num_dims == 2 and new_residual.num_dims == 2 and output.num_dims == 2 and weight.num_dims == 1
+        self._task("residual_rmsnorm", (1, 1, 1), (256, 1, 1),
+                   [(input, _REPL, -1), (residual, _REPL, -1), (weight, _REPL, -1), (new_residual, _REPL, -1), (output, _REPL, -1)],
+                   [output.dim(1) if width is None else int(width), _f32_bits(alpha), _f32_bits(eps), _f32_bits(weight_offset)])
+
+    def flex_attention_layer(self, input: DTensor, k_cache: DTensor, v_cache: DTensor, cos: DTensor, sin: DTensor, sink: DTensor, q_workspace: DTensor,
+                             output: DTensor, num_q_heads: int, num_kv_heads: int, head_dim: int, v_dim: int, rot_dims: int, scale: float,
+                             softcap: float = 0.0, unit_norm: bool = False, eps: float = 1e-6):
+        """Causal paged attention with rotary positions on the first `rot_dims` dims of each q/k head (rotate-half pairs;
+        cos / sin are fp32 [positions, rot_dims / 2]), heads divided by their root mean square after the rotation
+        (unit_norm), score = softcap * tanh(q.k * scale / softcap) (softcap 0: plain), and a per-head logit `sink` (fp32,
+        None: none) that only takes part in the softmax's denominator.  input rows: all q heads, all k heads, all v heads.
+        Caches: [pages, page_size, kv_heads, flex_cache_dims(...)], in the kernel's own order inside a page."""
+        assert input.num_dims == 2 and output.num_dims == 2 and q_workspace.num_dims == 2
+        assert k_cache.num_dims == 4 and v_cache.num_dims == 4
+        self._task("flex_attention", (1, 1, 1), (256, 1, 1),
+                   [(input, _REPL, -1), (k_cache, _REPL, -1), (v_cache, _REPL, -1), (cos, _REPL, -1), (sin, _REPL, -1), (sink, _REPL, -1),
+                    (q_workspace, _REPL, -1), (output, _REPL, -1)],
+                   [num_q_heads, num_kv_heads, head_dim, v_dim, rot_dims, int(unit_norm), _f32_bits(eps), _f32_bits(scale), _f32_bits(softcap or 0.0)])
+
     # layers of the reference that are outside the one-GPU decode path
     def tensor_init_layer(self, *args, **kwargs):
         raise NotImplementedError("tensor_init_layer registers a Blackwell-only task (tasks/blackwell/tensor_init.cuh); it has no MI300-family kernel in the reference either")
@@ -944,6 +985,13 @@ class PersistentKernel:
                 self.finalize()
         except Exception:
             pass
+
+
+def flex_cache_dims(head_dim: int, v_dim: int, dtype: torch.dtype = torch.bfloat16):
+    """(key, value) entries per position and kv head of the caches flex_attention_layer takes: the head sizes rounded up to
+    whole matrix-core operands."""
+    kw = 32 if dtype == torch.bfloat16 else 16
+    return -(-head_dim // kw) * kw, -(-v_dim // 16) * 16
 
 
 class _DevicePtr:
