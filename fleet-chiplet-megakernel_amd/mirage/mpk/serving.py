@@ -112,7 +112,7 @@ class ServingSession:
                 if places:
                     logits = self.logits() if logits is None else logits
                     for p in places:
-                        found[i][p] = logits[row + p - lo].to(torch.float32)
+                        found[i][p] = logits[row + p - lo].to(torch.float32, copy=True)
                 if hi == len(entries[i][1]):
                     sampled = self.mpk.output_tokens.view(-1).tolist() if sampled is None else sampled
                     greedy[i] = sampled[row + n - 1]
