@@ -212,6 +212,107 @@ def run_leg(torch, dec, shape, model, B, K, W, P, max_seq, mode, stage_profile=F
     }
 
 
+# ---- Suborax beside the closest model at equal size (bench.py --compare suborax) --------------------------------------
+# Both models with the same width, heads, head size, feed-forward, depth and vocabulary; random weights.
+COMPARE_SHAPES = {"8b": dict(width=4096, heads=32, kv_heads=8, ff=12288), "2k": dict(width=2048, heads=32, kv_heads=4, ff=6144)}
+
+
+def stage_times(dec):
+    """Microseconds per stage kind of the last iteration: last arrival of a stage after the last arrival of the stage before
+    it (device timestamps, all workgroups), averaged over the layers."""
+    G = dec.mpk.stats()["num_workgroups"]
+    prof = [dec.mpk.stage_profile(w, raw=True) for w in range(G)]
+    rows = [i for i in range(len(prof[0]) - 1) if prof[0][i][1] > 0]
+    newest = max(prof[0][i][4] for i in rows)
+    rows = [i for i in rows if newest - prof[0][i][4] < 10 ** 8]  # (stages an iteration skips keep an older record)
+    t_first = max(prof[w][rows[0]][1] for w in range(G))
+    rows = [i for i in rows if prof[0][i][4] >= t_first]
+    kinds, prev = {}, t_first
+    for i in rows:
+        end = max(prof[w][i][4] for w in range(G))
+        desc = prof[0][i][0].split()
+        op = desc[1]
+        n = next((d for d in desc if d.startswith("n=")), "")
+        k = next((d for d in desc if d.startswith("k=")), "")
+        kinds.setdefault(" ".join(x for x in (op.replace("[multi-token", "").replace("[portions]", ""), n, k) if x), []).append((end - prev) * 0.01)
+        prev = end
+    return {k: [round(sum(v) / len(v), 1), len(v)] for k, v in kinds.items()}
+
+
+def compare_decoder(torch, which, shape, layers, vocab, B, R, max_seq, page_size=4096):
+    """A decoder of either model with B token rows per iteration and R batch slots."""
+    per_req = min(B, 64)
+    if which == "qwen3":
+        from demo_qwen3 import Qwen3Decoder, Qwen3Shape, random_weights
+        s = Qwen3Shape(hidden_size=shape["width"], num_q_heads=shape["heads"], num_kv_heads=shape["kv_heads"], intermediate_size=shape["ff"], num_layers=layers, vocab_size=vocab)
+        return Qwen3Decoder(s, random_weights(s), max_num_batched_tokens=B, max_num_batched_requests=R, max_seq_length=max_seq, page_size=page_size,
+                            max_tokens_per_request=per_req), s.weight_bytes_per_token(), s.kv_bytes_per_position()
+    from generate import Generator, suborax_shape
+    from mirage.mpk import MirageModelConfig
+    from mirage.mpk.models.suborax.builder import SuboraxConfig, random_state_dict
+    c = suborax_shape(layers=layers, vocab=vocab, **shape)
+    sc = SuboraxConfig.from_dict(c)
+    g = Generator(max_seq, model_config=MirageModelConfig(architecture=c, state_dict=random_state_dict(sc)), batch=R, max_num_batched_tokens=B,
+                  max_tokens_per_request=per_req, page_size=page_size, eos_token_id=-1)
+    return g, sc.weight_bytes_per_token(), sc.kv_bytes_per_position()
+
+
+def compare_leg(torch, which, shape, layers, vocab, B, R, prompt, steps, stages):
+    """One model, one workload: the prefill rate of R prompts (64-row iterations), then `steps` decode steps in one launch."""
+    max_seq = prompt + steps + 24 + (0 if R == 1 else 8 * prompt)  # (the first of several requests decodes while the last still ingests)
+    dec, wbytes, kvbytes = compare_decoder(torch, which, shape, layers, vocab, B, R, max_seq)
+    prompts = [torch.randint(0, vocab, (prompt,), generator=torch.Generator().manual_seed(r)) for r in range(R)]
+    out = {"model": which, "batch": R, "rows_per_iteration": B, "context": prompt}
+    if B > R:  # prompt portions
+        for rep in range(2):  # (the first pass warms up)
+            dec.load_prompts(prompts)
+            n = -(-prompt // min(B, 64)) * R if B < 64 * R else -(-prompt // 64)
+            torch.cuda.synchronize()
+            dec.mpk.run_steps(n)
+            ms = dec.mpk.stats()["last_launch_ms"]
+        out["prefill_tokens_per_s"] = round(prompt * R / ms * 1e3)
+        out["prefill_us_per_iteration"] = round(ms / n * 1e3, 1)
+        if stages:
+            out["prefill_stages_us"] = stage_times(dec)
+    else:
+        dec.load_prompts(prompts)
+    it = 0
+    while int(dec.meta["step"].min().item()) < prompt:
+        dec.mpk.run_steps(16)
+        it += 1
+        assert it < prompt * R, "prompt ingestion did not finish"
+    s0 = dec.meta["step"].cpu().tolist()
+    torch.cuda.synchronize()
+    dec.mpk.run_steps(steps)
+    ms = dec.mpk.stats()["last_launch_ms"] / steps
+    assert dec.meta["step"].cpu().tolist() == [s + steps for s in s0]
+    kv = sum(s + 1 + i for s in s0 for i in range(steps)) * kvbytes / steps
+    out["decode_ms_per_step"] = round(ms, 4)
+    out["decode_tokens_per_s"] = round(R / ms * 1e3)
+    out["decode_hbm_frac"] = round((wbytes + kv) / (ms * 1e-3) / 1e9 / HBM_PEAK_GBS, 4)
+    if stages:
+        out["decode_stages_us"] = stage_times(dec)
+    (dec.mpk if which == "qwen3" else dec).finalize()
+    return out
+
+
+def compare_main(torch, args):
+    vocab, layers = 32768, min(args.layers, 8)
+    legs = []
+    for name, shape in COMPARE_SHAPES.items():
+        # (rows per iteration, batch slots, prompt): single-token kernel short and long, long prompt in portions, batches
+        for B, R, prompt in ((1, 1, 80), (1, 1, 4096), (64, 1, 4096), (8, 8, 80), (64, 64, 80)):
+            for which in ("qwen3", "suborax"):
+                leg = dict(shape=name, **compare_leg(torch, which, shape, layers, vocab, B, R, prompt, 64, args.stage_profile))
+                print(json.dumps(leg), file=sys.stderr, flush=True)
+                legs.append(leg)
+                torch.cuda.empty_cache()
+    worst = max(b["decode_ms_per_step"] / a["decode_ms_per_step"] for a, b in zip(legs[::2], legs[1::2]))
+    print(json.dumps({"metric": "Suborax decode time relative to a Qwen3 stack of equal size (worst leg)", "value": round(worst, 3), "unit": "x", "n_gpus": 1,
+                      "higher_is_better": False, "dtype": "bf16", "data": "synthetic (random-init weights, seeded random prompts)",
+                      "config": {"layers": layers, "vocab": vocab, "shapes": COMPARE_SHAPES}, "legs": legs}), flush=True)
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -228,6 +329,8 @@ def main():
     ap.add_argument("--single-weight-copy", action="store_true",
                     help="keep every linear weight once, in matrix-core tile order (BS >= 2): what the memory saving costs iterations of one or two tokens")
     ap.add_argument("--calib-copy", action="store_true", help="also run one 1 GiB device-to-device copy (scale for rocprofv3 FETCH_SIZE / WRITE_SIZE)")
+    ap.add_argument("--compare", choices=["suborax"], default=None,
+                    help="instead of the headline workload: prefill and decode of this model beside the closest one at equal size (8 layers)")
     ap.add_argument("--stage-profile", action="store_true",
                     help="after each timed launch, print its last iteration's per-stage timeline over all workgroups to stderr")
     args = ap.parse_args()
@@ -247,6 +350,9 @@ def main():
     from mirage import _capi
     # where the library is mapped (a crash report of the process can be matched against it)
     print(f"bench.py: pid {os.getpid()}, {_capi.LIB_PATH} at {_capi.load_address():#x}", file=sys.stderr, flush=True)
+    if args.compare:
+        compare_main(torch, args)
+        return
     moe = args.model == "qwen3-30b-a3b"
     shape = Qwen3Shape.qwen3_30b_a3b(min(args.layers, 48) if args.layers != 36 else 48) if moe else Qwen3Shape(num_layers=args.layers)
     K, W, P = args.steps, args.warmup, args.prompt_length

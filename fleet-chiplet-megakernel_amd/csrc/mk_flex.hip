@@ -216,36 +216,49 @@ template <typename E> __device__ __forceinline__ FxRows<E> fx_rows(CStage &st, C
 }
 #define MK_FX_HEAD_REGS (MK_FX_MAX_HEAD_DIM / 64)
 // One query or key head row by one wavefront: dims [0, rot) are rotated (dim i < rot / 2 pairs with i + rot / 2), then the
-// row is divided by sqrt(mean(x^2) + eps) when the stage asks for it.  put(d, value) for every d < D.
-template <typename E, typename Put>
-__device__ __forceinline__ void fx_head_row(CStage &st, const FxRows<E> &rows, int tok, int col, int pos, int lane, Put put) {
+// row is divided by sqrt(mean(x^2) + eps) when the stage asks for it.  Split in a half that requests everything and a half
+// that computes, so that a wavefront can have the requests of two rows in flight; put(d, value) for every d < D.
+struct FxHead {
+  float x[MK_FX_HEAD_REGS], xp[MK_FX_HEAD_REGS], cs[MK_FX_HEAD_REGS], sn[MK_FX_HEAD_REGS];
+};
+template <typename E>
+__device__ __forceinline__ void fx_head_load(CStage &st, const FxRows<E> &rows, int tok, int col, int pos, int lane, FxHead &h) {
   const int D = st.head_dim, rot = (st.flags & MK_F_ROPE) ? st.rot_dims : 0, half = rot >> 1;
   const float *ct = (const float *)st.cos_tab + (size_t)pos * st.ld_cos, *sn = (const float *)st.sin_tab + (size_t)pos * st.ld_cos;
-  float y[MK_FX_HEAD_REGS];
-  float ss = 0.f;
 #pragma unroll
   for (int j = 0; j < MK_FX_HEAD_REGS; j++)
     if (j * 64 < D) {
       const int d = min(j * 64 + lane, D - 1);
-      y[j] = rows.get(tok, col + d);
+      h.x[j] = rows.get(tok, col + d);
       if (j * 64 < rot) {
         const bool in = d < rot, lo = d < half;
-        const float xp = rows.get(tok, col + (in ? (lo ? d + half : d - half) : d));
+        h.xp[j] = rows.get(tok, col + (in ? (lo ? d + half : d - half) : d));
         const int ci = in ? (lo ? d : d - half) : 0;
-        const float cs = ct[ci], s = sn[ci];
-        y[j] = in ? (lo ? y[j] * cs - xp * s : y[j] * cs + xp * s) : y[j];
+        h.cs[j] = ct[ci];
+        h.sn[j] = sn[ci];
       }
-      ss += j * 64 + lane < D ? y[j] * y[j] : 0.f;
+    }
+}
+template <typename Put>
+__device__ __forceinline__ void fx_head_finish(CStage &st, int lane, FxHead &h, Put put) {
+  const int D = st.head_dim, rot = (st.flags & MK_F_ROPE) ? st.rot_dims : 0, half = rot >> 1;
+  float ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < MK_FX_HEAD_REGS; j++)
+    if (j * 64 < D) {
+      const int d = j * 64 + lane;
+      if (j * 64 < rot && d < rot) h.x[j] = d < half ? h.x[j] * h.cs[j] - h.xp[j] * h.sn[j] : h.x[j] * h.cs[j] + h.xp[j] * h.sn[j];
+      ss += d < D ? h.x[j] * h.x[j] : 0.f;
     }
   if (st.flags & MK_F_QK_NORM) {
     const float r = 1.f / sqrtf(wave_sum(ss) / (float)D + st.eps);
 #pragma unroll
     for (int j = 0; j < MK_FX_HEAD_REGS; j++)
-      if (j * 64 < D) y[j] *= r;
+      if (j * 64 < D) h.x[j] *= r;
   }
 #pragma unroll
   for (int j = 0; j < MK_FX_HEAD_REGS; j++)
-    if (j * 64 + lane < D) put(j * 64 + lane, y[j]);
+    if (j * 64 + lane < D) put(j * 64 + lane, h.x[j]);
 }
 
 // Cache layout, chosen for the matrix cores (a page is page_size positions of all kv heads):
@@ -277,23 +290,44 @@ __device__ __forceinline__ void stage_fx_prep(CStage &st, Ctx &c, const MkRuntim
   const int nkc = (D + KW - 1) / KW, nvb = (DV + 15) / 16, ps = rt.page_size;
   const int per = H + 2 * nkv, total = M * per;
   E *kc = (E *)st.k_cache, *vc = (E *)st.v_cache;
-  for (int i = c.vid * MK_WAVES + wave; i < total; i += c.G * MK_WAVES) {
+  const int stride = c.G * MK_WAVES;
+  auto load = [&](int i, FxHead &h, int &page) {
     const int t = i / per, s = i - t * per;
     const int pos = __builtin_amdgcn_readfirstlane(c.sh_tok[t]);
+    page = s < H ? 0 : rt.kv_indices[__builtin_amdgcn_readfirstlane(c.sh_tok[3 * MK_MAX_TOKENS + t]) + pos / ps];
+    if (s < H + nkv) {
+      fx_head_load<E>(st, rows, t, s * D, pos, lane, h);
+    } else {
+      const int col = (H + nkv) * D + (s - H - nkv) * DV;
+#pragma unroll
+      for (int j = 0; j < MK_FX_HEAD_REGS; j++)
+        if (j * 64 < DV) h.x[j] = rows.get(t, col + min(j * 64 + lane, DV - 1));
+    }
+  };
+  auto finish = [&](int i, FxHead &h, int page) {
+    const int t = i / per, s = i - t * per;
+    const int pp = __builtin_amdgcn_readfirstlane(c.sh_tok[t]) % ps;
     if (s < H) {
       E *q = (E *)st.q_ws + (size_t)t * st.ld_qws + (size_t)s * nkc * KW;
-      fx_head_row<E>(st, rows, t, s * D, pos, lane, [&](int d, float v) { fx_stc(q + d, fx_round<E>(v)); });
+      fx_head_finish(st, lane, h, [&](int d, float v) { fx_stc(q + d, fx_round<E>(v)); });
       for (int d = D + lane; d < nkc * KW; d += 64) fx_stc(q + d, (E)0);
+    } else if (s < H + nkv) {
+      fx_head_finish(st, lane, h, [&](int d, float v) { fx_stc(kc + fx_k_at<E>(page, pp, ps, nkv, s - H, nkc, d), fx_round<E>(v)); });
     } else {
-      const int pg = pos / ps, pp = pos - pg * ps;
-      const int page = rt.kv_indices[__builtin_amdgcn_readfirstlane(c.sh_tok[3 * MK_MAX_TOKENS + t]) + pg];
-      if (s < H + nkv) {
-        fx_head_row<E>(st, rows, t, s * D, pos, lane, [&](int d, float v) { fx_stc(kc + fx_k_at<E>(page, pp, ps, nkv, s - H, nkc, d), fx_round<E>(v)); });
-      } else {
-        const int g = s - H - nkv, col = (H + nkv) * D + g * DV;
-        for (int d = lane; d < DV; d += 64) fx_stc(vc + fx_v_at<E>(page, pp, ps, nkv, g, nvb, d), fx_round<E>(rows.get(t, col + d)));
-      }
+      const int g = s - H - nkv, col = (H + nkv) * D + g * DV;
+#pragma unroll
+      for (int j = 0; j < MK_FX_HEAD_REGS; j++)
+        if (j * 64 + lane < DV) fx_stc(vc + fx_v_at<E>(page, pp, ps, nkv, g, nvb, j * 64 + lane), fx_round<E>(h.x[j]));
+      for (int d = MK_FX_HEAD_REGS * 64 + lane; d < DV; d += 64) fx_stc(vc + fx_v_at<E>(page, pp, ps, nkv, g, nvb, d), fx_round<E>(rows.get(t, col + d)));
     }
+  };
+  for (int i = c.vid * MK_WAVES + wave; i < total; i += 2 * stride) {
+    FxHead h0, h1;
+    int p0, p1 = 0;
+    load(i, h0, p0);
+    if (i + stride < total) load(i + stride, h1, p1);
+    finish(i, h0, p0);
+    if (i + stride < total) finish(i + stride, h1, p1);
   }
   c.wrote_through = true;
 }
@@ -322,6 +356,12 @@ __device__ __forceinline__ float fx_exp2(float, float x) { return exp2f(x); }
 // from memory), and the first tiles' rows, which earlier iterations wrote, are requested before the barrier is awaited.
 // Otherwise the prep stage has written queries, keys and values.
 #define MK_FX_NEG (-1e30f)
+#ifndef MK_TUNE_FX_ONE
+#define MK_TUNE_FX_ONE 2  // tiles per wavefront up to which a unit is not split into chunks (a hand-over costs about two tiles)
+#endif
+#ifndef MK_TUNE_FX_TPW
+#define MK_TUNE_FX_TPW 1  // tiles per wavefront a chunk aims for
+#endif
 template <typename E, int KC, int VB>
 __device__ __forceinline__ void stage_fx_attn_t(CStage &st, Ctx &c, const MkRuntime &rt, int M, bool single, char *smem) {
   using X = FxType<E>;
@@ -373,7 +413,7 @@ __device__ __forceinline__ void stage_fx_attn_t(CStage &st, Ctx &c, const MkRunt
     a.p0 = __builtin_amdgcn_readfirstlane(c.sh_tok[a.t0]);
     a.p = a.p0 + (a.r0 + a.nrows - 1) / qpk;  // newest position any of the rows sees
     const int NT = a.p / TP + 1;
-    a.C = min(cmax, (NT + MK_WAVES - 1) / MK_WAVES);
+    a.C = NT <= MK_TUNE_FX_ONE * MK_WAVES ? 1 : min(cmax, (NT + MK_TUNE_FX_TPW * MK_WAVES - 1) / (MK_TUNE_FX_TPW * MK_WAVES));
     if (a.cidx >= a.C) return false;
     a.tb = (int)(((long long)NT * a.cidx) / a.C);
     a.te = (int)(((long long)NT * (a.cidx + 1)) / a.C);
@@ -434,20 +474,47 @@ __device__ __forceinline__ void stage_fx_attn_t(CStage &st, Ctx &c, const MkRunt
     const bool newest = single && a.cidx == a.C - 1;
     // ---- query rows into operand order (and the new key and value)
     if (single) {
+      // (everything the row writers below leave out is zeroed: unused query columns, padding dims)
       const u32x4 z = {0u, 0u, 0u, 0u};
-      for (int i = tid; i < nkg * KC * 64; i += MK_THREADS) qs[i] = z;
+      for (int i = tid; i < nkg * KC * 64; i += MK_THREADS)
+        if ((i & 15) >= a.nrows || (i >> 6) >= nkc) qs[i] = z;
+      E *q = (E *)qs;
+      for (int i = tid; i < 16 * (nkc * KW - D); i += MK_THREADS) {
+        const int d = D + i / 16;
+        if ((i & 15) < a.nrows) q[((d / KW) * 64 + ((d % KW) / EPC) * 16 + (i & 15)) * EPC + d % EPC] = (E)0;
+      }
       for (int i = D + tid; i < nkc * KW; i += MK_THREADS) kn[i] = (E)0;
       for (int i = DV + tid; i < nvb * 16; i += MK_THREADS) vn[i] = (E)0;
-      __syncthreads();
-      E *q = (E *)qs;
-      for (int r = wave; r < a.nrows; r += MK_WAVES)
-        fx_head_row<E>(st, rows, a.t0, (a.g * qpk + a.r0 + r) * D, a.p, lane,
-                       [&](int d, float v) { q[((d / KW) * 64 + ((d % KW) / EPC) * 16 + r) * EPC + d % EPC] = fx_round<E>(v); });
-      if (newest) {
-        if (wave == MK_WAVES - 1)
-          fx_head_row<E>(st, rows, a.t0, (st.num_q_heads + a.g) * D, a.p, lane, [&](int d, float v) { kn[d] = fx_round<E>(v); });
-        if (wave == MK_WAVES - 2)
-          for (int d = lane; d < DV; d += 64) vn[d] = fx_round<E>(rows.get(a.t0, (st.num_q_heads + nkv) * D + a.g * DV + d));
+      // rows 0 .. nrows - 1 are queries, row nrows (the chunk that owns the new position) is the new key; the last
+      // wavefront, whose tile has been in flight longest, takes row 0 and with it the first of the second round
+      const int n_rows = a.nrows + (newest ? 1 : 0), w_ = MK_WAVES - 1 - wave;
+      const bool v_row = newest && w_ == 1;
+      const int v_col = (st.num_q_heads + nkv) * D + a.g * DV;
+      float vv[MK_FX_HEAD_REGS];
+      if (v_row) {
+#pragma unroll
+        for (int j = 0; j < MK_FX_HEAD_REGS; j++)
+          if (j * 64 < DV) vv[j] = rows.get(a.t0, v_col + min(j * 64 + lane, DV - 1));
+      }
+      auto load_row = [&](int r, FxHead &h) {
+        fx_head_load<E>(st, rows, a.t0, (r < a.nrows ? a.g * qpk + a.r0 + r : st.num_q_heads + a.g) * D, a.p, lane, h);
+      };
+      auto put_row = [&](int r, FxHead &h) {
+        if (r < a.nrows) fx_head_finish(st, lane, h, [&](int d, float v) { q[((d / KW) * 64 + ((d % KW) / EPC) * 16 + r) * EPC + d % EPC] = fx_round<E>(v); });
+        else fx_head_finish(st, lane, h, [&](int d, float v) { kn[d] = fx_round<E>(v); });
+      };
+      for (int r = w_; r < n_rows; r += 2 * MK_WAVES) {
+        FxHead h0, h1;
+        load_row(r, h0);
+        if (r + MK_WAVES < n_rows) load_row(r + MK_WAVES, h1);
+        put_row(r, h0);
+        if (r + MK_WAVES < n_rows) put_row(r + MK_WAVES, h1);
+      }
+      if (v_row) {
+#pragma unroll
+        for (int j = 0; j < MK_FX_HEAD_REGS; j++)
+          if (j * 64 + lane < DV) vn[j * 64 + lane] = fx_round<E>(vv[j]);
+        for (int d = MK_FX_HEAD_REGS * 64 + lane; d < DV; d += 64) vn[d] = fx_round<E>(rows.get(a.t0, v_col + d));
       }
     } else {
       for (int i = tid; i < nkg * KC * 64; i += MK_THREADS) {
