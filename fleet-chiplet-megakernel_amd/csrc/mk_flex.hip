@@ -146,13 +146,17 @@ __device__ __forceinline__ void stage_fx_addnorm_t(CStage &st, Ctx &c, int M, ch
         f32x4 y = {0.f, 0.f, 0.f, 0.f};
         if (dS) {
           const float *p = dpart + (size_t)t * c.defer_n + 4 * s;
-          f32x4 q[8];
+          auto sum_slices = [&](auto ns) {  // all slices requested at once, summed in slice order
+            constexpr int Q = decltype(ns)::value;
+            f32x4 q[Q];
 #pragma unroll
-          for (int b = 0; b < 8; b++)
-            if (b < dS) q[b] = fx_ldc_quad(p + b * dslice);
+            for (int b = 0; b < Q; b++) q[b] = fx_ldc_quad(p + b * dslice);
 #pragma unroll
-          for (int b = 0; b < 8; b++)
-            if (b < dS) y += q[b];
+            for (int b = 0; b < Q; b++) y += q[b];
+          };
+          if (dS == 2) sum_slices(std::integral_constant<int, 2>{});
+          else if (dS == 4) sum_slices(std::integral_constant<int, 4>{});
+          else sum_slices(std::integral_constant<int, 8>{});
         } else if (st.in) {
           y = fx_ldc_quad((const E *)st.in + (size_t)t * st.ld_in + 4 * s);
         }
@@ -196,17 +200,25 @@ template <typename E> struct FxRows {
   int S;
   const float *part;
   size_t slice, ldp;
-  __device__ __forceinline__ float get(int tok, int col) const {
-    if (S == 0) return fx_ldc(in + (size_t)tok * ld + col);
-    const float *p = part + (size_t)tok * ldp + col;
-    float q[8], s = 0.f;
+  template <int NS> __device__ __forceinline__ float get(int tok, int col) const {
+    if constexpr (NS == 0) {
+      return fx_ldc(in + (size_t)tok * ld + col);
+    } else {
+      const float *p = part + (size_t)tok * ldp + col;
+      float q[NS], s = 0.f;
 #pragma unroll
-    for (int b = 0; b < 8; b++)
-      if (b < S) q[b] = ldc_f32(p + b * slice);
+      for (int b = 0; b < NS; b++) q[b] = ldc_f32(p + b * slice);
 #pragma unroll
-    for (int b = 0; b < 8; b++)
-      if (b < S) s += q[b];
-    return fx_val(fx_round<E>(s));
+      for (int b = 0; b < NS; b++) s += q[b];
+      return fx_val(fx_round<E>(s));
+    }
+  }
+  // f(slices) with the slice count as a compile-time constant: one branch per row instead of one per element
+  template <typename F> __device__ __forceinline__ void with_slices(F f) const {
+    if (S == 0) f(std::integral_constant<int, 0>{});
+    else if (S == 2) f(std::integral_constant<int, 2>{});
+    else if (S == 4) f(std::integral_constant<int, 4>{});
+    else f(std::integral_constant<int, 8>{});
   }
 };
 template <typename E> __device__ __forceinline__ FxRows<E> fx_rows(CStage &st, Ctx &c) {
@@ -225,19 +237,31 @@ template <typename E>
 __device__ __forceinline__ void fx_head_load(CStage &st, const FxRows<E> &rows, int tok, int col, int pos, int lane, FxHead &h) {
   const int D = st.head_dim, rot = (st.flags & MK_F_ROPE) ? st.rot_dims : 0, half = rot >> 1;
   const float *ct = (const float *)st.cos_tab + (size_t)pos * st.ld_cos, *sn = (const float *)st.sin_tab + (size_t)pos * st.ld_cos;
+  rows.with_slices([&](auto ns) {
+    constexpr int NS = decltype(ns)::value;
 #pragma unroll
-  for (int j = 0; j < MK_FX_HEAD_REGS; j++)
-    if (j * 64 < D) {
-      const int d = min(j * 64 + lane, D - 1);
-      h.x[j] = rows.get(tok, col + d);
-      if (j * 64 < rot) {
-        const bool in = d < rot, lo = d < half;
-        h.xp[j] = rows.get(tok, col + (in ? (lo ? d + half : d - half) : d));
-        const int ci = in ? (lo ? d : d - half) : 0;
-        h.cs[j] = ct[ci];
-        h.sn[j] = sn[ci];
+    for (int j = 0; j < MK_FX_HEAD_REGS; j++)
+      if (j * 64 < D) {
+        const int d = min(j * 64 + lane, D - 1);
+        h.x[j] = rows.template get<NS>(tok, col + d);
+        if (j * 64 < rot) {
+          const bool in = d < rot, lo = d < half;
+          h.xp[j] = rows.template get<NS>(tok, col + (in ? (lo ? d + half : d - half) : d));
+          const int ci = in ? (lo ? d : d - half) : 0;
+          h.cs[j] = ct[ci];
+          h.sn[j] = sn[ci];
+        }
       }
-    }
+  });
+}
+// ... and a value row, which is copied as it is: columns [0, n) of it, lane l holds every 64th
+template <typename E>
+__device__ __forceinline__ void fx_value_load(const FxRows<E> &rows, int tok, int col, int n, int lane, float (&v)[MK_FX_HEAD_REGS]) {
+  rows.with_slices([&](auto ns) {
+#pragma unroll
+    for (int j = 0; j < MK_FX_HEAD_REGS; j++)
+      if (j * 64 < n) v[j] = rows.template get<decltype(ns)::value>(tok, col + min(j * 64 + lane, n - 1));
+  });
 }
 template <typename Put>
 __device__ __forceinline__ void fx_head_finish(CStage &st, int lane, FxHead &h, Put put) {
@@ -298,10 +322,7 @@ __device__ __forceinline__ void stage_fx_prep(CStage &st, Ctx &c, const MkRuntim
     if (s < H + nkv) {
       fx_head_load<E>(st, rows, t, s * D, pos, lane, h);
     } else {
-      const int col = (H + nkv) * D + (s - H - nkv) * DV;
-#pragma unroll
-      for (int j = 0; j < MK_FX_HEAD_REGS; j++)
-        if (j * 64 < DV) h.x[j] = rows.get(t, col + min(j * 64 + lane, DV - 1));
+      fx_value_load<E>(rows, t, (H + nkv) * D + (s - H - nkv) * DV, DV, lane, h.x);
     }
   };
   auto finish = [&](int i, FxHead &h, int page) {
@@ -314,11 +335,10 @@ __device__ __forceinline__ void stage_fx_prep(CStage &st, Ctx &c, const MkRuntim
     } else if (s < H + nkv) {
       fx_head_finish(st, lane, h, [&](int d, float v) { fx_stc(kc + fx_k_at<E>(page, pp, ps, nkv, s - H, nkc, d), fx_round<E>(v)); });
     } else {
-      const int g = s - H - nkv, col = (H + nkv) * D + g * DV;
+      const int g = s - H - nkv;
 #pragma unroll
       for (int j = 0; j < MK_FX_HEAD_REGS; j++)
         if (j * 64 + lane < DV) fx_stc(vc + fx_v_at<E>(page, pp, ps, nkv, g, nvb, j * 64 + lane), fx_round<E>(h.x[j]));
-      for (int d = MK_FX_HEAD_REGS * 64 + lane; d < DV; d += 64) fx_stc(vc + fx_v_at<E>(page, pp, ps, nkv, g, nvb, d), fx_round<E>(rows.get(t, col + d)));
     }
   };
   for (int i = c.vid * MK_WAVES + wave; i < total; i += 2 * stride) {
@@ -356,12 +376,12 @@ __device__ __forceinline__ float fx_exp2(float, float x) { return exp2f(x); }
 // from memory), and the first tiles' rows, which earlier iterations wrote, are requested before the barrier is awaited.
 // Otherwise the prep stage has written queries, keys and values.
 #define MK_FX_NEG (-1e30f)
-#ifndef MK_TUNE_FX_ONE
-#define MK_TUNE_FX_ONE 2  // tiles per wavefront up to which a unit is not split into chunks (a hand-over costs about two tiles)
-#endif
-#ifndef MK_TUNE_FX_TPW
-#define MK_TUNE_FX_TPW 1  // tiles per wavefront a chunk aims for
-#endif
+// Chunks a unit of NT tiles is split into: none while every wavefront has at most two tiles (a hand-over costs about as
+// much), else one tile per wavefront, and two once that would make more than 16 chunks to combine.
+__device__ __forceinline__ int fx_chunks(int NT, int cmax) {
+  const int rounds = (NT + MK_WAVES - 1) / MK_WAVES;  // tiles of the busiest wavefront without a split
+  return rounds <= 2 ? 1 : min(cmax, rounds <= 16 ? rounds : max(16, (rounds + 1) / 2));
+}
 template <typename E, int KC, int VB>
 __device__ __forceinline__ void stage_fx_attn_t(CStage &st, Ctx &c, const MkRuntime &rt, int M, bool single, char *smem) {
   using X = FxType<E>;
@@ -413,7 +433,7 @@ __device__ __forceinline__ void stage_fx_attn_t(CStage &st, Ctx &c, const MkRunt
     a.p0 = __builtin_amdgcn_readfirstlane(c.sh_tok[a.t0]);
     a.p = a.p0 + (a.r0 + a.nrows - 1) / qpk;  // newest position any of the rows sees
     const int NT = a.p / TP + 1;
-    a.C = NT <= MK_TUNE_FX_ONE * MK_WAVES ? 1 : min(cmax, (NT + MK_TUNE_FX_TPW * MK_WAVES - 1) / (MK_TUNE_FX_TPW * MK_WAVES));
+    a.C = fx_chunks(NT, cmax);
     if (a.cidx >= a.C) return false;
     a.tb = (int)(((long long)NT * a.cidx) / a.C);
     a.te = (int)(((long long)NT * (a.cidx + 1)) / a.C);
@@ -491,11 +511,7 @@ __device__ __forceinline__ void stage_fx_attn_t(CStage &st, Ctx &c, const MkRunt
       const bool v_row = newest && w_ == 1;
       const int v_col = (st.num_q_heads + nkv) * D + a.g * DV;
       float vv[MK_FX_HEAD_REGS];
-      if (v_row) {
-#pragma unroll
-        for (int j = 0; j < MK_FX_HEAD_REGS; j++)
-          if (j * 64 < DV) vv[j] = rows.get(a.t0, v_col + min(j * 64 + lane, DV - 1));
-      }
+      if (v_row) fx_value_load<E>(rows, a.t0, v_col, DV, lane, vv);
       auto load_row = [&](int r, FxHead &h) {
         fx_head_load<E>(st, rows, a.t0, (r < a.nrows ? a.g * qpk + a.r0 + r : st.num_q_heads + a.g) * D, a.p, lane, h);
       };
@@ -514,7 +530,6 @@ __device__ __forceinline__ void stage_fx_attn_t(CStage &st, Ctx &c, const MkRunt
 #pragma unroll
         for (int j = 0; j < MK_FX_HEAD_REGS; j++)
           if (j * 64 + lane < DV) vn[j * 64 + lane] = fx_round<E>(vv[j]);
-        for (int d = MK_FX_HEAD_REGS * 64 + lane; d < DV; d += 64) vn[d] = fx_round<E>(rows.get(a.t0, v_col + d));
       }
     } else {
       for (int i = tid; i < nkg * KC * 64; i += MK_THREADS) {

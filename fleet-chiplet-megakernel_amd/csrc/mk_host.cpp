@@ -746,7 +746,7 @@ int lower_flex_attention(mk_graph *g, size_t &i) {
   const bool f32 = in.dtype == MK_DT_F32;
   const int es = f32 ? 4 : 2, KW = f32 ? 16 : 32, TP = f32 ? 16 : 32;
   if (H < 1 || G < 1 || H % G || D < 1 || DV < 1 || rot < 0 || rot > D || rot % 2) return fail(MK_EINVAL, "flex_attention: heads %d / %d, dims %d / %d, rotated %d", H, G, D, DV, rot);
-  if (D > MK_FX_MAX_HEAD_DIM) return fail(MK_EUNSUPPORTED, "flex_attention: head dim %d (most %d)", D, MK_FX_MAX_HEAD_DIM);
+  if (D > MK_FX_MAX_HEAD_DIM || DV > MK_FX_MAX_HEAD_DIM) return fail(MK_EUNSUPPORTED, "flex_attention: head dims %d / %d (most %d)", D, DV, MK_FX_MAX_HEAD_DIM);
   const int dk = (D + KW - 1) / KW * KW, dv = (DV + 15) / 16 * 16;
   if (in.ndims != 2 || in.dims[0] < B || in.dims[1] < (int64_t)H * D + (int64_t)G * (D + DV)) return fail(MK_EINVAL, "flex_attention: input must be [tokens, >= (q + kv) * dim + kv * value dim]");
   if (o.ndims != 2 || o.dims[0] < B || o.dims[1] < (int64_t)H * DV || o.dtype != in.dtype) return fail(MK_EINVAL, "flex_attention: output must be [tokens, >= q heads * value dim] of the input's type");
