@@ -76,7 +76,7 @@ class Generator:
         self.model.finalize()
 
 
-def main():
+def main(argv=None):
     ap = argparse.ArgumentParser(description="Greedy generation on the MI355X persistent megakernel")
     src = ap.add_mutually_exclusive_group(required=True)
     src.add_argument("--model-path", help="checkpoint directory (config.json + *.safetensors)")
@@ -91,7 +91,7 @@ def main():
     ap.add_argument("--max-num-batched-tokens", type=int, default=None, help="token rows per iteration (default 64, or 1 for a single request of one token)")
     ap.add_argument("--page-size", type=int, default=64)
     ap.add_argument("--eos-token-id", type=int, default=None)
-    args = ap.parse_args()
+    args = ap.parse_args(argv)
     dtype = getattr(torch, args.dtype)
     if args.model_path:
         with open(os.path.join(args.model_path, "config.json")) as f:
