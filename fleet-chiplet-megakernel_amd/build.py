@@ -3,7 +3,7 @@
 Usage: python build.py            (from anywhere; output lands next to this file: the library, then the Cython binding
                                    mirage/_cython/core.*.so that links against it)
 
-Every kernel instantiation is a translation unit of its own; they compile side by side.  `build(kernels=...)` makes a
+The kernels are translation units of their own (build.KERNELS) and compile side by side.  `build(kernels=...)` makes a
 library with only some of them (a graph that needs a missing one is refused by mk_compile); `ensure_library()` is what a
 program calls that wants to run one kind of graph from a fresh checkout.
 """
@@ -18,8 +18,8 @@ HERE = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(HERE, "csrc")
 LIB = os.path.join(HERE, "libfleet_mk.so")
 
-# kernel instantiations of mk_kernel.hip (-DMK_KERNEL_<name>)
-KERNELS = ("GENERAL", "M1", "FLEX", "FLEX_M1", "FLEX_F32")
+# kernels of mk_kernel.hip (-DMK_KERNEL_<name>): the fixed-shape pair, and the flex ones
+KERNELS = ("DENSE", "FLEX", "FLEX_M1", "FLEX_F32")
 
 HIPCC_FLAGS = [
     "--offload-arch=gfx950",

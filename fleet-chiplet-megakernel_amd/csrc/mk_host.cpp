@@ -27,10 +27,8 @@ typedef unsigned u32x4 __attribute__((ext_vector_type(4)));
 // the kernels, each from a translation unit of its own (build.py); a library may be built without some of them
 extern "C" __global__ void mk_pack_weights_kernel(const MkWeight w, int n, int k, int silu, int half, u32x4 *dst, long long total);
 #define MK_DECLARE_KERNEL(name) extern "C" __global__ void name(const MkRuntime rt, const MkRuntime *rtp, int max_iters, int run_scheduler)
-#ifdef MK_HAVE_KERNEL_GENERAL
+#ifdef MK_HAVE_KERNEL_DENSE
 MK_DECLARE_KERNEL(mk_persistent_kernel);
-#endif
-#ifdef MK_HAVE_KERNEL_M1
 MK_DECLARE_KERNEL(mk_persistent_kernel_m1);
 #endif
 #ifdef MK_HAVE_KERNEL_FLEX
@@ -1692,11 +1690,8 @@ static const void *kernel_of(const mk_graph *g) {
   const bool m1 = g->cfg.max_num_batched_tokens == 1;
   const void *k = nullptr;
   if (g->flex == FLEX_NONE) {
-#ifdef MK_HAVE_KERNEL_GENERAL
-    if (!m1) k = (const void *)mk_persistent_kernel;
-#endif
-#ifdef MK_HAVE_KERNEL_M1
-    if (m1) k = (const void *)mk_persistent_kernel_m1;
+#ifdef MK_HAVE_KERNEL_DENSE
+    k = m1 ? (const void *)mk_persistent_kernel_m1 : (const void *)mk_persistent_kernel;
 #endif
   } else if (g->flex == FLEX_BF16) {
 #ifdef MK_HAVE_KERNEL_FLEX

@@ -4368,15 +4368,15 @@ __device__ __forceinline__ void mk_kernel_body(const MkRuntime &rt, const MkRunt
   if (c.vid == 0 && threadIdx.x == 0 && rt.timing) rt.timing[0] = (long long)wall_clock64();
 }
 
-// Each instantiation is a translation unit of its own (build.py compiles this file once per -DMK_KERNEL_*), so they
-// compile side by side and a build may leave out the ones it does not need.
+// build.py compiles this file once per -DMK_KERNEL_*, so that the kernels compile side by side and a build may leave out
+// the ones it does not need.  The two fixed-shape instantiations share a translation unit: compiled alone, the single-token
+// one gets another register assignment (about a thousand more moves and exec-mask instructions) and is 1.3 % slower.
 #define MK_KERNEL_ARGS const MkRuntime rt, const MkRuntime *rtp, int max_iters, int run_scheduler
-#ifdef MK_KERNEL_GENERAL
+#ifdef MK_KERNEL_DENSE
 extern "C" __global__ __launch_bounds__(MK_THREADS, 1) void mk_persistent_kernel(MK_KERNEL_ARGS) {
   mk_kernel_body<MK_MAX_TOKENS, void>(rt, rtp, max_iters, run_scheduler);
 }
-#endif
-#ifdef MK_KERNEL_M1  // graphs with max_num_batched_tokens == 1
+// graphs with max_num_batched_tokens == 1
 extern "C" __global__ __launch_bounds__(MK_THREADS, 1) void mk_persistent_kernel_m1(MK_KERNEL_ARGS) {
   mk_kernel_body<1, void>(rt, rtp, max_iters, run_scheduler);
 }

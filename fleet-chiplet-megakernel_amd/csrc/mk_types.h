@@ -132,19 +132,21 @@ struct MkStage {
   void *out2;
   int num_experts, topk, ld_logits, ld_topk_w;
   int ld_routing, ld_in_slot, ld_out_slot, ld_out2;
-  int ld_out2_slot, pad4, pad5, pad6;
-  // flex stages.  FX_ADDNORM and LINEAR+ADDNORM: rows are `n_pad` long in memory with `k_real` of them real (a linear's
-  // k is n_pad then); y_in / ld_y: the rows added to alpha * res (null: none); out2 / ld_out2: the 32-bit result.
+  int ld_out2_slot;
+  // flex stages (mk_flex.hip)
+  int k_tiles, v_tiles;  // FX_ATTN: instantiation -- operand rows of a key / 16-wide value blocks held at a time
+  int rot_dims;          // FX_ATTN: rotated dims of a head (head_dim: query/key size)
+  // FX_ADDNORM and LINEAR+ADDNORM: rows are padded with zeros to `n` / `k` entries, `k` / `k_real` of them are real; y_in: the
+  // rows added to alpha * res (null: none); out2: the 32-bit result.
   const void *y_in;
-  const void *sink;      // [num_q_heads] fp32, null: none
+  const void *sink;      // FX_ATTN: [num_q_heads] fp32, null: none
   float alpha, w_offset; // residual (or embedding) factor; constant added to the norm weight
   float sm_scale, softcap;  // FX_ATTN: score factor, tanh cap (0: none)
-  int k_real, ld_y;
-  int v_dim, rot_dims;   // FX_ATTN: value size per head, rotated dims (head_dim: query/key size)
-  int k_tiles, v_tiles;  // FX_ATTN: instantiation -- operand rows of a key / 16-wide value blocks held at a time
   float norm_eps;        // LINEAR+ADDNORM: eps of the fused norm
-  int pad7;
+  int k_real, ld_y;
+  int v_dim;             // FX_ATTN: value size per head
 };
+static_assert(sizeof(MkStage) % 64 == 0, "a descriptor is whole scalar-cache lines");
 
 // Hierarchical barrier state.  One 128-byte line per counter so that XCD-local
 // counters stay in that XCD's L2.

@@ -56,8 +56,8 @@ class GraphBuilder(abc.ABC):
 
     @classmethod
     def kernels(cls, dtype: torch.dtype, max_num_batched_tokens: int):
-        """Kernel instantiations of the library (build.py: KERNELS) a graph of this builder runs on."""
-        return ("M1",) if max_num_batched_tokens == 1 else ("GENERAL",)
+        """Kernels of the library (build.py: KERNELS) a graph of this builder runs on."""
+        return ("DENSE",)
 
     @abc.abstractmethod
     def build_from_model(self, model_name: str = None, model_path: str = None):
