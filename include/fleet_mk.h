@@ -123,7 +123,11 @@ void *mk_tensor_ptr(mk_graph *g, int id);
 
 /* Replaces TBGraph.new_input per operand + KNGraph.customized + Graph::register_task(name, params)
  * (core.pyx:1023-1059,817,1011; src/kernel/graph.cc:439-848).  Operands are given inputs first, outputs last,
- * in the order the reference layer builders use; `input_maps` holds 3 ints per operand, `forloop_dims` one. */
+ * in the order the reference layer builders use; `input_maps` holds 3 ints per operand, `forloop_dims` one.
+ * Besides the reference's task names: "embedding_scaled", "residual_rmsnorm" and "flex_attention" (sizes and constants are
+ * parameters, floats as their bits; operands -1 = absent where optional), and "linear" / "silu_mul" / "argmax" over fp32
+ * tensors.  A graph that uses them runs on the flex kernels and holds none of the fixed-shape norm / attention /
+ * mixture-of-experts tasks. */
 int mk_add_task(mk_graph *g, const char *task_name, const int grid_dim[3], const int block_dim[3], int n_operands,
                 const int *tensor_ids, const int *input_maps, const int *forloop_dims, int n_params, const int *params);
 
