@@ -40,6 +40,15 @@ MK_DECLARE_KERNEL(mk_persistent_kernel_flex_m1);
 #ifdef MK_HAVE_KERNEL_FLEX_F32
 MK_DECLARE_KERNEL(mk_persistent_kernel_flex_f32);
 #endif
+#ifdef MK_HAVE_KERNEL_MIX
+MK_DECLARE_KERNEL(mk_persistent_kernel_mix);
+#endif
+#ifdef MK_HAVE_KERNEL_MIX_M1
+MK_DECLARE_KERNEL(mk_persistent_kernel_mix_m1);
+#endif
+#ifdef MK_HAVE_KERNEL_MIX_F32
+MK_DECLARE_KERNEL(mk_persistent_kernel_mix_f32);
+#endif
 
 namespace {
 
@@ -147,7 +156,9 @@ struct mk_graph {
   int64_t row_major_bytes = 0;
   int flex = FLEX_NONE;
   size_t flex_items = 0;     // most work items of a flex attention stage (row tiles x kv heads x value slices)
-  size_t flex_part = 0;      // floats of split-KV partials the flex attention stages need
+  size_t flex_part = 0;      // floats of split-KV partials the flex and latent attention stages need
+  bool mix = false;          // some stage is one of mk_mix.hip's
+  int *state_ids = nullptr;  // batch slot -> recurrent-state slot (the caller's tensor); null: no recurrence
 };
 
 namespace {
@@ -252,7 +263,7 @@ int num_outputs(const Task &t) {
   if (t.name == "gang_attn_split_kv_mi300") return 3;
   if (t.name == "paged_attention_ck_fmha_split_kv_mi300" || t.name == "paged_attention_split_kv_mi300") return 2;
   if (t.name == "moe_topk_softmax_mi300") return 3;
-  if (t.name == "embedding_scaled" || t.name == "residual_rmsnorm") return 2;
+  if (t.name == "embedding_scaled" || t.name == "residual_rmsnorm" || t.name == "residual_prenorm" || t.name == "latent_prep" || t.name == "general_delta") return 2;
   return 1;
 }
 
@@ -816,6 +827,332 @@ int lower_flex_attention(mk_graph *g, size_t &i) {
   return MK_OK;
 }
 
+// ---- mix tasks (mk_mix.hip) --------------------------------------------------------------------------------------------
+bool rows_ok(const Tensor &t, int B, int64_t cols, int dtype) { return t.ndims == 2 && t.dims[0] >= B && t.dims[1] >= cols && t.dtype == dtype && !(t.strides[0] & 3); }
+bool vector_ok(const Tensor &t, int64_t n) { return t.dtype == MK_DT_F32 && (int64_t)t.elems() >= n; }
+
+int set_mix(mk_graph *g, int dtype, const char *task) {
+  g->mix = true;
+  return set_flex(g, dtype, task);
+}
+
+// residual_prenorm [y (optional), y weight (fp32, optional), residual (fp32), weight (fp32, optional), new residual (fp32), rows]
+// params [width, groups, alpha bits, eps bits, y eps bits]: v = residual + alpha * y (with a y weight: of the RMS-normalised
+// y); new residual = v, rows = the RMS norm of v in `groups` equal parts times weight (no weight: v).  A bf16 linear that
+// reads the rows next forms them itself when an iteration has one token.
+int lower_residual_prenorm(mk_graph *g, size_t &i) {
+  const Task t = g->ltasks[i];
+  if (t.ops.size() != 6 || t.params.size() != 5) return fail(MK_EINVAL, "residual_prenorm expects 6 operands / 5 params");
+  auto opt = [&](int k) { return t.ops[k] >= 0 ? &g->tensors[t.ops[k]] : nullptr; };
+  const Tensor *y = opt(0), *yw = opt(1), *w = opt(3);
+  const Tensor x = g->tensors[t.ops[2]], xo = g->tensors[t.ops[4]], o = g->tensors[t.ops[5]];
+  const int B = g->cfg.max_num_batched_tokens, width = t.params[0], groups = t.params[1];
+  const int64_t n = o.ndims == 2 ? o.dims[1] : 0;
+  int rc = set_mix(g, o.dtype, "residual_prenorm");
+  if (rc) return rc;
+  if (n < 4 || n % 4 || width < 1 || width > n || !rows_ok(o, B, n, o.dtype) || !rows_ok(x, B, n, MK_DT_F32) || !rows_ok(xo, B, n, MK_DT_F32) || x.dims[1] != n || xo.dims[1] != n ||
+      (y && (!rows_ok(*y, B, n, o.dtype) || y->dims[1] != n)) || (w && !vector_ok(*w, n)) || (yw && (!y || !vector_ok(*yw, n))))
+    return fail(MK_EINVAL, "residual_prenorm: every row tensor is [tokens, %lld] (a multiple of 4; residual fp32), weights are fp32 of that size, width=%d of it real", (long long)n, width);
+  if (w && (groups < 1 || groups > MK_MX_MAX_GROUPS || width % groups)) return fail(MK_EINVAL, "residual_prenorm: %d parts of a row of %d (at most %d)", groups, width, MK_MX_MAX_GROUPS);
+  if (n > 12 * 4 * MK_THREADS) return fail(MK_EUNSUPPORTED, "residual_prenorm: rows of %lld values (most %d)", (long long)n, 12 * 4 * MK_THREADS);
+  if (x.ptr == xo.ptr || (xo.ptr == o.ptr && w)) return fail(MK_EINVAL, "residual_prenorm: the new residual rows must not overwrite the old ones (other workgroups may still read them), nor the rows them");
+  MkStage st;
+  memset(&st, 0, sizeof(st));
+  st.op = MK_OP_MX_PRENORM;
+  st.n = (int)n;
+  st.k = width;
+  st.norm_groups = w ? groups : 0;
+  st.alpha = bits_f32(t.params[2]);
+  st.eps = bits_f32(t.params[3]);
+  st.norm_eps = bits_f32(t.params[4]);
+  st.in = y ? y->ptr : nullptr;
+  st.ld_in = y ? (int)y->strides[0] : 0;
+  st.y_norm_w = yw ? yw->ptr : nullptr;
+  st.res = x.ptr;
+  st.ld_res = (int)x.strides[0];
+  st.norm_w = w ? w->ptr : nullptr;
+  st.out = xo.ptr == o.ptr ? nullptr : o.ptr;
+  st.ld_out = (int)o.strides[0];
+  st.out2 = xo.ptr;
+  st.ld_out2 = (int)xo.strides[0];
+  if (!g->stages.empty()) {
+    const MkStage &pl = g->stages.back();
+    if (pl.out != st.res && pl.out2 != st.res && pl.norm_out != st.res) st.flags |= MK_F_RES_EARLY;
+  }
+  bool res, silu;
+  int extra;
+  const bool fuse = g->flex == FLEX_BF16 && w && i + 1 < g->ltasks.size() && linear_kind(g->ltasks[i + 1].name, &res, &silu, &extra) && !res && g->ltasks[i + 1].ops[0] == t.ops[5];
+  if (fuse) st.flags |= MK_F_ONLY_MULTI;
+  g->stages.push_back(st);
+  g->stage_desc.push_back(fmt("MX_PRENORM%s %s + %g * %s%s -> %s, %s k=%d parts=%d", fuse ? "[multi-token only]" : "", x.name.c_str(), st.alpha, yw ? "norm of " : "", y ? y->name.c_str() : "0", xo.name.c_str(),
+                              o.name.c_str(), width, st.norm_groups));
+  i++;
+  if (!fuse) return MK_OK;
+  rc = lower_linear(g, i);
+  if (rc) return rc;
+  MkStage &l = g->stages.back();
+  l.flags |= MK_F_NORM | MK_F_PRENORM | (st.flags & MK_F_RES_EARLY);
+  l.y_in = st.in;
+  l.ld_y = st.ld_in;
+  l.y_norm_w = st.y_norm_w;
+  l.res = st.res;
+  l.ld_res = st.ld_res;
+  l.norm_w = st.norm_w;
+  l.norm_out = st.out;
+  l.ld_norm = st.ld_out;
+  l.out2 = st.out2;
+  l.ld_out2 = st.ld_out2;
+  l.alpha = st.alpha;
+  l.norm_groups = st.norm_groups;
+  l.eps = st.eps;
+  l.norm_eps = st.norm_eps;
+  l.k_real = width;
+  return MK_OK;
+}
+
+// gated activation beside another stage: params [output column, n, gate column, up column, limit bits, beta bits, bias bits]
+int lower_glu(mk_graph *g, const Task &t, int out_op, size_t p, const Tensor &in, MkStage *st) {
+  if (t.ops[out_op] < 0) return MK_OK;
+  const Tensor &o = g->tensors[t.ops[out_op]];
+  const int at = t.params[p], n = t.params[p + 1], a = t.params[p + 2], b = t.params[p + 3];
+  if (at < 0 || at % 4 || n < 4 || n % 4 || a < 0 || b < 0 || a % 4 || b % 4 || a + n > in.dims[1] || b + n > in.dims[1] || !rows_ok(o, g->cfg.max_num_batched_tokens, at + n, in.dtype))
+    return fail(MK_EINVAL, "%s: gated activation of %d columns at %d / %d does not fit its rows (multiples of 4)", t.name.c_str(), n, a, b);
+  st->glu_out = (char *)o.ptr + (size_t)at * dtype_size(o.dtype);
+  st->ld_glu = (int)o.strides[0];
+  st->glu_n = n;
+  st->glu_gate = a;
+  st->glu_up = b;
+  st->glu_limit = bits_f32(t.params[p + 4]);
+  st->glu_beta = bits_f32(t.params[p + 5]);
+  st->glu_bias = bits_f32(t.params[p + 6]);
+  return MK_OK;
+}
+
+int lower_rotary_tables(mk_graph *g, const Task &t, int op, int rot, MkStage *st) {
+  if (rot == 0) return MK_OK;
+  if (t.ops[op] < 0 || t.ops[op + 1] < 0) return fail(MK_EINVAL, "%s: rotated dims without cos / sin tables", t.name.c_str());
+  const Tensor &c = g->tensors[t.ops[op]], &s = g->tensors[t.ops[op + 1]];
+  if (c.dtype != MK_DT_F32 || s.dtype != MK_DT_F32 || c.ndims != 2 || s.ndims != 2 || c.dims[1] != rot / 2 || s.dims[1] != rot / 2 || c.dims[0] < g->cfg.max_seq_length ||
+      s.dims[0] < g->cfg.max_seq_length || c.strides[0] != s.strides[0])
+    return fail(MK_EINVAL, "%s: cos / sin tables must be fp32 [>= max_seq_length, rotated dims / 2]", t.name.c_str());
+  st->cos_tab = c.ptr;
+  st->sin_tab = s.ptr;
+  st->ld_cos = (int)c.strides[0];
+  return MK_OK;
+}
+
+struct LatentDims {
+  int kw, nrc, nkc, rp;
+};
+LatentDims latent_dims(int dtype, int rank, int rot) {
+  LatentDims d;
+  d.kw = dtype == MK_DT_F32 ? 16 : 32;
+  d.nrc = (rank + d.kw - 1) / d.kw;
+  d.nkc = d.nrc + (rot + d.kw - 1) / d.kw;
+  d.rp = d.nrc * d.kw;
+  return d;
+}
+int check_latent_cache(mk_graph *g, const Tensor &kc, int dtype, const LatentDims &d, const char *task) {
+  if (kc.ndims != 3 || kc.dtype != dtype || kc.dims[0] < g->cfg.max_num_pages || kc.dims[1] != g->cfg.page_size || kc.dims[2] != d.nkc * d.kw)
+    return fail(MK_EINVAL, "%s: the cache must be [>= %d pages, %d, %d], of the rows' type", task, g->cfg.max_num_pages, g->cfg.page_size, d.nkc * d.kw);
+  return MK_OK;
+}
+
+// latent_prep [rows, q norm (fp32), latent norm (fp32, optional), cos (optional), sin (optional), cache (optional), activation
+// (optional), q latents] params [q column, q rank, latent column, latent rank, rotated column, rotated dims, eps bits, then the
+// gated activation's seven]
+int lower_latent_prep(mk_graph *g, size_t &i) {
+  const Task &t = g->ltasks[i];
+  if (t.ops.size() != 8 || t.params.size() != 14) return fail(MK_EINVAL, "latent_prep expects 8 operands / 14 params");
+  const Tensor &in = g->tensors[t.ops[0]], &qn = g->tensors[t.ops[1]], &o = g->tensors[t.ops[7]];
+  const int B = g->cfg.max_num_batched_tokens, qc = t.params[0], qr = t.params[1], kc = t.params[2], R = t.params[3], rc_ = t.params[4], rot = t.params[5];
+  int rc = set_mix(g, in.dtype, "latent_prep");
+  if (rc) return rc;
+  auto up4 = [](int n) { return (n + 3) / 4 * 4; };
+  if (qr < 1 || qc < 0 || qc % 4 || qr > MK_MX_MAX_NORM_ROW || !rows_ok(in, B, qc + up4(qr), in.dtype) || !rows_ok(o, B, up4(qr), in.dtype) || !vector_ok(qn, up4(qr)))
+    return fail(MK_EINVAL, "latent_prep: query latent of %d values at column %d (at most %d, columns multiples of 4, weights padded to 4)", qr, qc, MK_MX_MAX_NORM_ROW);
+  MkStage st;
+  memset(&st, 0, sizeof(st));
+  st.op = MK_OP_MX_LATENT_PREP;
+  st.in = in.ptr;
+  st.ld_in = (int)in.strides[0];
+  st.n = qr;
+  st.cols[0] = qc;
+  st.q_norm_w = qn.ptr;
+  st.out = o.ptr;
+  st.ld_out = (int)o.strides[0];
+  st.eps = bits_f32(t.params[6]);
+  if (t.ops[5] >= 0) {
+    const LatentDims d = latent_dims(in.dtype, R, rot);
+    if (t.ops[2] < 0 || R < 1 || R > MK_MX_MAX_LATENT || kc < 0 || kc % 4 || rot < 0 || rot % 2 || rc_ < 0 || kc + up4(R) > in.dims[1] || rc_ + rot > in.dims[1] ||
+        !vector_ok(g->tensors[t.ops[2]], up4(R)))
+      return fail(MK_EINVAL, "latent_prep: latent of %d values (at most %d) at column %d, %d rotated at %d", R, MK_MX_MAX_LATENT, kc, rot, rc_);
+    if ((rc = check_latent_cache(g, g->tensors[t.ops[5]], in.dtype, d, "latent_prep"))) return rc;
+    if ((rc = lower_rotary_tables(g, t, 3, rot, &st))) return rc;
+    st.k_cache = g->tensors[t.ops[5]].ptr;
+    st.k_norm_w = g->tensors[t.ops[2]].ptr;
+    st.rank = R;
+    st.rot_dims = rot;
+    st.cols[1] = kc;
+    st.cols[2] = rc_;
+  }
+  if ((rc = lower_glu(g, t, 6, 7, in, &st))) return rc;
+  g->stages.push_back(st);
+  g->stage_desc.push_back(fmt("MX_LATENT_PREP %s -> %s q=%d latent=%d rot=%d glu=%d", in.name.c_str(), o.name.c_str(), qr, st.rank, st.rot_dims, st.glu_n));
+  i++;
+  return MK_OK;
+}
+
+// head_linear [rows, weights, ids (optional), table (optional), output] params [heads, n, k, input columns per head, output
+// columns per head, table column]: one n x k matrix per head, weights in matrix-core operand order (see mk_mix.hip); with a
+// table: out = gelu(.) * table[id][column + n].
+int lower_head_linear(mk_graph *g, size_t &i) {
+  const Task &t = g->ltasks[i];
+  if (t.ops.size() != 5 || t.params.size() != 6) return fail(MK_EINVAL, "head_linear expects 5 operands / 6 params");
+  const Tensor &in = g->tensors[t.ops[0]], &w = g->tensors[t.ops[1]], &o = g->tensors[t.ops[4]];
+  const int B = g->cfg.max_num_batched_tokens, H = t.params[0], n = t.params[1], k = t.params[2], is = t.params[3], os = t.params[4], tc = t.params[5];
+  int rc = set_mix(g, in.dtype, "head_linear");
+  if (rc) return rc;
+  const int es = in.dtype == MK_DT_F32 ? 4 : 2, kw = 64 / es, epc = 16 / es;
+  if (H < 1 || n < 1 || k < kw || k % kw || is < 0 || is % epc || os < 0 || in.strides[0] % epc || !rows_ok(in, B, (int64_t)(H - 1) * is + k, in.dtype) ||
+      o.ndims != 2 || o.dims[0] < B || o.dims[1] < (int64_t)(H - 1) * os + n || o.dtype != in.dtype || w.dtype != in.dtype || (int64_t)w.elems() != (int64_t)H * ((n + 15) / 16 * 16) * k)
+    return fail(MK_EINVAL, "head_linear: %d heads of %d x %d (whole operand rows of %d), input columns %d and output columns %d per head do not fit the operands", H, n, k, kw, is, os);
+  MkStage st;
+  memset(&st, 0, sizeof(st));
+  st.op = MK_OP_MX_HEAD_LINEAR;
+  st.groups = H;
+  st.n = n;
+  st.k = k;
+  st.in = in.ptr;
+  st.ld_in = (int)in.strides[0];
+  st.ld_in_slot = is;
+  st.out = o.ptr;
+  st.ld_out = (int)o.strides[0];
+  st.ld_out_slot = os;
+  st.w.nseg = 1;
+  st.w.seg[0] = w.ptr;
+  if (t.ops[3] >= 0) {
+    const Tensor &tab = g->tensors[t.ops[3]];
+    if (t.ops[2] < 0 || H != 1 || tab.ndims != 2 || tab.dtype != in.dtype || tc < 0 || tc + n > tab.dims[1] || g->tensors[t.ops[2]].dtype != MK_DT_I64 || (int64_t)g->tensors[t.ops[2]].elems() < B)
+      return fail(MK_EINVAL, "head_linear: a table needs int64 ids, one per token row, one head and %d columns from %d on", n, tc);
+    st.flags |= MK_F_GELU_TABLE;
+    st.aux0 = g->tensors[t.ops[2]].ptr;
+    st.aux1 = (char *)tab.ptr + (size_t)tc * es;
+    st.ld_res = (int)tab.strides[0];
+  }
+  g->stages.push_back(st);
+  g->stage_desc.push_back(fmt("MX_HEAD_LINEAR %s x %s -> %s heads=%d n=%d k=%d%s", in.name.c_str(), w.name.c_str(), o.name.c_str(), H, n, k, t.ops[3] >= 0 ? " gelu * table" : ""));
+  g->weight_bytes += (int64_t)w.elems() * es;
+  i++;
+  return MK_OK;
+}
+
+// latent_attention [query rows, query latents, cache, cos (optional), sin (optional), output] params [heads, latent rank, rotated
+// dims, query columns per head, rotated column of a head, scale bits]
+int lower_latent_attention(mk_graph *g, size_t &i) {
+  const Task &t = g->ltasks[i];
+  if (t.ops.size() != 6 || t.params.size() != 6) return fail(MK_EINVAL, "latent_attention expects 6 operands / 6 params");
+  const Tensor &q = g->tensors[t.ops[0]], &ql = g->tensors[t.ops[1]], &kc = g->tensors[t.ops[2]], &o = g->tensors[t.ops[5]];
+  const int B = g->cfg.max_num_batched_tokens, ps = g->cfg.page_size, H = t.params[0], R = t.params[1], rot = t.params[2], hs = t.params[3], ro = t.params[4];
+  int rc = set_mix(g, q.dtype, "latent_attention");
+  if (rc) return rc;
+  const bool f32 = q.dtype == MK_DT_F32;
+  if (H < 1 || R < 1 || R > MK_MX_MAX_LATENT || rot < 0 || rot % 2) return fail(MK_EINVAL, "latent_attention: %d heads, latent of %d values (at most %d), %d rotated", H, R, MK_MX_MAX_LATENT, rot);
+  const LatentDims d = latent_dims(q.dtype, R, rot);
+  if (hs < 0 || ro < 0 || !rows_ok(q, B, (int64_t)(H - 1) * hs + ro + rot, q.dtype) || !rows_ok(ql, B, (int64_t)H * d.rp, q.dtype) || (ql.strides[0] * (f32 ? 4 : 2)) % 16 || !rows_ok(o, B, (int64_t)H * d.rp, q.dtype))
+    return fail(MK_EINVAL, "latent_attention: query latents and output are [tokens, >= heads * %d], the query rows hold %d columns per head", d.rp, hs);
+  if ((rc = check_latent_cache(g, kc, q.dtype, d, "latent_attention"))) return rc;
+  MkStage st;
+  memset(&st, 0, sizeof(st));
+  st.op = MK_OP_MX_LATENT_ATTN;
+  st.in = q.ptr;
+  st.ld_in = (int)q.strides[0];
+  st.ld_in_slot = hs;
+  st.cols[0] = ro;
+  st.q_ws = ql.ptr;
+  st.ld_qws = (int)ql.strides[0];
+  st.k_cache = kc.ptr;
+  st.out = o.ptr;
+  st.ld_out = (int)o.strides[0];
+  st.num_q_heads = H;
+  st.rank = R;
+  st.rot_dims = rot;
+  st.sm_scale = bits_f32(t.params[5]);
+  if ((rc = lower_rotary_tables(g, t, 3, rot, &st))) return rc;
+  // a tile is 16 SUB positions of one page; the kernel's register copy of it holds 20 (short latents: 6) operand rows per wavefront
+  const bool small_ = !f32 && R <= 128 && rot <= 64;
+  const int kcap = small_ ? 6 : 20;
+  st.v_tiles = f32 ? 1 : 2;  // 16-row query tiles per unit
+  const int pages = (g->cfg.max_seq_length + ps - 1) / ps;
+  int sub = 4;
+  auto fits = [&](int s) { return ps % (16 * s) == 0 && d.nkc <= kcap * (MK_WAVES / s) && mk_latent_lds(f32 ? 4 : 2, st.v_tiles, d.nkc, s, pages).bytes <= MK_LDS_BYTES; };
+  while (sub > (f32 ? 1 : 2) && !fits(sub)) sub /= 2;
+  if (!fits(sub)) return fail(MK_EUNSUPPORTED, "latent_attention: page_size %d (a multiple of %d is needed), latent %d + %d or %d pages per request do not fit", ps, f32 ? 16 : 32, R, rot, pages);
+  st.k_tiles = sub;
+  g->flex_part = std::max(g->flex_part, (size_t)g->G * 16 * st.v_tiles * (d.rp + 32));
+  g->stages.push_back(st);
+  g->stage_desc.push_back(fmt("MX_LATENT_ATTN %s, %s -> %s heads=%d latent=%d rot=%d scale=%g", q.name.c_str(), ql.name.c_str(), o.name.c_str(), H, R, rot, st.sm_scale));
+  st.op = MK_OP_MX_LATENT_MERGE;
+  g->stages.push_back(st);
+  g->stage_desc.push_back(fmt("MX_LATENT_MERGE[split requests] -> %s", o.name.c_str()));
+  i++;
+  return MK_OK;
+}
+
+// general_delta [rows, decay weights, decay offset (fp32), removal offset (fp32), norm (fp32), state (fp32), state slots (int32),
+// activation (optional), output] params [heads, dim, low rank (whole operand rows), columns of r k v g a and the low-rank
+// projection, eps bits, then the gated activation's seven]
+int lower_general_delta(mk_graph *g, size_t &i) {
+  const Task &t = g->ltasks[i];
+  if (t.ops.size() != 9 || t.params.size() != 17) return fail(MK_EINVAL, "general_delta expects 9 operands / 17 params");
+  const Tensor &in = g->tensors[t.ops[0]], &w2 = g->tensors[t.ops[1]], &state = g->tensors[t.ops[5]], &ids = g->tensors[t.ops[6]], &o = g->tensors[t.ops[8]];
+  const int B = g->cfg.max_num_batched_tokens, slots = g->cfg.max_num_batched_requests, H = t.params[0], D = t.params[1], rank = t.params[2];
+  int rc = set_mix(g, in.dtype, "general_delta");
+  if (rc) return rc;
+  const int es = in.dtype == MK_DT_F32 ? 4 : 2, kw = 64 / es;
+  if (H < 1 || D < 1 || D > MK_MX_MAX_DELTA_DIM || rank < kw || rank % kw || rank > MK_MX_MAX_RANK)
+    return fail(MK_EUNSUPPORTED, "general_delta: %d heads of %d (at most %d), low rank %d (whole operand rows of %d, at most %d)", H, D, MK_MX_MAX_DELTA_DIM, rank, kw, MK_MX_MAX_RANK);
+  const int nd = (D + 15) / 16, dp = D <= 64 ? 64 : D <= 128 ? 128 : 256;
+  if (!rows_ok(in, B, 1, in.dtype) || !rows_ok(o, B, (int64_t)H * D, in.dtype)) return fail(MK_EINVAL, "general_delta: bad row tensors");
+  for (int a = 0; a < 6; a++) {
+    const int col = t.params[3 + a], n = a == 5 ? rank : H * D;
+    if (col < 0 || col + n > in.dims[1] || (a == 5 && col % 4)) return fail(MK_EINVAL, "general_delta: columns %d .. %d lie outside the rows", col, col + n);
+  }
+  if (w2.dtype != in.dtype || (int64_t)w2.elems() != (int64_t)H * nd * 16 * rank || !vector_ok(g->tensors[t.ops[2]], (int64_t)H * D) || !vector_ok(g->tensors[t.ops[3]], (int64_t)H * D) ||
+      !vector_ok(g->tensors[t.ops[4]], (int64_t)H * D))
+    return fail(MK_EINVAL, "general_delta: decay weights are %d x %d per head in operand order, the three vectors fp32 of %d", nd * 16, rank, H * D);
+  if (state.dtype != MK_DT_F32 || state.ndims != 4 || state.dims[0] < slots || state.dims[1] != H || state.dims[2] != nd * 16 || state.dims[3] != nd * 16)
+    return fail(MK_EINVAL, "general_delta: the state is fp32 [>= %d slots, %d, %d, %d]", slots, H, nd * 16, nd * 16);
+  if (ids.dtype != MK_DT_I32 || (int)ids.elems() < slots) return fail(MK_EINVAL, "general_delta: one int32 state slot per batch slot");
+  if (g->state_ids && g->state_ids != (int *)ids.ptr) return fail(MK_EINVAL, "general_delta: every recurrence of a graph uses the same state-slot tensor");
+  g->state_ids = (int *)ids.ptr;
+  if ((int64_t)6 * 16 * (dp + 4) * 4 + (int64_t)rank / kw * 2048 > MK_LDS_BYTES) return fail(MK_EUNSUPPORTED, "general_delta: head size %d with low rank %d needs too much LDS", D, rank);
+  MkStage st;
+  memset(&st, 0, sizeof(st));
+  st.op = MK_OP_MX_DELTA;
+  st.in = in.ptr;
+  st.ld_in = (int)in.strides[0];
+  st.out = o.ptr;
+  st.ld_out = (int)o.strides[0];
+  st.num_q_heads = H;
+  st.head_dim = D;
+  st.rank = rank;
+  for (int a = 0; a < 6; a++) st.cols[a] = t.params[3 + a];
+  st.eps = bits_f32(t.params[9]);
+  st.w.nseg = 1;
+  st.w.seg[0] = w2.ptr;
+  st.q_norm_w = g->tensors[t.ops[2]].ptr;
+  st.k_norm_w = g->tensors[t.ops[3]].ptr;
+  st.norm_w = g->tensors[t.ops[4]].ptr;
+  st.k_cache = state.ptr;
+  if ((rc = lower_glu(g, t, 7, 10, in, &st))) return rc;
+  g->stages.push_back(st);
+  g->stage_desc.push_back(fmt("MX_DELTA %s -> %s heads=%d d=%d rank=%d glu=%d", in.name.c_str(), o.name.c_str(), H, D, rank, st.glu_n));
+  g->weight_bytes += (int64_t)w2.elems() * es;
+  i++;
+  return MK_OK;
+}
+
 bool is_moe_linear(const std::string &n) {
   return n == "moe_w13_linear_mi300" || n == "moe_w2_linear_mi300" || n == "gang_moe_w13_linear_mi300" || n == "gang_moe_w2_linear_mi300";
 }
@@ -995,6 +1332,8 @@ int lower(mk_graph *g) {
   g->last_linear_task = g->last_linear_stage = -1;
   g->flex = FLEX_NONE;
   g->flex_items = g->flex_part = 0;
+  g->mix = false;
+  g->state_ids = nullptr;
   const int B = g->cfg.max_num_batched_tokens;
   // The list that is lowered: the recorded tasks, with the composite ones spelt out as the tasks they stand for (the
   // task graph handed back to the caller keeps them as recorded).
@@ -1126,6 +1465,21 @@ int lower(mk_graph *g) {
       if (rc) return rc;
     } else if (t.name == "flex_attention") {
       int rc = lower_flex_attention(g, i);
+      if (rc) return rc;
+    } else if (t.name == "residual_prenorm") {
+      int rc = lower_residual_prenorm(g, i);
+      if (rc) return rc;
+    } else if (t.name == "latent_prep") {
+      int rc = lower_latent_prep(g, i);
+      if (rc) return rc;
+    } else if (t.name == "head_linear") {
+      int rc = lower_head_linear(g, i);
+      if (rc) return rc;
+    } else if (t.name == "latent_attention") {
+      int rc = lower_latent_attention(g, i);
+      if (rc) return rc;
+    } else if (t.name == "general_delta") {
+      int rc = lower_general_delta(g, i);
       if (rc) return rc;
     } else if (t.name == "moe_topk_softmax_mi300") {
       bool inline_next = false;
@@ -1312,6 +1666,7 @@ int lower(mk_graph *g) {
       return fail(MK_EUNSUPPORTED, "task '%s' has no MI355X lowering", t.name.c_str());
     }
   }
+  if (g->spec_len && g->state_ids) return fail(MK_EUNSUPPORTED, "speculative decoding with a recurrence: rows of rejected guesses cannot be taken back out of its state");
   g->stage_weight.resize(g->stages.size(), -1);
   for (size_t s = 0; s < g->stages.size(); s++) {
     const int op = g->stages[s].op;
@@ -1336,7 +1691,13 @@ int lower(mk_graph *g) {
       case MK_OP_FX_ADDNORM: st.prof_event = 119; break;
       case MK_OP_FX_PREP:
       case MK_OP_FX_ATTN: st.prof_event = 116; break;
-      case MK_OP_LINEAR_F32: st.prof_event = 120; break;
+      case MK_OP_LINEAR_F32:
+      case MK_OP_MX_HEAD_LINEAR: st.prof_event = 120; break;
+      case MK_OP_MX_PRENORM: st.prof_event = 119; break;
+      case MK_OP_MX_LATENT_PREP:
+      case MK_OP_MX_LATENT_ATTN:
+      case MK_OP_MX_LATENT_MERGE:
+      case MK_OP_MX_DELTA: st.prof_event = 116; break;
       case MK_OP_FX_ARGMAX_F32: st.prof_event = 110; break;
       case MK_OP_NGRAM_PARTIAL: st.prof_event = 112; break;
       case MK_OP_NGRAM_GLOBAL: st.prof_event = 113; break;
@@ -1392,7 +1753,8 @@ int task_type_id(const std::string &n) {
       {"paged_attention_ck_fmha_merge_mi300", 131}, {"gang_attn_merge_mi300", 139}, {"splitk_reduce_mi300", 132},
       {"silu_mul_linear_with_residual", 105}, {"rmsnorm_linear", 102}, {"identity", 121}, {"argmax", 109}, {"attention", 103},
       {"find_ngram_partial", 112}, {"find_ngram_global", 113}, {"target_verify_greedy", 114}, {"single_batch_extend_attention", 115},
-      {"embedding_scaled", 101}, {"residual_rmsnorm", 119}, {"flex_attention", 116}};
+      {"embedding_scaled", 101}, {"residual_rmsnorm", 119}, {"flex_attention", 116},
+      {"residual_prenorm", 119}, {"latent_prep", 116}, {"head_linear", 120}, {"latent_attention", 116}, {"general_delta", 116}};
   auto it = ids.find(n);
   return it == ids.end() ? 0 : it->second;
 }
@@ -1692,6 +2054,16 @@ static const void *kernel_of(const mk_graph *g) {
   if (g->flex == FLEX_NONE) {
 #ifdef MK_HAVE_KERNEL_DENSE
     k = m1 ? (const void *)mk_persistent_kernel_m1 : (const void *)mk_persistent_kernel;
+#endif
+  } else if (g->mix) {
+#ifdef MK_HAVE_KERNEL_MIX
+    if (g->flex == FLEX_BF16 && !m1) k = (const void *)mk_persistent_kernel_mix;
+#endif
+#ifdef MK_HAVE_KERNEL_MIX_M1
+    if (g->flex == FLEX_BF16 && m1) k = (const void *)mk_persistent_kernel_mix_m1;
+#endif
+#ifdef MK_HAVE_KERNEL_MIX_F32
+    if (g->flex == FLEX_F32) k = (const void *)mk_persistent_kernel_mix_f32;
 #endif
   } else if (g->flex == FLEX_BF16) {
 #ifdef MK_HAVE_KERNEL_FLEX
@@ -1995,10 +2367,12 @@ int mk_add_task(mk_graph *g, const char *task_name, const int grid_dim[3], const
   }
   for (int i = 0; i < n_operands; i++) {
     // id -1 = optional operand that is absent: only the q/k-norm weights and the cos/sin tables of the attention tasks
-    // (and the sink of flex_attention, the summand of residual_rmsnorm)
+    // (and the sink of flex_attention, the summand of residual_rmsnorm, what the mix tasks may leave out)
     const bool optional = ((t.name == "gang_attn_split_kv_mi300" || t.name == "kv_cache_update_mi300" || t.name == "paged_attention" ||
                            t.name == "paged_attention_split_kv_mi300" || t.name == "attention" || t.name == "single_batch_extend_attention") && i >= 3 && i <= 6) ||
-                          (t.name == "flex_attention" && i >= 3 && i <= 5) || (t.name == "residual_rmsnorm" && i == 0);
+                          (t.name == "flex_attention" && i >= 3 && i <= 5) || (t.name == "residual_rmsnorm" && i == 0) ||
+                          (t.name == "residual_prenorm" && (i == 0 || i == 1 || i == 3)) || (t.name == "latent_prep" && i >= 2 && i <= 6) ||
+                          (t.name == "head_linear" && (i == 2 || i == 3)) || (t.name == "latent_attention" && (i == 3 || i == 4)) || (t.name == "general_delta" && i == 7);
     if (tensor_ids[i] >= (int)g->tensors.size() || tensor_ids[i] < (optional ? -1 : 0))
       return fail(MK_EINVAL, "task '%s': bad tensor id %d for operand %d", task_name, tensor_ids[i], i);
     t.ops.push_back(tensor_ids[i]);
@@ -2017,7 +2391,7 @@ int mk_add_task(mk_graph *g, const char *task_name, const int grid_dim[3], const
                                 "paged_attention", "paged_attention_split_kv_mi300", "paged_attention_split_kv_merge_mi300",
                                 "paged_attention_ck_fmha_merge_mi300", "gang_attn_merge_mi300", "splitk_reduce_mi300", "silu_mul_linear_with_residual", "rmsnorm_linear", "identity", "argmax", "attention",
                                 "find_ngram_partial", "find_ngram_global", "target_verify_greedy", "single_batch_extend_attention",
-                                "embedding_scaled", "residual_rmsnorm", "flex_attention"};
+                                "embedding_scaled", "residual_rmsnorm", "flex_attention", "residual_prenorm", "latent_prep", "head_linear", "latent_attention", "general_delta"};
   bool ok = linear_kind(t.name, &a, &b, &c);
   for (auto k : known) ok = ok || t.name == k;
   if (!ok) return fail(MK_EUNSUPPORTED, "Unsupported task name: %s", task_name);
@@ -2110,6 +2484,7 @@ int mk_compile(mk_graph *g) {
   rt.total_requests = c.total_num_requests;
   rt.max_new_per_req = c.max_tokens_per_request > 0 ? c.max_tokens_per_request : 8;
   rt.spec_len = g->spec_len;
+  rt.state_ids = g->state_ids;
   rt.eos_token_id = c.eos_token_id;
   rt.step = c.step;
   rt.tokens = (long long *)c.tokens;
@@ -2248,6 +2623,11 @@ int mk_init_requests(mk_graph *g) {
   HIP_TRY(hipDeviceSynchronize());
   HIP_TRY(hipMemset(rt.step, 0, sizeof(int) * rt.total_requests));
   HIP_TRY(hipMemset(rt.request_ids, 0xFF, sizeof(int) * rt.max_requests));
+  if (rt.state_ids) {
+    std::vector<int> ids(rt.max_requests);
+    for (int i = 0; i < rt.max_requests; i++) ids[i] = i;
+    HIP_TRY(hipMemcpy(rt.state_ids, ids.data(), sizeof(int) * rt.max_requests, hipMemcpyHostToDevice));
+  }
   HIP_TRY(hipMemset(rt.qo_indptr, 0, sizeof(int) * (rt.max_requests + 1)));
   HIP_TRY(hipMemset(rt.kv_indptr, 0, sizeof(int) * (rt.max_requests + 1)));
   std::vector<int> pq(rt.max_pages);

@@ -74,6 +74,12 @@ typedef const __attribute__((address_space(4))) MkWeight CWeight;
 #define MK_TUNE_R24 2
 #endif
 
+#if defined(MK_KERNEL_MIX) || defined(MK_KERNEL_MIX_M1) || defined(MK_KERNEL_MIX_F32)
+#define MK_HAVE_MIX 1  // this translation unit holds a kernel with the mix stages (mk_mix.hip) beside the flex ones
+#else
+#define MK_HAVE_MIX 0
+#endif
+
 struct Ctx {
   int vid;   // virtual workgroup id: xcd-major, so vids [x*quota, (x+1)*quota) share an L2
   int G;     // workgroups in the grid
@@ -106,6 +112,9 @@ struct Ctx {
   const float *defer_part;  // [slice][row][n] fp32
   const void *defer_res;  // residual rows of that linear (null: none)
   int defer_ld_res;
+#if MK_HAVE_MIX
+  bool mx_split;  // the latent attention that just ran left some request in chunks
+#endif
 #ifdef MK_TRACE
   long long mark[4];  // (tracing builds) wall-clock marks the running stage sets, stored next to its stage timing
 #endif
@@ -386,6 +395,14 @@ __device__ __attribute__((noinline)) int mk_prepare_next_batch(const MkRuntime &
       }
     }
   }
+  if (rt.state_ids) {
+    // recurrent-state slots move with their requests: the survivors' in front, in order, then the free ones
+    int n = 0;
+    for (int pass = 0; pass < 2; pass++)
+      for (int i = 0; i < R; i++)
+        if ((rt.request_ids[i] >= 0) == (pass == 0)) scratch_pages[n++] = rt.state_ids[i];
+    for (int i = 0; i < R; i++) rt.state_ids[i] = scratch_pages[i];
+  }
   // 2. snapshot the page table (it is compacted in place below)
   const int old_pages = rt.kv_indptr[R];
   for (int i = 0; i < old_pages; i++) scratch_pages[i] = rt.kv_indices[i];
@@ -535,6 +552,10 @@ __device__ __attribute__((noinline)) int mk_prepare_next_batch_wave(const MkRunt
   const unsigned long long alive_mask = __ballot(alive);
   const int rank = __popcll(alive_mask & ((1ull << lane) - 1ull));
   const int nrun = __popcll(alive_mask);
+  if (rt.state_ids && slot) {  // recurrent-state slots: the survivors' in front, in order, then the free ones
+    const int id = rt.state_ids[lane];
+    rt.state_ids[alive ? rank : nrun + (lane - rank)] = id;
+  }
   const int wish = alive ? (plen - st > 0 ? min(plen - st, rt.max_new_per_req) : 1) : 0;
   const int wish_incl = wave_incl_scan(wish, lane);
   const int tok0 = min(wish_incl - wish, B), n = min(wish_incl, B) - tok0;
@@ -885,6 +906,13 @@ __device__ __forceinline__ void stage_norm(CStage &st, Ctx &c, int M, char *smem
 
 __device__ __forceinline__ float silu_mul(float g, float u) { return g / (1.f + __expf(-g)) * u; }
 
+#if MK_HAVE_MIX  // a residual_prenorm in front of a single-token linear (mk_mix.hip): by the workgroup, by the control wavefront
+__device__ __forceinline__ void mx_x_m1_prenorm(CStage &st, const Ctx &c, uint32_t *xs, float *red);
+template <int KL> __device__ __forceinline__ void mx_x_m1_prenorm_wave(CStage &st, Ctx &c, uint32_t *xs, int lane);
+// the control wavefront wants whole 16-byte segments in one part of the norm, and few parts
+__device__ __forceinline__ bool mx_prenorm_by_wave(CStage &st) { return st.k <= 4096 && st.norm_groups <= 8 && (st.k_real / st.norm_groups & 7) == 0; }
+#endif
+
 // Stage the single input row of a one-token linear in LDS as packed bf16, applying the fused RMSNorm when the
 // stage asks for it (virtual workgroup 0 also stores the normalised row, which is the norm task's output tensor).
 // FX: the norm in front may be an FX_ADDNORM (see mk_flex.hip): alpha * residual + y, both rows in memory, then the norm.
@@ -894,6 +922,12 @@ __device__ __forceinline__ void stage_x_m1(CStage &st, const Ctx &c, uint32_t *x
   const unsigned long long *xin = (const unsigned long long *)st.in;
   unsigned long long *xs2 = (unsigned long long *)xs;
   if constexpr (FX) {
+#if MK_HAVE_MIX
+    if (st.flags & MK_F_PRENORM) {
+      mx_x_m1_prenorm(st, c, xs, red);
+      return;
+    }
+#endif
     if (st.flags & MK_F_ADDNORM) {
       f32x4 *vs = (f32x4 *)((char *)xs + MK_MOE_OFFSET);  // the sum, 32-bit
       float ss = 0.f;
@@ -1124,6 +1158,10 @@ __device__ __forceinline__ void stage_linear_m1_t(CStage &st, Ctx &c, char *smem
         if (uo[j] >= 0) load_unit(uo[j], buf[j]);
       }
     }
+#if MK_HAVE_MIX
+  } else if (FX && (st.flags & MK_F_PRENORM)) {
+    if constexpr (FX && KL <= 8) mx_x_m1_prenorm_wave<KL>(st, c, xs, lane);
+#endif
   } else if (FX && (st.flags & MK_F_ADDNORM)) {
     if constexpr (FX && KL <= 8) stage_x_m1_addnorm_wave<KL>(st, c, xs, lane);  // (longer rows take the generic form)
   } else {
@@ -1284,6 +1322,10 @@ __device__ __forceinline__ void stage_linear_m1(CStage &st, Ctx &c, char *smem) 
   const bool fits = ((silu ? st.n / 2 : st.n) / c.G + 1) * 2 <= MK_MOE_OFFSET - MK_OUT_OFFSET;
   if (!fits || (FX && (st.flags & MK_F_ADDNORM) && st.k > 4096)) {
     stage_linear_m1_generic<FX>(st, c, smem);
+#if MK_HAVE_MIX
+  } else if (FX && (st.flags & MK_F_PRENORM) && !mx_prenorm_by_wave(st)) {
+    stage_linear_m1_generic<FX>(st, c, smem);
+#endif
   } else if (st.k == 4096) {
     if (silu) stage_linear_m1_t<8, MK_TUNE_R8, true, W0OK, FX>(st, c, smem);
     else stage_linear_m1_t<8, MK_TUNE_R8N, false, W0OK, FX>(st, c, smem);
@@ -1501,7 +1543,7 @@ __device__ __forceinline__ void stage_linear_small(CStage &st, Ctx &c, int M, ch
 #define MK_TUNE_SMALL_MAX 2
 #endif
 __device__ __forceinline__ bool linear_small_ok(CStage &st, const Ctx &c, int M) {
-  if (M > MK_TUNE_SMALL_MAX || (st.k != 4096 && st.k != 2048) || (st.flags & MK_F_ADDNORM)) return false;
+  if (M > MK_TUNE_SMALL_MAX || (st.k != 4096 && st.k != 2048) || (st.flags & (MK_F_ADDNORM | MK_F_PRENORM))) return false;
   const int n_out = (st.flags & MK_F_SILU) ? st.n / 2 : st.n;
   return (size_t)M * st.k * 2 <= (size_t)(MK_LDS_BYTES - MK_MOE_X_OFFSET) && (size_t)M * (n_out / c.G + 1) * 2 <= (size_t)MK_MOE_OFFSET;
 }
@@ -4081,8 +4123,11 @@ __device__ __attribute__((noinline)) void mk_verify_greedy(int stage, const MkRu
   }
 }
 
-#if defined(MK_KERNEL_FLEX) || defined(MK_KERNEL_FLEX_M1) || defined(MK_KERNEL_FLEX_F32)
+#if defined(MK_KERNEL_FLEX) || defined(MK_KERNEL_FLEX_M1) || defined(MK_KERNEL_FLEX_F32) || MK_HAVE_MIX
 #include "mk_flex.hip"
+#if MK_HAVE_MIX
+#include "mk_mix.hip"
+#endif
 #define MK_HAVE_FLEX 1
 #else
 #define MK_HAVE_FLEX 0
@@ -4104,8 +4149,11 @@ __device__ __forceinline__ void run_stage_program(const MkRuntime &rt, const MkR
       // (a handle that holds only the matrix-core copies of its weights runs every linear in a matrix-core form, which
       // reads normalised rows from the NORM stage's output: that stage then runs for one and two tokens as well)
       const bool packed_only = MAXM > 1 && rt.packed_only;
-      if ((flags & MK_F_ONLY_MULTI) && M == 1 && !(packed_only && (op == MK_OP_NORM || (FX && op == MK_OP_FX_ADDNORM)))) continue;
+      if ((flags & MK_F_ONLY_MULTI) && M == 1 && !(packed_only && (op == MK_OP_NORM || (FX && (op == MK_OP_FX_ADDNORM || op == MK_OP_MX_PRENORM))))) continue;
       if (FX && op == MK_OP_FX_PREP && single) continue;
+#if MK_HAVE_MIX
+      if (op == MK_OP_MX_LATENT_MERGE && !c.mx_split) continue;
+#endif
       if ((flags & MK_F_ONLY_MULTI) && op == MK_OP_NORM && s + 1 < rt.num_stages && !packed_only) {
         // the few-token linear normalises its rows itself
         CStage &nx = ((CStage *)(unsigned long long)rt.stages)[s + 1];
@@ -4126,6 +4174,14 @@ __device__ __forceinline__ void run_stage_program(const MkRuntime &rt, const MkR
           }
           break;
         case MK_OP_FX_ARGMAX_F32: if constexpr (F32) stage_fx_argmax_f32(st, c, rt, M); break;
+#endif
+#if MK_HAVE_MIX
+        case MK_OP_MX_PRENORM: stage_mx_prenorm<E>(st, c, M, smem); break;
+        case MK_OP_MX_LATENT_PREP: stage_mx_latent_prep<E>(st, c, rt, M); break;
+        case MK_OP_MX_HEAD_LINEAR: stage_mx_head_linear<E, MAXM>(st, c, M, smem); break;
+        case MK_OP_MX_LATENT_ATTN: stage_mx_latent_attn<E>(st, c, rt, M, smem); break;
+        case MK_OP_MX_LATENT_MERGE: stage_mx_latent_merge<E>(st, c, rt, M); break;
+        case MK_OP_MX_DELTA: stage_mx_delta<E>(st, c, rt, M, smem); break;
 #endif
         case MK_OP_EMBED: if constexpr (!FX) stage_embed(st, c, rt, M); break;
         case MK_OP_NORM: if constexpr (!FX) stage_norm(st, c, M, smem); break;
@@ -4389,6 +4445,21 @@ extern "C" __global__ __launch_bounds__(MK_THREADS, 1) void mk_persistent_kernel
 #ifdef MK_KERNEL_FLEX_M1
 extern "C" __global__ __launch_bounds__(MK_THREADS, 1) void mk_persistent_kernel_flex_m1(MK_KERNEL_ARGS) {
   mk_kernel_body<1, uint16_t>(rt, rtp, max_iters, run_scheduler);
+}
+#endif
+#ifdef MK_KERNEL_MIX  // graphs with mix stages (mk_mix.hip): the flex stages and those
+extern "C" __global__ __launch_bounds__(MK_THREADS, 1) void mk_persistent_kernel_mix(MK_KERNEL_ARGS) {
+  mk_kernel_body<MK_MAX_TOKENS, uint16_t>(rt, rtp, max_iters, run_scheduler);
+}
+#endif
+#ifdef MK_KERNEL_MIX_M1
+extern "C" __global__ __launch_bounds__(MK_THREADS, 1) void mk_persistent_kernel_mix_m1(MK_KERNEL_ARGS) {
+  mk_kernel_body<1, uint16_t>(rt, rtp, max_iters, run_scheduler);
+}
+#endif
+#ifdef MK_KERNEL_MIX_F32
+extern "C" __global__ __launch_bounds__(MK_THREADS, 1) void mk_persistent_kernel_mix_f32(MK_KERNEL_ARGS) {
+  mk_kernel_body<MK_MAX_TOKENS, float>(rt, rtp, max_iters, run_scheduler);
 }
 #endif
 #ifdef MK_KERNEL_FLEX_F32  // 32-bit activations, weights and caches

@@ -10,6 +10,12 @@
 #pragma once
 #include <stdint.h>
 
+#ifdef __HIP__
+#define MK_HOST_DEVICE __host__ __device__
+#else
+#define MK_HOST_DEVICE
+#endif
+
 #define MK_THREADS 256        // threads per workgroup (4 wavefronts of 64)
 #define MK_WAVES 4
 #define MK_MAX_XCD 16
@@ -58,6 +64,13 @@ enum MkOp {
   MK_OP_FX_ATTN = 18,        // paged attention with softcap and sink (single-token iterations: preparation and append included)
   MK_OP_LINEAR_F32 = 19,     // LINEAR with 32-bit operands
   MK_OP_FX_ARGMAX_F32 = 20,  // ARGMAX_PARTIAL over 32-bit logits
+  // latent attention, recurrence and what goes with them (mk_mix.hip); a graph that holds one runs on the mix kernels
+  MK_OP_MX_PRENORM = 21,     // v = res + alpha * in (in: optionally RMS-normalised first); out2 = v in 32 bits, out = group RMS norm of v (or v), rounded
+  MK_OP_MX_LATENT_PREP = 22, // normalised query latents, normalised + rotated key latents into their pages, gated activation
+  MK_OP_MX_HEAD_LINEAR = 23, // one small matrix per head; optionally gelu(...) * a per-token table row
+  MK_OP_MX_LATENT_ATTN = 24, // attention in the latent space, one shared key/value row per position
+  MK_OP_MX_LATENT_MERGE = 25,  // chunks of the latent attention (iterations in which some request was split)
+  MK_OP_MX_DELTA = 26,       // generalised delta rule: recurrent state per request and head, gated activation beside it
 };
 
 enum MkStageFlags {
@@ -72,8 +85,17 @@ enum MkStageFlags {
   MK_F_MOE_COMBINE = 256,       // MOE_LINEAR: a single-token iteration also forms res + sum_k w_k * y_k (the MOE_COMBINE stage after it is multi-token only)
   MK_F_DEFER_SUM = 512,  // LINEAR: the next stage is a full-row NORM over this stage's output, which may be handed the K-slice partials to sum
   MK_F_ADDNORM = 1024,   // LINEAR (set together with MK_F_NORM): the norm in front is an FX_ADDNORM; a single-token iteration forms it inside this stage
+  MK_F_PRENORM = 4096,   // LINEAR (set together with MK_F_NORM): the norm in front is an MX_PRENORM; a single-token iteration forms it inside this stage
+  MK_F_GELU_TABLE = 8192,  // MX_HEAD_LINEAR: out = gelu(acc) * table[id][n]
   MK_F_RES_EARLY = 2048, // FX_ADDNORM / LINEAR+ADDNORM: the stage before this one does not write the residual rows, so they may be requested before its barrier
 };
+
+#define MK_MX_MAX_GROUPS 256     // parts of a row with a norm of their own
+#define MK_MX_MAX_NORM_ROW 4096  // longest query latent / key latent row a wavefront normalises
+#define MK_MX_MAX_LATENT 512     // key latent size of the latent attention
+#define MK_MX_MAX_LATENT_CHUNKS 40  // 64-byte operand rows of a cached latent (latent + rotated part)
+#define MK_MX_MAX_DELTA_DIM 256  // head size of the recurrence
+#define MK_MX_MAX_RANK 1024      // low-rank decay projection
 
 #define MK_FX_MAX_HEAD_DIM 512  // largest q/k head the flex attention keeps in a wavefront's registers
 
@@ -145,8 +167,33 @@ struct MkStage {
   float norm_eps;        // LINEAR+ADDNORM: eps of the fused norm
   int k_real, ld_y;
   int v_dim;             // FX_ATTN: value size per head
+  // mix stages (mk_mix.hip)
+  const void *y_norm_w;  // MX_PRENORM / LINEAR+PRENORM: fp32 weight of the RMS norm of the summand (null: none)
+  int norm_groups;       // ... parts of the output norm (0: no norm)
+  int rank;              // key latent size (latent stages); padded low rank of the decay projection (MX_DELTA)
+  int cols[6];           // columns of `in`: MX_LATENT_PREP q latent, k latent; MX_LATENT_ATTN rotated query part of a head; MX_DELTA r k v g a w1
+  // gated activation beside MX_LATENT_PREP / MX_DELTA: out = a / (1 + exp(-beta a)) * (b + bias), a = min(gate, limit), b = clamp(up, -limit, limit)
+  void *glu_out;
+  int glu_n, ld_glu, glu_gate, glu_up;
+  float glu_limit, glu_beta, glu_bias;
+  int pad_mx[13];
 };
 static_assert(sizeof(MkStage) % 64 == 0, "a descriptor is whole scalar-cache lines");
+
+// LDS map of MX_LATENT_ATTN, in bytes: query operands, one tile of cached rows, weights of the tile's positions, row statistics,
+// page-table entries.  RT: 16-row query tiles per unit; nkc: operand rows of a cached latent; sub: 16-position sub-tiles of a tile.
+struct MkLatentLds {
+  int kt, pb, mx, pages, bytes;
+};
+MK_HOST_DEVICE inline MkLatentLds mk_latent_lds(int es, int rt, int nkc, int sub, int max_pages) {
+  MkLatentLds l;
+  l.kt = rt * nkc * 1024;
+  l.pb = l.kt + sub * nkc * 1024;
+  l.mx = l.pb + rt * 1024 * (es == 2 ? (sub + 1) / 2 * 2 : sub);
+  l.pages = l.mx + 2 * 4 * rt * 16 * 4;
+  l.bytes = l.pages + (max_pages + 1) * 4;
+  return l;
+}
 
 // Hierarchical barrier state.  One 128-byte line per counter so that XCD-local
 // counters stay in that XCD's L2.
@@ -167,11 +214,6 @@ struct MkSync {
 // Barrier completion test.  Arrival counters and their targets (quota x epoch) are 32-bit and only ever grow during a
 // launch, so on a long launch both wrap; their difference taken as a signed number stays correct as long as the two
 // are less than 2^31 apart, and they are never more than one stage apart.
-#ifdef __HIP__
-#define MK_HOST_DEVICE __host__ __device__
-#else
-#define MK_HOST_DEVICE
-#endif
 MK_HOST_DEVICE inline bool mk_counter_reached(unsigned counter, unsigned target) { return (int)(counter - target) >= 0; }
 
 // Who describes the batch of an iteration (the kernel's `run_scheduler` argument).
@@ -210,6 +252,7 @@ struct MkRuntime {
   int *kv_last_page_len;
   // library-owned scheduler memory
   int *request_ids;   // [max_requests] request id per batch slot, -1 = free
+  int *state_ids;     // [max_requests] recurrent-state slot per batch slot, a permutation (null: the graph has no recurrence)
   int *page_queue;    // [max_pages] ring of free page ids
   int *tok_slot;      // [max_tokens] batch slot of each token of this iteration
   int *tok_pos;       // [max_tokens] absolute position of each token

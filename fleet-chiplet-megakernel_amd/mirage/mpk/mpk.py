@@ -56,6 +56,7 @@ class MPKMetadata:
     paged_kv_indptr_buffer: Optional[torch.Tensor] = None
     paged_kv_indices_buffer: Optional[torch.Tensor] = None
     paged_kv_last_page_len_buffer: Optional[torch.Tensor] = None
+    state_slots_buffer: Optional[torch.Tensor] = None  # recurrent models: int32, the state slot of every batch slot (None: the builder's)
     # MirageModelConfig
     model_config: Optional[MirageModelConfig] = None
     # profiling
@@ -174,7 +175,8 @@ class MPK:
                 "step": self.step, "tokens": self.tokens, "input_tokens": self.input_tokens, "output_tokens": self.output_tokens,
                 "num_new_tokens": self.num_new_tokens, "prompt_lengths": self.prompt_lengths, "qo_indptr_buffer": self.qo_indptr_buffer,
                 "paged_kv_indptr_buffer": self.paged_kv_indptr_buffer, "paged_kv_indices_buffer": self.paged_kv_indices_buffer,
-                "paged_kv_last_page_len_buffer": self.paged_kv_last_page_len_buffer},
+                "paged_kv_last_page_len_buffer": self.paged_kv_last_page_len_buffer,
+                **({} if meta.state_slots_buffer is None else {"state_slots_buffer": meta.state_slots_buffer})},
             profiler_tensor=self.profiler_tensor, trace_name=meta.trace_name, spec_decode_config=meta.spec_decode_config,
             use_cutlass_kernel=False, eos_token_id=next(e for e in (meta.eos_token_id, builder_cls.default_eos_token_id, -1) if e is not None),
             max_tokens_per_request=meta.max_tokens_per_request, single_weight_copy=meta.single_weight_copy)

@@ -663,6 +663,69 @@ class PersistentKernel:
                     (q_workspace, _REPL, -1), (output, _REPL, -1)],
                    [num_q_heads, num_kv_heads, head_dim, v_dim, rot_dims, int(unit_norm), _f32_bits(eps), _f32_bits(scale), _f32_bits(softcap or 0.0)])
 
+    # ------------------------------------------------------------------ mix layers (csrc/mk_mix.hip)
+    # Like the flex layers above (and usable in one graph with them): constants are arguments, one activation type per graph.
+    @staticmethod
+    def _glu_params(glu):
+        """`glu`: None, or (output rows, output column, columns, gate column, up column, limit, beta, bias) of a gated activation
+        the stage runs beside its own work: out = a / (1 + exp(-beta a)) * (b + bias), a = min(gate, limit), b = clamp(up,
+        -limit, limit)."""
+        if glu is None:
+            return None, [0] * 7
+        out, at, n, gate, up, limit, beta, bias = glu
+        return out, [at, n, gate, up, _f32_bits(limit), _f32_bits(beta), _f32_bits(bias)]
+
+    def residual_prenorm_layer(self, input: DTensor, residual: DTensor, new_residual: DTensor, output: DTensor, weight: DTensor = None, input_weight: DTensor = None,
+                               width: int = None, groups: int = 1, alpha: float = 1.0, eps: float = 1e-6, input_eps: float = 1e-6):
+        """new_residual (fp32) = v = residual + alpha * input (input None: a copy; with `input_weight`: the input is divided by
+        its root mean square and multiplied by that weight first); output = v in `groups` equal parts, each divided by its
+        own root mean square, times weight (weight None: v itself), rounded to the activation type.  A linear_layer over
+        `output` right behind forms it itself when an iteration has one token."""
+        assert residual.num_dims == 2 and new_residual.num_dims == 2 and output.num_dims == 2
+        self._task("residual_prenorm", (1, 1, 1), (256, 1, 1),
+                   [(input, _REPL, -1), (input_weight, _REPL, -1), (residual, _REPL, -1), (weight, _REPL, -1), (new_residual, _REPL, -1), (output, _REPL, -1)],
+                   [output.dim(1) if width is None else int(width), groups, _f32_bits(alpha), _f32_bits(eps), _f32_bits(input_eps)])
+
+    def latent_prep_layer(self, input: DTensor, q_weight: DTensor, output: DTensor, q_column: int, q_rank: int, eps: float, cache: DTensor = None,
+                          latent_weight: DTensor = None, cos: DTensor = None, sin: DTensor = None, latent_column: int = 0, latent_rank: int = 0, rot_column: int = 0,
+                          rot_dims: int = 0, glu: tuple = None):
+        """output = RMS norm of the query latent in columns [q_column, q_column + q_rank) of the input rows.  With a `cache`
+        ([pages, page_size, latent_row_dim(...)]): the RMS-normalised key latent and the rotated shared key part
+        (rotate-half pairs) are appended to the request's page."""
+        out, p = self._glu_params(glu)
+        self._task("latent_prep", (1, 1, 1), (256, 1, 1),
+                   [(input, _REPL, -1), (q_weight, _REPL, -1), (latent_weight, _REPL, -1), (cos, _REPL, -1), (sin, _REPL, -1), (cache, _REPL, -1), (out, _REPL, -1),
+                    (output, _REPL, -1)], [q_column, q_rank, latent_column, latent_rank, rot_column, rot_dims, _f32_bits(eps)] + p)
+
+    def head_linear_layer(self, input: DTensor, weight: DTensor, output: DTensor, heads: int, n: int, k: int, in_stride: int, out_stride: int, ids: DTensor = None,
+                          table: DTensor = None, table_column: int = 0):
+        """output[t, h * out_stride + j] = sum_i input[t, h * in_stride + i] W[h][j][i], j < n, i < k; `weight` is
+        operand_tiles(W).  With a table: gelu(tanh form) of the sum times table[ids[t], table_column + j]."""
+        self._task("head_linear", (1, 1, 1), (256, 1, 1), [(input, _REPL, -1), (weight, _REPL, -1), (ids, _REPL, -1), (table, _REPL, -1), (output, _REPL, -1)],
+                   [heads, n, k, in_stride, out_stride, table_column])
+
+    def latent_attention_layer(self, input: DTensor, q_latent: DTensor, cache: DTensor, cos: DTensor, sin: DTensor, output: DTensor, num_heads: int, latent_rank: int,
+                               rot_dims: int, head_stride: int, rot_column: int, scale: float):
+        """Causal paged attention over cached latents: every head's query is the latent q_latent[t, h] and the part of
+        input[t, h * head_stride + rot_column ...] that is rotated here; output[t, h] is the weighted sum of latents.
+        q_latent and output rows hold heads x (latent_rank rounded up to whole operand rows)."""
+        self._task("latent_attention", (1, 1, 1), (256, 1, 1),
+                   [(input, _REPL, -1), (q_latent, _REPL, -1), (cache, _REPL, -1), (cos, _REPL, -1), (sin, _REPL, -1), (output, _REPL, -1)],
+                   [num_heads, latent_rank, rot_dims, head_stride, rot_column, _f32_bits(scale)])
+
+    def general_delta_layer(self, input: DTensor, decay_weight: DTensor, decay_offset: DTensor, removal_offset: DTensor, norm_weight: DTensor, state: DTensor,
+                            state_slots: DTensor, output: DTensor, heads: int, dim: int, low_rank: int, columns: tuple, eps: float, glu: tuple = None):
+        """Generalised delta rule per head, state S [dim, dim] carried from iteration to iteration in fp32 (zero where a request
+        begins): S <- diag(w) S - (a u)(u^T S) + k v^T, o = S^T r, u = k / sqrt(sum k^2 + 1e-6), a = sigmoid(input + removal_offset),
+        w = exp(-exp(-1/2) sigmoid(W2 tanh(low-rank input) + decay_offset)); output = o / rms(o) * norm_weight * sigmoid(gate
+        input).  `columns`: where r, k, v, gate, a and the low-rank projection (low_rank wide, whole operand rows) begin in the
+        input rows.  decay_weight: operand_tiles of W2 per head.  state: [slots, heads, dim and dim rounded up to 16];
+        state_slots: int32, the state slot of every batch slot (the on-GPU schedulers permute it, a host fills it per pass)."""
+        out, p = self._glu_params(glu)
+        self._task("general_delta", (1, 1, 1), (256, 1, 1),
+                   [(input, _REPL, -1), (decay_weight, _REPL, -1), (decay_offset, _REPL, -1), (removal_offset, _REPL, -1), (norm_weight, _REPL, -1), (state, _REPL, -1),
+                    (state_slots, _REPL, -1), (out, _REPL, -1), (output, _REPL, -1)], [heads, dim, low_rank, *columns, _f32_bits(eps)] + p)
+
     # layers of the reference that are outside the one-GPU decode path
     def tensor_init_layer(self, *args, **kwargs):
         raise NotImplementedError("tensor_init_layer registers a Blackwell-only task (tasks/blackwell/tensor_init.cuh); it has no MI300-family kernel in the reference either")
@@ -992,6 +1055,28 @@ def flex_cache_dims(head_dim: int, v_dim: int, dtype: torch.dtype = torch.bfloat
     whole matrix-core operands."""
     kw = 32 if dtype == torch.bfloat16 else 16
     return -(-head_dim // kw) * kw, -(-v_dim // 16) * 16
+
+
+def operand_row(dtype: torch.dtype) -> int:
+    """Values along the reduction one matrix-core operand row holds (head_linear_layer, latent caches)."""
+    return 32 if dtype == torch.bfloat16 else 16
+
+
+def operand_tiles(w: torch.Tensor) -> torch.Tensor:
+    """[heads, n, k] matrices in the order head_linear_layer and general_delta_layer read them: per head and 16 rows, operand
+    row by operand row, 64 lanes of 16 bytes (lane l: row l % 16, a sixteenth-and-quarter of the operand row).  Rows are padded
+    with zeros to 16, k to whole operand rows.  Returns [heads * row tiles, values of a tile]."""
+    kw = operand_row(w.dtype)
+    H, n, k = w.shape
+    w = torch.nn.functional.pad(w, (0, -k % kw, 0, -n % 16))
+    n, k = w.shape[1:]
+    return w.view(H, n // 16, 16, k // kw, 4, kw // 4).permute(0, 1, 3, 4, 2, 5).reshape(H * (n // 16), 16 * k).contiguous()
+
+
+def latent_row_dim(rank: int, rot_dims: int, dtype: torch.dtype) -> int:
+    """Values per position of the cache latent_prep_layer and latent_attention_layer share."""
+    kw = operand_row(dtype)
+    return (-(-rank // kw) + -(-rot_dims // kw)) * kw
 
 
 class _DevicePtr:

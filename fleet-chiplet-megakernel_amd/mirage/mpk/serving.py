@@ -3,8 +3,8 @@
 The caller says, step by step, which requests bring which tokens; the session keeps every live request's pages, packs the
 tokens of a step into passes of at most `max_num_batched_tokens` rows (single decoded tokens beside portions of prompts,
 at most `max_tokens_per_request` rows of one request per pass), describes each pass in the meta tensors and launches the
-megakernel once for it.  What a request has in the cache is its pages and its length, so a request may pause for any
-number of steps, and a portion may end anywhere.
+megakernel once for it.  What a request has in the cache is its pages, its length and, where the model has recurrent layers,
+its state slot, so a request may pause for any number of steps, and a portion may end anywhere.
 
 `generate` is the greedy loop on top: continuous batching over a list of prompts with as many live requests as there are
 batch slots and pages.
@@ -18,10 +18,10 @@ from .mpk import MPK, MPKMetadata
 
 
 class PagePool:
-    """Free list of cache pages.  Pages given back are handed out again first."""
+    """Free list of cache pages (or state slots).  What is given back is handed out again first."""
 
-    def __init__(self, num_pages: int):
-        self.num_pages = num_pages
+    def __init__(self, num_pages: int, what: str = "cache pages"):
+        self.num_pages, self.what = num_pages, what
         self._free = list(range(num_pages - 1, -1, -1))
 
     def __len__(self):
@@ -29,7 +29,7 @@ class PagePool:
 
     def take(self, n: int) -> List[int]:
         if n > len(self._free):
-            raise RuntimeError(f"out of cache pages: {n} asked for, {len(self._free)} of {self.num_pages} free")
+            raise RuntimeError(f"out of {self.what}: {n} asked for, {len(self._free)} of {self.num_pages} free")
         return [self._free.pop() for _ in range(n)]
 
     def give(self, pages: List[int]):
@@ -40,6 +40,7 @@ class PagePool:
 class _Request:
     pages: List[int] = field(default_factory=list)
     length: int = 0  # positions whose keys and values are in the cache
+    slot: int = -1   # recurrent-state slot (models with recurrent layers)
 
 
 class ServingSession:
@@ -51,6 +52,9 @@ class ServingSession:
         self.page_size, self.max_rows, self.max_requests = pk.page_size, pk.max_num_batched_tokens, pk.max_num_batched_requests
         self.rows_per_request, self.max_seq = pk.max_tokens_per_request, pk.max_seq_length
         self.pool = PagePool(pk.max_num_pages)
+        # one state slot per batch slot: the kernel starts a request's state from zero where its position is zero
+        self.state_slots = getattr(mpk.model_builder, "state_slots", None)
+        self.slots = PagePool(self.max_requests, "state slots") if self.state_slots is not None else None
         self.requests: Dict[object, _Request] = {}
         mpk._ensure_compiled()
 
@@ -61,14 +65,14 @@ class ServingSession:
         with a cache of `max_tokens` positions."""
         pages = max(1, max_tokens // page_size)
         max_seq = max_seq_length or pages * page_size
-        # the batch description of a pass travels in one copy: the four index tensors are slices of one buffer
+        # the batch description of a pass travels in one copy: the five index tensors are slices of one buffer
         R = max_requests
-        block = torch.zeros(3 * R + 2 + pages, dtype=torch.int32, device=device)
-        qo, kv, last, idx = block.split([R + 1, R + 1, R, pages])
+        block = torch.zeros(4 * R + 2 + pages, dtype=torch.int32, device=device)
+        qo, kv, last, slots, idx = block.split([R + 1, R + 1, R, R, pages])
         meta = MPKMetadata(mode="online_notoken", max_seq_length=max(2, max_seq), max_num_batched_requests=R, max_num_batched_tokens=max_rows, max_num_pages=pages,
                            page_size=page_size, device=device, weight_from_model=model_path is not None, model_path=model_path, model_name=model_name,
                            model_config=model_config, max_tokens_per_request=min(max_rows, 64), dtype=dtype, qo_indptr_buffer=qo, paged_kv_indptr_buffer=kv,
-                           paged_kv_last_page_len_buffer=last, paged_kv_indices_buffer=idx)
+                           paged_kv_last_page_len_buffer=last, paged_kv_indices_buffer=idx, state_slots_buffer=slots)
         mpk = MPK(meta)
         mpk.build()
         session = ServingSession(mpk)
@@ -122,9 +126,12 @@ class ServingSession:
 
     def _pass(self, batch):
         ps = self.page_size
-        ids, qo, kv, last, pages = [], [0], [0], [], []
+        ids, qo, kv, last, slots, pages = [], [0], [0], [], [], []
         for rid, toks in batch:
-            r = self.requests.setdefault(rid, _Request())
+            r = self.requests.get(rid)
+            if r is None:
+                r = _Request(slot=-1 if self.slots is None else self.slots.take(1)[0])
+                self.requests[rid] = r
             r.length += len(toks)
             need = -(-r.length // ps) - len(r.pages)
             if need > 0:
@@ -138,24 +145,28 @@ class ServingSession:
             qo.append(len(ids))
             kv.append(len(pages))
             last.append(r.length - (len(r.pages) - 1) * ps)
+            slots.append(max(r.slot, 0))
         R, m = self.max_requests, self.mpk
         pad = R - len(batch)
-        desc = qo + [qo[-1]] * pad + kv + [kv[-1]] * pad + last + [0] * pad + pages
+        desc = qo + [qo[-1]] * pad + kv + [kv[-1]] * pad + last + [0] * pad + slots + [0] * pad + pages
         if getattr(self, "_block", None) is not None:
             self._block[:len(desc)].copy_(torch.tensor(desc, dtype=torch.int32))
         else:
             t = torch.tensor(desc, dtype=torch.int32)
             for dst, lo, n in ((m.qo_indptr_buffer, 0, R + 1), (m.paged_kv_indptr_buffer, R + 1, R + 1), (m.paged_kv_last_page_len_buffer, 2 * R + 2, R),
-                               (m.paged_kv_indices_buffer, 3 * R + 2, len(pages))):
-                dst[:n].copy_(t[lo:lo + n])
+                               (self.state_slots, 3 * R + 2, R), (m.paged_kv_indices_buffer, 4 * R + 2, len(pages))):
+                if dst is not None:
+                    dst[:n].copy_(t[lo:lo + n])
         m.input_tokens.view(-1)[:len(ids)].copy_(torch.tensor(ids, dtype=torch.int64))
         m()
 
     def end(self, rid):
-        """The request is finished: its pages go back to the pool."""
+        """The request is finished: its pages and its state slot go back to their pools."""
         r = self.requests.pop(rid, None)
         if r is not None:
             self.pool.give(r.pages)
+            if r.slot >= 0:
+                self.slots.give([r.slot])
 
     # ------------------------------------------------------------------ greedy generation
     def generate(self, prompts: Sequence[Sequence[int]], max_new_tokens: int, eos_token_id: int = -1) -> List[List[int]]:
