@@ -212,8 +212,10 @@ def run_leg(torch, dec, shape, model, B, K, W, P, max_seq, mode, stage_profile=F
     }
 
 
-# ---- Suborax beside the closest model at equal size (bench.py --compare suborax) --------------------------------------
-# Both models with the same width, heads, head size, feed-forward, depth and vocabulary; random weights.
+# ---- a model beside the closest one at equal size (bench.py --compare suborax | dodonex) ------------------------------
+# Both models with the same width, heads, head size, feed-forward, depth and vocabulary; random weights.  (Dodonex: what the
+# closest model has no counterpart for -- latent sizes, recurrence, per-token vectors -- comes from generate.py's shapes.)
+CLOSEST = {"suborax": "qwen3", "dodonex": "suborax"}
 COMPARE_SHAPES = {"8b": dict(width=4096, heads=32, kv_heads=8, ff=12288), "2k": dict(width=2048, heads=32, kv_heads=4, ff=6144)}
 
 
@@ -234,27 +236,24 @@ def stage_times(dec):
         op = desc[1]
         n = next((d for d in desc if d.startswith("n=")), "")
         k = next((d for d in desc if d.startswith("k=")), "")
-        kinds.setdefault(" ".join(x for x in (op.replace("[multi-token", "").replace("[portions]", ""), n, k) if x), []).append((end - prev) * 0.01)
+        kinds.setdefault(" ".join(x for x in (op.replace("[multi-token", "").replace("[portions]", "").replace("[split", ""), n, k) if x), []).append((end - prev) * 0.01)
         prev = end
     return {k: [round(sum(v) / len(v), 1), len(v)] for k, v in kinds.items()}
 
 
 def compare_decoder(torch, which, shape, layers, vocab, B, R, max_seq, page_size=4096):
-    """A decoder of either model with B token rows per iteration and R batch slots."""
+    """A decoder of a model with B token rows per iteration and R batch slots."""
     per_req = min(B, 64)
     if which == "qwen3":
         from demo_qwen3 import Qwen3Decoder, Qwen3Shape, random_weights
         s = Qwen3Shape(hidden_size=shape["width"], num_q_heads=shape["heads"], num_kv_heads=shape["kv_heads"], intermediate_size=shape["ff"], num_layers=layers, vocab_size=vocab)
         return Qwen3Decoder(s, random_weights(s), max_num_batched_tokens=B, max_num_batched_requests=R, max_seq_length=max_seq, page_size=page_size,
                             max_tokens_per_request=per_req), s.weight_bytes_per_token(), s.kv_bytes_per_position()
-    from generate import Generator, suborax_shape
-    from mirage.mpk import MirageModelConfig
-    from mirage.mpk.models.suborax.builder import SuboraxConfig, random_state_dict
-    c = suborax_shape(layers=layers, vocab=vocab, **shape)
-    sc = SuboraxConfig.from_dict(c)
-    g = Generator(max_seq, model_config=MirageModelConfig(architecture=c, state_dict=random_state_dict(sc)), batch=R, max_num_batched_tokens=B,
-                  max_tokens_per_request=per_req, page_size=page_size, eos_token_id=-1)
-    return g, sc.weight_bytes_per_token(), sc.kv_bytes_per_position()
+    from generate import SHAPES, Generator, random_model
+    make, sizes = SHAPES[f"{which}-{'8b' if shape['width'] == 4096 else '2k'}"]
+    mc, sc = random_model(make(layers=layers, vocab=vocab, **sizes))
+    g = Generator(max_seq, model_config=mc, batch=R, max_num_batched_tokens=B, max_tokens_per_request=per_req, page_size=page_size, eos_token_id=-1)
+    return g, sc.weight_bytes_per_token() + (2 * R * sc.state_bytes() if which == "dodonex" else 0), sc.kv_bytes_per_position()
 
 
 def compare_leg(torch, which, shape, layers, vocab, B, R, prompt, steps, stages):
@@ -302,13 +301,13 @@ def compare_main(torch, args):
     for name, shape in COMPARE_SHAPES.items():
         # (rows per iteration, batch slots, prompt): single-token kernel short and long, long prompt in portions, batches
         for B, R, prompt in ((1, 1, 80), (1, 1, 4096), (64, 1, 4096), (8, 8, 80), (64, 64, 80)):
-            for which in ("qwen3", "suborax"):
+            for which in (CLOSEST[args.compare], args.compare):
                 leg = dict(shape=name, **compare_leg(torch, which, shape, layers, vocab, B, R, prompt, 64, args.stage_profile))
                 print(json.dumps(leg), file=sys.stderr, flush=True)
                 legs.append(leg)
                 torch.cuda.empty_cache()
     worst = max(b["decode_ms_per_step"] / a["decode_ms_per_step"] for a, b in zip(legs[::2], legs[1::2]))
-    print(json.dumps({"metric": "Suborax decode time relative to a Qwen3 stack of equal size (worst leg)", "value": round(worst, 3), "unit": "x", "n_gpus": 1,
+    print(json.dumps({"metric": f"{args.compare} decode time relative to a {CLOSEST[args.compare]} stack of equal size (worst leg)", "value": round(worst, 3), "unit": "x", "n_gpus": 1,
                       "higher_is_better": False, "dtype": "bf16", "data": "synthetic (random-init weights, seeded random prompts)",
                       "config": {"layers": layers, "vocab": vocab, "shapes": COMPARE_SHAPES}, "legs": legs}), flush=True)
 
@@ -329,7 +328,7 @@ def main():
     ap.add_argument("--single-weight-copy", action="store_true",
                     help="keep every linear weight once, in matrix-core tile order (BS >= 2): what the memory saving costs iterations of one or two tokens")
     ap.add_argument("--calib-copy", action="store_true", help="also run one 1 GiB device-to-device copy (scale for rocprofv3 FETCH_SIZE / WRITE_SIZE)")
-    ap.add_argument("--compare", choices=["suborax"], default=None,
+    ap.add_argument("--compare", choices=sorted(CLOSEST), default=None,
                     help="instead of the headline workload: prefill and decode of this model beside the closest one at equal size (8 layers)")
     ap.add_argument("--stage-profile", action="store_true",
                     help="after each timed launch, print its last iteration's per-stage timeline over all workgroups to stderr")

@@ -876,7 +876,19 @@ int lower_residual_prenorm(mk_graph *g, size_t &i) {
   st.out2 = xo.ptr;
   st.ld_out2 = (int)xo.strides[0];
   if (!g->stages.empty()) {
-    const MkStage &pl = g->stages.back();
+    MkStage &pl = g->stages.back();
+    if (!w && !yw && y && st.out && pl.op == MK_OP_LINEAR && !(pl.flags & (MK_F_SILU | MK_F_RES)) && pl.out == st.in && (pl.k & 63) == 0) {
+      // a plain linear in front adds its single-token result to the stream itself
+      pl.flags |= MK_F_JOIN;
+      pl.res = st.res;
+      pl.ld_res = st.ld_res;
+      pl.out2 = st.out2;
+      pl.ld_out2 = st.ld_out2;
+      pl.norm_out = st.out;
+      pl.ld_norm = st.ld_out;
+      pl.alpha = st.alpha;
+      st.flags |= MK_F_ONLY_MULTI;
+    }
     if (pl.out != st.res && pl.out2 != st.res && pl.norm_out != st.res) st.flags |= MK_F_RES_EARLY;
   }
   bool res, silu;
@@ -884,7 +896,7 @@ int lower_residual_prenorm(mk_graph *g, size_t &i) {
   const bool fuse = g->flex == FLEX_BF16 && w && i + 1 < g->ltasks.size() && linear_kind(g->ltasks[i + 1].name, &res, &silu, &extra) && !res && g->ltasks[i + 1].ops[0] == t.ops[5];
   if (fuse) st.flags |= MK_F_ONLY_MULTI;
   g->stages.push_back(st);
-  g->stage_desc.push_back(fmt("MX_PRENORM%s %s + %g * %s%s -> %s, %s k=%d parts=%d", fuse ? "[multi-token only]" : "", x.name.c_str(), st.alpha, yw ? "norm of " : "", y ? y->name.c_str() : "0", xo.name.c_str(),
+  g->stage_desc.push_back(fmt("MX_PRENORM%s %s + %g * %s%s -> %s, %s k=%d parts=%d", (st.flags & MK_F_ONLY_MULTI) ? "[multi-token only]" : "", x.name.c_str(), st.alpha, yw ? "norm of " : "", y ? y->name.c_str() : "0", xo.name.c_str(),
                               o.name.c_str(), width, st.norm_groups));
   i++;
   if (!fuse) return MK_OK;
@@ -1079,16 +1091,15 @@ int lower_latent_attention(mk_graph *g, size_t &i) {
   st.rot_dims = rot;
   st.sm_scale = bits_f32(t.params[5]);
   if ((rc = lower_rotary_tables(g, t, 3, rot, &st))) return rc;
-  // a tile is 16 SUB positions of one page; the kernel's register copy of it holds 20 (short latents: 6) operand rows per wavefront
-  const bool small_ = !f32 && R <= 128 && rot <= 64;
-  const int kcap = small_ ? 6 : 20;
-  st.v_tiles = f32 ? 1 : 2;  // 16-row query tiles per unit
+  // instantiation (mk_mix.hip: stage_mx_latent_attn): operand rows of a cached latent, 16-position sub-tiles of a tile, 16-row
+  // query tiles of a unit
+  st.nk = f32 ? (R <= 128 && d.nkc <= 12 ? 12 : 40) : (R <= 128 && d.nkc <= 6 ? 6 : d.nkc <= 18 ? 18 : 20);
+  st.k_tiles = f32 ? 2 : 4;
+  st.v_tiles = f32 ? 1 : 2;
+  if (d.nkc > st.nk) return fail(MK_EUNSUPPORTED, "latent_attention: latent of %d and rotated part of %d values (%d operand rows, at most %d)", R, rot, d.nkc, st.nk);
+  if (ps % (16 * st.k_tiles)) return fail(MK_EINVAL, "latent_attention: page_size %d must be a multiple of %d", ps, 16 * st.k_tiles);
   const int pages = (g->cfg.max_seq_length + ps - 1) / ps;
-  int sub = 4;
-  auto fits = [&](int s) { return ps % (16 * s) == 0 && d.nkc <= kcap * (MK_WAVES / s) && mk_latent_lds(f32 ? 4 : 2, st.v_tiles, d.nkc, s, pages).bytes <= MK_LDS_BYTES; };
-  while (sub > (f32 ? 1 : 2) && !fits(sub)) sub /= 2;
-  if (!fits(sub)) return fail(MK_EUNSUPPORTED, "latent_attention: page_size %d (a multiple of %d is needed), latent %d + %d or %d pages per request do not fit", ps, f32 ? 16 : 32, R, rot, pages);
-  st.k_tiles = sub;
+  if (mk_latent_lds(f32 ? 4 : 2, st.v_tiles, st.nk, st.k_tiles, pages).bytes > MK_LDS_BYTES) return fail(MK_EUNSUPPORTED, "latent_attention: %d pages per request need too much LDS", pages);
   g->flex_part = std::max(g->flex_part, (size_t)g->G * 16 * st.v_tiles * (d.rp + 32));
   g->stages.push_back(st);
   g->stage_desc.push_back(fmt("MX_LATENT_ATTN %s, %s -> %s heads=%d latent=%d rot=%d scale=%g", q.name.c_str(), ql.name.c_str(), o.name.c_str(), H, R, rot, st.sm_scale));
@@ -1100,54 +1111,73 @@ int lower_latent_attention(mk_graph *g, size_t &i) {
 }
 
 // general_delta [rows, decay weights, decay offset (fp32), removal offset (fp32), norm (fp32), state (fp32), state slots (int32),
-// activation (optional), output] params [heads, dim, low rank (whole operand rows), columns of r k v g a and the low-rank
-// projection, eps bits, then the gated activation's seven]
+// workspace (fp32), activation (optional), output] params [heads, dim, low rank (whole operand rows), columns of r k v g a and the
+// low-rank projection, eps bits, then the gated activation's seven].  A head's columns, offsets, norm and output are dim rounded
+// up to 16 wide; the workspace rows hold twice that for all heads.
 int lower_general_delta(mk_graph *g, size_t &i) {
   const Task &t = g->ltasks[i];
-  if (t.ops.size() != 9 || t.params.size() != 17) return fail(MK_EINVAL, "general_delta expects 9 operands / 17 params");
-  const Tensor &in = g->tensors[t.ops[0]], &w2 = g->tensors[t.ops[1]], &state = g->tensors[t.ops[5]], &ids = g->tensors[t.ops[6]], &o = g->tensors[t.ops[8]];
+  if (t.ops.size() != 10 || t.params.size() != 17) return fail(MK_EINVAL, "general_delta expects 10 operands / 17 params");
+  const Tensor &in = g->tensors[t.ops[0]], &w2 = g->tensors[t.ops[1]], &state = g->tensors[t.ops[5]], &ids = g->tensors[t.ops[6]], &ws = g->tensors[t.ops[7]], &o = g->tensors[t.ops[9]];
   const int B = g->cfg.max_num_batched_tokens, slots = g->cfg.max_num_batched_requests, H = t.params[0], D = t.params[1], rank = t.params[2];
   int rc = set_mix(g, in.dtype, "general_delta");
   if (rc) return rc;
   const int es = in.dtype == MK_DT_F32 ? 4 : 2, kw = 64 / es;
   if (H < 1 || D < 1 || D > MK_MX_MAX_DELTA_DIM || rank < kw || rank % kw || rank > MK_MX_MAX_RANK)
     return fail(MK_EUNSUPPORTED, "general_delta: %d heads of %d (at most %d), low rank %d (whole operand rows of %d, at most %d)", H, D, MK_MX_MAX_DELTA_DIM, rank, kw, MK_MX_MAX_RANK);
-  const int nd = (D + 15) / 16, dp = D <= 64 ? 64 : D <= 128 ? 128 : 256;
-  if (!rows_ok(in, B, 1, in.dtype) || !rows_ok(o, B, (int64_t)H * D, in.dtype)) return fail(MK_EINVAL, "general_delta: bad row tensors");
+  const int dp = (D + 15) / 16 * 16, cols = H * dp;
+  if (!rows_ok(in, B, 1, in.dtype) || (in.strides[0] * es) % 16 || !rows_ok(o, B, cols, in.dtype) || !rows_ok(ws, B, 2 * (int64_t)cols, MK_DT_F32)) return fail(MK_EINVAL, "general_delta: bad row tensors");
   for (int a = 0; a < 6; a++) {
-    const int col = t.params[3 + a], n = a == 5 ? rank : H * D;
-    if (col < 0 || col + n > in.dims[1] || (a == 5 && col % 4)) return fail(MK_EINVAL, "general_delta: columns %d .. %d lie outside the rows", col, col + n);
+    const int col = t.params[3 + a], n = a == 5 ? rank : cols;
+    if (col < 0 || col % (16 / es) || col + n > in.dims[1]) return fail(MK_EINVAL, "general_delta: columns %d .. %d lie outside the rows or begin inside a 16-byte word", col, col + n);
   }
-  if (w2.dtype != in.dtype || (int64_t)w2.elems() != (int64_t)H * nd * 16 * rank || !vector_ok(g->tensors[t.ops[2]], (int64_t)H * D) || !vector_ok(g->tensors[t.ops[3]], (int64_t)H * D) ||
-      !vector_ok(g->tensors[t.ops[4]], (int64_t)H * D))
-    return fail(MK_EINVAL, "general_delta: decay weights are %d x %d per head in operand order, the three vectors fp32 of %d", nd * 16, rank, H * D);
-  if (state.dtype != MK_DT_F32 || state.ndims != 4 || state.dims[0] < slots || state.dims[1] != H || state.dims[2] != nd * 16 || state.dims[3] != nd * 16)
-    return fail(MK_EINVAL, "general_delta: the state is fp32 [>= %d slots, %d, %d, %d]", slots, H, nd * 16, nd * 16);
+  if (w2.dtype != in.dtype || (int64_t)w2.elems() != (int64_t)cols * rank || !vector_ok(g->tensors[t.ops[2]], cols) || !vector_ok(g->tensors[t.ops[3]], cols) || !vector_ok(g->tensors[t.ops[4]], cols))
+    return fail(MK_EINVAL, "general_delta: decay weights are %d x %d in operand order, the three vectors fp32 of %d", cols, rank, cols);
+  if (state.dtype != MK_DT_F32 || state.ndims != 4 || state.dims[0] < slots || state.dims[1] != H || state.dims[2] != dp || state.dims[3] != dp)
+    return fail(MK_EINVAL, "general_delta: the state is fp32 [>= %d slots, %d, %d, %d]", slots, H, dp, dp);
   if (ids.dtype != MK_DT_I32 || (int)ids.elems() < slots) return fail(MK_EINVAL, "general_delta: one int32 state slot per batch slot");
   if (g->state_ids && g->state_ids != (int *)ids.ptr) return fail(MK_EINVAL, "general_delta: every recurrence of a graph uses the same state-slot tensor");
   g->state_ids = (int *)ids.ptr;
-  if ((int64_t)6 * 16 * (dp + 4) * 4 + (int64_t)rank / kw * 2048 > MK_LDS_BYTES) return fail(MK_EUNSUPPORTED, "general_delta: head size %d with low rank %d needs too much LDS", D, rank);
+  MkStage sd;  // decays
+  memset(&sd, 0, sizeof(sd));
+  sd.op = MK_OP_MX_DECAY;
+  sd.groups = 1;
+  sd.n = cols;
+  sd.k = rank;
+  sd.in = (const char *)in.ptr + (size_t)t.params[8] * es;
+  sd.ld_in = (int)in.strides[0];
+  sd.w.nseg = 1;
+  sd.w.seg[0] = w2.ptr;
+  sd.q_norm_w = g->tensors[t.ops[2]].ptr;
+  sd.out2 = ws.ptr;
+  sd.ld_out2 = (int)ws.strides[0];
+  if ((rc = lower_glu(g, t, 8, 10, in, &sd))) return rc;
+  sd.glu_gate -= t.params[8];  // (columns from the low-rank projection on)
+  sd.glu_up -= t.params[8];
+  g->stages.push_back(sd);
+  g->stage_desc.push_back(fmt("MX_DECAY %s x %s n=%d k=%d glu=%d", in.name.c_str(), w2.name.c_str(), cols, rank, sd.glu_n));
   MkStage st;
   memset(&st, 0, sizeof(st));
   st.op = MK_OP_MX_DELTA;
   st.in = in.ptr;
   st.ld_in = (int)in.strides[0];
+  st.in2 = ws.ptr;
+  st.ld_in2 = (int)ws.strides[0];
+  st.out2 = (float *)ws.ptr + cols;
+  st.ld_out2 = (int)ws.strides[0];
   st.out = o.ptr;
   st.ld_out = (int)o.strides[0];
   st.num_q_heads = H;
   st.head_dim = D;
-  st.rank = rank;
-  for (int a = 0; a < 6; a++) st.cols[a] = t.params[3 + a];
+  for (int a = 0; a < 5; a++) st.cols[a] = t.params[3 + a];
   st.eps = bits_f32(t.params[9]);
-  st.w.nseg = 1;
-  st.w.seg[0] = w2.ptr;
-  st.q_norm_w = g->tensors[t.ops[2]].ptr;
   st.k_norm_w = g->tensors[t.ops[3]].ptr;
   st.norm_w = g->tensors[t.ops[4]].ptr;
   st.k_cache = state.ptr;
-  if ((rc = lower_glu(g, t, 7, 10, in, &st))) return rc;
   g->stages.push_back(st);
-  g->stage_desc.push_back(fmt("MX_DELTA %s -> %s heads=%d d=%d rank=%d glu=%d", in.name.c_str(), o.name.c_str(), H, D, rank, st.glu_n));
+  g->stage_desc.push_back(fmt("MX_DELTA %s -> %s heads=%d d=%d", in.name.c_str(), o.name.c_str(), H, D));
+  st.op = MK_OP_MX_DELTA_OUT;
+  g->stages.push_back(st);
+  g->stage_desc.push_back(fmt("MX_DELTA_OUT[sliced] -> %s", o.name.c_str()));
   g->weight_bytes += (int64_t)w2.elems() * es;
   i++;
   return MK_OK;
@@ -1697,7 +1727,9 @@ int lower(mk_graph *g) {
       case MK_OP_MX_LATENT_PREP:
       case MK_OP_MX_LATENT_ATTN:
       case MK_OP_MX_LATENT_MERGE:
-      case MK_OP_MX_DELTA: st.prof_event = 116; break;
+      case MK_OP_MX_DECAY:
+      case MK_OP_MX_DELTA:
+      case MK_OP_MX_DELTA_OUT: st.prof_event = 116; break;
       case MK_OP_FX_ARGMAX_F32: st.prof_event = 110; break;
       case MK_OP_NGRAM_PARTIAL: st.prof_event = 112; break;
       case MK_OP_NGRAM_GLOBAL: st.prof_event = 113; break;
@@ -2372,7 +2404,7 @@ int mk_add_task(mk_graph *g, const char *task_name, const int grid_dim[3], const
                            t.name == "paged_attention_split_kv_mi300" || t.name == "attention" || t.name == "single_batch_extend_attention") && i >= 3 && i <= 6) ||
                           (t.name == "flex_attention" && i >= 3 && i <= 5) || (t.name == "residual_rmsnorm" && i == 0) ||
                           (t.name == "residual_prenorm" && (i == 0 || i == 1 || i == 3)) || (t.name == "latent_prep" && i >= 2 && i <= 6) ||
-                          (t.name == "head_linear" && (i == 2 || i == 3)) || (t.name == "latent_attention" && (i == 3 || i == 4)) || (t.name == "general_delta" && i == 7);
+                          (t.name == "head_linear" && (i == 2 || i == 3)) || (t.name == "latent_attention" && (i == 3 || i == 4)) || (t.name == "general_delta" && i == 8);
     if (tensor_ids[i] >= (int)g->tensors.size() || tensor_ids[i] < (optional ? -1 : 0))
       return fail(MK_EINVAL, "task '%s': bad tensor id %d for operand %d", task_name, tensor_ids[i], i);
     t.ops.push_back(tensor_ids[i]);

@@ -113,7 +113,7 @@ struct Ctx {
   const void *defer_res;  // residual rows of that linear (null: none)
   int defer_ld_res;
 #if MK_HAVE_MIX
-  bool mx_split;  // the latent attention that just ran left some request in chunks
+  bool mx_split;  // the latent attention (delta rule) that just ran left some request in chunks (its heads in slices)
 #endif
 #ifdef MK_TRACE
   long long mark[4];  // (tracing builds) wall-clock marks the running stage sets, stored next to its stage timing
@@ -909,6 +909,8 @@ __device__ __forceinline__ float silu_mul(float g, float u) { return g / (1.f + 
 #if MK_HAVE_MIX  // a residual_prenorm in front of a single-token linear (mk_mix.hip): by the workgroup, by the control wavefront
 __device__ __forceinline__ void mx_x_m1_prenorm(CStage &st, const Ctx &c, uint32_t *xs, float *red);
 template <int KL> __device__ __forceinline__ void mx_x_m1_prenorm_wave(CStage &st, Ctx &c, uint32_t *xs, int lane);
+__device__ __forceinline__ bool mx_linear_m1_form(CStage &st);
+__device__ __forceinline__ void stage_mx_linear_m1(CStage &st, Ctx &c, char *smem);
 // the control wavefront wants whole 16-byte segments in one part of the norm, and few parts
 __device__ __forceinline__ bool mx_prenorm_by_wave(CStage &st) { return st.k <= 4096 && st.norm_groups <= 8 && (st.k_real / st.norm_groups & 7) == 0; }
 #endif
@@ -1320,6 +1322,12 @@ __device__ __forceinline__ void stage_linear_m1(CStage &st, Ctx &c, char *smem) 
   const bool silu = st.flags & MK_F_SILU;
   // the tuned forms collect a workgroup's outputs in the LDS window [MK_OUT_OFFSET, MK_MOE_OFFSET)
   const bool fits = ((silu ? st.n / 2 : st.n) / c.G + 1) * 2 <= MK_MOE_OFFSET - MK_OUT_OFFSET;
+#if MK_HAVE_MIX
+  if (FX && mx_linear_m1_form(st)) {
+    stage_mx_linear_m1(st, c, smem);
+    return;
+  }
+#endif
   if (!fits || (FX && (st.flags & MK_F_ADDNORM) && st.k > 4096)) {
     stage_linear_m1_generic<FX>(st, c, smem);
 #if MK_HAVE_MIX
@@ -4152,7 +4160,7 @@ __device__ __forceinline__ void run_stage_program(const MkRuntime &rt, const MkR
       if ((flags & MK_F_ONLY_MULTI) && M == 1 && !(packed_only && (op == MK_OP_NORM || (FX && (op == MK_OP_FX_ADDNORM || op == MK_OP_MX_PRENORM))))) continue;
       if (FX && op == MK_OP_FX_PREP && single) continue;
 #if MK_HAVE_MIX
-      if (op == MK_OP_MX_LATENT_MERGE && !c.mx_split) continue;
+      if ((op == MK_OP_MX_LATENT_MERGE || op == MK_OP_MX_DELTA_OUT) && !c.mx_split) continue;
 #endif
       if ((flags & MK_F_ONLY_MULTI) && op == MK_OP_NORM && s + 1 < rt.num_stages && !packed_only) {
         // the few-token linear normalises its rows itself
@@ -4181,7 +4189,9 @@ __device__ __forceinline__ void run_stage_program(const MkRuntime &rt, const MkR
         case MK_OP_MX_HEAD_LINEAR: stage_mx_head_linear<E, MAXM>(st, c, M, smem); break;
         case MK_OP_MX_LATENT_ATTN: stage_mx_latent_attn<E>(st, c, rt, M, smem); break;
         case MK_OP_MX_LATENT_MERGE: stage_mx_latent_merge<E>(st, c, rt, M); break;
-        case MK_OP_MX_DELTA: stage_mx_delta<E>(st, c, rt, M, smem); break;
+        case MK_OP_MX_DECAY: stage_mx_decay<E, MAXM>(st, c, M, smem); break;
+        case MK_OP_MX_DELTA: stage_mx_delta<E>(st, c, rt, M, MAXM == 1 || single, smem); break;
+        case MK_OP_MX_DELTA_OUT: stage_mx_delta_out<E>(st, c, M); break;
 #endif
         case MK_OP_EMBED: if constexpr (!FX) stage_embed(st, c, rt, M); break;
         case MK_OP_NORM: if constexpr (!FX) stage_norm(st, c, M, smem); break;

@@ -28,13 +28,11 @@ __device__ __forceinline__ void stage_mx_prenorm_t(CStage &st, Ctx &c, int M, ch
   auto at = [&](int j) { return min(tid + j * MK_THREADS, n4 - 1); };
   auto load_x = [&](int t) {
 #pragma unroll
-    for (int j = 0; j < NS; j++)
-      if (j * MK_THREADS < n4) x[j] = fx_ldc_quad(xr + (size_t)t * st.ld_res + 4 * at(j));
+    for (int j = 0; j < NS; j++) x[j] = fx_ldc_quad(xr + (size_t)t * st.ld_res + 4 * at(j));
   };
   if (ng) {
 #pragma unroll
-    for (int j = 0; j < NS; j++)
-      if (j * MK_THREADS < n4) g[j] = w4[at(j)];
+    for (int j = 0; j < NS; j++) g[j] = w4[at(j)];
   }
   // the residual row was written at least one barrier earlier than y: requested before the barrier is awaited (not by the
   // wavefront that polls it)
@@ -46,8 +44,7 @@ __device__ __forceinline__ void stage_mx_prenorm_t(CStage &st, Ctx &c, int M, ch
     if (st.in) {
       f32x4 y[NS];
 #pragma unroll
-      for (int j = 0; j < NS; j++)
-        if (j * MK_THREADS < n4) y[j] = fx_ldc_quad((const E *)st.in + (size_t)t * st.ld_in + 4 * at(j));
+      for (int j = 0; j < NS; j++) y[j] = fx_ldc_quad((const E *)st.in + (size_t)t * st.ld_in + 4 * at(j));
       float f = st.alpha;
       if (yw4) {
         float ss = 0.f;
@@ -57,15 +54,12 @@ __device__ __forceinline__ void stage_mx_prenorm_t(CStage &st, Ctx &c, int M, ch
         ss = block_sum(ss, red);
         const float r = 1.f / sqrtf(ss / (float)st.k + st.norm_eps);
 #pragma unroll
-        for (int j = 0; j < NS; j++)
-          if (j * MK_THREADS < n4) y[j] = (y[j] * r) * yw4[at(j)];
+        for (int j = 0; j < NS; j++) y[j] = (y[j] * r) * yw4[at(j)];
       }
 #pragma unroll
       for (int j = 0; j < NS; j++)
-        if (j * MK_THREADS < n4) {
 #pragma unroll
-          for (int e = 0; e < 4; e++) x[j][e] = fmaf(f, y[j][e], x[j][e]);
-        }
+        for (int e = 0; e < 4; e++) x[j][e] = fmaf(f, y[j][e], x[j][e]);
     }
     if (ng > 1) {
 #pragma unroll
@@ -235,6 +229,86 @@ __device__ __forceinline__ void mx_x_m1_prenorm_wave(CStage &st, Ctx &c, uint32_
   }
 }
 
+// ----------------------------------------------------------------------------- single-token linear, any reduction length
+// out[n] = sum_k W[n, k] x[k], k a multiple of 64.  A wavefront owns a run of rows and takes R of them at a time, 512 U values of
+// k per step, two steps' loads in flight; the first step's are requested before the previous stage's barrier is awaited (not by
+// the wavefront that polls it).  MK_F_JOIN: the sum joins the residual stream, out2 = res + alpha * sum (32-bit), norm_out = the
+// same rounded, and st.out is not written.
+template <int R, int U>
+__device__ __forceinline__ void stage_mx_linear_m1_t(CStage &st, Ctx &c, char *smem) {
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int K = st.k, k8 = K / 8, nkb = (k8 + 64 * U - 1) / (64 * U), n = st.n;
+  u32x4 *xs4 = (u32x4 *)smem;
+  const int nw = c.G * MK_WAVES, id = c.vid * MK_WAVES + wave, q = n / nw, rem = n - q * nw;
+  const int r0 = id * q + min(id, rem), r1 = r0 + q + (id < rem ? 1 : 0);
+  const int steps = ((r1 - r0 + R - 1) / R) * nkb;
+  u32x4 A[R][U], B[R][U];
+  auto load = [&](int step, u32x4 (&b)[R][U]) {
+    const int rb = step / nkb, kb = step - rb * nkb;
+#pragma unroll
+    for (int r = 0; r < R; r++) {
+      const u32x4 *w = weight_row(st.w, min(r0 + rb * R + r, n - 1), k8);
+#pragma unroll
+      for (int u = 0; u < U; u++) b[r][u] = ldg_stream(w + min((kb * U + u) * 64 + lane, k8 - 1));
+    }
+  };
+  if (wave != 0) load(0, A);
+  barrier_wait(c);
+  for (int i = k8 + tid; i < nkb * U * 64; i += MK_THREADS) xs4[i] = (u32x4){0u, 0u, 0u, 0u};  // (nothing multiplies the repeated loads)
+  stage_x_m1<true>(st, c, (uint32_t *)smem, (float *)(smem + MK_RED_OFFSET));
+  if (wave == 0) load(0, A);
+  const bool join = st.flags & MK_F_JOIN;
+  float acc[R];
+#pragma unroll
+  for (int r = 0; r < R; r++) acc[r] = 0.f;
+  auto consume = [&](int step, const u32x4 (&b)[R][U]) {
+    const int rb = step / nkb, kb = step - rb * nkb;
+#pragma unroll
+    for (int u = 0; u < U; u++) {
+      const u32x4 x = xs4[(kb * U + u) * 64 + lane];
+#pragma unroll
+      for (int r = 0; r < R; r++) acc[r] = dot8(b[r][u], x, acc[r]);
+    }
+    if (kb + 1 < nkb) return;
+    const int row = r0 + rb * R + lane;
+    const bool mine = lane < R && row < r1;
+    const float x = join && mine ? ldc_f32((const float *)st.res + row) : 0.f;
+    float v = 0.f;
+#pragma unroll
+    for (int r = 0; r < R; r++) {
+      const float s = wave_sum(acc[r]);
+      v = lane == r ? s : v;
+      acc[r] = 0.f;
+    }
+    if (mine) {
+      if (join) {
+        v = fmaf(st.alpha, v, x);
+        stc_f32((float *)st.out2 + row, v);
+        stc_u16((uint16_t *)st.norm_out + row, (uint16_t)f2bf(v));
+      } else {
+        stc_u16((uint16_t *)st.out + row, (uint16_t)f2bf(v));
+      }
+    }
+  };
+  for (int s = 0; s < steps; s += 2) {
+    load(min(s + 1, steps - 1), B);
+    consume(s, A);
+    if (s + 1 >= steps) break;
+    load(min(s + 2, steps - 1), A);
+    consume(s + 1, B);
+  }
+  c.wrote_through = true;
+}
+// (which single-token linears: those that join the stream, and those no tuned instantiation exists for)
+__device__ __forceinline__ bool mx_linear_m1_form(CStage &st) {
+  return !(st.flags & (MK_F_SILU | MK_F_RES)) && (st.k & 63) == 0 && ((st.flags & MK_F_JOIN) || (st.k != 4096 && st.k != 2048 && st.k != 1024 && st.k != 12288));
+}
+__device__ __forceinline__ void stage_mx_linear_m1(CStage &st, Ctx &c, char *smem) {
+  if (st.k <= 512) stage_mx_linear_m1_t<4, 1>(st, c, smem);
+  else if (st.k <= 1536) stage_mx_linear_m1_t<4, 3>(st, c, smem);
+  else stage_mx_linear_m1_t<4, 4>(st, c, smem);
+}
+
 // ----------------------------------------------------------------------------- gated activation
 // Elements of the rows, 1024 per item, dealt from the last workgroup downwards (the stage's own units start at the first).
 template <typename E>
@@ -258,26 +332,32 @@ __device__ __forceinline__ void mx_glu(CStage &st, Ctx &c, int M) {
 }
 
 // ----------------------------------------------------------------------------- latent rows
-// One wavefront: row of n values (n4 quads are readable, those behind n are zero) / rms * w; put(quad index, values).
-template <typename E, typename Put>
-__device__ __forceinline__ void mx_norm_row(const E *src, const float *w, int n, float eps, int lane, Put put) {
-  constexpr int NQ = MK_MX_MAX_NORM_ROW / 256;
+// One wavefront: row of n values (n4 quads are readable, those behind n are zero) / rms * w; put(quad index, values).  NQ: quads
+// per lane, 256 NQ >= n; every load is unconditional (indices are clamped), so all of them are in flight together.
+template <typename E, int NQ, typename Put>
+__device__ __forceinline__ void mx_norm_row_t(const E *src, const float *w, int n, float eps, int lane, Put put) {
   const int n4 = (n + 3) / 4;
-  f32x4 v[NQ];
+  f32x4 v[NQ], g[NQ];
 #pragma unroll
-  for (int j = 0; j < NQ; j++)
-    if (j * 64 < n4) v[j] = fx_ldc_quad(src + 4 * min(j * 64 + lane, n4 - 1));
+  for (int j = 0; j < NQ; j++) v[j] = fx_ldc_quad(src + 4 * min(j * 64 + lane, n4 - 1));
+#pragma unroll
+  for (int j = 0; j < NQ; j++) g[j] = ((const f32x4 *)w)[min(j * 64 + lane, n4 - 1)];
   float ss = 0.f;
 #pragma unroll
-  for (int j = 0; j < NQ; j++)
-    if (j * 64 + lane < n4) ss += v[j][0] * v[j][0] + v[j][1] * v[j][1] + v[j][2] * v[j][2] + v[j][3] * v[j][3];
+  for (int j = 0; j < NQ; j++) {
+    const float q = v[j][0] * v[j][0] + v[j][1] * v[j][1] + v[j][2] * v[j][2] + v[j][3] * v[j][3];
+    ss += j * 64 + lane < n4 ? q : 0.f;
+  }
   const float r = 1.f / sqrtf(wave_sum(ss) / (float)n + eps);
 #pragma unroll
   for (int j = 0; j < NQ; j++)
-    if (j * 64 + lane < n4) {
-      const f32x4 g = ((const f32x4 *)w)[j * 64 + lane];
-      put(j * 64 + lane, (v[j] * r) * g);
-    }
+    if (j * 64 + lane < n4) put(j * 64 + lane, (v[j] * r) * g[j]);
+}
+template <typename E, typename Put>
+__device__ __forceinline__ void mx_norm_row(const E *src, const float *w, int n, float eps, int lane, Put put) {
+  if (n <= 512) mx_norm_row_t<E, 2>(src, w, n, eps, lane, put);
+  else if (n <= 2048) mx_norm_row_t<E, 8>(src, w, n, eps, lane, put);
+  else mx_norm_row_t<E, MK_MX_MAX_NORM_ROW / 256>(src, w, n, eps, lane, put);
 }
 // A cached latent: the normalised latent, padded with zeros to whole operand rows, then the rotated key part, padded likewise.
 // Inside a page: [position / 16][operand row][64 lanes][EPC], lane l holds position l % 16, dims (l / 16) * EPC .. of the row.
@@ -323,92 +403,129 @@ __device__ __forceinline__ void stage_mx_latent_prep(CStage &st, Ctx &c, const M
 
 // ----------------------------------------------------------------------------- a matrix per head
 // out[t, h * ld_out_slot + n] = sum_k in[t, h * ld_in_slot + k] W[h][n][k],  n < st.n,  k < st.k (whole operand rows).  Weights
-// are [head][n / 16][k / KW][64 lanes][EPC]: lane l holds row l % 16, k (l / 16) * EPC .. .  A wavefront per 16-row tile; few
-// tiles with long rows: a workgroup per tile, its wavefronts split K.  MK_F_GELU_TABLE: out = gelu(sum) * table[id(t)][n].
-template <typename E, int MT, bool SPLIT>
+// are [head][n / 16][k / KW][64 lanes][EPC]: lane l holds row l % 16, k (l / 16) * EPC .. .  A wavefront per 16-row tile and all
+// tokens; few tiles with long rows: a workgroup per tile and 16 tokens, its wavefronts split K.
+//   MX_GELU:   out = gelu(sum) * table[id(t)][n]
+//   MX_DECAY:  tanh is applied to the inputs (kept as value + remainder in bf16), out2 = exp(-exp(-1/2) sigmoid(sum + offset[n]))
+//              in 32 bits, and the gated activation runs beside it
+enum { MX_PLAIN, MX_GELU, MX_DECAY };
+template <typename E, int MT, int EPI, bool SPLIT>
 __device__ __forceinline__ void stage_mx_head_linear_t(CStage &st, Ctx &c, int M, char *smem) {
-  constexpr int EPC = FxType<E>::EPC, KW = FxType<E>::KW, KB = MT == 4 ? 4 : 8;
+  constexpr int EPC = FxType<E>::EPC, KW = FxType<E>::KW, KB = MT == 4 ? 4 : SPLIT ? 16 : EPI == MX_DECAY ? 4 : 8, B16 = sizeof(E) == 2;
+  static_assert(!SPLIT || MT == 1, "");
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lr = lane & 15, lg = lane >> 4;
-  const int N = st.n, nks = st.k / KW, nt = (N + 15) / 16, tiles = st.groups * nt;
+  const int N = st.n, nks = st.k / KW, nt = (N + 15) / 16, mts = SPLIT ? (M + 15) / 16 : 1, items = st.groups * nt * mts;
   const int kq = SPLIT ? (nks + MK_WAVES - 1) / MK_WAVES : nks;
   const int kb = SPLIT ? min(nks, wave * kq) : 0, ke = SPLIT ? min(nks, kb + kq) : nks;
   const u32x4 *W = (const u32x4 *)st.w.seg[0];
   const int i0 = SPLIT ? mx_spread(c) : mx_spread(c) + wave * c.G, di = SPLIT ? c.G : c.G * MK_WAVES;
   f32x4 *red = (f32x4 *)smem;
+  const u32x4 zero = {0u, 0u, 0u, 0u};
   u32x4 a[KB];
   auto load_w = [&](int i, int k0) {
 #pragma unroll
-    for (int j = 0; j < KB; j++) a[j] = ldg_stream(W + ((size_t)i * nks + min(k0 + j, nks - 1)) * 64 + lane);
+    for (int j = 0; j < KB; j++) a[j] = ldg_stream(W + ((size_t)(i / mts) * nks + min(k0 + j, nks - 1)) * 64 + lane);
   };
   // weights do not depend on the previous stage: the first tile's are requested before its barrier completes
-  const bool early = i0 < tiles && wave != 0;
+  const bool early = i0 < items && wave != 0;
   if (early) load_w(i0, kb);
   if (tid == 0) __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "agent");
   barrier_wait(c);
-  for (int i = i0; i < tiles; i += di) {
-    const int h = i / nt, n0 = (i - h * nt) * 16 + lg * 4;
+  for (int i = i0; i < items; i += di) {
+    const int tile = i / mts, mt0 = SPLIT ? i - tile * mts : 0, h = tile / nt, n0 = (tile - h * nt) * 16 + lg * 4;
     const E *xr[MT];
 #pragma unroll
-    for (int m = 0; m < MT; m++) xr[m] = (const E *)st.in + (size_t)min(m * 16 + lr, M - 1) * st.ld_in + (size_t)h * st.ld_in_slot + lg * EPC;
+    for (int m = 0; m < MT; m++) xr[m] = (const E *)st.in + (size_t)min((mt0 + m) * 16 + lr, M - 1) * st.ld_in + (size_t)h * st.ld_in_slot + lg * EPC;
     f32x4 acc[MT];
 #pragma unroll
     for (int m = 0; m < MT; m++) acc[m] = (f32x4){0.f, 0.f, 0.f, 0.f};
     for (int k0 = kb; k0 < ke; k0 += KB) {
       if (!(early && i == i0 && k0 == kb)) load_w(i, k0);
+      u32x4 b[KB][MT];
+#pragma unroll
+      for (int j = 0; j < KB; j++)
+#pragma unroll
+        for (int m = 0; m < MT; m++) b[j][m] = *(const u32x4 *)(xr[m] + (size_t)min(k0 + j, nks - 1) * KW);
 #pragma unroll
       for (int j = 0; j < KB; j++) {
-        const int ks = min(k0 + j, nks - 1);
-        u32x4 b[MT];
+        const u32x4 w = k0 + j < ke ? a[j] : zero;
 #pragma unroll
-        for (int m = 0; m < MT; m++) b[m] = *(const u32x4 *)(xr[m] + (size_t)ks * KW);
-        if (k0 + j < ke) {
+        for (int m = 0; m < MT; m++) {
+          if constexpr (EPI == MX_DECAY) {
+            u32x4 hi, lo;
 #pragma unroll
-          for (int m = 0; m < MT; m++) acc[m] = fx_mma_k(E(), a[j], b[m], acc[m]);
+            for (int q = 0; q < 4; q++) {
+              if constexpr (B16) {
+                const float x0 = tanhf(bf_lo(b[j][m][q])), x1 = tanhf(bf_hi(b[j][m][q]));
+                hi[q] = pack2(x0, x1);
+                lo[q] = pack2(x0 - bf_lo(hi[q]), x1 - bf_hi(hi[q]));
+              } else {
+                hi[q] = __float_as_uint(tanhf(__uint_as_float(b[j][m][q])));
+              }
+            }
+            acc[m] = fx_mma_k(E(), w, hi, acc[m]);
+            if constexpr (B16) acc[m] = fx_mma_k(E(), w, lo, acc[m]);
+          } else {
+            acc[m] = fx_mma_k(E(), w, b[j][m], acc[m]);
+          }
         }
       }
     }
     if constexpr (SPLIT) {
       __syncthreads();
-#pragma unroll
-      for (int m = 0; m < MT; m++) red[(wave * MT + m) * 64 + lane] = acc[m];
+      red[wave * 64 + lane] = acc[0];
       __syncthreads();
+      if (wave != 0) continue;
+      acc[0] = red[lane] + red[64 + lane] + red[128 + lane] + red[192 + lane];
     }
 #pragma unroll
     for (int m = 0; m < MT; m++) {
-      if (SPLIT && m % MK_WAVES != wave) continue;
-      f32x4 v = acc[m];
-      if constexpr (SPLIT) {
-        v = red[m * 64 + lane];
-#pragma unroll
-        for (int w = 1; w < MK_WAVES; w++) v += red[(w * MT + m) * 64 + lane];
-      }
-      const int t = m * 16 + lr;
+      const int t = (mt0 + m) * 16 + lr;
       if (t >= M) continue;
-      float r[4] = {v[0], v[1], v[2], v[3]};
-      if (st.flags & MK_F_GELU_TABLE) {
+      float r[4] = {acc[m][0], acc[m][1], acc[m][2], acc[m][3]};
+      if constexpr (EPI == MX_GELU) {
         const long long id = (long long)ldc_u64((const long long *)st.aux0 + t);
         const E *e = (const E *)st.aux1 + (size_t)(id < 0 ? 0 : id) * st.ld_res;
+        float f[4];
+#pragma unroll
+        for (int q = 0; q < 4; q++) f[q] = fx_val(e[min(n0 + q, N - 1)]);
 #pragma unroll
         for (int q = 0; q < 4; q++) {
           const float z = r[q], th = tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z));
-          r[q] = (id < 0 || n0 + q >= N) ? 0.f : 0.5f * z * (1.f + th) * fx_val(e[n0 + q]);
+          r[q] = id < 0 ? 0.f : 0.5f * z * (1.f + th) * f[q];
         }
       }
-      fx_stc4((E *)st.out + (size_t)t * st.ld_out + (size_t)h * st.ld_out_slot, n0, N, r);
+      if constexpr (EPI == MX_DECAY) {
+        const f32x4 w0 = *(const f32x4 *)((const float *)st.q_norm_w + n0);
+        f32x4 d;
+#pragma unroll
+        for (int q = 0; q < 4; q++) d[q] = expf(-0.6065306597126334f / (1.f + expf(-(r[q] + w0[q]))));
+        fx_stc_quad((float *)st.out2 + (size_t)t * st.ld_out2 + n0, d);
+      } else {
+        fx_stc4((E *)st.out + (size_t)t * st.ld_out + (size_t)h * st.ld_out_slot, n0, N, r);
+      }
     }
   }
+  if constexpr (EPI == MX_DECAY) mx_glu<E>(st, c, M);
   c.wrote_through = true;
 }
 template <typename E, int MAXM>
 __device__ __forceinline__ void stage_mx_head_linear(CStage &st, Ctx &c, int M, char *smem) {
-  const bool split = st.groups * ((st.n + 15) / 16) <= c.G && st.k / FxType<E>::KW >= 8;
-  if (split) {
-    if (MAXM == 1 || M <= 16) stage_mx_head_linear_t<E, 1, true>(st, c, M, smem);
-    else stage_mx_head_linear_t<E, 4, true>(st, c, M, smem);
+  if (st.groups * ((st.n + 15) / 16) * 4 <= c.G && st.k / FxType<E>::KW >= 8) {
+    if (st.flags & MK_F_GELU_TABLE) stage_mx_head_linear_t<E, 1, MX_GELU, true>(st, c, M, smem);
+    else stage_mx_head_linear_t<E, 1, MX_PLAIN, true>(st, c, M, smem);
+  } else if (st.flags & MK_F_GELU_TABLE) {
+    stage_mx_head_linear_t<E, MAXM == 1 ? 1 : 4, MX_GELU, false>(st, c, M, smem);
+  } else if (MAXM == 1 || M <= 16) {
+    stage_mx_head_linear_t<E, 1, MX_PLAIN, false>(st, c, M, smem);
   } else {
-    if (MAXM == 1 || M <= 16) stage_mx_head_linear_t<E, 1, false>(st, c, M, smem);
-    else stage_mx_head_linear_t<E, 4, false>(st, c, M, smem);
+    stage_mx_head_linear_t<E, 4, MX_PLAIN, false>(st, c, M, smem);
   }
+}
+template <typename E, int MAXM>
+__device__ __forceinline__ void stage_mx_decay(CStage &st, Ctx &c, int M, char *smem) {
+  if (MAXM == 1 || M <= 16) stage_mx_head_linear_t<E, 1, MX_DECAY, false>(st, c, M, smem);
+  else stage_mx_head_linear_t<E, 4, MX_DECAY, false>(st, c, M, smem);
 }
 
 // ----------------------------------------------------------------------------- latent attention
@@ -431,11 +548,11 @@ __device__ __forceinline__ MxLatentRows mx_latent_rows(const Ctx &c, int M, int 
   r.my_tiles = (r.my_n * H + unit_rows - 1) / unit_rows;
   r.tiles_incl = wave_incl_scan(r.my_tiles, lane);
   r.total = wave_bcast(r.tiles_incl, 63);
-  r.cmax = max(1, min(c.G / r.total, MK_ATTN_MAX_CHUNKS));
+  r.cmax = max(1, min(c.G / r.total, MK_MX_MAX_CHUNKS));
   return r;
 }
 // Chunks of a unit with NT tiles.
-__device__ __forceinline__ int mx_chunks(int NT, int cmax) { return NT <= 2 ? 1 : min(cmax, NT <= 16 ? NT : max(16, (NT + 1) / 2)); }
+__device__ __forceinline__ int mx_chunks(int NT, int cmax) { return NT <= 2 ? 1 : min(cmax, NT); }
 
 // 16-wide block of the latent, transposed out of the LDS tile: lane l gets dim l % 16 of the block at positions 4 (l / 16) .. + 3
 // of sub-tiles s and s + 1 (bf16) or of sub-tile s (32-bit).
@@ -457,16 +574,21 @@ __device__ __forceinline__ u32x4 mx_value_operand(float, const char *kt, int nkc
   return (u32x4){p[0], p[4], p[8], p[12]};
 }
 
-template <typename E, int KC, int VBW, int RT>
+// NK: operand rows of a cached latent the instantiation has room for (rows behind the real ones repeat one and meet zeros in the
+// query), SUB: sub-tiles per tile, VBW: 16-wide blocks per wavefront, RT: 16-row query tiles.  No loop of the tile walk has a
+// run-time bound or a branch, so that its loads and LDS reads are scheduled together.
+template <typename E, int NK, int SUB, int VBW, int RT>
 __device__ __forceinline__ void stage_mx_latent_attn_t(CStage &st, Ctx &c, const MkRuntime &rt, int M, char *smem) {
   using X = FxType<E>;
-  constexpr int EPC = X::EPC, KW = X::KW, B16 = sizeof(E) == 2;
+  constexpr int EPC = X::EPC, KW = X::KW, B16 = sizeof(E) == 2, TPOS = 16 * SUB, PARTS = MK_WAVES / SUB, KC = (NK + PARTS - 1) / PARTS;
+  constexpr int QN = RT * NK * 64 / MK_THREADS;
+  static_assert(RT * NK % 4 == 0, "whole rounds of query operands");
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lr = lane & 15, lg = lane >> 4;
   const int H = st.num_q_heads, R = st.rank, rot = st.rot_dims, half = rot / 2;
-  const int nrc = (R + KW - 1) / KW, nkc = nrc + (rot + KW - 1) / KW, nvb = nrc * KW / 16, Rp = nrc * KW, PST = Rp + 32;
-  const int SUB = st.k_tiles, TPOS = 16 * SUB, parts = MK_WAVES / SUB, ps = rt.page_size;
-  const int my_sub = wave & (SUB - 1), my_part = wave / SUB;
-  const MkLatentLds L = mk_latent_lds(sizeof(E), RT, nkc, SUB, 0);
+  const int nrc = (R + KW - 1) / KW, npc = (rot + KW - 1) / KW, nkc = nrc + npc, nvb = nrc * KW / 16, Rp = nrc * KW, PST = Rp + 32;
+  const int ps = rt.page_size;
+  const int my_sub = wave % SUB, my_part = wave / SUB;
+  const MkLatentLds L = mk_latent_lds(sizeof(E), RT, NK, SUB, 0);
   u32x4 *qs = (u32x4 *)smem;
   char *kt = smem + L.kt;
   u32x4 *pb = (u32x4 *)(smem + L.pb);
@@ -475,7 +597,6 @@ __device__ __forceinline__ void stage_mx_latent_attn_t(CStage &st, Ctx &c, const
   const u32x4 *kc = (const u32x4 *)st.k_cache;
   const MxLatentRows rw = mx_latent_rows(c, M, H, 16 * RT);
   const int cmax = rw.cmax, n_units = rw.total * cmax;
-  c.mx_split = false;
   {  // (every workgroup: will some request be split?  then the merge stage runs)
     const int NT = rw.my_n ? (c.sh_tok[lane] + rw.my_n - 1) / TPOS + 1 : 0;
     c.mx_split = __any(rw.my_n && mx_chunks(NT, cmax) > 1);
@@ -507,16 +628,13 @@ __device__ __forceinline__ void stage_mx_latent_attn_t(CStage &st, Ctx &c, const
     const int pp = (tile * TPOS) % ps;
     const u32x4 *p = kc + ((((size_t)page * ps + pp) / 16 + my_sub) * nkc) * 64 + lane;
 #pragma unroll
-    for (int j = 0; j < KC; j++)
-      if (j * parts < nkc) kv[j] = p[min(j * parts + my_part, nkc - 1) * 64];
+    for (int j = 0; j < KC; j++) kv[j] = p[min(j * PARTS + my_part, nkc - 1) * 64];
   };
   auto store_tile = [&](int tile, int newest) {
     const bool hidden = tile * TPOS + my_sub * 16 + lr > newest;  // rows behind the newest position belong to nobody
+    u32x4 *dst = (u32x4 *)kt + (my_sub * NK + my_part) * 64 + lane;
 #pragma unroll
-    for (int j = 0; j < KC; j++) {
-      const int ch = j * parts + my_part;
-      if (ch < nkc) ((u32x4 *)kt)[(my_sub * nkc + ch) * 64 + lane] = hidden ? (u32x4){0u, 0u, 0u, 0u} : kv[j];
-    }
+    for (int j = 0; j < KC; j++) dst[j * PARTS * 64] = hidden ? (u32x4){0u, 0u, 0u, 0u} : kv[j];
   };
   Unit a0;
   const int u0 = mx_spread(c);
@@ -539,39 +657,47 @@ __device__ __forceinline__ void stage_mx_latent_attn_t(CStage &st, Ctx &c, const
     __syncthreads();  // LDS reuse across units
     const int pg_lo = a.tb * TPOS / ps, npg = a.tb < a.te ? (a.te * TPOS - 1) / ps - pg_lo + 1 : 0;
     for (int i = tid; i < npg; i += MK_THREADS) spg[i] = rt.kv_indices[a.pages + min(pg_lo + i, a.p / ps)];
-    // ---- query rows in operand order, the rotated part on the way
-    for (int i = tid; i < RT * nkc * 64; i += MK_THREADS) {
-      const int rc = i >> 6, rtile = rc / nkc, ch = rc - rtile * nkc, r = rtile * 16 + (i & 15), g = (i & 63) >> 4, Rw = a.r0 + r;
-      u32x4 v = {0u, 0u, 0u, 0u};
-      if (r < a.nrows) {
-        const int t = a.t0 + Rw / H, h = Rw % H;
-        if (ch < nrc) {
-          v = ldc_16B((const u32x4 *)((const E *)st.q_ws + (size_t)t * st.ld_qws + (size_t)h * Rp + ch * KW + g * EPC));
-        } else {
-          const E *q = (const E *)st.in + (size_t)t * st.ld_in + (size_t)h * st.ld_in_slot + st.cols[0];
-          const int pos = c.sh_tok[t];
-          const float *ct = (const float *)st.cos_tab + (size_t)pos * st.ld_cos, *sn = (const float *)st.sin_tab + (size_t)pos * st.ld_cos;
-          float f[EPC];
+    // ---- query rows in operand order: latent parts, then (over the zeros left for it) the rotated part
+    {
+      u32x4 q[QN];
 #pragma unroll
-          for (int e = 0; e < EPC; e++) {
-            const int d = (ch - nrc) * KW + g * EPC + e;
-            f[e] = 0.f;
-            if (d < rot) {
-              const int k = d < half ? d : d - half;
-              const float x = fx_ldc(q + d), y = fx_ldc(q + (d < half ? d + half : k));
-              f[e] = d < half ? x * ct[k] - y * sn[k] : x * ct[k] + y * sn[k];
-            }
-          }
-          if constexpr (B16) {
-#pragma unroll
-            for (int w = 0; w < 4; w++) v[w] = pack2(f[(2 * w) % EPC], f[(2 * w + 1) % EPC]);
-          } else {
-#pragma unroll
-            for (int w = 0; w < 4; w++) v[w] = __float_as_uint(f[w % EPC]);
-          }
-        }
+      for (int k = 0; k < QN; k++) {
+        const int i = tid + k * MK_THREADS, rc = i >> 6, rtile = rc / NK, ch = rc - rtile * NK, Rw = a.r0 + min(rtile * 16 + (i & 15), a.nrows - 1);
+        q[k] = ldc_16B((const u32x4 *)((const E *)st.q_ws + (size_t)(a.t0 + Rw / H) * st.ld_qws + (size_t)(Rw % H) * Rp + min(ch, nrc - 1) * KW + ((i & 63) >> 4) * EPC));
       }
-      qs[i] = v;
+#pragma unroll
+      for (int k = 0; k < QN; k++) {
+        const int i = tid + k * MK_THREADS, rc = i >> 6, rtile = rc / NK, ch = rc - rtile * NK;
+        const bool real = ch < nrc && rtile * 16 + (i & 15) < a.nrows;
+        if (ch < nrc || ch >= nkc) qs[i] = real ? q[k] : (u32x4){0u, 0u, 0u, 0u};
+      }
+      for (int i = tid; i < RT * npc * 64; i += MK_THREADS) {
+        const int rc = i >> 6, rtile = rc / npc, ch = rc - rtile * npc, r = rtile * 16 + (i & 15), Rw = a.r0 + min(r, a.nrows - 1), t = a.t0 + Rw / H;
+        const E *qr = (const E *)st.in + (size_t)t * st.ld_in + (size_t)(Rw % H) * st.ld_in_slot + st.cols[0];
+        const int pos = c.sh_tok[t];
+        const float *ct = (const float *)st.cos_tab + (size_t)pos * st.ld_cos, *sn = (const float *)st.sin_tab + (size_t)pos * st.ld_cos;
+        float x[EPC], y[EPC], cs[EPC], sv[EPC];
+#pragma unroll
+        for (int e = 0; e < EPC; e++) {
+          const int d = min(ch * KW + ((i & 63) >> 4) * EPC + e, rot - 1), k = d < half ? d : d - half;
+          x[e] = fx_ldc(qr + d);
+          y[e] = fx_ldc(qr + (d < half ? d + half : k));
+          cs[e] = ct[k];
+          sv[e] = sn[k];
+        }
+#pragma unroll
+        for (int e = 0; e < EPC; e++) {
+          const int d = ch * KW + ((i & 63) >> 4) * EPC + e;
+          x[e] = d >= rot || r >= a.nrows ? 0.f : d < half ? x[e] * cs[e] - y[e] * sv[e] : x[e] * cs[e] + y[e] * sv[e];
+        }
+        u32x4 v;
+#pragma unroll
+        for (int w = 0; w < 4; w++) {
+          if constexpr (B16) v[w] = pack2(x[(2 * w) % EPC], x[(2 * w + 1) % EPC]);
+          else v[w] = __float_as_uint(x[w % EPC]);
+        }
+        qs[(rtile * NK + nrc + ch) * 64 + (i & 63)] = v;
+      }
     }
     // ---- tiles
     int plim[RT];
@@ -591,22 +717,23 @@ __device__ __forceinline__ void stage_mx_latent_attn_t(CStage &st, Ctx &c, const
       if (tile + 1 < a.te) load_tile(tile + 1, spg[(tile + 1) * TPOS / ps - pg_lo]);
       __syncthreads();
       float sc[RT][4];
-      if (wave < SUB) {
-        f32x4 S[RT];
+      if (SUB == MK_WAVES || wave < SUB) {
+        f32x4 S[RT][2];  // (two chains per row tile)
 #pragma unroll
-        for (int q = 0; q < RT; q++) S[q] = (f32x4){0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
-        for (int ch = 0; ch < nkc; ch++) {
-          const u32x4 k = ((const u32x4 *)kt)[(wave * nkc + ch) * 64 + lane];
+        for (int q = 0; q < RT; q++) S[q][0] = S[q][1] = (f32x4){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-          for (int q = 0; q < RT; q++) S[q] = fx_mma_k(E(), k, qs[(q * nkc + ch) * 64 + lane], S[q]);
+        for (int ch = 0; ch < NK; ch++) {
+          const u32x4 k = ((const u32x4 *)kt)[(wave * NK + ch) * 64 + lane];
+#pragma unroll
+          for (int q = 0; q < RT; q++) S[q][ch & 1] = fx_mma_k(E(), k, qs[(q * NK + ch) * 64 + lane], S[q][ch & 1]);
         }
 #pragma unroll
         for (int q = 0; q < RT; q++) {
+          const f32x4 s = S[q][0] + S[q][1];
           float tm = MK_FX_NEG;
 #pragma unroll
           for (int i = 0; i < 4; i++) {
-            sc[q][i] = tile * TPOS + wave * 16 + lg * 4 + i <= plim[q] ? S[q][i] * sc1 : MK_FX_NEG;
+            sc[q][i] = tile * TPOS + wave * 16 + lg * 4 + i <= plim[q] ? s[i] * sc1 : MK_FX_NEG;
             tm = fmaxf(tm, sc[q][i]);
           }
           tm = groups_max(tm);
@@ -614,21 +741,31 @@ __device__ __forceinline__ void stage_mx_latent_attn_t(CStage &st, Ctx &c, const
         }
       }
       __syncthreads();
+      float nm[RT];
+      bool grow = false;
 #pragma unroll
       for (int q = 0; q < RT; q++) {
-        float nm = m[q];
-        for (int s = 0; s < SUB; s++) nm = fmaxf(nm, mx[(s * RT + q) * 16 + lr]);
-        if (__any(nm > m[q])) {
-          const float corr = fx_exp2(E(), m[q] - nm);
-          m[q] = nm;
+        nm[q] = m[q];
+#pragma unroll
+        for (int s = 0; s < SUB; s++) nm[q] = fmaxf(nm[q], mx[(s * RT + q) * 16 + lr]);
+        grow = grow || nm[q] > m[q];
+      }
+      if (__any(grow)) {
+#pragma unroll
+        for (int q = 0; q < RT; q++) {
+          const float corr = fx_exp2(E(), m[q] - nm[q]);
+          m[q] = nm[q];
           l[q] *= corr;
 #pragma unroll
           for (int b = 0; b < VBW; b++) acc[q][b] *= corr;
         }
-        if (wave < SUB) {
+      }
+      if (SUB == MK_WAVES || wave < SUB) {
+#pragma unroll
+        for (int q = 0; q < RT; q++) {
 #pragma unroll
           for (int i = 0; i < 4; i++) {
-            sc[q][i] = sc[q][i] > 0.5f * MK_FX_NEG ? fx_exp2(E(), sc[q][i] - nm) : 0.f;
+            sc[q][i] = sc[q][i] > 0.5f * MK_FX_NEG ? fx_exp2(E(), sc[q][i] - m[q]) : 0.f;
             l[q] += sc[q][i];
           }
           if constexpr (B16) {
@@ -643,24 +780,25 @@ __device__ __forceinline__ void stage_mx_latent_attn_t(CStage &st, Ctx &c, const
         }
       }
       __syncthreads();
+#pragma unroll
       for (int s = 0; s < SUB; s += B16 ? 2 : 1) {
+        u32x4 p[RT][2];
+#pragma unroll
+        for (int q = 0; q < RT; q++) {
+          if constexpr (B16) {
+            p[q][0] = pb[(((s >> 1) * RT + q) * 2) * 64 + lane];
+            p[q][1] = pb[(((s >> 1) * RT + q) * 2 + 1) * 64 + lane];
+          } else {
+            p[q][0] = pb[(s * RT + q) * 64 + lane];
+          }
+        }
 #pragma unroll
         for (int j = 0; j < VBW; j++) {
-          const int b = wave + MK_WAVES * j;
-          if (b < nvb) {
-            const u32x4 v = mx_value_operand(E(), kt, nkc, s, b, lane);
+          const u32x4 v = mx_value_operand(E(), kt, NK, s, wave + MK_WAVES * j, lane);  // (blocks behind the last are finite and never stored)
 #pragma unroll
-            for (int q = 0; q < RT; q++) {
-              if (q * 16 < a.nrows) {
-                if constexpr (B16) {
-                  const u32x4 *p = pb + (((s >> 1) * RT + q) * 2) * 64 + lane;
-                  acc[q][j] = fx_mma_k(E(), v, p[0], acc[q][j]);
-                  acc[q][j] = fx_mma_k(E(), v, p[64], acc[q][j]);
-                } else {
-                  acc[q][j] = fx_mma_k(E(), v, pb[(s * RT + q) * 64 + lane], acc[q][j]);
-                }
-              }
-            }
+          for (int q = 0; q < RT; q++) {
+            acc[q][j] = fx_mma_k(E(), v, p[q][0], acc[q][j]);
+            if constexpr (B16) acc[q][j] = fx_mma_k(E(), v, p[q][1], acc[q][j]);
           }
         }
       }
@@ -742,229 +880,379 @@ __device__ __forceinline__ void stage_mx_latent_merge(CStage &st, Ctx &c, const 
 }
 template <typename E>
 __device__ __forceinline__ void stage_mx_latent_attn(CStage &st, Ctx &c, const MkRuntime &rt, int M, char *smem) {
+  // (the host picks st.nk, the operand rows of the instantiation, from this list)
   if constexpr (sizeof(E) == 2) {
-    if (st.rank <= 128 && st.rot_dims <= 64) stage_mx_latent_attn_t<E, 6, 2, 2>(st, c, rt, M, smem);
-    else stage_mx_latent_attn_t<E, 20, 8, 2>(st, c, rt, M, smem);
+    if (st.nk == 6) stage_mx_latent_attn_t<E, 6, 4, 2, 2>(st, c, rt, M, smem);
+    else if (st.nk == 18) stage_mx_latent_attn_t<E, 18, 4, 8, 2>(st, c, rt, M, smem);
+    else stage_mx_latent_attn_t<E, 20, 4, 8, 2>(st, c, rt, M, smem);
   } else {
-    stage_mx_latent_attn_t<E, 20, 8, 1>(st, c, rt, M, smem);
+    if (st.nk == 12) stage_mx_latent_attn_t<E, 12, 2, 2, 1>(st, c, rt, M, smem);
+    else stage_mx_latent_attn_t<E, 40, 2, 8, 1>(st, c, rt, M, smem);
   }
 }
 
 // ----------------------------------------------------------------------------- generalised delta rule
-// Unit = (request, head), a workgroup each; a token block of 16 rows at a time.  The columns of the state are independent of
-// each other given the block's key-side vectors, so a wavefront keeps 16-column blocks of it in registers (lane l: column
-// l % 16, channels 16 i + 4 (l / 16) .. + 3) and walks the tokens; the two sums over channels cross lanes with two swaps.
-// The key-side vectors (unit key, removal, decay) are formed first, the decay's low-rank product on the matrix cores.
-// State: [slot][head][column block][i][64 lanes] f32x4, 32-bit; zero where a request begins.
+// The columns of a head's state are independent of each other given the key-side vectors of a token.  A lane keeps NC columns x
+// 4 NI channels in registers: lane l of a wavefront holds columns (l / 16) NC .. + NC - 1 of its wavefront's 4 NC and channels
+// 64 i + 4 (l % 16) .. + 3, so the sums over channels stay inside a 16-lane row (four DPP additions).  State: 32-bit
+// [slot][head][column][channel], sizes rounded up to 16; zero where a request begins.  Row sections of a head are padded with
+// zeros to the same size Dp (D values count for the norm).  Decays come from the MX_DECAY form of the head linear.
+//
+// Iterations in which every request brings one token: a workgroup per (request, head), the next unit's state and rows in
+// flight while one is computed.  Otherwise the rows of 16 tokens at a time are put in LDS by all wavefronts (the next 16 are in
+// flight meanwhile) and every wavefront walks them; few units are dealt in slices of columns to several workgroups, which
+// leave their unnormalised outputs to the MX_DELTA_OUT stage.
 #define MX_TB 16
-template <typename E, int DQ, int NB>
-__device__ __forceinline__ void stage_mx_delta_t(CStage &st, Ctx &c, const MkRuntime &rt, int M, char *smem) {
-  constexpr int EPC = FxType<E>::EPC, KW = FxType<E>::KW, B16 = sizeof(E) == 2, DP = DQ * 16, DPS = DP + 4;
+struct MxDeltaUnits {
+  bool first;
+  int my_n, rank_of, nreq;
+};
+__device__ __forceinline__ MxDeltaUnits mx_delta_units(const Ctx &c, int M) {
+  const int lane = threadIdx.x & 63;
+  MxDeltaUnits r;
+  r.first = lane < M && c.sh_tok[2 * MK_MAX_TOKENS + lane] == lane;
+  const unsigned long long fm = __ballot(r.first), later = lane < 63 ? fm >> (lane + 1) : 0ull;
+  r.my_n = r.first ? (later ? (int)__ffsll(later) : M - lane) : 0;
+  r.rank_of = __popcll(fm & ((1ull << lane) - 1ull));
+  r.nreq = __popcll(fm);
+  return r;
+}
+struct MxDeltaUnit {
+  int h, t0, n, p0, col0;
+  float *state;
+};
+// unit u of `slices` per (request, head), cols columns each
+__device__ __forceinline__ MxDeltaUnit mx_delta_unit(CStage &st, const Ctx &c, const MkRuntime &rt, const MxDeltaUnits &us, int u, int slices, int cols, int Dp) {
+  MxDeltaUnit a;
+  const int uh = u / slices, H = st.num_q_heads, ri = uh / H;
+  a.col0 = (u - uh * slices) * cols;
+  a.h = uh - ri * H;
+  a.t0 = (int)__ffsll(__ballot(us.first && us.rank_of == ri)) - 1;
+  a.n = wave_bcast(us.my_n, a.t0);
+  a.p0 = __builtin_amdgcn_readfirstlane(c.sh_tok[a.t0]);
+  const int slot = __builtin_amdgcn_readfirstlane(c.sh_tok[MK_MAX_TOKENS + a.t0]);
+  a.state = (float *)st.k_cache + ((size_t)__builtin_amdgcn_readfirstlane(rt.state_ids[slot]) * H + a.h) * Dp * Dp;
+  return a;
+}
+template <int NI, int NC>
+__device__ __forceinline__ void mx_delta_load(f32x4 (&S)[NC][NI], const float *state, bool zero, int col, int lr, int Dp) {
+#pragma unroll
+  for (int j = 0; j < NC; j++)
+#pragma unroll
+    for (int i = 0; i < NI; i++) S[j][i] = fx_ldc_quad(state + (size_t)min(col + j, Dp - 1) * Dp + min(i * 64 + lr * 4, Dp - 4));
+#pragma unroll
+  for (int j = 0; j < NC; j++)
+#pragma unroll
+    for (int i = 0; i < NI; i++)
+      if (zero || col + j >= Dp || i * 64 + lr * 4 >= Dp) S[j][i] = (f32x4){0.f, 0.f, 0.f, 0.f};
+}
+template <int NI, int NC>
+__device__ __forceinline__ void mx_delta_store(const f32x4 (&S)[NC][NI], float *state, int col, int lr, int Dp) {
+#pragma unroll
+  for (int j = 0; j < NC; j++)
+#pragma unroll
+    for (int i = 0; i < NI; i++)
+      if (col + j < Dp && i * 64 + lr * 4 < Dp) fx_stc_quad(state + (size_t)(col + j) * Dp + i * 64 + lr * 4, S[j][i]);
+}
+template <int NI> struct MxDeltaVec {
+  f32x4 r[NI], k[NI], u[NI], au[NI], w[NI];
+};
+// one token: S <- diag(w) S - (a u)(u^T S) + k v^T, o = S^T r
+template <int NI, int NC>
+__device__ __forceinline__ void mx_delta_step(f32x4 (&S)[NC][NI], const MxDeltaVec<NI> &x, const float (&v)[NC], float (&o)[NC]) {
+  float su[NC];
+#pragma unroll
+  for (int j = 0; j < NC; j++) {
+    su[j] = 0.f;
+#pragma unroll
+    for (int i = 0; i < NI; i++)
+#pragma unroll
+      for (int e = 0; e < 4; e++) su[j] = fmaf(x.u[i][e], S[j][i][e], su[j]);
+  }
+#pragma unroll
+  for (int j = 0; j < NC; j++) su[j] = group16_sum(su[j]);
+#pragma unroll
+  for (int j = 0; j < NC; j++) {
+    o[j] = 0.f;
+#pragma unroll
+    for (int i = 0; i < NI; i++)
+#pragma unroll
+      for (int e = 0; e < 4; e++) {
+        S[j][i][e] = fmaf(x.k[i][e], v[j], fmaf(-x.au[i][e], su[j], x.w[i][e] * S[j][i][e]));
+        o[j] = fmaf(x.r[i][e], S[j][i][e], o[j]);
+      }
+  }
+#pragma unroll
+  for (int j = 0; j < NC; j++) o[j] = group16_sum(o[j]);
+}
+__device__ __forceinline__ float mx_sigmoid(float z) { return 1.f / (1.f + expf(-z)); }
+
+// every request brings one token
+template <typename E, int NI, int NC>
+__device__ __forceinline__ void stage_mx_delta_single(CStage &st, Ctx &c, const MkRuntime &rt, int M, char *smem) {
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lr = lane & 15, lg = lane >> 4;
-  const int D = st.head_dim, H = st.num_q_heads, nd = (D + 15) / 16, nks = st.rank / KW, passes = (nd + MK_WAVES * NB - 1) / (MK_WAVES * NB);
-  float *rv = (float *)smem, *kv = rv + MX_TB * DPS, *uv = kv + MX_TB * DPS, *av = uv + MX_TB * DPS, *wv = av + MX_TB * DPS, *vv = wv + MX_TB * DPS;
-  u32x4 *tw = (u32x4 *)(vv + MX_TB * DPS);  // [rank / KW][value, remainder][64] operands of tanh(low-rank projection)
-  const bool first = lane < M && c.sh_tok[2 * MK_MAX_TOKENS + lane] == lane;
-  const unsigned long long fm = __ballot(first), later = lane < 63 ? fm >> (lane + 1) : 0ull;
-  const int my_n = first ? (later ? (int)__ffsll(later) : M - lane) : 0;
-  const int rank_of = __popcll(fm & ((1ull << lane) - 1ull)), n_units = __popcll(fm) * H;
-  struct Unit {
-    int h, t0, n, p0;
-    f32x4 *state;
+  const int D = st.head_dim, Dp = (D + 15) / 16 * 16, H = st.num_q_heads, n_units = M * H, col = (wave * 4 + lg) * NC;
+  const MxDeltaUnits us = mx_delta_units(c, M);
+  const E *in = (const E *)st.in;
+  const float *ab = (const float *)st.k_norm_w, *nw = (const float *)st.norm_w;
+  float *red = (float *)smem;
+  struct Raw {
+    f32x4 r[NI], k[NI], a[NI], w[NI], ab[NI], v[NC / 4], g[NC / 4], nw[NC / 4];
   };
-  auto decode = [&](int u) {
-    Unit a;
-    const int ri = u / H;
-    a.h = u - ri * H;
-    a.t0 = (int)__ffsll(__ballot(first && rank_of == ri)) - 1;
-    a.n = wave_bcast(my_n, a.t0);
-    a.p0 = __builtin_amdgcn_readfirstlane(c.sh_tok[a.t0]);
-    const int slot = __builtin_amdgcn_readfirstlane(c.sh_tok[MK_MAX_TOKENS + a.t0]);
-    a.state = (f32x4 *)st.k_cache + ((size_t)rt.state_ids[slot] * H + a.h) * nd * nd * 64 + lane;
-    return a;
+  auto load_raw = [&](const MxDeltaUnit &a, Raw &x) {
+    const E *row = in + (size_t)a.t0 * st.ld_in + a.h * Dp;
+    const float *wr = (const float *)st.in2 + (size_t)a.t0 * st.ld_in2 + a.h * Dp;
+#pragma unroll
+    for (int i = 0; i < NI; i++) {
+      const int d = min(i * 64 + lr * 4, Dp - 4);
+      x.r[i] = fx_ldc_quad(row + st.cols[0] + d);
+      x.k[i] = fx_ldc_quad(row + st.cols[1] + d);
+      x.a[i] = fx_ldc_quad(row + st.cols[4] + d);
+      x.w[i] = fx_ldc_quad(wr + d);
+      x.ab[i] = *(const f32x4 *)(ab + a.h * Dp + d);
+    }
+#pragma unroll
+    for (int j = 0; j < NC / 4; j++) {
+      const int d = min(col + 4 * j, Dp - 4);
+      x.v[j] = fx_ldc_quad(row + st.cols[2] + d);
+      x.g[j] = fx_ldc_quad(row + st.cols[3] + d);
+      x.nw[j] = *(const f32x4 *)(nw + a.h * Dp + d);
+    }
   };
-  f32x4 S[NB][DQ];
-  auto load_state = [&](const Unit &a, int pass, bool zero) {
+  f32x4 S[NC][NI];
+  const int u0 = mx_spread(c);
+  MxDeltaUnit a{};
+  // earlier iterations wrote the state: the first unit's is requested before the barrier is awaited
+  const bool early = u0 < n_units && wave != 0;
+  if (u0 < n_units) a = mx_delta_unit(st, c, rt, us, u0, 1, 0, Dp);
+  if (early) mx_delta_load<NI, NC>(S, a.state, a.p0 == 0, col, lr, Dp);
+  barrier_wait(c);
+  Raw x;
+  if (u0 < n_units) {
+    if (!early) mx_delta_load<NI, NC>(S, a.state, a.p0 == 0, col, lr, Dp);
+    load_raw(a, x);
+  }
+  int par = 0;
+  for (int u = u0; u < n_units; u += c.G, par ^= 4) {
+    MxDeltaUnit nx = a;
+    f32x4 Sn[NC][NI];
+    Raw xn;
+    if (u + c.G < n_units) nx = mx_delta_unit(st, c, rt, us, u + c.G, 1, 0, Dp);
+    mx_delta_load<NI, NC>(Sn, nx.state, nx.p0 == 0, col, lr, Dp);  // (the last unit's again when there is no other)
+    load_raw(nx, xn);
+    MxDeltaVec<NI> y;
+    float ss = 0.f;
 #pragma unroll
-    for (int b = 0; b < NB; b++) {
-      const int cb = (pass * NB + b) * MK_WAVES + wave;
+    for (int i = 0; i < NI; i++)
 #pragma unroll
-      for (int i = 0; i < DQ; i++) {
-        S[b][i] = (f32x4){0.f, 0.f, 0.f, 0.f};
-        if (!zero && i < nd && cb < nd) S[b][i] = fx_ldc_quad((const float *)(a.state + (size_t)(cb * nd + i) * 64));
+      for (int e = 0; e < 4; e++) {
+        if (i * 64 + lr * 4 >= Dp) x.r[i][e] = x.k[i][e] = 0.f;
+        ss += x.k[i][e] * x.k[i][e];
+      }
+    const float inv = 1.f / sqrtf(group16_sum(ss) + 1e-6f);
+#pragma unroll
+    for (int i = 0; i < NI; i++)
+#pragma unroll
+      for (int e = 0; e < 4; e++) {
+        y.r[i][e] = x.r[i][e];
+        y.k[i][e] = x.k[i][e];
+        y.u[i][e] = x.k[i][e] * inv;
+        y.au[i][e] = mx_sigmoid(x.a[i][e] + x.ab[i][e]) * y.u[i][e];
+        y.w[i][e] = x.w[i][e];
+      }
+    float v[NC], o[NC];
+#pragma unroll
+    for (int j = 0; j < NC; j++) v[j] = col + j < Dp ? x.v[j / 4][j & 3] : 0.f;
+    mx_delta_step<NI, NC>(S, y, v, o);
+    mx_delta_store<NI, NC>(S, a.state, col, lr, Dp);
+    float so = 0.f;
+#pragma unroll
+    for (int j = 0; j < NC; j++) so += o[j] * o[j];
+    so = groups_sum(so);
+    if (lane == 0) red[par + wave] = so;
+    __syncthreads();
+    const float rn = 1.f / sqrtf(((red[par] + red[par + 1]) + (red[par + 2] + red[par + 3])) / (float)D + st.eps);
+    if (lr == 0) {
+#pragma unroll
+      for (int j = 0; j < NC / 4; j++) {
+        f32x4 q;
+#pragma unroll
+        for (int e = 0; e < 4; e++) q[e] = (o[4 * j + e] * rn) * x.nw[j][e] * mx_sigmoid(x.g[j][e]);
+        if (col + 4 * j < Dp) fx_stc_quad((E *)st.out + (size_t)a.t0 * st.ld_out + a.h * Dp + col + 4 * j, q);
       }
     }
-  };
-  auto store_state = [&](const Unit &a, int pass) {
+    a = nx;
+    x = xn;
 #pragma unroll
-    for (int b = 0; b < NB; b++) {
-      const int cb = (pass * NB + b) * MK_WAVES + wave;
+    for (int j = 0; j < NC; j++)
 #pragma unroll
-      for (int i = 0; i < DQ; i++)
-        if (i < nd && cb < nd) fx_stc_quad((float *)(a.state + (size_t)(cb * nd + i) * 64), S[b][i]);
-    }
-  };
+      for (int i = 0; i < NI; i++) S[j][i] = Sn[j][i];
+  }
+  c.wrote_through = true;
+}
+
+// some request brings several tokens: `slices` workgroups per (request, head), 16 NC columns each
+template <typename E, int NI, int NC>
+__device__ __forceinline__ void stage_mx_delta_multi(CStage &st, Ctx &c, const MkRuntime &rt, int M, int slices, char *smem) {
+  constexpr int DPS = NI * 64 + 4, TW = MX_TB / MK_WAVES;
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lr = lane & 15, lg = lane >> 4;
+  const int D = st.head_dim, Dp = (D + 15) / 16 * 16, H = st.num_q_heads, cw = (wave * 4 + lg) * NC, d4 = min(4 * lane, Dp - 4);
+  float *rv = (float *)smem, *kv = rv + MX_TB * DPS, *uv = kv + MX_TB * DPS, *av = uv + MX_TB * DPS, *wv = av + MX_TB * DPS, *vv = wv + MX_TB * DPS, *ov = vv + MX_TB * DPS;
+  const MxDeltaUnits us = mx_delta_units(c, M);
+  const int n_units = us.nreq * H * slices;
+  const E *in = (const E *)st.in;
+  const float *ab = (const float *)st.k_norm_w, *nw = (const float *)st.norm_w;
+  f32x4 S[NC][NI];
   const int u0 = mx_spread(c);
-  // earlier iterations wrote the state: the first unit's is requested before the barrier is awaited
-  const bool early = passes == 1 && u0 < n_units && wave != 0;
+  const bool early = u0 < n_units && wave != 0;
   if (early) {
-    const Unit a = decode(u0);
-    load_state(a, 0, a.p0 == 0);
+    const MxDeltaUnit a = mx_delta_unit(st, c, rt, us, u0, slices, 16 * NC, Dp);
+    mx_delta_load<NI, NC>(S, a.state, a.p0 == 0, a.col0 + cw, lr, Dp);
   }
   barrier_wait(c);
-  const E *in = (const E *)st.in;
-  const float *w0 = (const float *)st.q_norm_w, *ab = (const float *)st.k_norm_w, *nw = (const float *)st.norm_w;
   for (int u = u0; u < n_units; u += c.G) {
-    const Unit a = decode(u);
-    if (passes == 1 && !(u == u0 && early)) load_state(a, 0, a.p0 == 0);
+    const MxDeltaUnit a = mx_delta_unit(st, c, rt, us, u, slices, 16 * NC, Dp);
+    const int col = a.col0 + cw;
+    if (!(u == u0 && early)) mx_delta_load<NI, NC>(S, a.state, a.p0 == 0, col, lr, Dp);
+    // lane l of a wavefront takes channels 4 l .. + 3 of tokens wave, wave + 4, ... of the block
+    f32x4 xr[TW], xk[TW], xv[TW], xa[TW], xw[TW];
+    const f32x4 xab = *(const f32x4 *)(ab + a.h * Dp + d4), xnw = *(const f32x4 *)(nw + a.h * Dp + d4);
+    auto load_rows = [&](int tb) {
+#pragma unroll
+      for (int j = 0; j < TW; j++) {
+        const int t = a.t0 + min(tb + wave + j * MK_WAVES, a.n - 1);
+        const E *row = in + (size_t)t * st.ld_in + a.h * Dp + d4;
+        xr[j] = fx_ldc_quad(row + st.cols[0]);
+        xk[j] = fx_ldc_quad(row + st.cols[1]);
+        xv[j] = fx_ldc_quad(row + st.cols[2]);
+        xa[j] = fx_ldc_quad(row + st.cols[4]);
+        xw[j] = fx_ldc_quad((const float *)st.in2 + (size_t)t * st.ld_in2 + a.h * Dp + d4);
+      }
+    };
+    load_rows(0);
     for (int tb = 0; tb < a.n; tb += MX_TB) {
       const int nt = min(MX_TB, a.n - tb);
       __syncthreads();  // LDS reuse
-      // ---- rows: r, k, v as they are, u = k / |k|, a u
-      for (int j = wave; j < nt; j += MK_WAVES) {
-        const E *row = in + (size_t)(a.t0 + tb + j) * st.ld_in + a.h * D;
-        float xr[DP / 64], xk[DP / 64], xv[DP / 64], xa[DP / 64], ss = 0.f;
 #pragma unroll
-        for (int i = 0; i < DP / 64; i++) {
-          const int d = min(i * 64 + lane, D - 1);
-          xr[i] = fx_ldc(row + st.cols[0] + d);
-          xk[i] = fx_ldc(row + st.cols[1] + d);
-          xv[i] = fx_ldc(row + st.cols[2] + d);
-          xa[i] = fx_ldc(row + st.cols[4] + d);
-        }
-#pragma unroll
-        for (int i = 0; i < DP / 64; i++) {
-          if (i * 64 + lane >= D) xr[i] = xk[i] = xv[i] = 0.f;
-          ss += xk[i] * xk[i];
-        }
+      for (int j = 0; j < TW; j++) {
+        const bool real = 4 * lane < Dp;
+        float ss = real ? xk[j][0] * xk[j][0] + xk[j][1] * xk[j][1] + xk[j][2] * xk[j][2] + xk[j][3] * xk[j][3] : 0.f;
         const float inv = 1.f / sqrtf(wave_sum(ss) + 1e-6f);
+        if (4 * lane < NI * 64) {
+          f32x4 un, au;
 #pragma unroll
-        for (int i = 0; i < DP / 64; i++) {
-          const int d = i * 64 + lane, at = j * DPS + d;
-          const float un = xk[i] * inv, rem = d < D ? 1.f / (1.f + expf(-(xa[i] + ab[a.h * D + min(d, D - 1)]))) : 0.f;
-          rv[at] = xr[i];
-          kv[at] = xk[i];
-          vv[at] = xv[i];
-          uv[at] = un;
-          av[at] = rem * un;
-        }
-      }
-      for (int i = tid; i < nks * 64; i += MK_THREADS) {
-        const int ks = i >> 6, t = i & 15, k = ks * KW + ((i & 63) >> 4) * EPC;
-        const E *row = in + (size_t)(a.t0 + tb + min(t, nt - 1)) * st.ld_in + st.cols[5] + k;
-        float f[EPC];
-#pragma unroll
-        for (int e = 0; e < EPC; e += 4) {
-          const f32x4 q = fx_ldc_quad(row + e);
-#pragma unroll
-          for (int y = 0; y < 4; y++) f[e + y] = tanhf(q[y]);
-        }
-        u32x4 hi, lo;
-#pragma unroll
-        for (int w = 0; w < 4; w++) {
-          if constexpr (B16) {
-            const float x0 = f[(2 * w) % EPC], x1 = f[(2 * w + 1) % EPC];
-            hi[w] = pack2(x0, x1);
-            lo[w] = pack2(x0 - bf_lo(hi[w]), x1 - bf_hi(hi[w]));
-          } else {
-            hi[w] = __float_as_uint(f[w % EPC]);
-            lo[w] = 0u;
+          for (int e = 0; e < 4; e++) {
+            if (!real) xr[j][e] = xk[j][e] = xv[j][e] = xw[j][e] = 0.f;
+            un[e] = xk[j][e] * inv;
+            au[e] = mx_sigmoid(xa[j][e] + xab[e]) * un[e];
           }
+          const int at = (wave + j * MK_WAVES) * DPS + 4 * lane;
+          *(f32x4 *)(rv + at) = xr[j];
+          *(f32x4 *)(kv + at) = xk[j];
+          *(f32x4 *)(uv + at) = un;
+          *(f32x4 *)(av + at) = au;
+          *(f32x4 *)(wv + at) = xw[j];
+          *(f32x4 *)(vv + at) = xv[j];
         }
-        tw[(ks * 2) * 64 + (i & 63)] = hi;
-        if constexpr (B16) tw[(ks * 2 + 1) * 64 + (i & 63)] = lo;
       }
+      load_rows(min(tb + MX_TB, a.n - 1));
       __syncthreads();
-      // ---- decays of 16 channels x 16 tokens at a time
-      for (int ct = wave; ct < DQ; ct += MK_WAVES) {
-        f32x4 z = {0.f, 0.f, 0.f, 0.f};
-        if (ct < nd) {
-          const u32x4 *wt = (const u32x4 *)st.w.seg[0] + ((size_t)a.h * nd + ct) * nks * 64 + lane;
-          for (int ks = 0; ks < nks; ks++) {
-            const u32x4 w = wt[ks * 64];
-            z = fx_mma_k(E(), w, tw[(ks * 2) * 64 + lane], z);
-            if constexpr (B16) z = fx_mma_k(E(), w, tw[(ks * 2 + 1) * 64 + lane], z);
-          }
-        }
-        f32x4 w;
+      auto load_vec = [&](int j, MxDeltaVec<NI> &y, float (&v)[NC]) {
 #pragma unroll
-        for (int i = 0; i < 4; i++) {
-          const int d = ct * 16 + lg * 4 + i;
-          w[i] = d < D ? expf(-0.6065306597126334f / (1.f + expf(-(z[i] + w0[a.h * D + min(d, D - 1)])))) : 0.f;
+        for (int i = 0; i < NI; i++) {
+          const int at = j * DPS + i * 64 + lr * 4;
+          y.r[i] = *(const f32x4 *)(rv + at);
+          y.k[i] = *(const f32x4 *)(kv + at);
+          y.u[i] = *(const f32x4 *)(uv + at);
+          y.au[i] = *(const f32x4 *)(av + at);
+          y.w[i] = *(const f32x4 *)(wv + at);
         }
-        *(f32x4 *)(wv + lr * DPS + ct * 16 + lg * 4) = w;
+#pragma unroll
+        for (int q = 0; q < NC; q++) v[q] = vv[j * DPS + min(col + q, NI * 64 - 1)];
+      };
+      MxDeltaVec<NI> y;
+      float v[NC];
+      load_vec(0, y, v);
+      for (int j = 0; j < nt; j++) {
+        MxDeltaVec<NI> yn;
+        float vn[NC], o[NC];
+        load_vec(min(j + 1, nt - 1), yn, vn);
+        mx_delta_step<NI, NC>(S, y, v, o);
+        if (slices > 1) {
+          float *row = (float *)st.out2 + (size_t)(a.t0 + tb + j) * st.ld_out2 + a.h * Dp;
+          if (lr == 0) {
+#pragma unroll
+            for (int q = 0; q < NC; q++)
+              if (col + q < Dp) stc_f32(row + col + q, o[q]);
+          }
+        } else if (lr == 0) {
+#pragma unroll
+          for (int q = 0; q < NC; q++) ov[j * DPS + min(col + q, NI * 64 - 1)] = o[q];
+        }
+        y = yn;
+#pragma unroll
+        for (int q = 0; q < NC; q++) v[q] = vn[q];
       }
+      if (slices > 1) continue;
       __syncthreads();
-      // ---- tokens
-      for (int pass = 0; pass < passes; pass++) {
-        if (passes > 1) load_state(a, pass, a.p0 == 0 && tb == 0);
-        for (int j = 0; j < nt; j++) {
-          const size_t o4 = (size_t)(j * DPS + lg * 4);
-          float su[NB], so[NB], v[NB];
-#pragma unroll
-          for (int b = 0; b < NB; b++) {
-            su[b] = so[b] = 0.f;
-            v[b] = vv[j * DPS + min(((pass * NB + b) * MK_WAVES + wave) * 16, DP - 16) + lr];
-          }
-#pragma unroll
-          for (int i = 0; i < DQ; i++) {
-            const f32x4 q = *(const f32x4 *)(uv + o4 + i * 16);
-#pragma unroll
-            for (int b = 0; b < NB; b++)
-#pragma unroll
-              for (int e = 0; e < 4; e++) su[b] = fmaf(q[e], S[b][i][e], su[b]);
-          }
-#pragma unroll
-          for (int b = 0; b < NB; b++) su[b] = groups_sum(su[b]);
-#pragma unroll
-          for (int i = 0; i < DQ; i++) {
-            const f32x4 w = *(const f32x4 *)(wv + o4 + i * 16), q = *(const f32x4 *)(av + o4 + i * 16), k = *(const f32x4 *)(kv + o4 + i * 16),
-                        r = *(const f32x4 *)(rv + o4 + i * 16);
-#pragma unroll
-            for (int b = 0; b < NB; b++)
-#pragma unroll
-              for (int e = 0; e < 4; e++) {
-                S[b][i][e] = fmaf(k[e], v[b], fmaf(-q[e], su[b], w[e] * S[b][i][e]));
-                so[b] = fmaf(r[e], S[b][i][e], so[b]);
-              }
-          }
-#pragma unroll
-          for (int b = 0; b < NB; b++) {
-            so[b] = groups_sum(so[b]);
-            const int cb = (pass * NB + b) * MK_WAVES + wave;
-            if (lg == 0 && cb < nd) vv[j * DPS + cb * 16 + lr] = so[b];  // (v of these columns is this wavefront's own)
-          }
-        }
-        if (passes > 1) store_state(a, pass);
-      }
-      __syncthreads();
-      // ---- each head's output divided by its root mean square, weight, gate
+      // ---- the head's outputs divided by their root mean square, weight, gate
       for (int j = wave; j < nt; j += MK_WAVES) {
         const size_t t = a.t0 + tb + j;
-        float o[DP / 64], g[DP / 64], ss = 0.f;
+        const f32x4 g = fx_ldc_quad(in + t * st.ld_in + st.cols[3] + a.h * Dp + d4);
+        const f32x4 o = *(const f32x4 *)(ov + j * DPS + d4);
+        const float ss = 4 * lane < Dp ? o[0] * o[0] + o[1] * o[1] + o[2] * o[2] + o[3] * o[3] : 0.f;
+        const float rn = 1.f / sqrtf(wave_sum(ss) / (float)D + st.eps);
+        f32x4 q;
 #pragma unroll
-        for (int i = 0; i < DP / 64; i++) {
-          const int d = i * 64 + lane;
-          g[i] = fx_ldc(in + t * st.ld_in + st.cols[3] + a.h * D + min(d, D - 1));
-          o[i] = d < D ? vv[j * DPS + d] : 0.f;
-          ss += o[i] * o[i];
-        }
-        const float inv = 1.f / sqrtf(wave_sum(ss) / (float)D + st.eps);
-#pragma unroll
-        for (int i = 0; i < DP / 64; i++) {
-          const int d = i * 64 + lane;
-          if (d < D) fx_stc((E *)st.out + t * st.ld_out + a.h * D + d, fx_round<E>((o[i] * inv) * nw[a.h * D + d] / (1.f + expf(-g[i]))));
-        }
+        for (int e = 0; e < 4; e++) q[e] = (o[e] * rn) * xnw[e] * mx_sigmoid(g[e]);
+        if (4 * lane < Dp) fx_stc_quad((E *)st.out + t * st.ld_out + a.h * Dp + 4 * lane, q);
       }
     }
-    if (passes == 1) store_state(a, 0);
+    mx_delta_store<NI, NC>(S, a.state, col, lr, Dp);
   }
-  mx_glu<E>(st, c, M);
+  c.wrote_through = true;
+}
+// Head outputs of an iteration whose units were dealt in slices: a wavefront per (token, head).
+template <typename E>
+__device__ __forceinline__ void stage_mx_delta_out(CStage &st, Ctx &c, int M) {
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int D = st.head_dim, Dp = (D + 15) / 16 * 16, H = st.num_q_heads, d4 = min(4 * lane, Dp - 4);
+  barrier_wait(c);
+  for (int i = mx_spread(c) + wave * c.G; i < M * H; i += c.G * MK_WAVES) {
+    const int t = i / H, h = i - t * H;
+    const f32x4 o = fx_ldc_quad((const float *)st.out2 + (size_t)t * st.ld_out2 + h * Dp + d4), g = fx_ldc_quad((const E *)st.in + (size_t)t * st.ld_in + st.cols[3] + h * Dp + d4),
+                w = *(const f32x4 *)((const float *)st.norm_w + h * Dp + d4);
+    const float ss = 4 * lane < Dp ? o[0] * o[0] + o[1] * o[1] + o[2] * o[2] + o[3] * o[3] : 0.f;
+    const float rn = 1.f / sqrtf(wave_sum(ss) / (float)D + st.eps);
+    f32x4 q;
+#pragma unroll
+    for (int e = 0; e < 4; e++) q[e] = (o[e] * rn) * w[e] * mx_sigmoid(g[e]);
+    if (4 * lane < Dp) fx_stc_quad((E *)st.out + (size_t)t * st.ld_out + h * Dp + 4 * lane, q);
+  }
   c.wrote_through = true;
 }
 template <typename E>
-__device__ __forceinline__ void stage_mx_delta(CStage &st, Ctx &c, const MkRuntime &rt, int M, char *smem) {
-  if (st.head_dim <= 64) stage_mx_delta_t<E, 4, 1>(st, c, rt, M, smem);
-  else if (st.head_dim <= 128) stage_mx_delta_t<E, 8, 2>(st, c, rt, M, smem);
-  else stage_mx_delta_t<E, 16, 1>(st, c, rt, M, smem);
+__device__ __forceinline__ void stage_mx_delta(CStage &st, Ctx &c, const MkRuntime &rt, int M, bool single, char *smem) {
+  const int D = st.head_dim, Dp = (D + 15) / 16 * 16;
+  c.mx_split = false;
+  if (single && D <= 128) {
+    if (D <= 64) stage_mx_delta_single<E, 1, 4>(st, c, rt, M, smem);
+    else stage_mx_delta_single<E, 2, 8>(st, c, rt, M, smem);
+    return;
+  }
+  // workgroups per (request, head) if every wavefront took as few columns as it can, and if they took all
+  const int units = mx_delta_units(c, M).nreq * st.num_q_heads, fine = D <= 64 ? (Dp + 15) / 16 : (Dp + 31) / 32;
+  const bool deal = units * fine <= c.G;
+  if (D <= 64) {
+    c.mx_split = deal && fine > 1;
+    if (deal) stage_mx_delta_multi<E, 1, 1>(st, c, rt, M, fine, smem);
+    else stage_mx_delta_multi<E, 1, 4>(st, c, rt, M, 1, smem);
+  } else if (D <= 128) {
+    c.mx_split = deal && fine > 1;
+    if (deal) stage_mx_delta_multi<E, 2, 2>(st, c, rt, M, fine, smem);
+    else stage_mx_delta_multi<E, 2, 8>(st, c, rt, M, 1, smem);
+  } else {
+    c.mx_split = true;
+    stage_mx_delta_multi<E, 4, 2>(st, c, rt, M, fine, smem);
+  }
 }

@@ -70,7 +70,9 @@ enum MkOp {
   MK_OP_MX_HEAD_LINEAR = 23, // one small matrix per head; optionally gelu(...) * a per-token table row
   MK_OP_MX_LATENT_ATTN = 24, // attention in the latent space, one shared key/value row per position
   MK_OP_MX_LATENT_MERGE = 25,  // chunks of the latent attention (iterations in which some request was split)
-  MK_OP_MX_DELTA = 26,       // generalised delta rule: recurrent state per request and head, gated activation beside it
+  MK_OP_MX_DECAY = 26,       // decays of the delta rule (low-rank product of tanh), gated activation beside it
+  MK_OP_MX_DELTA = 27,       // generalised delta rule: recurrent state per request and head
+  MK_OP_MX_DELTA_OUT = 28,   // norm and gate of its outputs (iterations that dealt heads in slices)
 };
 
 enum MkStageFlags {
@@ -87,13 +89,14 @@ enum MkStageFlags {
   MK_F_ADDNORM = 1024,   // LINEAR (set together with MK_F_NORM): the norm in front is an FX_ADDNORM; a single-token iteration forms it inside this stage
   MK_F_PRENORM = 4096,   // LINEAR (set together with MK_F_NORM): the norm in front is an MX_PRENORM; a single-token iteration forms it inside this stage
   MK_F_GELU_TABLE = 8192,  // MX_HEAD_LINEAR: out = gelu(acc) * table[id][n]
+  MK_F_JOIN = 16384,     // LINEAR: a single-token iteration adds the result to the residual stream itself (the MX_PRENORM behind is multi-token only)
   MK_F_RES_EARLY = 2048, // FX_ADDNORM / LINEAR+ADDNORM: the stage before this one does not write the residual rows, so they may be requested before its barrier
 };
 
 #define MK_MX_MAX_GROUPS 256     // parts of a row with a norm of their own
 #define MK_MX_MAX_NORM_ROW 4096  // longest query latent / key latent row a wavefront normalises
 #define MK_MX_MAX_LATENT 512     // key latent size of the latent attention
-#define MK_MX_MAX_LATENT_CHUNKS 40  // 64-byte operand rows of a cached latent (latent + rotated part)
+#define MK_MX_MAX_CHUNKS 64      // split of a request's cached latents (one lane of the merging wavefront each)
 #define MK_MX_MAX_DELTA_DIM 256  // head size of the recurrence
 #define MK_MX_MAX_RANK 1024      // low-rank decay projection
 
@@ -170,13 +173,16 @@ struct MkStage {
   // mix stages (mk_mix.hip)
   const void *y_norm_w;  // MX_PRENORM / LINEAR+PRENORM: fp32 weight of the RMS norm of the summand (null: none)
   int norm_groups;       // ... parts of the output norm (0: no norm)
-  int rank;              // key latent size (latent stages); padded low rank of the decay projection (MX_DELTA)
-  int cols[6];           // columns of `in`: MX_LATENT_PREP q latent, k latent; MX_LATENT_ATTN rotated query part of a head; MX_DELTA r k v g a w1
-  // gated activation beside MX_LATENT_PREP / MX_DELTA: out = a / (1 + exp(-beta a)) * (b + bias), a = min(gate, limit), b = clamp(up, -limit, limit)
+  int rank;              // key latent size (latent stages)
+  int nk;                // MX_LATENT_ATTN: operand rows of a cached latent its instantiation holds
+  int cols[5];           // columns of `in`: MX_LATENT_PREP q latent, k latent, rotated key part; MX_LATENT_ATTN rotated query part of a head; MX_DELTA r k v g a
+  const void *in2;       // MX_DELTA: decays, 32-bit rows (out2 / ld_out2: unnormalised outputs)
+  int ld_in2, pad_in2;
+  // gated activation beside MX_LATENT_PREP / MX_DECAY: out = a / (1 + exp(-beta a)) * (b + bias), a = min(gate, limit), b = clamp(up, -limit, limit)
   void *glu_out;
   int glu_n, ld_glu, glu_gate, glu_up;
   float glu_limit, glu_beta, glu_bias;
-  int pad_mx[13];
+  int pad_mx[9];
 };
 static_assert(sizeof(MkStage) % 64 == 0, "a descriptor is whole scalar-cache lines");
 

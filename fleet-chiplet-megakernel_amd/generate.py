@@ -14,7 +14,7 @@ import time
 import torch
 
 from mirage.mpk import MPK, MirageModelConfig, MPKMetadata, ServingSession
-from mirage.mpk.models.suborax.builder import SuboraxConfig, random_state_dict
+from mirage.mpk.models import dodonex, suborax
 
 
 def suborax_shape(width=4096, heads=32, kv_heads=8, dim=128, vdim=128, ff=12288, layers=36, vocab=151936) -> dict:
@@ -26,7 +26,27 @@ def suborax_shape(width=4096, heads=32, kv_heads=8, dim=128, vdim=128, ff=12288,
             "layers": [layer] * layers}
 
 
-SHAPES = {"suborax-8b": dict(), "suborax-2k": dict(width=2048, heads=32, kv_heads=4, ff=6144)}
+def dodonex_shape(width=4096, heads=32, dim=128, rot_dim=64, vdim=128, q_rank=1536, kv_rank=512, delta_heads=32, delta_dim=128, low_rank=128, ff=12288, side=256, layers=36,
+                  vocab=151936) -> dict:
+    """A Dodonex config.json of the given sizes, latent attention and delta rule by turns."""
+    mlp = {"kind": "dense", "ff": ff, "limit": 7.0}
+    latent = {"type": "latent_attention", "mlp": mlp, "mixer": {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim, "q_rank": q_rank, "kv_rank": kv_rank,
+                                                               "rot": {"base": 5e5, "dims": rot_dim}, "scale": (dim + rot_dim) ** -0.5}}
+    delta = {"type": "general_delta", "mlp": mlp, "mixer": {"heads": delta_heads, "dim": delta_dim, "low_rank": low_rank}}
+    return {"architecture": "Dodonex", "vocab": vocab, "width": width, "norm": {"eps": 1e-6, "groups": 4}, "residual_mult": 1.0, "embedding": {"scale": 1.0}, "logit_scale": 1.0,
+            "token_side": {"dim": side}, "layers": [delta if i % 2 else latent for i in range(layers)]}
+
+
+# name -> (config.json of a shape, its sizes)
+SHAPES = {"suborax-8b": (suborax_shape, {}), "suborax-2k": (suborax_shape, dict(width=2048, heads=32, kv_heads=4, ff=6144)),
+          "dodonex-8b": (dodonex_shape, {}), "dodonex-2k": (dodonex_shape, dict(width=2048, heads=16, q_rank=768, delta_heads=32, delta_dim=64, low_rank=64, ff=6144))}
+
+
+def random_model(config: dict):
+    """(MirageModelConfig with random-init weights, the reader's form of the config) of a parsed config.json."""
+    kind, module = {"Suborax": (suborax.SuboraxConfig, suborax), "Dodonex": (dodonex.DodonexConfig, dodonex)}[config["architecture"]]
+    sizes = kind.from_dict(config)
+    return MirageModelConfig(architecture=config, state_dict=module.random_state_dict(sizes)), sizes
 
 
 class Generator:
@@ -98,11 +118,9 @@ def main(argv=None):
             cfg = json.load(f)
         vocab, source = cfg.get("vocab") or cfg["vocab_size"], dict(model_path=args.model_path)
     else:
-        shape = dict(SHAPES[args.random])
-        if args.layers:
-            shape["layers"] = args.layers
-        cfg = suborax_shape(**shape)
-        vocab, source = cfg["vocab"], dict(model_config=MirageModelConfig(architecture=cfg, state_dict=random_state_dict(SuboraxConfig.from_dict(cfg))))
+        make, shape = SHAPES[args.random]
+        cfg = make(**shape, **({"layers": args.layers} if args.layers else {}))
+        vocab, source = cfg["vocab"], dict(model_config=random_model(cfg)[0])
     prompts = [[int(x) for x in p.split(",")] for p in args.prompt_ids]
     if not prompts:
         prompts = [torch.randint(0, vocab, (args.prompt_length,), generator=torch.Generator().manual_seed(r)).tolist() for r in range(args.batch or 1)]

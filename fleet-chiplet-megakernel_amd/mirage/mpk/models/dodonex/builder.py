@@ -31,6 +31,10 @@ from ...persistent_kernel import PersistentKernel, latent_row_dim, operand_row, 
 from ....kernel import bfloat16, float32, int64
 from ..graph_builder import GraphBuilder, MirageModelConfig
 
+def _up(n: int, m: int) -> int:
+    return -(-n // m) * m
+
+
 GLU_BETA, GLU_BIAS = 1.702, 1.0  # feed-forward: g sigmoid(1.702 g) (u + 1)
 
 
@@ -66,8 +70,12 @@ class DeltaMixer:
     low_rank: Optional[int]  # None until the weights are seen: the shape of w1 gives it
 
     @property
+    def padded_dim(self):
+        return _up(self.dim, 16)
+
+    @property
     def out_cols(self):
-        return self.heads * self.dim
+        return self.heads * self.padded_dim
 
     def tensor_shapes(self, W):
         n = self.heads * self.dim
@@ -167,10 +175,6 @@ def random_state_dict(cfg: DodonexConfig, seed: int = 0, device="cuda", std: flo
     return out
 
 
-def _up(n: int, m: int) -> int:
-    return -(-n // m) * m
-
-
 @register_model_builder("Dodonex")
 class DodonexBuilder(GraphBuilder):
     owns_kv_cache = True
@@ -227,6 +231,11 @@ class DodonexBuilder(GraphBuilder):
             w = torch.nn.functional.pad(w, (0, cols - w.shape[1], 0, rows - w.shape[0]))
         return w
 
+    def _head_vector(self, name: str, m: DeltaMixer):
+        """Attach a per-channel vector in fp32, every head zero-padded to a multiple of 16."""
+        v = self._w(name).to(torch.float32).view(m.heads, m.dim)
+        return self._attach(torch.nn.functional.pad(v, (0, m.padded_dim - m.dim)).reshape(-1), name)
+
     def _vector(self, name: str, size: int = None, factor: float = 1.0):
         """Attach a norm weight or an offset in fp32, zero-padded to `size`."""
         v = self._w(name).to(torch.float32) * factor
@@ -262,7 +271,7 @@ class DodonexBuilder(GraphBuilder):
         for i, l in enumerate(self.config.layers):
             m = l.mixer
             if isinstance(m, DeltaMixer):
-                d = _up(m.dim, 16)
+                d = m.padded_dim
                 self.state[i] = torch.zeros(mpk.max_num_batched_requests, m.heads, d, d, dtype=torch.float32, device=mpk.device)
             elif m.kv_from is None:
                 self.latent_cache[i] = torch.zeros(mpk.max_num_pages, mpk.page_size, latent_row_dim(m.kv_rank, m.rot_dim, self.dtype), dtype=self.dtype, device=mpk.device)
@@ -323,7 +332,8 @@ class DodonexBuilder(GraphBuilder):
                     dkv = self._w(p + "mix.dkv")
                     sections += [("c", dkv[:m.kv_rank], _up(m.kv_rank, 16)), ("rot", dkv[m.kv_rank:], _up(m.rot_dim, 16))]
             else:
-                sections += [(n, self._w(p + "mix." + n), _up(m.out_cols, 16)) for n in "rkvga"]
+                by_head = lambda w: torch.nn.functional.pad(w.view(m.heads, m.dim, -1), (0, 0, 0, m.padded_dim - m.dim)).reshape(m.out_cols, -1)
+                sections += [(n, by_head(self._w(p + "mix." + n)), m.out_cols) for n in "rkvga"]
                 sections.append(("w1", self._w(p + "mix.w1"), _up(m.low_rank, KW)))
             if F:
                 sections += [(n, self._w(p + "mlp." + n), F) for n in ("gate", "up")]
@@ -365,12 +375,16 @@ class DodonexBuilder(GraphBuilder):
                 uv = operand_tiles(self._w(p + "mix.uv").to(self.dtype).view(m.heads, m.vdim, m.kv_rank))
                 mpk.head_linear_layer(input=ol, weight=self._attach(uv, p + "mix.uv"), output=both, heads=m.heads, n=m.vdim, k=Rp, in_stride=Rp, out_stride=m.vdim)
             else:
-                w2 = operand_tiles(self._w(p + "mix.w2").to(self.dtype).view(m.heads, m.dim, m.low_rank))
-                mpk.general_delta_layer(input=rows, decay_weight=self._attach(w2, p + "mix.w2"), decay_offset=self._vector(p + "mix.w0"),
-                                        removal_offset=self._vector(p + "mix.a.b"), norm_weight=self._vector(p + "mix.norm"),
-                                        state=self._attach(self.state[i], p + "state"), state_slots=slots, output=both, heads=m.heads, dim=m.dim,
-                                        low_rank=_up(m.low_rank, KW), columns=tuple(col[n] for n in ("r", "k", "v", "g", "a", "w1")), eps=c.eps, glu=glu)
-            w_out = self._matrix(p + "mix.o", cols=A)
+                w2 = operand_tiles(by_head(self._w(p + "mix.w2").to(self.dtype))[None])
+                mpk.general_delta_layer(input=rows, decay_weight=self._attach(w2, p + "mix.w2"), decay_offset=self._head_vector(p + "mix.w0", m),
+                                        removal_offset=self._head_vector(p + "mix.a.b", m), norm_weight=self._head_vector(p + "mix.norm", m),
+                                        state=self._attach(self.state[i], p + "state"), state_slots=slots, workspace=self._rows("delta_work", 2 * m.out_cols, float32),
+                                        output=both, heads=m.heads, dim=m.dim, low_rank=_up(m.low_rank, KW),
+                                        columns=tuple(col[n] for n in ("r", "k", "v", "g", "a", "w1")), eps=c.eps, glu=glu)
+            w_out = self._matrix(p + "mix.o")
+            if not latent:
+                w_out = by_head(w_out.T).T
+            w_out = torch.nn.functional.pad(w_out, (0, A - w_out.shape[1]))
             if F:
                 w_out = torch.cat([w_out, self._matrix(p + "mlp.down", cols=F)], dim=1)
             mpk.linear_layer(input=both, weight=self._attach(w_out, p + "out"), output=y, **one)

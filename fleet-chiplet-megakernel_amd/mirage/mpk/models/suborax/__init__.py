@@ -1,3 +1,3 @@
-from .builder import SuboraxBuilder, SuboraxConfig
+from .builder import SuboraxBuilder, SuboraxConfig, random_state_dict
 
-__all__ = ["SuboraxBuilder", "SuboraxConfig"]
+__all__ = ["SuboraxBuilder", "SuboraxConfig", "random_state_dict"]

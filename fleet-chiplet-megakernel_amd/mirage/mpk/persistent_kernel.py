@@ -714,17 +714,20 @@ class PersistentKernel:
                    [num_heads, latent_rank, rot_dims, head_stride, rot_column, _f32_bits(scale)])
 
     def general_delta_layer(self, input: DTensor, decay_weight: DTensor, decay_offset: DTensor, removal_offset: DTensor, norm_weight: DTensor, state: DTensor,
-                            state_slots: DTensor, output: DTensor, heads: int, dim: int, low_rank: int, columns: tuple, eps: float, glu: tuple = None):
+                            state_slots: DTensor, workspace: DTensor, output: DTensor, heads: int, dim: int, low_rank: int, columns: tuple, eps: float,
+                            glu: tuple = None):
         """Generalised delta rule per head, state S [dim, dim] carried from iteration to iteration in fp32 (zero where a request
         begins): S <- diag(w) S - (a u)(u^T S) + k v^T, o = S^T r, u = k / sqrt(sum k^2 + 1e-6), a = sigmoid(input + removal_offset),
         w = exp(-exp(-1/2) sigmoid(W2 tanh(low-rank input) + decay_offset)); output = o / rms(o) * norm_weight * sigmoid(gate
         input).  `columns`: where r, k, v, gate, a and the low-rank projection (low_rank wide, whole operand rows) begin in the
-        input rows.  decay_weight: operand_tiles of W2 per head.  state: [slots, heads, dim and dim rounded up to 16];
-        state_slots: int32, the state slot of every batch slot (the on-GPU schedulers permute it, a host fills it per pass)."""
+        input rows.  A head takes `dim` rounded up to 16 columns there, in the vectors and in the output; what is behind `dim` is
+        zero in r, k and v.  decay_weight: operand_tiles of W2 padded likewise; workspace: fp32 rows of 2 x heads x that size;
+        state: [slots, heads, that size, that size]; state_slots: int32, the state slot of every batch slot (the on-GPU
+        schedulers permute it, a host fills it per pass)."""
         out, p = self._glu_params(glu)
         self._task("general_delta", (1, 1, 1), (256, 1, 1),
                    [(input, _REPL, -1), (decay_weight, _REPL, -1), (decay_offset, _REPL, -1), (removal_offset, _REPL, -1), (norm_weight, _REPL, -1), (state, _REPL, -1),
-                    (state_slots, _REPL, -1), (out, _REPL, -1), (output, _REPL, -1)], [heads, dim, low_rank, *columns, _f32_bits(eps)] + p)
+                    (state_slots, _REPL, -1), (workspace, _REPL, -1), (out, _REPL, -1), (output, _REPL, -1)], [heads, dim, low_rank, *columns, _f32_bits(eps)] + p)
 
     # layers of the reference that are outside the one-GPU decode path
     def tensor_init_layer(self, *args, **kwargs):
