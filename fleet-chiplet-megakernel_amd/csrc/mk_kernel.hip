@@ -4189,7 +4189,7 @@ __device__ __forceinline__ void run_stage_program(const MkRuntime &rt, const MkR
         case MK_OP_MX_HEAD_LINEAR: stage_mx_head_linear<E, MAXM>(st, c, M, smem); break;
         case MK_OP_MX_LATENT_ATTN: stage_mx_latent_attn<E>(st, c, rt, M, smem); break;
         case MK_OP_MX_LATENT_MERGE: stage_mx_latent_merge<E>(st, c, rt, M); break;
-        case MK_OP_MX_DECAY: stage_mx_decay<E, MAXM>(st, c, M, smem); break;
+        case MK_OP_MX_DECAY: stage_mx_head_linear_t<E, 1, MX_DECAY, false>(st, c, M, smem); break;
         case MK_OP_MX_DELTA: stage_mx_delta<E>(st, c, rt, M, MAXM == 1 || single, smem); break;
         case MK_OP_MX_DELTA_OUT: stage_mx_delta_out<E>(st, c, M); break;
 #endif

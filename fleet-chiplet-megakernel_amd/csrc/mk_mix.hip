@@ -12,6 +12,20 @@
 // Index that deals consecutive work over the dies first (a handful of units then spreads over all of them).
 __device__ __forceinline__ int mx_spread(const Ctx &c) { return c.even_xcds ? c.rank * c.nxcd + c.xi : c.vid; }
 
+// Index of a wavefront among those of the grid, the wavefronts that do not poll the barrier first.
+__device__ __forceinline__ int mx_wave_item(const Ctx &c, int wave) { return mx_spread(c) + (MK_WAVES - 1 - wave) * c.G; }
+
+// 1 / (1 + exp(-z)) and tanh(z): hardware exp2 and reciprocal next to 16-bit operands, library functions in the 32-bit build
+__device__ __forceinline__ float mx_sigmoid(uint16_t, float z) { return __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z)); }
+__device__ __forceinline__ float mx_sigmoid(float, float z) { return 1.f / (1.f + expf(-z)); }
+__device__ __forceinline__ float mx_tanh(uint16_t, float z) { return 1.f - 2.f * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(2.8853900817779268f * z)); }
+__device__ __forceinline__ float mx_tanh(float, float z) { return tanhf(z); }
+
+// A quad of 32-bit values written through to memory in one store (the same visibility as stc_f32).
+__device__ __forceinline__ void mx_stc_quad(float *p, f32x4 v) {
+  asm volatile("global_store_dwordx4 %0, %1, off sc1" ::"v"((const MK_GLOBAL void *)(unsigned long long)p), "v"(v) : "memory");
+}
+
 // ----------------------------------------------------------------------------- residual sum + norm in parts
 // v = x + alpha * f(y),  f(y) = y or y / sqrt(mean(y^2) + norm_eps) * y_norm_w;  out2 = v (32-bit);  out = the RMS norm of v in
 // st.norm_groups equal parts times norm_w (norm_groups 0: v itself), rounded to E.  Rows are st.n long, st.k of them real (the
@@ -325,7 +339,7 @@ __device__ __forceinline__ void mx_glu(CStage &st, Ctx &c, int M) {
 #pragma unroll
     for (int e = 0; e < 4; e++) {
       const float g = fminf(a[e], lim), u = fminf(fmaxf(b[e], -lim), lim);
-      o[e] = g / (1.f + expf(-beta * g)) * (u + bias);
+      o[e] = g * mx_sigmoid(E(), beta * g) * (u + bias);
     }
     fx_stc_quad((E *)st.glu_out + (size_t)t * st.ld_glu + d, o);
   }
@@ -370,8 +384,8 @@ __device__ __forceinline__ void stage_mx_latent_prep(CStage &st, Ctx &c, const M
   constexpr int KW = FxType<E>::KW;
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int R = st.rank, rot = st.rot_dims, half = rot / 2, nrc = (R + KW - 1) / KW, nkc = nrc + (rot + KW - 1) / KW, ps = rt.page_size;
-  const int per = st.k_cache ? 2 : 1, total = M * per, w0 = mx_spread(c);
-  for (int i = w0 + wave * c.G; i < total; i += c.G * MK_WAVES) {
+  const int per = st.k_cache ? 2 : 1, total = M * per;
+  for (int i = mx_wave_item(c, wave); i < total; i += c.G * MK_WAVES) {
     const int t = i / per;
     const E *row = (const E *)st.in + (size_t)t * st.ld_in;
     if (i - t * per == 0) {
@@ -414,11 +428,11 @@ __device__ __forceinline__ void stage_mx_head_linear_t(CStage &st, Ctx &c, int M
   constexpr int EPC = FxType<E>::EPC, KW = FxType<E>::KW, KB = MT == 4 ? 4 : SPLIT ? 16 : EPI == MX_DECAY ? 4 : 8, B16 = sizeof(E) == 2;
   static_assert(!SPLIT || MT == 1, "");
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lr = lane & 15, lg = lane >> 4;
-  const int N = st.n, nks = st.k / KW, nt = (N + 15) / 16, mts = SPLIT ? (M + 15) / 16 : 1, items = st.groups * nt * mts;
+  const int N = st.n, nks = st.k / KW, nt = (N + 15) / 16, mts = MT == 1 ? (M + 15) / 16 : 1, items = st.groups * nt * mts;
   const int kq = SPLIT ? (nks + MK_WAVES - 1) / MK_WAVES : nks;
   const int kb = SPLIT ? min(nks, wave * kq) : 0, ke = SPLIT ? min(nks, kb + kq) : nks;
   const u32x4 *W = (const u32x4 *)st.w.seg[0];
-  const int i0 = SPLIT ? mx_spread(c) : mx_spread(c) + wave * c.G, di = SPLIT ? c.G : c.G * MK_WAVES;
+  const int i0 = SPLIT ? mx_spread(c) : mx_wave_item(c, wave), di = SPLIT ? c.G : c.G * MK_WAVES;
   f32x4 *red = (f32x4 *)smem;
   const u32x4 zero = {0u, 0u, 0u, 0u};
   u32x4 a[KB];
@@ -432,7 +446,7 @@ __device__ __forceinline__ void stage_mx_head_linear_t(CStage &st, Ctx &c, int M
   if (tid == 0) __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "agent");
   barrier_wait(c);
   for (int i = i0; i < items; i += di) {
-    const int tile = i / mts, mt0 = SPLIT ? i - tile * mts : 0, h = tile / nt, n0 = (tile - h * nt) * 16 + lg * 4;
+    const int tile = i / mts, mt0 = i - tile * mts, h = tile / nt, n0 = (tile - h * nt) * 16 + lg * 4;
     const E *xr[MT];
 #pragma unroll
     for (int m = 0; m < MT; m++) xr[m] = (const E *)st.in + (size_t)min((mt0 + m) * 16 + lr, M - 1) * st.ld_in + (size_t)h * st.ld_in_slot + lg * EPC;
@@ -456,11 +470,11 @@ __device__ __forceinline__ void stage_mx_head_linear_t(CStage &st, Ctx &c, int M
 #pragma unroll
             for (int q = 0; q < 4; q++) {
               if constexpr (B16) {
-                const float x0 = tanhf(bf_lo(b[j][m][q])), x1 = tanhf(bf_hi(b[j][m][q]));
+                const float x0 = mx_tanh(E(), bf_lo(b[j][m][q])), x1 = mx_tanh(E(), bf_hi(b[j][m][q]));
                 hi[q] = pack2(x0, x1);
                 lo[q] = pack2(x0 - bf_lo(hi[q]), x1 - bf_hi(hi[q]));
               } else {
-                hi[q] = __float_as_uint(tanhf(__uint_as_float(b[j][m][q])));
+                hi[q] = __float_as_uint(mx_tanh(E(), __uint_as_float(b[j][m][q])));
               }
             }
             acc[m] = fx_mma_k(E(), w, hi, acc[m]);
@@ -491,7 +505,7 @@ __device__ __forceinline__ void stage_mx_head_linear_t(CStage &st, Ctx &c, int M
         for (int q = 0; q < 4; q++) f[q] = fx_val(e[min(n0 + q, N - 1)]);
 #pragma unroll
         for (int q = 0; q < 4; q++) {
-          const float z = r[q], th = tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z));
+          const float z = r[q], th = mx_tanh(E(), 0.7978845608028654f * (z + 0.044715f * z * z * z));
           r[q] = id < 0 ? 0.f : 0.5f * z * (1.f + th) * f[q];
         }
       }
@@ -499,7 +513,7 @@ __device__ __forceinline__ void stage_mx_head_linear_t(CStage &st, Ctx &c, int M
         const f32x4 w0 = *(const f32x4 *)((const float *)st.q_norm_w + n0);
         f32x4 d;
 #pragma unroll
-        for (int q = 0; q < 4; q++) d[q] = expf(-0.6065306597126334f / (1.f + expf(-(r[q] + w0[q]))));
+        for (int q = 0; q < 4; q++) d[q] = expf(-0.6065306597126334f * mx_sigmoid(E(), r[q] + w0[q]));
         fx_stc_quad((float *)st.out2 + (size_t)t * st.ld_out2 + n0, d);
       } else {
         fx_stc4((E *)st.out + (size_t)t * st.ld_out + (size_t)h * st.ld_out_slot, n0, N, r);
@@ -515,17 +529,12 @@ __device__ __forceinline__ void stage_mx_head_linear(CStage &st, Ctx &c, int M, 
     if (st.flags & MK_F_GELU_TABLE) stage_mx_head_linear_t<E, 1, MX_GELU, true>(st, c, M, smem);
     else stage_mx_head_linear_t<E, 1, MX_PLAIN, true>(st, c, M, smem);
   } else if (st.flags & MK_F_GELU_TABLE) {
-    stage_mx_head_linear_t<E, MAXM == 1 ? 1 : 4, MX_GELU, false>(st, c, M, smem);
-  } else if (MAXM == 1 || M <= 16) {
+    stage_mx_head_linear_t<E, 1, MX_GELU, false>(st, c, M, smem);
+  } else if (MAXM == 1 || st.groups * ((st.n + 15) / 16) * ((M + 15) / 16) <= MK_WAVES * c.G) {
     stage_mx_head_linear_t<E, 1, MX_PLAIN, false>(st, c, M, smem);
   } else {
     stage_mx_head_linear_t<E, 4, MX_PLAIN, false>(st, c, M, smem);
   }
-}
-template <typename E, int MAXM>
-__device__ __forceinline__ void stage_mx_decay(CStage &st, Ctx &c, int M, char *smem) {
-  if (MAXM == 1 || M <= 16) stage_mx_head_linear_t<E, 1, MX_DECAY, false>(st, c, M, smem);
-  else stage_mx_head_linear_t<E, 4, MX_DECAY, false>(st, c, M, smem);
 }
 
 // ----------------------------------------------------------------------------- latent attention
@@ -581,7 +590,7 @@ template <typename E, int NK, int SUB, int VBW, int RT>
 __device__ __forceinline__ void stage_mx_latent_attn_t(CStage &st, Ctx &c, const MkRuntime &rt, int M, char *smem) {
   using X = FxType<E>;
   constexpr int EPC = X::EPC, KW = X::KW, B16 = sizeof(E) == 2, TPOS = 16 * SUB, PARTS = MK_WAVES / SUB, KC = (NK + PARTS - 1) / PARTS;
-  constexpr int QN = RT * NK * 64 / MK_THREADS;
+  constexpr int QN = RT * NK * 64 / MK_THREADS, GRP = NK % 6 == 0 ? 6 : 5;
   static_assert(RT * NK % 4 == 0, "whole rounds of query operands");
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lr = lane & 15, lg = lane >> 4;
   const int H = st.num_q_heads, R = st.rank, rot = st.rot_dims, half = rot / 2;
@@ -655,50 +664,80 @@ __device__ __forceinline__ void stage_mx_latent_attn_t(CStage &st, Ctx &c, const
     }
     if (a.tb < a.te && !(u == u0 && early)) load_tile(a.tb, rt.kv_indices[a.pages + a.tb * TPOS / ps]);
     __syncthreads();  // LDS reuse across units
-    const int pg_lo = a.tb * TPOS / ps, npg = a.tb < a.te ? (a.te * TPOS - 1) / ps - pg_lo + 1 : 0;
+    const int pg_lo = a.tb * TPOS / ps, npg = a.tb + 1 < a.te ? (a.te * TPOS - 1) / ps - pg_lo + 1 : 0;  // (pages of the tiles behind the first)
     for (int i = tid; i < npg; i += MK_THREADS) spg[i] = rt.kv_indices[a.pages + min(pg_lo + i, a.p / ps)];
-    // ---- query rows in operand order: latent parts, then (over the zeros left for it) the rotated part
+    // ---- query rows in operand order: latent parts, and (in the zeros left for it) the rotated part.  A wavefront takes every
+    // fourth operand row, so which one it is and where it goes are scalars; a lane always has the same query row of a row tile.
     {
-      u32x4 q[QN];
+      const E *ql[RT], *qr[RT];
+      const float *ct[RT], *sn[RT];
+      bool real[RT];
+#pragma unroll
+      for (int q = 0; q < RT; q++) {
+        const int r = q * 16 + lr, Rw = a.r0 + min(r, a.nrows - 1), t = a.t0 + Rw / H, h = Rw % H, pos = c.sh_tok[t];
+        real[q] = r < a.nrows;
+        ql[q] = (const E *)st.q_ws + (size_t)t * st.ld_qws + (size_t)h * Rp + lg * EPC;
+        qr[q] = (const E *)st.in + (size_t)t * st.ld_in + (size_t)h * st.ld_in_slot + st.cols[0];
+        ct[q] = (const float *)st.cos_tab + (size_t)pos * st.ld_cos;
+        sn[q] = (const float *)st.sin_tab + (size_t)pos * st.ld_cos;
+      }
+      u32x4 v[QN];
 #pragma unroll
       for (int k = 0; k < QN; k++) {
-        const int i = tid + k * MK_THREADS, rc = i >> 6, rtile = rc / NK, ch = rc - rtile * NK, Rw = a.r0 + min(rtile * 16 + (i & 15), a.nrows - 1);
-        q[k] = ldc_16B((const u32x4 *)((const E *)st.q_ws + (size_t)(a.t0 + Rw / H) * st.ld_qws + (size_t)(Rw % H) * Rp + min(ch, nrc - 1) * KW + ((i & 63) >> 4) * EPC));
+        const int rc = wave + k * MK_WAVES, q = rc >= NK, ch = rc - q * NK;
+        v[k] = ldc_16B((const u32x4 *)(ql[RT == 1 ? 0 : q] + min(ch, nrc - 1) * KW));
+      }
+      // parts of 16-byte words: dims d0 .. of the rotated part and their partners half a part away
+      if ((half % EPC) == 0) {
+        for (int rc = wave; rc < RT * npc; rc += MK_WAVES) {
+          const int q = rc >= npc, d0 = (rc - q * npc) * KW + lg * EPC, dc = min(d0, rot - EPC), k0 = dc < half ? dc : dc - half;
+          const E *x = qr[RT == 1 ? 0 : q];
+          const float *cs = ct[RT == 1 ? 0 : q] + k0, *sv = sn[RT == 1 ? 0 : q] + k0;
+          const f32x4 x0 = fx_ldc_quad(x + dc), y0 = fx_ldc_quad(x + (dc < half ? dc + half : k0)), c0 = *(const f32x4 *)cs, s0 = *(const f32x4 *)sv;
+          f32x4 x1, y1, c1, s1;
+          if constexpr (B16) {
+            x1 = fx_ldc_quad(x + dc + 4);
+            y1 = fx_ldc_quad(x + (dc < half ? dc + half : k0) + 4);
+            c1 = *(const f32x4 *)(cs + 4);
+            s1 = *(const f32x4 *)(sv + 4);
+          }
+          const float sgn = dc < half ? -1.f : 1.f;
+          const bool on = d0 < rot && real[RT == 1 ? 0 : q];
+          u32x4 w;
+#pragma unroll
+          for (int e = 0; e < 4; e++) {
+            const float z0 = on ? fmaf(sgn * y0[e], s0[e], x0[e] * c0[e]) : 0.f;
+            if constexpr (B16) {
+              const float z1 = on ? fmaf(sgn * y1[e], s1[e], x1[e] * c1[e]) : 0.f;
+              ((uint16_t *)&w)[e] = (uint16_t)f2bf(z0);
+              ((uint16_t *)&w)[4 + e] = (uint16_t)f2bf(z1);
+            } else {
+              w[e] = __float_as_uint(z0);
+            }
+          }
+          qs[(q * NK + nrc + rc - q * npc) * 64 + lane] = w;
+        }
+      } else {
+        for (int rc = wave; rc < RT * npc; rc += MK_WAVES) {
+          const int q = rc >= npc;
+          E *dst = (E *)(qs + (q * NK + nrc + rc - q * npc) * 64 + lane);
+#pragma unroll 1
+          for (int e = 0; e < EPC; e++) {
+            const int d = (rc - q * npc) * KW + lg * EPC + e, dc = min(d, rot - 1), k = dc < half ? dc : dc - half;
+            const E *x = qr[RT == 1 ? 0 : q];
+            const float xv = fx_ldc(x + dc), yv = fx_ldc(x + (dc < half ? dc + half : k)), cv = ct[RT == 1 ? 0 : q][k], sv = sn[RT == 1 ? 0 : q][k];
+            dst[e] = fx_round<E>(d < rot && real[RT == 1 ? 0 : q] ? (dc < half ? xv * cv - yv * sv : xv * cv + yv * sv) : 0.f);
+          }
+        }
       }
 #pragma unroll
       for (int k = 0; k < QN; k++) {
-        const int i = tid + k * MK_THREADS, rc = i >> 6, rtile = rc / NK, ch = rc - rtile * NK;
-        const bool real = ch < nrc && rtile * 16 + (i & 15) < a.nrows;
-        if (ch < nrc || ch >= nkc) qs[i] = real ? q[k] : (u32x4){0u, 0u, 0u, 0u};
-      }
-      for (int i = tid; i < RT * npc * 64; i += MK_THREADS) {
-        const int rc = i >> 6, rtile = rc / npc, ch = rc - rtile * npc, r = rtile * 16 + (i & 15), Rw = a.r0 + min(r, a.nrows - 1), t = a.t0 + Rw / H;
-        const E *qr = (const E *)st.in + (size_t)t * st.ld_in + (size_t)(Rw % H) * st.ld_in_slot + st.cols[0];
-        const int pos = c.sh_tok[t];
-        const float *ct = (const float *)st.cos_tab + (size_t)pos * st.ld_cos, *sn = (const float *)st.sin_tab + (size_t)pos * st.ld_cos;
-        float x[EPC], y[EPC], cs[EPC], sv[EPC];
-#pragma unroll
-        for (int e = 0; e < EPC; e++) {
-          const int d = min(ch * KW + ((i & 63) >> 4) * EPC + e, rot - 1), k = d < half ? d : d - half;
-          x[e] = fx_ldc(qr + d);
-          y[e] = fx_ldc(qr + (d < half ? d + half : k));
-          cs[e] = ct[k];
-          sv[e] = sn[k];
-        }
-#pragma unroll
-        for (int e = 0; e < EPC; e++) {
-          const int d = ch * KW + ((i & 63) >> 4) * EPC + e;
-          x[e] = d >= rot || r >= a.nrows ? 0.f : d < half ? x[e] * cs[e] - y[e] * sv[e] : x[e] * cs[e] + y[e] * sv[e];
-        }
-        u32x4 v;
-#pragma unroll
-        for (int w = 0; w < 4; w++) {
-          if constexpr (B16) v[w] = pack2(x[(2 * w) % EPC], x[(2 * w + 1) % EPC]);
-          else v[w] = __float_as_uint(x[w % EPC]);
-        }
-        qs[(rtile * NK + nrc + ch) * 64 + (i & 63)] = v;
+        const int rc = wave + k * MK_WAVES, q = rc >= NK, ch = rc - q * NK;
+        const bool on = ch < nrc && real[RT == 1 ? 0 : q];
+        if (ch < nrc || ch >= nkc) qs[rc * 64 + lane] = on ? v[k] : (u32x4){0u, 0u, 0u, 0u};
       }
     }
+    MK_MARK(c, 0);
     // ---- tiles
     int plim[RT];
     float m[RT], l[RT];
@@ -721,11 +760,21 @@ __device__ __forceinline__ void stage_mx_latent_attn_t(CStage &st, Ctx &c, const
         f32x4 S[RT][2];  // (two chains per row tile)
 #pragma unroll
         for (int q = 0; q < RT; q++) S[q][0] = S[q][1] = (f32x4){0.f, 0.f, 0.f, 0.f};
+        // (operands are fetched a group at a time and held back from the products: left alone they are fetched one by one)
 #pragma unroll
-        for (int ch = 0; ch < NK; ch++) {
-          const u32x4 k = ((const u32x4 *)kt)[(wave * NK + ch) * 64 + lane];
+        for (int c0 = 0; c0 < NK; c0 += GRP) {
+          u32x4 k[GRP], b[RT][GRP];
 #pragma unroll
-          for (int q = 0; q < RT; q++) S[q][ch & 1] = fx_mma_k(E(), k, qs[(q * NK + ch) * 64 + lane], S[q][ch & 1]);
+          for (int y = 0; y < GRP; y++) {
+            k[y] = ((const u32x4 *)kt)[(wave * NK + c0 + y) * 64 + lane];
+#pragma unroll
+            for (int q = 0; q < RT; q++) b[q][y] = qs[(q * NK + c0 + y) * 64 + lane];
+          }
+          __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+          for (int y = 0; y < GRP; y++)
+#pragma unroll
+            for (int q = 0; q < RT; q++) S[q][y & 1] = fx_mma_k(E(), k[y], b[q][y], S[q][y & 1]);
         }
 #pragma unroll
         for (int q = 0; q < RT; q++) {
@@ -782,7 +831,7 @@ __device__ __forceinline__ void stage_mx_latent_attn_t(CStage &st, Ctx &c, const
       __syncthreads();
 #pragma unroll
       for (int s = 0; s < SUB; s += B16 ? 2 : 1) {
-        u32x4 p[RT][2];
+        u32x4 p[RT][2], v[VBW];
 #pragma unroll
         for (int q = 0; q < RT; q++) {
           if constexpr (B16) {
@@ -793,16 +842,17 @@ __device__ __forceinline__ void stage_mx_latent_attn_t(CStage &st, Ctx &c, const
           }
         }
 #pragma unroll
-        for (int j = 0; j < VBW; j++) {
-          const u32x4 v = mx_value_operand(E(), kt, NK, s, wave + MK_WAVES * j, lane);  // (blocks behind the last are finite and never stored)
+        for (int j = 0; j < VBW; j++) v[j] = mx_value_operand(E(), kt, NK, s, wave + MK_WAVES * j, lane);  // (blocks behind the last are finite and never stored)
+        __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-          for (int q = 0; q < RT; q++) {
-            acc[q][j] = fx_mma_k(E(), v, p[q][0], acc[q][j]);
-            if constexpr (B16) acc[q][j] = fx_mma_k(E(), v, p[q][1], acc[q][j]);
-          }
-        }
+        for (int w = 0; w < (B16 ? 2 : 1); w++)
+#pragma unroll
+          for (int j = 0; j < VBW; j++)
+#pragma unroll
+            for (int q = 0; q < RT; q++) acc[q][j] = fx_mma_k(E(), v[j], p[q][w], acc[q][j]);
       }
     }
+    MK_MARK(c, 1);
     // ---- sums of the wavefronts, then out (one chunk) or to the partial buffer
 #pragma unroll
     for (int q = 0; q < RT; q++) {
@@ -828,7 +878,7 @@ __device__ __forceinline__ void stage_mx_latent_attn_t(CStage &st, Ctx &c, const
           float *o = (float *)rt.attn_part + ((size_t)u * 16 * RT + r) * PST;
 #pragma unroll
           for (int j = 0; j < VBW; j++)
-            if (wave + MK_WAVES * j < nvb) fx_stc_quad(o + (wave + MK_WAVES * j) * 16 + lg * 4, acc[q][j]);
+            if (wave + MK_WAVES * j < nvb) mx_stc_quad(o + (wave + MK_WAVES * j) * 16 + lg * 4, acc[q][j]);
           if (wave == 0 && lg == 0) {
             stc_f32(o + Rp, m[q]);
             stc_f32(o + Rp + 1, Lr);
@@ -839,42 +889,55 @@ __device__ __forceinline__ void stage_mx_latent_attn_t(CStage &st, Ctx &c, const
   }
   c.wrote_through = true;
 }
-// Rows of split requests: a wavefront per (token, head).
+// Rows of split requests.  Few chunks: a wavefront per (token, head), 256 values and eight chunks at a time.  Many chunks (few
+// rows then): a wavefront per (token, head) and 64 values, a 16-lane row per chunk.
 template <typename E>
 __device__ __forceinline__ void stage_mx_latent_merge(CStage &st, Ctx &c, const MkRuntime &rt, int M) {
   barrier_wait(c);
   constexpr int KW = FxType<E>::KW;
-  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lr = lane & 15, lg = lane >> 4;
   const int H = st.num_q_heads, Rp = (st.rank + KW - 1) / KW * KW, PST = Rp + 32, UR = 16 * st.v_tiles, TPOS = 16 * st.k_tiles;
   const MxLatentRows rw = mx_latent_rows(c, M, H, UR);
-  for (int i = mx_spread(c) + wave * c.G; i < M * H; i += c.G * MK_WAVES) {
-    const int t = i / H, h = i - t * H, t0 = __builtin_amdgcn_readfirstlane(c.sh_tok[2 * MK_MAX_TOKENS + t]), Rw = (t - t0) * H + h;
+  const bool few = rw.cmax <= 8;
+  const int bw = few ? 256 : 64, nb = (Rp + bw - 1) / bw;
+  for (int ib = mx_wave_item(c, wave); ib < M * H * nb; ib += c.G * MK_WAVES) {
+    const int i = ib / nb, blk = ib - i * nb, t = i / H, h = i - t * H, t0 = __builtin_amdgcn_readfirstlane(c.sh_tok[2 * MK_MAX_TOKENS + t]), Rw = (t - t0) * H + h;
     const int n = wave_bcast(rw.my_n, t0), item = wave_bcast(rw.tiles_incl, t0) - wave_bcast(rw.my_tiles, t0) + Rw / UR;
     const int C = mx_chunks((__builtin_amdgcn_readfirstlane(c.sh_tok[t0]) + n - 1) / TPOS + 1, rw.cmax);
     if (C == 1) continue;
     const float *p = (const float *)rt.attn_part + ((size_t)item * rw.cmax * UR + Rw % UR) * PST;
     const size_t step = (size_t)UR * PST;
+    E *out = (E *)st.out + (size_t)t * st.ld_out + (size_t)h * Rp;
     // lane q holds chunk q's statistics
-    const float mq = lane < C ? ldc_f32(p + lane * step + Rp) : MK_FX_NEG, lq = lane < C ? ldc_f32(p + lane * step + Rp + 1) : 0.f;
-    float mm = mq;
+    const float mq = ldc_f32(p + min(lane, C - 1) * step + Rp), lq = ldc_f32(p + min(lane, C - 1) * step + Rp + 1);
+    const int d = blk * bw + 4 * (few ? lane : lr), dc = min(d, Rp - 4);
+    f32x4 x[8];
+    auto load = [&](int q0) {
+#pragma unroll
+      for (int q = 0; q < 8; q++) x[q] = fx_ldc_quad(p + (size_t)min(few ? q0 + q : q0 + q * 4 + lg, C - 1) * step + dc);
+    };
+    load(0);
+    float mm = lane < C ? mq : MK_FX_NEG;
 #pragma unroll
     for (int o = 32; o > 0; o >>= 1) mm = fmaxf(mm, __shfl_xor(mm, o));
     const float e = lane < C ? exp2f(mq - mm) : 0.f, inv = 1.f / wave_sum(lq * e);
-    E *out = (E *)st.out + (size_t)t * st.ld_out + (size_t)h * Rp;
-    for (int d = 4 * lane; d < (Rp + 255) / 256 * 256; d += 256) {
-      f32x4 o = {0.f, 0.f, 0.f, 0.f};
-      for (int q0 = 0; q0 < C; q0 += 8) {
-        f32x4 x[8];
+    f32x4 o = {0.f, 0.f, 0.f, 0.f};
+    for (int q0 = 0;;) {
 #pragma unroll
-        for (int q = 0; q < 8; q++) x[q] = fx_ldc_quad(p + min(q0 + q, C - 1) * step + min(d, Rp - 4));
-#pragma unroll
-        for (int q = 0; q < 8; q++) {
-          const float f = lane_f32(e, min(q0 + q, C - 1));
-          if (q0 + q < C) o += x[q] * f;
-        }
+      for (int q = 0; q < 8; q++) {
+        const int at = few ? q0 + q : q0 + q * 4 + lg;
+        const float f = __builtin_bit_cast(float, __builtin_amdgcn_ds_bpermute((at & 63) << 2, __builtin_bit_cast(int, e)));
+        o += x[q] * (at < C ? f : 0.f);
       }
-      if (d < Rp) fx_stc_quad(out + d, o * inv);
+      q0 += few ? 8 : 32;
+      if (q0 >= C) break;
+      load(q0);
     }
+    if (!few) {
+#pragma unroll
+      for (int y = 0; y < 4; y++) o[y] = groups_sum(o[y]);
+    }
+    if ((few || lg == 0) && d < Rp) fx_stc_quad(out + d, o * inv);
   }
   c.wrote_through = true;
 }
@@ -939,7 +1002,7 @@ __device__ __forceinline__ void mx_delta_load(f32x4 (&S)[NC][NI], const float *s
 #pragma unroll
   for (int j = 0; j < NC; j++)
 #pragma unroll
-    for (int i = 0; i < NI; i++) S[j][i] = fx_ldc_quad(state + (size_t)min(col + j, Dp - 1) * Dp + min(i * 64 + lr * 4, Dp - 4));
+    for (int i = 0; i < NI; i++) S[j][i] = __builtin_nontemporal_load((const f32x4 *)(state + (size_t)min(col + j, Dp - 1) * Dp + min(i * 64 + lr * 4, Dp - 4)));
 #pragma unroll
   for (int j = 0; j < NC; j++)
 #pragma unroll
@@ -952,7 +1015,7 @@ __device__ __forceinline__ void mx_delta_store(const f32x4 (&S)[NC][NI], float *
   for (int j = 0; j < NC; j++)
 #pragma unroll
     for (int i = 0; i < NI; i++)
-      if (col + j < Dp && i * 64 + lr * 4 < Dp) fx_stc_quad(state + (size_t)(col + j) * Dp + i * 64 + lr * 4, S[j][i]);
+      if (col + j < Dp && i * 64 + lr * 4 < Dp) mx_stc_quad(state + (size_t)(col + j) * Dp + i * 64 + lr * 4, S[j][i]);
 }
 template <int NI> struct MxDeltaVec {
   f32x4 r[NI], k[NI], u[NI], au[NI], w[NI];
@@ -985,8 +1048,6 @@ __device__ __forceinline__ void mx_delta_step(f32x4 (&S)[NC][NI], const MxDeltaV
 #pragma unroll
   for (int j = 0; j < NC; j++) o[j] = group16_sum(o[j]);
 }
-__device__ __forceinline__ float mx_sigmoid(float z) { return 1.f / (1.f + expf(-z)); }
-
 // every request brings one token
 template <typename E, int NI, int NC>
 __device__ __forceinline__ void stage_mx_delta_single(CStage &st, Ctx &c, const MkRuntime &rt, int M, char *smem) {
@@ -1037,9 +1098,11 @@ __device__ __forceinline__ void stage_mx_delta_single(CStage &st, Ctx &c, const 
     MxDeltaUnit nx = a;
     f32x4 Sn[NC][NI];
     Raw xn;
-    if (u + c.G < n_units) nx = mx_delta_unit(st, c, rt, us, u + c.G, 1, 0, Dp);
-    mx_delta_load<NI, NC>(Sn, nx.state, nx.p0 == 0, col, lr, Dp);  // (the last unit's again when there is no other)
-    load_raw(nx, xn);
+    if (u + c.G < n_units) {
+      nx = mx_delta_unit(st, c, rt, us, u + c.G, 1, 0, Dp);
+      mx_delta_load<NI, NC>(Sn, nx.state, nx.p0 == 0, col, lr, Dp);
+      load_raw(nx, xn);
+    }
     MxDeltaVec<NI> y;
     float ss = 0.f;
 #pragma unroll
@@ -1057,7 +1120,7 @@ __device__ __forceinline__ void stage_mx_delta_single(CStage &st, Ctx &c, const 
         y.r[i][e] = x.r[i][e];
         y.k[i][e] = x.k[i][e];
         y.u[i][e] = x.k[i][e] * inv;
-        y.au[i][e] = mx_sigmoid(x.a[i][e] + x.ab[i][e]) * y.u[i][e];
+        y.au[i][e] = mx_sigmoid(E(), x.a[i][e] + x.ab[i][e]) * y.u[i][e];
         y.w[i][e] = x.w[i][e];
       }
     float v[NC], o[NC];
@@ -1077,7 +1140,7 @@ __device__ __forceinline__ void stage_mx_delta_single(CStage &st, Ctx &c, const 
       for (int j = 0; j < NC / 4; j++) {
         f32x4 q;
 #pragma unroll
-        for (int e = 0; e < 4; e++) q[e] = (o[4 * j + e] * rn) * x.nw[j][e] * mx_sigmoid(x.g[j][e]);
+        for (int e = 0; e < 4; e++) q[e] = (o[4 * j + e] * rn) * x.nw[j][e] * mx_sigmoid(E(), x.g[j][e]);
         if (col + 4 * j < Dp) fx_stc_quad((E *)st.out + (size_t)a.t0 * st.ld_out + a.h * Dp + col + 4 * j, q);
       }
     }
@@ -1144,7 +1207,7 @@ __device__ __forceinline__ void stage_mx_delta_multi(CStage &st, Ctx &c, const M
           for (int e = 0; e < 4; e++) {
             if (!real) xr[j][e] = xk[j][e] = xv[j][e] = xw[j][e] = 0.f;
             un[e] = xk[j][e] * inv;
-            au[e] = mx_sigmoid(xa[j][e] + xab[e]) * un[e];
+            au[e] = mx_sigmoid(E(), xa[j][e] + xab[e]) * un[e];
           }
           const int at = (wave + j * MK_WAVES) * DPS + 4 * lane;
           *(f32x4 *)(rv + at) = xr[j];
@@ -1204,7 +1267,7 @@ __device__ __forceinline__ void stage_mx_delta_multi(CStage &st, Ctx &c, const M
         const float rn = 1.f / sqrtf(wave_sum(ss) / (float)D + st.eps);
         f32x4 q;
 #pragma unroll
-        for (int e = 0; e < 4; e++) q[e] = (o[e] * rn) * xnw[e] * mx_sigmoid(g[e]);
+        for (int e = 0; e < 4; e++) q[e] = (o[e] * rn) * xnw[e] * mx_sigmoid(E(), g[e]);
         if (4 * lane < Dp) fx_stc_quad((E *)st.out + t * st.ld_out + a.h * Dp + 4 * lane, q);
       }
     }
@@ -1218,7 +1281,7 @@ __device__ __forceinline__ void stage_mx_delta_out(CStage &st, Ctx &c, int M) {
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int D = st.head_dim, Dp = (D + 15) / 16 * 16, H = st.num_q_heads, d4 = min(4 * lane, Dp - 4);
   barrier_wait(c);
-  for (int i = mx_spread(c) + wave * c.G; i < M * H; i += c.G * MK_WAVES) {
+  for (int i = mx_wave_item(c, wave); i < M * H; i += c.G * MK_WAVES) {
     const int t = i / H, h = i - t * H;
     const f32x4 o = fx_ldc_quad((const float *)st.out2 + (size_t)t * st.ld_out2 + h * Dp + d4), g = fx_ldc_quad((const E *)st.in + (size_t)t * st.ld_in + st.cols[3] + h * Dp + d4),
                 w = *(const f32x4 *)((const float *)st.norm_w + h * Dp + d4);
@@ -1226,7 +1289,7 @@ __device__ __forceinline__ void stage_mx_delta_out(CStage &st, Ctx &c, int M) {
     const float rn = 1.f / sqrtf(wave_sum(ss) / (float)D + st.eps);
     f32x4 q;
 #pragma unroll
-    for (int e = 0; e < 4; e++) q[e] = (o[e] * rn) * w[e] * mx_sigmoid(g[e]);
+    for (int e = 0; e < 4; e++) q[e] = (o[e] * rn) * w[e] * mx_sigmoid(E(), g[e]);
     if (4 * lane < Dp) fx_stc_quad((E *)st.out + (size_t)t * st.ld_out + h * Dp + 4 * lane, q);
   }
   c.wrote_through = true;
