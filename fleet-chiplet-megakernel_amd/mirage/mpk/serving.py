@@ -44,6 +44,9 @@ class _Request:
 
 
 class ServingSession:
+    # models with recurrent layers: the tensor that names every batch slot's state slot, and the pool of state slots
+    state_slots = slots = None
+
     def __init__(self, mpk: MPK):
         if mpk.metadata.mode != "online_notoken":
             raise ValueError("a serving session drives an MPK in online_notoken mode")
@@ -54,7 +57,8 @@ class ServingSession:
         self.pool = PagePool(pk.max_num_pages)
         # one state slot per batch slot: the kernel starts a request's state from zero where its position is zero
         self.state_slots = getattr(mpk.model_builder, "state_slots", None)
-        self.slots = PagePool(self.max_requests, "state slots") if self.state_slots is not None else None
+        if self.state_slots is not None:
+            self.slots = PagePool(self.max_requests, "state slots")
         self.requests: Dict[object, _Request] = {}
         mpk._ensure_compiled()
 
@@ -165,7 +169,7 @@ class ServingSession:
         r = self.requests.pop(rid, None)
         if r is not None:
             self.pool.give(r.pages)
-            if r.slot >= 0:
+            if self.slots is not None:
                 self.slots.give([r.slot])
 
     # ------------------------------------------------------------------ greedy generation

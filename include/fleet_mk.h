@@ -126,8 +126,11 @@ void *mk_tensor_ptr(mk_graph *g, int id);
  * in the order the reference layer builders use; `input_maps` holds 3 ints per operand, `forloop_dims` one.
  * Besides the reference's task names: "embedding_scaled", "residual_rmsnorm" and "flex_attention" (sizes and constants are
  * parameters, floats as their bits; operands -1 = absent where optional), and "linear" / "silu_mul" / "argmax" over fp32
- * tensors.  A graph that uses them runs on the flex kernels and holds none of the fixed-shape norm / attention /
- * mixture-of-experts tasks. */
+ * tensors; "residual_prenorm", "latent_prep", "head_linear", "latent_attention" and "general_delta" (csrc/mk_mix.hip; operands
+ * and parameters are listed at their lowering in mk_host.cpp).  A graph that uses them runs on the flex (mix) kernels and holds
+ * none of the fixed-shape norm / attention / mixture-of-experts tasks.  general_delta: the state-slot tensor (int32, one entry
+ * per batch slot) is a permutation the on-GPU schedulers keep; mk_init_requests resets it; with host-described batches the
+ * caller fills it before each pass. */
 int mk_add_task(mk_graph *g, const char *task_name, const int grid_dim[3], const int block_dim[3], int n_operands,
                 const int *tensor_ids, const int *input_maps, const int *forloop_dims, int n_params, const int *params);
 
