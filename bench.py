@@ -212,10 +212,10 @@ def run_leg(torch, dec, shape, model, B, K, W, P, max_seq, mode, stage_profile=F
     }
 
 
-# ---- a model beside the closest one at equal size (bench.py --compare suborax | dodonex) ------------------------------
+# ---- a model beside the closest one at equal size (bench.py --compare suborax | dodonex | bukatar) ------------------------------
 # Both models with the same width, heads, head size, feed-forward, depth and vocabulary; random weights.  (Dodonex: what the
 # closest model has no counterpart for -- latent sizes, recurrence, per-token vectors -- comes from generate.py's shapes.)
-CLOSEST = {"suborax": "qwen3", "dodonex": "suborax"}
+CLOSEST = {"suborax": "qwen3", "dodonex": "suborax", "bukatar": "dodonex"}
 COMPARE_SHAPES = {"8b": dict(width=4096, heads=32, kv_heads=8, ff=12288), "2k": dict(width=2048, heads=32, kv_heads=4, ff=6144)}
 
 
@@ -253,7 +253,7 @@ def compare_decoder(torch, which, shape, layers, vocab, B, R, max_seq, page_size
     make, sizes = SHAPES[f"{which}-{'8b' if shape['width'] == 4096 else '2k'}"]
     mc, sc = random_model(make(layers=layers, vocab=vocab, **sizes))
     g = Generator(max_seq, model_config=mc, batch=R, max_num_batched_tokens=B, max_tokens_per_request=per_req, page_size=page_size, eos_token_id=-1)
-    return g, sc.weight_bytes_per_token() + (2 * R * sc.state_bytes() if which == "dodonex" else 0), sc.kv_bytes_per_position()
+    return g, sc.weight_bytes_per_token() + (2 * R * sc.state_bytes() if hasattr(sc, "state_bytes") else 0), sc.kv_bytes_per_position()
 
 
 def compare_leg(torch, which, shape, layers, vocab, B, R, prompt, steps, stages):

@@ -18,8 +18,9 @@ HERE = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(HERE, "csrc")
 LIB = os.path.join(HERE, "libfleet_mk.so")
 
-# kernels of mk_kernel.hip (-DMK_KERNEL_<name>): the fixed-shape pair, the flex ones, and those with the mix stages beside them
-KERNELS = ("DENSE", "FLEX", "FLEX_M1", "FLEX_F32", "MIX", "MIX_M1", "MIX_F32")
+# kernels of mk_kernel.hip (-DMK_KERNEL_<name>): the fixed-shape pair, the flex ones, those with the mix stages beside them,
+# and those with the hybrid stages beside both
+KERNELS = ("DENSE", "FLEX", "FLEX_M1", "FLEX_F32", "MIX", "MIX_M1", "MIX_F32", "HYB", "HYB_M1", "HYB_F32")
 
 HIPCC_FLAGS = [
     "--offload-arch=gfx950",

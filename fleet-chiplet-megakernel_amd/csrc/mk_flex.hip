@@ -200,7 +200,16 @@ template <typename E> struct FxRows {
   int S;
   const float *part;
   size_t slice, ldp;
+  const float *bias;  // (hybrid kernels) added to every row, null: none
   template <int NS> __device__ __forceinline__ float get(int tok, int col) const {
+#if MK_HAVE_HYB
+    const float b = bias ? bias[col] : 0.f;
+    return sum<NS>(tok, col) + b;
+#else
+    return sum<NS>(tok, col);
+#endif
+  }
+  template <int NS> __device__ __forceinline__ float sum(int tok, int col) const {
     if constexpr (NS == 0) {
       return fx_ldc(in + (size_t)tok * ld + col);
     } else {
@@ -222,7 +231,7 @@ template <typename E> struct FxRows {
   }
 };
 template <typename E> __device__ __forceinline__ FxRows<E> fx_rows(CStage &st, Ctx &c) {
-  FxRows<E> r{(const E *)st.in, st.ld_in, c.defer_S, c.defer_part, (size_t)c.defer_rows * c.defer_n, (size_t)c.defer_n};
+  FxRows<E> r{(const E *)st.in, st.ld_in, c.defer_S, c.defer_part, (size_t)c.defer_rows * c.defer_n, (size_t)c.defer_n, MK_HAVE_HYB ? st.in_bias : nullptr};
   c.defer_S = 0;
   return r;
 }
@@ -301,6 +310,15 @@ __device__ __forceinline__ size_t fx_v_at(int page, int pp, int ps, int nkv, int
   return ((((((size_t)page * ps + pp) / TP) * nkv + g) * nvb + d / 16) * 64 + ((pp & 15) >> 2) * 16 + (d & 15)) * EPC + ((pp % TP) / 16) * 4 + (pp & 3);
 }
 
+// Column the value heads begin at (hybrid kernels: the keys' where a model's values are its keys before rotation).
+__device__ __forceinline__ int fx_value_col(CStage &st) {
+#if MK_HAVE_HYB
+  return st.v_col;
+#else
+  return (st.num_q_heads + st.num_kv_heads) * st.head_dim;
+#endif
+}
+
 // Query, key and value rows of an iteration in which some request brings several tokens: a wavefront per (token, head)
 // row.  Queries go to the workspace, keys and values to their pages.  (When every request brings one token the attention
 // stage does this itself and the stage is skipped.)
@@ -322,7 +340,7 @@ __device__ __forceinline__ void stage_fx_prep(CStage &st, Ctx &c, const MkRuntim
     if (s < H + nkv) {
       fx_head_load<E>(st, rows, t, s * D, pos, lane, h);
     } else {
-      fx_value_load<E>(rows, t, (H + nkv) * D + (s - H - nkv) * DV, DV, lane, h.x);
+      fx_value_load<E>(rows, t, fx_value_col(st) + (s - H - nkv) * DV, DV, lane, h.x);
     }
   };
   auto finish = [&](int i, FxHead &h, int page) {
@@ -417,8 +435,11 @@ __device__ __forceinline__ void stage_fx_attn_t(CStage &st, Ctx &c, const MkRunt
   const int cmax = max(1, min(c.G / n_items, MK_ATTN_MAX_CHUNKS));
   const int n_units = n_items * cmax;
   struct Unit {
-    int item, cidx, C, g, vs, t0, r0, nrows, p0, p, tb, te, pages;
+    int item, cidx, C, g, vs, t0, r0, nrows, p0, p, tb, te, pages, kept, gap;
   };
+  // Tiles of a unit are counted without those that none of its rows sees: with a window, `kept` first ones, then `gap` left out.
+  const int win = MK_HAVE_HYB ? st.window : 0, keep = MK_HAVE_HYB ? st.keep_first : 0;
+  auto phys = [](const Unit &a, int tile) { return MK_HAVE_HYB && tile >= a.kept ? tile + a.gap : tile; };
   auto decode = [&](int u, Unit &a) -> bool {
     a.item = u / cmax;
     a.cidx = u - a.item * cmax;
@@ -432,7 +453,13 @@ __device__ __forceinline__ void stage_fx_attn_t(CStage &st, Ctx &c, const MkRunt
     a.nrows = min(16, n * qpk - a.r0);
     a.p0 = __builtin_amdgcn_readfirstlane(c.sh_tok[a.t0]);
     a.p = a.p0 + (a.r0 + a.nrows - 1) / qpk;  // newest position any of the rows sees
-    const int NT = a.p / TP + 1;
+    int NT = a.p / TP + 1;
+    if (MK_HAVE_HYB) {
+      const int oldest = win ? max(0, a.p0 + a.r0 / qpk - win + 1) : 0;  // oldest position inside the window of the unit's first row
+      a.kept = win ? min((keep + TP - 1) / TP, NT) : NT;
+      a.gap = max(0, oldest / TP - a.kept);
+      NT -= a.gap;
+    }
     a.C = fx_chunks(NT, cmax);
     if (a.cidx >= a.C) return false;
     a.tb = (int)(((long long)NT * a.cidx) / a.C);
@@ -460,8 +487,8 @@ __device__ __forceinline__ void stage_fx_attn_t(CStage &st, Ctx &c, const MkRunt
   auto load_first = [&](const Unit &a) {
     const int tile = a.tb + wave;
     const bool ok = tile < a.te;
-    const int page = rt.kv_indices[a.pages + (ok ? tile * TP : a.tb * TP) / ps];
-    load_tile(a, tile, 0, page, ok, kA, vA);
+    const int page = rt.kv_indices[a.pages + phys(a, ok ? tile : a.tb) * TP / ps];
+    load_tile(a, phys(a, tile), 0, page, ok, kA, vA);
   };
   const bool early = single && have0 && wave != 0;  // (the polling wavefront keeps its memory queue empty)
   if (early) load_first(a0);
@@ -489,7 +516,7 @@ __device__ __forceinline__ void stage_fx_attn_t(CStage &st, Ctx &c, const MkRunt
     }
     if (!(first && early)) load_first(a);
     __syncthreads();  // LDS reuse across units
-    const int pg_lo = a.tb * TP / ps, npg = min((a.te * TP - 1) / ps, a.p / ps) - pg_lo + 1;
+    const int pg_lo = phys(a, a.tb) * TP / ps, npg = min((phys(a, a.te - 1) * TP + TP - 1) / ps, a.p / ps) - pg_lo + 1;
     for (int i = tid; i < npg; i += MK_THREADS) spg[i] = rt.kv_indices[a.pages + pg_lo + i];
     const bool newest = single && a.cidx == a.C - 1;
     // ---- query rows into operand order (and the new key and value)
@@ -509,7 +536,7 @@ __device__ __forceinline__ void stage_fx_attn_t(CStage &st, Ctx &c, const MkRunt
       // wavefront, whose tile has been in flight longest, takes row 0 and with it the first of the second round
       const int n_rows = a.nrows + (newest ? 1 : 0), w_ = MK_WAVES - 1 - wave;
       const bool v_row = newest && w_ == 1;
-      const int v_col = (st.num_q_heads + nkv) * D + a.g * DV;
+      const int v_col = fx_value_col(st) + a.g * DV;
       float vv[MK_FX_HEAD_REGS];
       if (v_row) fx_value_load<E>(rows, a.t0, v_col, DV, lane, vv);
       auto load_row = [&](int r, FxHead &h) {
@@ -597,7 +624,10 @@ __device__ __forceinline__ void stage_fx_attn_t(CStage &st, Ctx &c, const MkRunt
           } else {
             s *= LOG2E;
           }
-          s = tile * TP + u_ * 16 + lg * 4 + i <= plim ? s : MK_FX_NEG;
+          const int at = tile * TP + u_ * 16 + lg * 4 + i;
+          bool seen = at <= plim;
+          if (MK_HAVE_HYB) seen = seen && (win == 0 || plim - at < win || at < keep);
+          s = seen ? s : MK_FX_NEG;
           sc[u_][i] = s;
           tm = fmaxf(tm, s);
         }
@@ -682,15 +712,15 @@ __device__ __forceinline__ void stage_fx_attn_t(CStage &st, Ctx &c, const MkRunt
       int tl = tile, kk = kg;
       next(tl, kk);
       bool ok = it + 1 < n_it;
-      load_tile(a, tl, kk, ok ? spg[tl * TP / ps - pg_lo] : 0, ok, kB, vB);
-      compute(tile, kg, kA, vA);
+      load_tile(a, phys(a, tl), kk, ok ? spg[phys(a, tl) * TP / ps - pg_lo] : 0, ok, kB, vB);
+      compute(phys(a, tile), kg, kA, vA);
       if (!ok) break;
       tile = tl;
       kg = kk;
       next(tl, kk);
       ok = it + 2 < n_it;
-      load_tile(a, tl, kk, ok ? spg[tl * TP / ps - pg_lo] : 0, ok, kA, vA);
-      compute(tile, kg, kB, vB);
+      load_tile(a, phys(a, tl), kk, ok ? spg[phys(a, tl) * TP / ps - pg_lo] : 0, ok, kA, vA);
+      compute(phys(a, tile), kg, kB, vB);
       tile = tl;
       kg = kk;
     }
@@ -861,7 +891,7 @@ __device__ __forceinline__ void stage_fx_linear_f32(CStage &st, Ctx &c, int M, c
       if (m < M) {
         float r[4];
 #pragma unroll
-        for (int i = 0; i < 4; i++) r[i] = silu ? v[i] / (1.f + expf(-v[i])) * g[i] : v[i];
+        for (int i = 0; i < 4; i++) r[i] = silu ? v[i] / (1.f + expf(-v[i])) * g[i] : linear_act(st, v[i]);
         fx_stc4((float *)st.out + (size_t)m * st.ld_out, ot * 16 + (l >> 4) * 4, n_out, r);
       }
     }

@@ -49,6 +49,15 @@ MK_DECLARE_KERNEL(mk_persistent_kernel_mix_m1);
 #ifdef MK_HAVE_KERNEL_MIX_F32
 MK_DECLARE_KERNEL(mk_persistent_kernel_mix_f32);
 #endif
+#ifdef MK_HAVE_KERNEL_HYB
+MK_DECLARE_KERNEL(mk_persistent_kernel_hyb);
+#endif
+#ifdef MK_HAVE_KERNEL_HYB_M1
+MK_DECLARE_KERNEL(mk_persistent_kernel_hyb_m1);
+#endif
+#ifdef MK_HAVE_KERNEL_HYB_F32
+MK_DECLARE_KERNEL(mk_persistent_kernel_hyb_f32);
+#endif
 
 namespace {
 
@@ -158,6 +167,7 @@ struct mk_graph {
   size_t flex_items = 0;     // most work items of a flex attention stage (row tiles x kv heads x value slices)
   size_t flex_part = 0;      // floats of split-KV partials the flex and latent attention stages need
   bool mix = false;          // some stage is one of mk_mix.hip's
+  bool hyb = false;          // ... of mk_hybrid.hip's, or an older stage has an option only the hybrid kernels know
   int *state_ids = nullptr;  // batch slot -> recurrent-state slot (the caller's tensor); null: no recurrence
 };
 
@@ -263,7 +273,7 @@ int num_outputs(const Task &t) {
   if (t.name == "gang_attn_split_kv_mi300") return 3;
   if (t.name == "paged_attention_ck_fmha_split_kv_mi300" || t.name == "paged_attention_split_kv_mi300") return 2;
   if (t.name == "moe_topk_softmax_mi300") return 3;
-  if (t.name == "embedding_scaled" || t.name == "residual_rmsnorm" || t.name == "residual_prenorm" || t.name == "latent_prep" || t.name == "general_delta") return 2;
+  if (t.name == "embedding_scaled" || t.name == "residual_rmsnorm" || t.name == "residual_prenorm" || t.name == "latent_prep" || t.name == "general_delta" || t.name == "expert_route") return 2;
   return 1;
 }
 
@@ -273,6 +283,9 @@ float bits_f32(int bits) {
   memcpy(&f, &bits, sizeof(f));
   return f;
 }
+
+bool rows_ok(const Tensor &t, int B, int64_t cols, int dtype) { return t.ndims == 2 && t.dims[0] >= B && t.dims[1] >= cols && t.dtype == dtype && !(t.strides[0] & 3); }
+bool vector_ok(const Tensor &t, int64_t n) { return t.dtype == MK_DT_F32 && (int64_t)t.elems() >= n; }
 
 // a graph holds flex stages of one activation type, and none of the fixed-shape stages next to them (checked after lowering)
 int set_flex(mk_graph *g, int dtype, const char *task) {
@@ -339,6 +352,15 @@ int lower_linear(mk_graph *g, size_t &i) {
     act = &g->ltasks[i + 1];
   }
   int final_out = out_id;
+  const Task *sq = nullptr;  // a following relu_squared likewise
+  if (!silu && !res && i + 1 < g->ltasks.size() && g->ltasks[i + 1].name == "relu_squared" && g->ltasks[i + 1].ops.size() == 2 && g->ltasks[i + 1].ops[0] == out_id && tout.kind == T_OWNED) {
+    sq = &g->ltasks[i + 1];
+    st.flags |= MK_F_RELU2;
+    final_out = sq->ops[1];
+    g->mix = g->hyb = true;
+    int rc2 = set_flex(g, tin.dtype, "relu_squared");
+    if (rc2) return rc2;
+  }
   if (silu || act) {
     st.flags |= MK_F_SILU;
     if (act) {
@@ -405,14 +427,14 @@ int lower_linear(mk_graph *g, size_t &i) {
   }
   g->stages.push_back(st);
   g->stage_desc.push_back(fmt("LINEAR%s%s%s%s %s x %s -> %s n=%d k=%d segs=%d", f32 ? "_F32" : "", (st.flags & MK_F_NORM) ? "+norm" : "", (st.flags & MK_F_RES) ? "+res" : "",
-                              (st.flags & MK_F_SILU) ? "+silu" : "", tin.name.c_str(), g->tensors[w_id].name.c_str(), tfo.name.c_str(), st.n, st.k,
+                              (st.flags & MK_F_SILU) ? "+silu" : sq ? "+relu2" : "", tin.name.c_str(), g->tensors[w_id].name.c_str(), tfo.name.c_str(), st.n, st.k,
                               st.w.nseg));
   g->weight_bytes += (int64_t)st.n * st.k * (int64_t)dtype_size(tin.dtype);
   g->stage_weight.resize(g->stages.size(), -1);
   g->stage_weight.back() = w_id;
   g->last_linear_task = (int)i;
   g->last_linear_stage = (int)g->stages.size() - 1;
-  i += act ? 2 : consumed_linear;
+  i += act || sq ? 2 : consumed_linear;
   return MK_OK;
 }
 
@@ -743,11 +765,15 @@ int lower_residual_rmsnorm(mk_graph *g, size_t &i) {
 // flex_attention [qkv rows, k cache, v cache, cos (optional), sin (optional), sink (optional), q workspace, output]
 // params [q heads, kv heads, head dim, value dim, rotated dims, unit norm 0/1, eps bits, scale bits, softcap bits].  The
 // qkv rows are all query heads, then all key heads, then all value heads; caches are [pages, page_size, kv heads, padded
-// dim] with a layout of the library's own inside a page.
+// dim] with a layout of the library's own inside a page.  With three more params [window, kept first positions, values from
+// keys 0/1] and one more operand behind the sink, fp32 [input columns] added to the rows: a position sees the `window` newest
+// ones and the kept first ones; the value heads are the key heads before rotation (the rows hold no others).
 int lower_flex_attention(mk_graph *g, size_t &i) {
   const Task &t = g->ltasks[i];
-  if (t.ops.size() != 8 || t.params.size() != 9) return fail(MK_EINVAL, "flex_attention expects 8 operands / 9 params");
-  const Tensor &in = g->tensors[t.ops[0]], &kc = g->tensors[t.ops[1]], &vc = g->tensors[t.ops[2]], &qw = g->tensors[t.ops[6]], &o = g->tensors[t.ops[7]];
+  const bool ext = t.ops.size() == 9 && t.params.size() == 12;
+  if (!ext && (t.ops.size() != 8 || t.params.size() != 9)) return fail(MK_EINVAL, "flex_attention expects 8 operands / 9 params, or 9 / 12");
+  const Tensor &in = g->tensors[t.ops[0]], &kc = g->tensors[t.ops[1]], &vc = g->tensors[t.ops[2]], &qw = g->tensors[t.ops[6 + ext]], &o = g->tensors[t.ops[7 + ext]];
+  const int window = ext ? t.params[9] : 0, keep = ext ? t.params[10] : 0, own_v = !(ext && t.params[11]);
   const int B = g->cfg.max_num_batched_tokens, ps = g->cfg.page_size;
   const int H = t.params[0], G = t.params[1], D = t.params[2], DV = t.params[3], rot = t.params[4];
   int rc = set_flex(g, in.dtype, "flex_attention");
@@ -757,7 +783,10 @@ int lower_flex_attention(mk_graph *g, size_t &i) {
   if (H < 1 || G < 1 || H % G || D < 1 || DV < 1 || rot < 0 || rot > D || rot % 2) return fail(MK_EINVAL, "flex_attention: heads %d / %d, dims %d / %d, rotated %d", H, G, D, DV, rot);
   if (D > MK_FX_MAX_HEAD_DIM || DV > MK_FX_MAX_HEAD_DIM) return fail(MK_EUNSUPPORTED, "flex_attention: head dims %d / %d (most %d)", D, DV, MK_FX_MAX_HEAD_DIM);
   const int dk = (D + KW - 1) / KW * KW, dv = (DV + 15) / 16 * 16;
-  if (in.ndims != 2 || in.dims[0] < B || in.dims[1] < (int64_t)H * D + (int64_t)G * (D + DV)) return fail(MK_EINVAL, "flex_attention: input must be [tokens, >= (q + kv) * dim + kv * value dim]");
+  const int64_t cols = (int64_t)H * D + (int64_t)G * (D + own_v * DV);
+  if (window < 0 || keep < 0 || (!own_v && D != DV)) return fail(MK_EINVAL, "flex_attention: window %d, %d kept positions, key / value size %d / %d", window, keep, D, DV);
+  if (ext && t.ops[6] >= 0 && !vector_ok(g->tensors[t.ops[6]], cols)) return fail(MK_EINVAL, "flex_attention: the bias holds one fp32 value per input column");
+  if (in.ndims != 2 || in.dims[0] < B || in.dims[1] < (int64_t)H * D + (int64_t)G * (D + own_v * DV)) return fail(MK_EINVAL, "flex_attention: input must be [tokens, >= (q + kv) * dim + kv * value dim]");
   if (o.ndims != 2 || o.dims[0] < B || o.dims[1] < (int64_t)H * DV || o.dtype != in.dtype) return fail(MK_EINVAL, "flex_attention: output must be [tokens, >= q heads * value dim] of the input's type");
   if (qw.ndims != 2 || qw.dims[0] < B || qw.dims[1] < (int64_t)H * dk || qw.dtype != in.dtype || (qw.strides[0] * es) % 16) return fail(MK_EINVAL, "flex_attention: q workspace must be [tokens, >= q heads * %d]", dk);
   if (kc.ndims != 4 || vc.ndims != 4 || kc.dtype != in.dtype || vc.dtype != in.dtype || kc.dims[0] < g->cfg.max_num_pages || vc.dims[0] < g->cfg.max_num_pages || kc.dims[1] != ps ||
@@ -780,6 +809,11 @@ int lower_flex_attention(mk_graph *g, size_t &i) {
   st.num_kv_heads = G;
   st.head_dim = D;
   st.v_dim = DV;
+  st.v_col = own_v ? (H + G) * D : H * D;
+  st.window = window;
+  st.keep_first = window ? keep : 0;
+  st.in_bias = ext && t.ops[6] >= 0 ? (const float *)g->tensors[t.ops[6]].ptr : nullptr;
+  if (ext) g->mix = g->hyb = true;
   st.rot_dims = rot;
   st.eps = bits_f32(t.params[6]);
   st.sm_scale = bits_f32(t.params[7]);
@@ -813,7 +847,7 @@ int lower_flex_attention(mk_graph *g, size_t &i) {
   g->flex_part = std::max(g->flex_part, (size_t)g->G * 16 * (st.v_tiles * 16 + 32));
   if (!g->stages.empty()) {
     MkStage &pl = g->stages.back();  // the q/k/v linear may leave its K-slice sum to this stage's row fetch
-    if (pl.op == MK_OP_LINEAR && !(pl.flags & (MK_F_SILU | MK_F_RES)) && pl.out == st.in && pl.ld_out == st.ld_in && pl.n >= H * D + G * (D + DV)) pl.flags |= MK_F_DEFER_SUM;
+    if (pl.op == MK_OP_LINEAR && !(pl.flags & (MK_F_SILU | MK_F_RES)) && pl.out == st.in && pl.ld_out == st.ld_in && pl.n >= cols) pl.flags |= MK_F_DEFER_SUM;
   }
   if (B > 1) {
     MkStage sp = st;
@@ -822,14 +856,12 @@ int lower_flex_attention(mk_graph *g, size_t &i) {
     g->stage_desc.push_back(fmt("FX_PREP[portions] %s", in.name.c_str()));
   }
   g->stages.push_back(st);
-  g->stage_desc.push_back(fmt("FX_ATTN %s -> %s q=%d kv=%d d=%d dv=%d rot=%d norm=%d softcap=%g sink=%d", in.name.c_str(), o.name.c_str(), H, G, D, DV, rot, t.params[5], st.softcap, t.ops[5] >= 0));
+  g->stage_desc.push_back(fmt("FX_ATTN %s -> %s q=%d kv=%d d=%d dv=%d rot=%d norm=%d softcap=%g sink=%d window=%d+%d bias=%d", in.name.c_str(), o.name.c_str(), H, G, D, DV, rot, t.params[5], st.softcap, t.ops[5] >= 0, st.window, st.keep_first, st.in_bias != nullptr));
   i++;
   return MK_OK;
 }
 
 // ---- mix tasks (mk_mix.hip) --------------------------------------------------------------------------------------------
-bool rows_ok(const Tensor &t, int B, int64_t cols, int dtype) { return t.ndims == 2 && t.dims[0] >= B && t.dims[1] >= cols && t.dtype == dtype && !(t.strides[0] & 3); }
-bool vector_ok(const Tensor &t, int64_t n) { return t.dtype == MK_DT_F32 && (int64_t)t.elems() >= n; }
 
 int set_mix(mk_graph *g, int dtype, const char *task) {
   g->mix = true;
@@ -840,20 +872,27 @@ int set_mix(mk_graph *g, int dtype, const char *task) {
 // params [width, groups, alpha bits, eps bits, y eps bits]: v = residual + alpha * y (with a y weight: of the RMS-normalised
 // y); new residual = v, rows = the RMS norm of v in `groups` equal parts times weight (no weight: v).  A bf16 linear that
 // reads the rows next forms them itself when an iteration has one token.
+// With two more operands behind the y weight (fp32 [columns] added to y, optional; fp32 [tokens, >= slots] weights, optional) and
+// two more params [slots, columns per slot]: y is the weighted sum of `slots` rows that lie side by side.
 int lower_residual_prenorm(mk_graph *g, size_t &i) {
   const Task t = g->ltasks[i];
-  if (t.ops.size() != 6 || t.params.size() != 5) return fail(MK_EINVAL, "residual_prenorm expects 6 operands / 5 params");
+  const bool ext = t.ops.size() == 8 && t.params.size() == 7;
+  const int e2 = ext ? 2 : 0;
+  if (!ext && (t.ops.size() != 6 || t.params.size() != 5)) return fail(MK_EINVAL, "residual_prenorm expects 6 operands / 5 params, or 8 / 7");
   auto opt = [&](int k) { return t.ops[k] >= 0 ? &g->tensors[t.ops[k]] : nullptr; };
-  const Tensor *y = opt(0), *yw = opt(1), *w = opt(3);
-  const Tensor x = g->tensors[t.ops[2]], xo = g->tensors[t.ops[4]], o = g->tensors[t.ops[5]];
+  const Tensor *y = opt(0), *yw = opt(1), *yb = ext ? opt(2) : nullptr, *sw = ext ? opt(3) : nullptr, *w = opt(3 + e2);
+  const Tensor x = g->tensors[t.ops[2 + e2]], xo = g->tensors[t.ops[4 + e2]], o = g->tensors[t.ops[5 + e2]];
+  const int slots = sw ? t.params[5] : 0, ld_slot = sw ? t.params[6] : 0;
   const int B = g->cfg.max_num_batched_tokens, width = t.params[0], groups = t.params[1];
   const int64_t n = o.ndims == 2 ? o.dims[1] : 0;
   int rc = set_mix(g, o.dtype, "residual_prenorm");
   if (rc) return rc;
   if (n < 4 || n % 4 || width < 1 || width > n || !rows_ok(o, B, n, o.dtype) || !rows_ok(x, B, n, MK_DT_F32) || !rows_ok(xo, B, n, MK_DT_F32) || x.dims[1] != n || xo.dims[1] != n ||
-      (y && (!rows_ok(*y, B, n, o.dtype) || y->dims[1] != n)) || (w && !vector_ok(*w, n)) || (yw && (!y || !vector_ok(*yw, n))))
+      (y && (!rows_ok(*y, B, n, o.dtype) || (!sw && y->dims[1] != n))) || (w && !vector_ok(*w, n)) || (yw && (!y || !vector_ok(*yw, n))))
     return fail(MK_EINVAL, "residual_prenorm: every row tensor is [tokens, %lld] (a multiple of 4; residual fp32), weights are fp32 of that size, width=%d of it real", (long long)n, width);
   if (w && (groups < 1 || groups > MK_MX_MAX_GROUPS || width % groups)) return fail(MK_EINVAL, "residual_prenorm: %d parts of a row of %d (at most %d)", groups, width, MK_MX_MAX_GROUPS);
+  if ((yb && (!y || !vector_ok(*yb, n))) || (sw && (!y || yb || slots < 1 || slots > MK_MOE_MAX_TOPK + 1 || ld_slot < n || ld_slot % 8 || y->dims[1] < (int64_t)(slots - 1) * ld_slot + n || !rows_ok(*sw, B, slots, MK_DT_F32))))
+    return fail(MK_EINVAL, "residual_prenorm: a bias has %lld entries; %d slots of %d columns with fp32 weights of that many columns (and no bias)", (long long)n, slots, ld_slot);
   if (n > 12 * 4 * MK_THREADS) return fail(MK_EUNSUPPORTED, "residual_prenorm: rows of %lld values (most %d)", (long long)n, 12 * 4 * MK_THREADS);
   if (x.ptr == xo.ptr || (xo.ptr == o.ptr && w)) return fail(MK_EINVAL, "residual_prenorm: the new residual rows must not overwrite the old ones (other workgroups may still read them), nor the rows them");
   MkStage st;
@@ -868,6 +907,12 @@ int lower_residual_prenorm(mk_graph *g, size_t &i) {
   st.in = y ? y->ptr : nullptr;
   st.ld_in = y ? (int)y->strides[0] : 0;
   st.y_norm_w = yw ? yw->ptr : nullptr;
+  st.in_bias = yb ? (const float *)yb->ptr : nullptr;
+  st.slots = slots;
+  st.ld_slot = ld_slot;
+  st.slot_w = sw ? (const float *)sw->ptr : nullptr;
+  st.ld_slot_w = sw ? (int)sw->strides[0] : 0;
+  if (yb || sw) g->hyb = true;
   st.res = x.ptr;
   st.ld_res = (int)x.strides[0];
   st.norm_w = w ? w->ptr : nullptr;
@@ -877,7 +922,7 @@ int lower_residual_prenorm(mk_graph *g, size_t &i) {
   st.ld_out2 = (int)xo.strides[0];
   if (!g->stages.empty()) {
     MkStage &pl = g->stages.back();
-    if (!w && !yw && y && st.out && pl.op == MK_OP_LINEAR && !(pl.flags & (MK_F_SILU | MK_F_RES)) && pl.out == st.in && (pl.k & 63) == 0) {
+    if (!w && !yw && !yb && !sw && y && st.out && pl.op == MK_OP_LINEAR && !(pl.flags & (MK_F_SILU | MK_F_RES)) && pl.out == st.in && (pl.k & 63) == 0) {
       // a plain linear in front adds its single-token result to the stream itself
       pl.flags |= MK_F_JOIN;
       pl.res = st.res;
@@ -893,7 +938,7 @@ int lower_residual_prenorm(mk_graph *g, size_t &i) {
   }
   bool res, silu;
   int extra;
-  const bool fuse = g->flex == FLEX_BF16 && w && i + 1 < g->ltasks.size() && linear_kind(g->ltasks[i + 1].name, &res, &silu, &extra) && !res && g->ltasks[i + 1].ops[0] == t.ops[5];
+  const bool fuse = g->flex == FLEX_BF16 && w && i + 1 < g->ltasks.size() && linear_kind(g->ltasks[i + 1].name, &res, &silu, &extra) && !res && g->ltasks[i + 1].ops[0] == t.ops[5 + e2];
   if (fuse) st.flags |= MK_F_ONLY_MULTI;
   g->stages.push_back(st);
   g->stage_desc.push_back(fmt("MX_PRENORM%s %s + %g * %s%s -> %s, %s k=%d parts=%d", (st.flags & MK_F_ONLY_MULTI) ? "[multi-token only]" : "", x.name.c_str(), st.alpha, yw ? "norm of " : "", y ? y->name.c_str() : "0", xo.name.c_str(),
@@ -907,6 +952,11 @@ int lower_residual_prenorm(mk_graph *g, size_t &i) {
   l.y_in = st.in;
   l.ld_y = st.ld_in;
   l.y_norm_w = st.y_norm_w;
+  l.in_bias = st.in_bias;
+  l.slots = st.slots;
+  l.ld_slot = st.ld_slot;
+  l.slot_w = st.slot_w;
+  l.ld_slot_w = st.ld_slot_w;
   l.res = st.res;
   l.ld_res = st.ld_res;
   l.norm_w = st.norm_w;
@@ -976,12 +1026,14 @@ int check_latent_cache(mk_graph *g, const Tensor &kc, int dtype, const LatentDim
 int lower_latent_prep(mk_graph *g, size_t &i) {
   const Task &t = g->ltasks[i];
   if (t.ops.size() != 8 || t.params.size() != 14) return fail(MK_EINVAL, "latent_prep expects 8 operands / 14 params");
-  const Tensor &in = g->tensors[t.ops[0]], &qn = g->tensors[t.ops[1]], &o = g->tensors[t.ops[7]];
+  const bool q = t.ops[1] >= 0;  // (without a query latent: operands 1 and 7 are absent)
+  const Tensor &in = g->tensors[t.ops[0]];
   const int B = g->cfg.max_num_batched_tokens, qc = t.params[0], qr = t.params[1], kc = t.params[2], R = t.params[3], rc_ = t.params[4], rot = t.params[5];
   int rc = set_mix(g, in.dtype, "latent_prep");
   if (rc) return rc;
   auto up4 = [](int n) { return (n + 3) / 4 * 4; };
-  if (qr < 1 || qc < 0 || qc % 4 || qr > MK_MX_MAX_NORM_ROW || !rows_ok(in, B, qc + up4(qr), in.dtype) || !rows_ok(o, B, up4(qr), in.dtype) || !vector_ok(qn, up4(qr)))
+  if (q != (t.ops[7] >= 0) || (!q && (t.ops[5] < 0 || qr || !rows_ok(in, B, 4, in.dtype)))) return fail(MK_EINVAL, "latent_prep: nothing to do, or half a query latent");
+  if (q && (qr < 1 || qc < 0 || qc % 4 || qr > MK_MX_MAX_NORM_ROW || !rows_ok(in, B, qc + up4(qr), in.dtype) || !rows_ok(g->tensors[t.ops[7]], B, up4(qr), in.dtype) || !vector_ok(g->tensors[t.ops[1]], up4(qr))))
     return fail(MK_EINVAL, "latent_prep: query latent of %d values at column %d (at most %d, columns multiples of 4, weights padded to 4)", qr, qc, MK_MX_MAX_NORM_ROW);
   MkStage st;
   memset(&st, 0, sizeof(st));
@@ -990,9 +1042,11 @@ int lower_latent_prep(mk_graph *g, size_t &i) {
   st.ld_in = (int)in.strides[0];
   st.n = qr;
   st.cols[0] = qc;
-  st.q_norm_w = qn.ptr;
-  st.out = o.ptr;
-  st.ld_out = (int)o.strides[0];
+  if (q) {
+    st.q_norm_w = g->tensors[t.ops[1]].ptr;
+    st.out = g->tensors[t.ops[7]].ptr;
+    st.ld_out = (int)g->tensors[t.ops[7]].strides[0];
+  }
   st.eps = bits_f32(t.params[6]);
   if (t.ops[5] >= 0) {
     const LatentDims d = latent_dims(in.dtype, R, rot);
@@ -1010,7 +1064,7 @@ int lower_latent_prep(mk_graph *g, size_t &i) {
   }
   if ((rc = lower_glu(g, t, 6, 7, in, &st))) return rc;
   g->stages.push_back(st);
-  g->stage_desc.push_back(fmt("MX_LATENT_PREP %s -> %s q=%d latent=%d rot=%d glu=%d", in.name.c_str(), o.name.c_str(), qr, st.rank, st.rot_dims, st.glu_n));
+  g->stage_desc.push_back(fmt("MX_LATENT_PREP %s -> %s q=%d latent=%d rot=%d glu=%d", in.name.c_str(), q ? g->tensors[t.ops[7]].name.c_str() : "cache", qr, st.rank, st.rot_dims, st.glu_n));
   i++;
   return MK_OK;
 }
@@ -1026,8 +1080,9 @@ int lower_head_linear(mk_graph *g, size_t &i) {
   int rc = set_mix(g, in.dtype, "head_linear");
   if (rc) return rc;
   const int es = in.dtype == MK_DT_F32 ? 4 : 2, kw = 64 / es, epc = 16 / es;
+  const bool out32 = o.dtype == MK_DT_F32 && in.dtype == MK_DT_BF16 && H == 1 && t.ops[3] < 0;  // 32-bit sums
   if (H < 1 || n < 1 || k < kw || k % kw || is < 0 || is % epc || os < 0 || in.strides[0] % epc || !rows_ok(in, B, (int64_t)(H - 1) * is + k, in.dtype) ||
-      o.ndims != 2 || o.dims[0] < B || o.dims[1] < (int64_t)(H - 1) * os + n || o.dtype != in.dtype || w.dtype != in.dtype || (int64_t)w.elems() != (int64_t)H * ((n + 15) / 16 * 16) * k)
+      o.ndims != 2 || o.dims[0] < B || o.dims[1] < (int64_t)(H - 1) * os + n || (o.dtype != in.dtype && !out32) || w.dtype != in.dtype || (int64_t)w.elems() != (int64_t)H * ((n + 15) / 16 * 16) * k)
     return fail(MK_EINVAL, "head_linear: %d heads of %d x %d (whole operand rows of %d), input columns %d and output columns %d per head do not fit the operands", H, n, k, kw, is, os);
   MkStage st;
   memset(&st, 0, sizeof(st));
@@ -1043,6 +1098,12 @@ int lower_head_linear(mk_graph *g, size_t &i) {
   st.ld_out_slot = os;
   st.w.nseg = 1;
   st.w.seg[0] = w.ptr;
+  if (out32) {
+    st.flags |= MK_F_OUT32;
+    st.out2 = o.ptr;
+    st.ld_out2 = (int)o.strides[0];
+    g->hyb = true;
+  }
   if (t.ops[3] >= 0) {
     const Tensor &tab = g->tensors[t.ops[3]];
     if (t.ops[2] < 0 || H != 1 || tab.ndims != 2 || tab.dtype != in.dtype || tc < 0 || tc + n > tab.dims[1] || g->tensors[t.ops[2]].dtype != MK_DT_I64 || (int64_t)g->tensors[t.ops[2]].elems() < B)
@@ -1179,6 +1240,223 @@ int lower_general_delta(mk_graph *g, size_t &i) {
   g->stages.push_back(st);
   g->stage_desc.push_back(fmt("MX_DELTA_OUT[sliced] -> %s", o.name.c_str()));
   g->weight_bytes += (int64_t)w2.elems() * es;
+  i++;
+  return MK_OK;
+}
+
+// ---- hybrid tasks (mk_hybrid.hip) --------------------------------------------------------------------------------------
+int set_hyb(mk_graph *g, int dtype, const char *task) {
+  g->hyb = true;
+  return set_mix(g, dtype, task);
+}
+int set_state_slots(mk_graph *g, const Tensor &ids, const char *task) {
+  if (ids.dtype != MK_DT_I32 || (int)ids.elems() < g->cfg.max_num_batched_requests) return fail(MK_EINVAL, "%s: one int32 state slot per batch slot", task);
+  if (g->state_ids && g->state_ids != (int *)ids.ptr) return fail(MK_EINVAL, "%s: every recurrence of a graph uses the same state-slot tensor", task);
+  g->state_ids = (int *)ids.ptr;
+  return MK_OK;
+}
+bool tail_ok(const mk_graph *g, const Tensor &t, int taps, int n, int dtype) {
+  return t.ndims == 3 && t.dtype == dtype && t.dims[0] >= g->cfg.max_num_batched_requests && t.dims[1] >= (taps > 1 ? taps - 1 : 1) && t.dims[2] == n && t.strides[1] == n &&
+         (taps == 1 || t.dims[1] == taps - 1);
+}
+
+// short_conv [rows, weights (fp32 [taps, channels]), bias (fp32), tail, state slots (int32), output] params [column]
+int lower_short_conv(mk_graph *g, size_t &i) {
+  const Task &t = g->ltasks[i];
+  if (t.ops.size() != 6 || t.params.size() != 1) return fail(MK_EINVAL, "short_conv expects 6 operands / 1 param");
+  const Tensor &in = g->tensors[t.ops[0]], &w = g->tensors[t.ops[1]], &b = g->tensors[t.ops[2]], &tail = g->tensors[t.ops[3]], &o = g->tensors[t.ops[5]];
+  const int B = g->cfg.max_num_batched_tokens, col = t.params[0], taps = w.ndims == 2 ? (int)w.dims[0] : 0, n = w.ndims == 2 ? (int)w.dims[1] : 0;
+  int rc = set_hyb(g, in.dtype, "short_conv");
+  if (rc) return rc;
+  if (taps < 1 || n < 4 || n % 4 || col < 0 || col % 4 || w.dtype != MK_DT_F32 || w.strides[0] != n || !vector_ok(b, n) || !rows_ok(in, B, (int64_t)col + n, in.dtype) || !rows_ok(o, B, n, in.dtype) ||
+      !tail_ok(g, tail, taps, n, in.dtype))
+    return fail(MK_EINVAL, "short_conv: %d taps over %d channels (a multiple of 4) at column %d do not fit the operands", taps, n, col);
+  if ((rc = set_state_slots(g, g->tensors[t.ops[4]], "short_conv"))) return rc;
+  MkStage st;
+  memset(&st, 0, sizeof(st));
+  st.op = MK_OP_HY_CONV;
+  st.n = n;
+  st.taps = taps;
+  st.in = in.ptr;
+  st.ld_in = (int)in.strides[0];
+  st.cols[0] = col;
+  st.norm_w = w.ptr;
+  st.in_bias = (const float *)b.ptr;
+  st.tail = tail.ptr;
+  st.out = o.ptr;
+  st.ld_out = (int)o.strides[0];
+  g->stages.push_back(st);
+  g->stage_desc.push_back(fmt("HY_CONV %s -> %s n=%d taps=%d", in.name.c_str(), o.name.c_str(), n, taps));
+  i++;
+  return MK_OK;
+}
+
+// scan_step [rows, weights (operand order), offset (fp32), output (fp32)] params [n, k, column]: softplus(W x + offset)
+int lower_scan_step(mk_graph *g, size_t &i) {
+  const Task &t = g->ltasks[i];
+  if (t.ops.size() != 4 || t.params.size() != 3) return fail(MK_EINVAL, "scan_step expects 4 operands / 3 params");
+  const Tensor &in = g->tensors[t.ops[0]], &w = g->tensors[t.ops[1]], &b = g->tensors[t.ops[2]], &o = g->tensors[t.ops[3]];
+  const int B = g->cfg.max_num_batched_tokens, n = t.params[0], k = t.params[1], col = t.params[2];
+  int rc = set_hyb(g, in.dtype, "scan_step");
+  if (rc) return rc;
+  const int es = in.dtype == MK_DT_F32 ? 4 : 2, kw = 64 / es, epc = 16 / es;
+  if (n < 16 || n % 16 || k < kw || k % kw || col < 0 || col % epc || in.strides[0] % epc || !rows_ok(in, B, (int64_t)col + k, in.dtype) || !rows_ok(o, B, n, MK_DT_F32) || !vector_ok(b, n) ||
+      w.dtype != in.dtype || (int64_t)w.elems() != (int64_t)n * k)
+    return fail(MK_EINVAL, "scan_step: %d x %d weights (multiples of 16 and %d) at column %d do not fit the operands", n, k, kw, col);
+  MkStage st;
+  memset(&st, 0, sizeof(st));
+  st.op = MK_OP_HY_STEP;
+  st.groups = 1;
+  st.n = n;
+  st.k = k;
+  st.in = (const char *)in.ptr + (size_t)col * es;
+  st.ld_in = (int)in.strides[0];
+  st.w.nseg = 1;
+  st.w.seg[0] = w.ptr;
+  st.in_bias = (const float *)b.ptr;
+  st.out2 = o.ptr;
+  st.ld_out2 = (int)o.strides[0];
+  g->stages.push_back(st);
+  g->stage_desc.push_back(fmt("HY_STEP %s x %s -> %s n=%d k=%d", in.name.c_str(), w.name.c_str(), o.name.c_str(), n, k));
+  g->weight_bytes += (int64_t)w.elems() * es;
+  i++;
+  return MK_OK;
+}
+
+// selective_scan [rows, convolved rows, step sizes (fp32), B / C rows, A (fp32 [channels, states up to 4]), D (fp32), state (fp32), tail,
+// state slots (int32), output] params [states, taps, x column, z column of the rows, B column, C column of the B / C rows]
+int lower_selective_scan(mk_graph *g, size_t &i) {
+  const Task &t = g->ltasks[i];
+  if (t.ops.size() != 10 || t.params.size() != 6) return fail(MK_EINVAL, "selective_scan expects 10 operands / 6 params");
+  const Tensor &in = g->tensors[t.ops[0]], &xc = g->tensors[t.ops[1]], &dt = g->tensors[t.ops[2]], &bc = g->tensors[t.ops[3]], &A = g->tensors[t.ops[4]], &D = g->tensors[t.ops[5]],
+               &state = g->tensors[t.ops[6]], &tail = g->tensors[t.ops[7]], &o = g->tensors[t.ops[9]];
+  const int B = g->cfg.max_num_batched_tokens, N = t.params[0], taps = t.params[1], xcol = t.params[2], zcol = t.params[3], bcol = t.params[4], ccol = t.params[5], np = (N + 3) / 4 * 4;
+  int rc = set_hyb(g, in.dtype, "selective_scan");
+  if (rc) return rc;
+  const int n = A.ndims == 2 ? (int)A.dims[0] : 0;
+  if (N < 1 || N > MK_HY_MAX_STATES || taps < 1 || n < 4) return fail(MK_EUNSUPPORTED, "selective_scan: %d channels, %d states (at most %d), %d taps", n, N, MK_HY_MAX_STATES, taps);
+  if (A.dtype != MK_DT_F32 || A.dims[1] != np || A.strides[0] != np || !vector_ok(D, n) || xcol < 0 || zcol < 0 || bcol < 0 || ccol < 0 || bcol % 4 || ccol % 4 ||
+      !rows_ok(in, B, (int64_t)std::max(xcol, zcol) + n, in.dtype) || !rows_ok(xc, B, n, in.dtype) || !rows_ok(dt, B, n, MK_DT_F32) || !rows_ok(bc, B, (int64_t)std::max(bcol, ccol) + np, in.dtype) ||
+      !rows_ok(o, B, n, in.dtype) || !tail_ok(g, tail, taps, n, in.dtype))
+    return fail(MK_EINVAL, "selective_scan: %d channels of %d states and %d taps do not fit the operands", n, N, taps);
+  if (state.dtype != MK_DT_F32 || state.ndims != 3 || state.dims[0] < g->cfg.max_num_batched_requests || state.dims[1] != n || state.dims[2] != np || state.strides[1] != np)
+    return fail(MK_EINVAL, "selective_scan: the state is fp32 [>= %d slots, %d, %d]", g->cfg.max_num_batched_requests, n, np);
+  if ((rc = set_state_slots(g, g->tensors[t.ops[8]], "selective_scan"))) return rc;
+  MkStage st;
+  memset(&st, 0, sizeof(st));
+  st.op = MK_OP_HY_SCAN;
+  st.n = n;
+  st.states = N;
+  st.taps = taps;
+  st.in = in.ptr;
+  st.ld_in = (int)in.strides[0];
+  st.cols[0] = xcol;
+  st.cols[1] = bcol;
+  st.cols[2] = ccol;
+  st.cols[3] = zcol;
+  st.q_ws = xc.ptr;
+  st.ld_qws = (int)xc.strides[0];
+  st.in2 = dt.ptr;
+  st.ld_in2 = (int)dt.strides[0];
+  st.in3 = bc.ptr;
+  st.ld_in3 = (int)bc.strides[0];
+  st.a_tab = (const float *)A.ptr;
+  st.d_tab = (const float *)D.ptr;
+  st.k_cache = state.ptr;
+  st.tail = tail.ptr;
+  st.out = o.ptr;
+  st.ld_out = (int)o.strides[0];
+  g->stages.push_back(st);
+  g->stage_desc.push_back(fmt("HY_SCAN %s -> %s n=%d states=%d taps=%d", in.name.c_str(), o.name.c_str(), n, N, taps));
+  i++;
+  return MK_OK;
+}
+
+// expert_route [logits (fp32), ids (int32 [tokens, top]), shares (fp32)] params [experts, top, shared 0/1]: the stage runs for
+// iterations of several tokens; the expert_linear behind it routes a single one itself.
+// expert_linear [rows, weights, shared weights (optional), ids, output] params [experts, top, n, k, shared n, shared k, gated 0/1, input
+// columns per place (0: one row for all), output columns per place]
+bool route_ok(int experts, int top) { return experts >= 1 && experts <= MK_MOE_MAX_EXPERTS && top >= 1 && top <= experts && top <= MK_MOE_MAX_TOPK; }
+int lower_expert_route(mk_graph *g, size_t &i) {
+  const Task &t = g->ltasks[i];
+  if (t.ops.size() != 3 || t.params.size() != 3) return fail(MK_EINVAL, "expert_route expects 3 operands / 3 params");
+  const Tensor &z = g->tensors[t.ops[0]], &ids = g->tensors[t.ops[1]], &w = g->tensors[t.ops[2]];
+  const int B = g->cfg.max_num_batched_tokens, E = t.params[0], top = t.params[1], sh = t.params[2] ? 1 : 0;
+  g->mix = g->hyb = true;
+  if (!route_ok(E, top)) return fail(MK_EUNSUPPORTED, "expert_route: %d of %d experts (at most %d of %d)", top, E, MK_MOE_MAX_TOPK, MK_MOE_MAX_EXPERTS);
+  if (!rows_ok(z, B, E + sh, MK_DT_F32) || ids.ndims != 2 || ids.dtype != MK_DT_I32 || ids.dims[0] < B || ids.dims[1] != top || ids.strides[0] != top || !rows_ok(w, B, top + sh, MK_DT_F32))
+    return fail(MK_EINVAL, "expert_route: logits fp32 [tokens, %d], ids int32 [tokens, %d], shares fp32 [tokens, >= %d]", E + sh, top, top + sh);
+  if (i + 1 >= g->ltasks.size() || g->ltasks[i + 1].name != "expert_linear" || g->ltasks[i + 1].ops.size() != 5 || g->ltasks[i + 1].ops[3] != t.ops[1] ||
+      (g->ltasks[i + 1].ops[2] >= 0) != (sh != 0))
+    return fail(MK_EUNSUPPORTED, "expert_route is followed by the expert_linear that reads its ids");
+  MkStage st;
+  memset(&st, 0, sizeof(st));
+  st.op = MK_OP_HY_ROUTE;
+  st.flags = MK_F_ONLY_MULTI;
+  st.num_experts = E;
+  st.topk = top;
+  st.moe_logits = z.ptr;
+  st.ld_logits = (int)z.strides[0];
+  st.ids = (int *)ids.ptr;
+  st.slot_w = (const float *)w.ptr;
+  st.ld_slot_w = (int)w.strides[0];
+  st.w_shared = sh ? z.ptr : nullptr;  // (only its presence counts here)
+  g->stages.push_back(st);
+  g->stage_desc.push_back(fmt("HY_ROUTE[multi-token only] %s -> %s experts=%d top=%d shared=%d", z.name.c_str(), w.name.c_str(), E, top, sh));
+  i++;
+  return MK_OK;
+}
+int lower_expert_linear(mk_graph *g, size_t &i) {
+  const Task &t = g->ltasks[i];
+  if (t.ops.size() != 5 || t.params.size() != 9) return fail(MK_EINVAL, "expert_linear expects 5 operands / 9 params");
+  const Tensor &in = g->tensors[t.ops[0]], &w = g->tensors[t.ops[1]], &ids = g->tensors[t.ops[3]], &o = g->tensors[t.ops[4]];
+  const Tensor *ws = t.ops[2] >= 0 ? &g->tensors[t.ops[2]] : nullptr;
+  const int B = g->cfg.max_num_batched_tokens, E = t.params[0], top = t.params[1], n = t.params[2], k = t.params[3], ns = ws ? t.params[4] : 0, ks = ws ? t.params[5] : 0, glu = t.params[6] ? 2 : 1,
+            is = t.params[7], os = t.params[8];
+  int rc = set_hyb(g, in.dtype, "expert_linear");
+  if (rc) return rc;
+  const int es = in.dtype == MK_DT_F32 ? 4 : 2, kw = 64 / es, epc = 16 / es;
+  auto up32 = [](int64_t x) { return (x + 31) / 32 * 32; };
+  const int last = top + (ws ? 1 : 0) - 1;
+  if (!route_ok(E, top)) return fail(MK_EUNSUPPORTED, "expert_linear: %d of %d experts (at most %d of %d)", top, E, MK_MOE_MAX_TOPK, MK_MOE_MAX_EXPERTS);
+  if (n < 1 || k < kw || k % kw || is < 0 || is % epc || os < 4 || os % 4 || in.strides[0] % epc || (glu == 2 && (n % 32 || ns % 32)) || (ws && (ns < 1 || ks < kw || ks % kw)) ||
+      !rows_ok(in, B, (int64_t)last * is + std::max(k, ks), in.dtype) || !rows_ok(o, B, (int64_t)last * os + std::max(n, ns) / glu, in.dtype) || os < std::max(n, ns) / glu ||
+      w.dtype != in.dtype || (int64_t)w.elems() != E * up32(n) * k || (ws && (ws->dtype != in.dtype || (int64_t)ws->elems() != up32(ns) * ks)))
+    return fail(MK_EINVAL, "expert_linear: %d experts of %d x %d (reductions in whole operand rows of %d, outputs padded to 32 rows), a shared one of %d x %d, do not fit the operands", E, n, k, kw, ns, ks);
+  if (ids.ndims != 2 || ids.dtype != MK_DT_I32 || ids.dims[0] < B || ids.dims[1] != top || ids.strides[0] != top) return fail(MK_EINVAL, "expert_linear: ids are int32 [tokens, %d]", top);
+  MkStage st;
+  memset(&st, 0, sizeof(st));
+  st.op = MK_OP_HY_EXPERTS;
+  if (glu == 2) st.flags |= MK_F_SILU;
+  st.num_experts = E;
+  st.topk = top;
+  st.n = n;
+  st.k = k;
+  st.n_shared = ns;
+  st.k_shared = ks;
+  st.in = in.ptr;
+  st.ld_in = (int)in.strides[0];
+  st.ld_in_slot = is;
+  st.out = o.ptr;
+  st.ld_out = (int)o.strides[0];
+  st.ld_out_slot = os;
+  st.w.nseg = 1;
+  st.w.seg[0] = w.ptr;
+  st.w_shared = ws ? ws->ptr : nullptr;
+  st.ids = (int *)ids.ptr;
+  if (!g->stages.empty() && g->stages.back().op == MK_OP_HY_ROUTE && g->stages.back().ids == st.ids) {
+    const MkStage &r = g->stages.back();
+    if (r.num_experts != E) return fail(MK_EINVAL, "expert_linear: %d experts, the routing has %d", E, r.num_experts);
+    st.flags |= MK_F_MOE_INLINE_TOPK;
+    st.moe_logits = r.moe_logits;
+    st.ld_logits = r.ld_logits;
+    st.slot_w = r.slot_w;
+    st.ld_slot_w = r.ld_slot_w;
+  }
+  g->stages.push_back(st);
+  g->stage_desc.push_back(fmt("HY_EXPERTS%s%s %s -> %s experts=%d top=%d n=%d k=%d shared=%dx%d", (st.flags & MK_F_MOE_INLINE_TOPK) ? "+route" : "", glu == 2 ? "+silu" : "", in.name.c_str(), o.name.c_str(), E,
+                              top, n, k, ns, ks));
+  g->weight_bytes += ((int64_t)top * n * k + (int64_t)ns * ks) * es;
   i++;
   return MK_OK;
 }
@@ -1362,7 +1640,7 @@ int lower(mk_graph *g) {
   g->last_linear_task = g->last_linear_stage = -1;
   g->flex = FLEX_NONE;
   g->flex_items = g->flex_part = 0;
-  g->mix = false;
+  g->mix = g->hyb = false;
   g->state_ids = nullptr;
   const int B = g->cfg.max_num_batched_tokens;
   // The list that is lowered: the recorded tasks, with the composite ones spelt out as the tasks they stand for (the
@@ -1510,6 +1788,21 @@ int lower(mk_graph *g) {
       if (rc) return rc;
     } else if (t.name == "general_delta") {
       int rc = lower_general_delta(g, i);
+      if (rc) return rc;
+    } else if (t.name == "short_conv") {
+      int rc = lower_short_conv(g, i);
+      if (rc) return rc;
+    } else if (t.name == "scan_step") {
+      int rc = lower_scan_step(g, i);
+      if (rc) return rc;
+    } else if (t.name == "selective_scan") {
+      int rc = lower_selective_scan(g, i);
+      if (rc) return rc;
+    } else if (t.name == "expert_route") {
+      int rc = lower_expert_route(g, i);
+      if (rc) return rc;
+    } else if (t.name == "expert_linear") {
+      int rc = lower_expert_linear(g, i);
       if (rc) return rc;
     } else if (t.name == "moe_topk_softmax_mi300") {
       bool inline_next = false;
@@ -1729,7 +2022,12 @@ int lower(mk_graph *g) {
       case MK_OP_MX_LATENT_MERGE:
       case MK_OP_MX_DECAY:
       case MK_OP_MX_DELTA:
-      case MK_OP_MX_DELTA_OUT: st.prof_event = 116; break;
+      case MK_OP_MX_DELTA_OUT:
+      case MK_OP_HY_CONV:
+      case MK_OP_HY_SCAN: st.prof_event = 116; break;
+      case MK_OP_HY_STEP: st.prof_event = 120; break;
+      case MK_OP_HY_ROUTE: st.prof_event = 172; break;
+      case MK_OP_HY_EXPERTS: st.prof_event = (st.flags & MK_F_SILU) ? 170 : 171; break;
       case MK_OP_FX_ARGMAX_F32: st.prof_event = 110; break;
       case MK_OP_NGRAM_PARTIAL: st.prof_event = 112; break;
       case MK_OP_NGRAM_GLOBAL: st.prof_event = 113; break;
@@ -1786,7 +2084,8 @@ int task_type_id(const std::string &n) {
       {"silu_mul_linear_with_residual", 105}, {"rmsnorm_linear", 102}, {"identity", 121}, {"argmax", 109}, {"attention", 103},
       {"find_ngram_partial", 112}, {"find_ngram_global", 113}, {"target_verify_greedy", 114}, {"single_batch_extend_attention", 115},
       {"embedding_scaled", 101}, {"residual_rmsnorm", 119}, {"flex_attention", 116},
-      {"residual_prenorm", 119}, {"latent_prep", 116}, {"head_linear", 120}, {"latent_attention", 116}, {"general_delta", 116}};
+      {"residual_prenorm", 119}, {"latent_prep", 116}, {"head_linear", 120}, {"latent_attention", 116}, {"general_delta", 116},
+      {"relu_squared", 118}, {"short_conv", 116}, {"scan_step", 120}, {"selective_scan", 116}, {"expert_route", 172}, {"expert_linear", 170}};
   auto it = ids.find(n);
   return it == ids.end() ? 0 : it->second;
 }
@@ -2086,6 +2385,16 @@ static const void *kernel_of(const mk_graph *g) {
   if (g->flex == FLEX_NONE) {
 #ifdef MK_HAVE_KERNEL_DENSE
     k = m1 ? (const void *)mk_persistent_kernel_m1 : (const void *)mk_persistent_kernel;
+#endif
+  } else if (g->hyb) {
+#ifdef MK_HAVE_KERNEL_HYB
+    if (g->flex == FLEX_BF16 && !m1) k = (const void *)mk_persistent_kernel_hyb;
+#endif
+#ifdef MK_HAVE_KERNEL_HYB_M1
+    if (g->flex == FLEX_BF16 && m1) k = (const void *)mk_persistent_kernel_hyb_m1;
+#endif
+#ifdef MK_HAVE_KERNEL_HYB_F32
+    if (g->flex == FLEX_F32) k = (const void *)mk_persistent_kernel_hyb_f32;
 #endif
   } else if (g->mix) {
 #ifdef MK_HAVE_KERNEL_MIX
@@ -2402,8 +2711,8 @@ int mk_add_task(mk_graph *g, const char *task_name, const int grid_dim[3], const
     // (and the sink of flex_attention, the summand of residual_rmsnorm, what the mix tasks may leave out)
     const bool optional = ((t.name == "gang_attn_split_kv_mi300" || t.name == "kv_cache_update_mi300" || t.name == "paged_attention" ||
                            t.name == "paged_attention_split_kv_mi300" || t.name == "attention" || t.name == "single_batch_extend_attention") && i >= 3 && i <= 6) ||
-                          (t.name == "flex_attention" && i >= 3 && i <= 5) || (t.name == "residual_rmsnorm" && i == 0) ||
-                          (t.name == "residual_prenorm" && (i == 0 || i == 1 || i == 3)) || (t.name == "latent_prep" && i >= 2 && i <= 6) ||
+                          (t.name == "flex_attention" && i >= 3 && i <= (n_operands == 9 ? 6 : 5)) || (t.name == "expert_linear" && i == 2) || (t.name == "residual_rmsnorm" && i == 0) ||
+                          (t.name == "residual_prenorm" && (i == 0 || i == 1 || i == 3 || (n_operands == 8 && (i == 2 || i == 5)))) || (t.name == "latent_prep" && i >= 1 && i <= 7) ||
                           (t.name == "head_linear" && (i == 2 || i == 3)) || (t.name == "latent_attention" && (i == 3 || i == 4)) || (t.name == "general_delta" && i == 8);
     if (tensor_ids[i] >= (int)g->tensors.size() || tensor_ids[i] < (optional ? -1 : 0))
       return fail(MK_EINVAL, "task '%s': bad tensor id %d for operand %d", task_name, tensor_ids[i], i);
@@ -2423,7 +2732,8 @@ int mk_add_task(mk_graph *g, const char *task_name, const int grid_dim[3], const
                                 "paged_attention", "paged_attention_split_kv_mi300", "paged_attention_split_kv_merge_mi300",
                                 "paged_attention_ck_fmha_merge_mi300", "gang_attn_merge_mi300", "splitk_reduce_mi300", "silu_mul_linear_with_residual", "rmsnorm_linear", "identity", "argmax", "attention",
                                 "find_ngram_partial", "find_ngram_global", "target_verify_greedy", "single_batch_extend_attention",
-                                "embedding_scaled", "residual_rmsnorm", "flex_attention", "residual_prenorm", "latent_prep", "head_linear", "latent_attention", "general_delta"};
+                                "embedding_scaled", "residual_rmsnorm", "flex_attention", "residual_prenorm", "latent_prep", "head_linear", "latent_attention", "general_delta",
+                                "relu_squared", "short_conv", "scan_step", "selective_scan", "expert_route", "expert_linear"};
   bool ok = linear_kind(t.name, &a, &b, &c);
   for (auto k : known) ok = ok || t.name == k;
   if (!ok) return fail(MK_EUNSUPPORTED, "Unsupported task name: %s", task_name);

@@ -74,7 +74,12 @@ typedef const __attribute__((address_space(4))) MkWeight CWeight;
 #define MK_TUNE_R24 2
 #endif
 
-#if defined(MK_KERNEL_MIX) || defined(MK_KERNEL_MIX_M1) || defined(MK_KERNEL_MIX_F32)
+#if defined(MK_KERNEL_HYB) || defined(MK_KERNEL_HYB_M1) || defined(MK_KERNEL_HYB_F32)
+#define MK_HAVE_HYB 1
+#else
+#define MK_HAVE_HYB 0
+#endif
+#if defined(MK_KERNEL_MIX) || defined(MK_KERNEL_MIX_M1) || defined(MK_KERNEL_MIX_F32) || MK_HAVE_HYB
 #define MK_HAVE_MIX 1  // this translation unit holds a kernel with the mix stages (mk_mix.hip) beside the flex ones
 #else
 #define MK_HAVE_MIX 0
@@ -905,6 +910,15 @@ __device__ __forceinline__ void stage_norm(CStage &st, Ctx &c, int M, char *smem
 }
 
 __device__ __forceinline__ float silu_mul(float g, float u) { return g / (1.f + __expf(-g)) * u; }
+// activation of a plain linear's outputs (hybrid kernels: the square of relu where the stage asks for it)
+__device__ __forceinline__ float linear_act(CStage &st, float v) {
+#if MK_HAVE_HYB
+  const float p = fmaxf(v, 0.f);
+  return (st.flags & MK_F_RELU2) ? p * p : v;
+#else
+  return v;
+#endif
+}
 
 #if MK_HAVE_MIX  // a residual_prenorm in front of a single-token linear (mk_mix.hip): by the workgroup, by the control wavefront
 __device__ __forceinline__ void mx_x_m1_prenorm(CStage &st, const Ctx &c, uint32_t *xs, float *red);
@@ -1235,7 +1249,7 @@ __device__ __forceinline__ void stage_linear_m1_t(CStage &st, Ctx &c, char *smem
         }
 #pragma unroll
         for (int h = 0; h < NROW; h++) a[h] = wave_sum(a[h]);
-        const float v = SILU ? silu_mul(a[0], a[NROW - 1]) : a[0] + lres[i];
+        const float v = SILU ? silu_mul(a[0], a[NROW - 1]) : linear_act(st, a[0] + lres[i]);
         if (lane == 0) so[lo_[i] - o_begin] = (uint16_t)f2bf(v);
       }
     }
@@ -1262,7 +1276,7 @@ __device__ __forceinline__ void stage_linear_m1_t(CStage &st, Ctx &c, char *smem
         }
 #pragma unroll
         for (int h = 0; h < NROW; h++) a[h] = wave_sum(a[h]);
-        const float v = SILU ? silu_mul(a[0], a[NROW - 1]) : a[0] + r;
+        const float v = SILU ? silu_mul(a[0], a[NROW - 1]) : linear_act(st, a[0] + r);
         if (lane == 0) so[o - o_begin] = (uint16_t)f2bf(v);
       }
     }
@@ -1312,6 +1326,7 @@ __device__ __forceinline__ void stage_linear_m1_generic(CStage &st, Ctx &c, char
       for (int kc = lane; kc < k8; kc += 64) a0 = dot8(ldg_stream(w0 + kc), xs4[kc], a0);
       v = wave_sum(a0);
       if (st.flags & MK_F_RES) v += bf2f(ldc_u16(res + r));
+      v = linear_act(st, v);
     }
     if (lane == 0) out[r] = (uint16_t)f2bf(v);
   }
@@ -1522,7 +1537,7 @@ __device__ __forceinline__ void stage_linear_small(CStage &st, Ctx &c, int M, ch
     const int m = lane & (MB - 1), q = SILU ? 0 : lane / MB;
     float v;
     if (SILU) v = silu_mul(tot, dpp_f32<0x100 + MB>(tot));  // row_shl:MB: the up sum sits MB lanes above the gate sum
-    else v = tot + rf;
+    else v = linear_act(st, tot + rf);
     if (lane < Q * MB && m < M && o + q < o_end) so[m * n_loc + (o + q - o_begin)] = (uint16_t)f2bf(v);
   };
   // two groups in flight: while one is reduced the other one's rows are landing; tickets only grow, so the first
@@ -1826,7 +1841,7 @@ __device__ __forceinline__ void stage_linear_mfma_tiles(CStage &st, Ctx &c, cons
             if (silu) r = TW >= 2 ? silu_mul(acc[(2 * u) % TW][mt][i], acc[(2 * u + 1) % TW][mt][i]) : 0.f;
             else r = acc[u][mt][i];
             if ((st.flags & MK_F_RES) && n < n_out) r += bf2f(rrow[n]);
-            rr[i] = r;
+            rr[i] = linear_act(st, r);
           }
           stc_bf16x4(orow, otile * 16 + lg * 4, n_out, rr);
         }
@@ -2143,7 +2158,7 @@ __device__ __forceinline__ void stage_linear_mfma_xres(CStage &st, Ctx &c, const
             const int n = otile * 16 + lg * 4 + i;
             float r = v[mt][i];
             if ((st.flags & MK_F_RES) && n < n_out) r += bf2f(rrow[n]);
-            rr[i] = r;
+            rr[i] = linear_act(st, r);
           }
           stc_bf16x4(orow, otile * 16 + lg * 4, n_out, rr);
         }
@@ -2341,7 +2356,7 @@ __device__ __forceinline__ void stage_linear_mfma(CStage &st, Ctx &c, int M, cha
           const int n = n0 + i;
           float r = silu ? silu_mul(v[i], v2[i]) : v[i];
           if ((st.flags & MK_F_RES) && n < n_out) r += bf2f(rrow[n]);
-          rr[i] = r;
+          rr[i] = linear_act(st, r);
         }
         stc_bf16x4(orow, n0, n_out, rr);
       }
@@ -4136,6 +4151,9 @@ __device__ __attribute__((noinline)) void mk_verify_greedy(int stage, const MkRu
 #if MK_HAVE_MIX
 #include "mk_mix.hip"
 #endif
+#if MK_HAVE_HYB
+#include "mk_hybrid.hip"
+#endif
 #define MK_HAVE_FLEX 1
 #else
 #define MK_HAVE_FLEX 0
@@ -4192,6 +4210,13 @@ __device__ __forceinline__ void run_stage_program(const MkRuntime &rt, const MkR
         case MK_OP_MX_DECAY: stage_mx_head_linear_t<E, 1, MX_DECAY, false>(st, c, M, smem); break;
         case MK_OP_MX_DELTA: stage_mx_delta<E>(st, c, rt, M, MAXM == 1 || single, smem); break;
         case MK_OP_MX_DELTA_OUT: stage_mx_delta_out<E>(st, c, M); break;
+#endif
+#if MK_HAVE_HYB
+        case MK_OP_HY_CONV: stage_hy_conv<E>(st, c, rt, M); break;
+        case MK_OP_HY_STEP: stage_mx_head_linear_t<E, 1, MX_STEP, false>(st, c, M, smem); break;
+        case MK_OP_HY_SCAN: stage_hy_scan<E>(st, c, rt, M, MAXM == 1 || single); break;
+        case MK_OP_HY_ROUTE: stage_hy_route(st, c, M); break;
+        case MK_OP_HY_EXPERTS: stage_hy_experts<E, MAXM>(st, c, M, smem); break;
 #endif
         case MK_OP_EMBED: if constexpr (!FX) stage_embed(st, c, rt, M); break;
         case MK_OP_NORM: if constexpr (!FX) stage_norm(st, c, M, smem); break;
@@ -4469,6 +4494,21 @@ extern "C" __global__ __launch_bounds__(MK_THREADS, 1) void mk_persistent_kernel
 #endif
 #ifdef MK_KERNEL_MIX_F32
 extern "C" __global__ __launch_bounds__(MK_THREADS, 1) void mk_persistent_kernel_mix_f32(MK_KERNEL_ARGS) {
+  mk_kernel_body<MK_MAX_TOKENS, float>(rt, rtp, max_iters, run_scheduler);
+}
+#endif
+#ifdef MK_KERNEL_HYB  // graphs with hybrid stages (mk_hybrid.hip): the flex and mix stages and those
+extern "C" __global__ __launch_bounds__(MK_THREADS, 1) void mk_persistent_kernel_hyb(MK_KERNEL_ARGS) {
+  mk_kernel_body<MK_MAX_TOKENS, uint16_t>(rt, rtp, max_iters, run_scheduler);
+}
+#endif
+#ifdef MK_KERNEL_HYB_M1
+extern "C" __global__ __launch_bounds__(MK_THREADS, 1) void mk_persistent_kernel_hyb_m1(MK_KERNEL_ARGS) {
+  mk_kernel_body<1, uint16_t>(rt, rtp, max_iters, run_scheduler);
+}
+#endif
+#ifdef MK_KERNEL_HYB_F32
+extern "C" __global__ __launch_bounds__(MK_THREADS, 1) void mk_persistent_kernel_hyb_f32(MK_KERNEL_ARGS) {
   mk_kernel_body<MK_MAX_TOKENS, float>(rt, rtp, max_iters, run_scheduler);
 }
 #endif

@@ -26,6 +26,35 @@ __device__ __forceinline__ void mx_stc_quad(float *p, f32x4 v) {
   asm volatile("global_store_dwordx4 %0, %1, off sc1" ::"v"((const MK_GLOBAL void *)(unsigned long long)p), "v"(v) : "memory");
 }
 
+// Four values of a norm stage's summand: row `y` from value 4 s on.  Hybrid kernels: plus a bias, and st.slots rows of the token,
+// st.ld_slot apart, weighted by `w` (four of them requested at once).
+template <typename E>
+__device__ __forceinline__ f32x4 mx_summand(CStage &st, const E *y, const float *w, int s) {
+#if MK_HAVE_HYB
+  if (st.slots) {
+    f32x4 v = {0.f, 0.f, 0.f, 0.f};
+    for (int q0 = 0; q0 < st.slots; q0 += 4) {
+      f32x4 x[4];
+      float f[4];
+#pragma unroll
+      for (int q = 0; q < 4; q++) {
+        const int at = min(q0 + q, st.slots - 1);
+        x[q] = fx_ldc_quad(y + (size_t)at * st.ld_slot + 4 * s);
+        f[q] = q0 + q < st.slots ? ldc_f32(w + at) : 0.f;
+      }
+#pragma unroll
+      for (int q = 0; q < 4; q++) v += x[q] * f[q];
+    }
+    return v;
+  }
+  f32x4 v = fx_ldc_quad(y + 4 * s);
+  if (st.in_bias) v += *(const f32x4 *)(st.in_bias + 4 * s);
+  return v;
+#else
+  return fx_ldc_quad(y + 4 * s);
+#endif
+}
+
 // ----------------------------------------------------------------------------- residual sum + norm in parts
 // v = x + alpha * f(y),  f(y) = y or y / sqrt(mean(y^2) + norm_eps) * y_norm_w;  out2 = v (32-bit);  out = the RMS norm of v in
 // st.norm_groups equal parts times norm_w (norm_groups 0: v itself), rounded to E.  Rows are st.n long, st.k of them real (the
@@ -58,7 +87,7 @@ __device__ __forceinline__ void stage_mx_prenorm_t(CStage &st, Ctx &c, int M, ch
     if (st.in) {
       f32x4 y[NS];
 #pragma unroll
-      for (int j = 0; j < NS; j++) y[j] = fx_ldc_quad((const E *)st.in + (size_t)t * st.ld_in + 4 * at(j));
+      for (int j = 0; j < NS; j++) y[j] = mx_summand<E>(st, (const E *)st.in + (size_t)t * st.ld_in, MK_HAVE_HYB ? st.slot_w + (size_t)t * st.ld_slot_w : nullptr, at(j));
       float f = st.alpha;
       if (yw4) {
         float ss = 0.f;
@@ -128,7 +157,7 @@ __device__ __forceinline__ void mx_x_m1_prenorm(CStage &st, const Ctx &c, uint32
   if (st.y_in && st.y_norm_w) {
     float ss = 0.f;
     for (int i = tid; i < k4; i += MK_THREADS) {
-      const f32x4 y = fx_ldc_quad((const uint16_t *)st.y_in + 4 * i);
+      const f32x4 y = mx_summand<uint16_t>(st, (const uint16_t *)st.y_in, MK_HAVE_HYB ? st.slot_w : nullptr, i);
       ss += y[0] * y[0] + y[1] * y[1] + y[2] * y[2] + y[3] * y[3];
     }
     f = 1.f / sqrtf(block_sum(ss, red) / (float)st.k_real + st.norm_eps);
@@ -136,7 +165,7 @@ __device__ __forceinline__ void mx_x_m1_prenorm(CStage &st, const Ctx &c, uint32
   for (int i = tid; i < k4; i += MK_THREADS) {
     f32x4 v = fx_ldc_quad((const float *)st.res + 4 * i);
     if (st.y_in) {
-      f32x4 y = fx_ldc_quad((const uint16_t *)st.y_in + 4 * i);
+      f32x4 y = mx_summand<uint16_t>(st, (const uint16_t *)st.y_in, MK_HAVE_HYB ? st.slot_w : nullptr, i);
       if (st.y_norm_w) y = (y * f) * ((const f32x4 *)st.y_norm_w)[i];
 #pragma unroll
       for (int e = 0; e < 4; e++) v[e] = fmaf(st.alpha, y[e], v[e]);
@@ -188,10 +217,51 @@ __device__ __forceinline__ void mx_x_m1_prenorm_wave(CStage &st, Ctx &c, uint32_
   if (c.pending && lane == 0) barrier_poll(c);
   if (!early) load_x();
   if (st.y_in) {
+#if MK_HAVE_HYB
+    f32x4 y[KL][2];
+    if (st.slots == 0) {
+      u32x4 raw[KL];
+#pragma unroll
+      for (int kc = 0; kc < KL; kc++) raw[kc] = ldc_16B((const u32x4 *)st.y_in + kc * 64 + lane);
+#pragma unroll
+      for (int kc = 0; kc < KL; kc++)
+#pragma unroll
+        for (int h = 0; h < 2; h++) {
+          y[kc][h] = (f32x4){bf_lo(raw[kc][2 * h]), bf_hi(raw[kc][2 * h]), bf_lo(raw[kc][2 * h + 1]), bf_hi(raw[kc][2 * h + 1])};
+          if (st.in_bias) y[kc][h] += *(const f32x4 *)(st.in_bias + ((kc * 64 + lane) * 2 + h) * 4);
+        }
+    } else {
+#pragma unroll
+      for (int kc = 0; kc < KL; kc++)
+#pragma unroll
+        for (int h = 0; h < 2; h++) y[kc][h] = (f32x4){0.f, 0.f, 0.f, 0.f};
+      u32x4 raw[2][KL];
+      float f[2];
+      auto fetch = [&](int q, u32x4 (&r)[KL], float &g_) {
+        const int at = min(q, st.slots - 1);
+#pragma unroll
+        for (int kc = 0; kc < KL; kc++) r[kc] = ldc_16B((const u32x4 *)((const uint16_t *)st.y_in + (size_t)at * st.ld_slot) + kc * 64 + lane);
+        g_ = q < st.slots ? ldc_f32(st.slot_w + at) : 0.f;
+      };
+      for (int q = 0; q < st.slots; q += 2) {
+        fetch(q, raw[0], f[0]);
+        fetch(q + 1, raw[1], f[1]);
+#pragma unroll
+        for (int z = 0; z < 2; z++)
+#pragma unroll
+          for (int kc = 0; kc < KL; kc++)
+#pragma unroll
+            for (int h = 0; h < 2; h++)
+              y[kc][h] += (f32x4){bf_lo(raw[z][kc][2 * h]), bf_hi(raw[z][kc][2 * h]), bf_lo(raw[z][kc][2 * h + 1]), bf_hi(raw[z][kc][2 * h + 1])} * f[z];
+      }
+    }
+    auto ye = [&](int kc, int h, int e) { return y[kc][h][e]; };
+#else
     u32x4 y[KL];
 #pragma unroll
     for (int kc = 0; kc < KL; kc++) y[kc] = ldc_16B((const u32x4 *)st.y_in + kc * 64 + lane);
     auto ye = [&](int kc, int h, int e) { return (e & 1) ? bf_hi(y[kc][h * 2 + (e >> 1)]) : bf_lo(y[kc][h * 2 + (e >> 1)]); };
+#endif
     float r = 1.f;
     if (yw4) {
       float ss = 0.f;
@@ -300,7 +370,7 @@ __device__ __forceinline__ void stage_mx_linear_m1_t(CStage &st, Ctx &c, char *s
         stc_f32((float *)st.out2 + row, v);
         stc_u16((uint16_t *)st.norm_out + row, (uint16_t)f2bf(v));
       } else {
-        stc_u16((uint16_t *)st.out + row, (uint16_t)f2bf(v));
+        stc_u16((uint16_t *)st.out + row, (uint16_t)f2bf(linear_act(st, v)));
       }
     }
   };
@@ -384,11 +454,11 @@ __device__ __forceinline__ void stage_mx_latent_prep(CStage &st, Ctx &c, const M
   constexpr int KW = FxType<E>::KW;
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int R = st.rank, rot = st.rot_dims, half = rot / 2, nrc = (R + KW - 1) / KW, nkc = nrc + (rot + KW - 1) / KW, ps = rt.page_size;
-  const int per = st.k_cache ? 2 : 1, total = M * per;
+  const int nq = st.n > 0, per = nq + (st.k_cache ? 1 : 0), total = M * per;  // (a model may form its queries without a latent)
   for (int i = mx_wave_item(c, wave); i < total; i += c.G * MK_WAVES) {
     const int t = i / per;
     const E *row = (const E *)st.in + (size_t)t * st.ld_in;
-    if (i - t * per == 0) {
+    if (i - t * per < nq) {
       E *o = (E *)st.out + (size_t)t * st.ld_out;
       mx_norm_row<E>(row + st.cols[0], (const float *)st.q_norm_w, st.n, st.eps, lane, [&](int q, f32x4 v) { fx_stc_quad(o + 4 * q, v); });
     } else {
@@ -420,9 +490,11 @@ __device__ __forceinline__ void stage_mx_latent_prep(CStage &st, Ctx &c, const M
 // are [head][n / 16][k / KW][64 lanes][EPC]: lane l holds row l % 16, k (l / 16) * EPC .. .  A wavefront per 16-row tile and all
 // tokens; few tiles with long rows: a workgroup per tile and 16 tokens, its wavefronts split K.
 //   MX_GELU:   out = gelu(sum) * table[id(t)][n]
+//   MX_OUT32:  out2 = sum in 32 bits
+//   MX_STEP:   out2 = softplus(sum + in_bias[n]) in 32 bits
 //   MX_DECAY:  tanh is applied to the inputs (kept as value + remainder in bf16), out2 = exp(-exp(-1/2) sigmoid(sum + offset[n]))
 //              in 32 bits, and the gated activation runs beside it
-enum { MX_PLAIN, MX_GELU, MX_DECAY };
+enum { MX_PLAIN, MX_GELU, MX_DECAY, MX_OUT32, MX_STEP };
 template <typename E, int MT, int EPI, bool SPLIT>
 __device__ __forceinline__ void stage_mx_head_linear_t(CStage &st, Ctx &c, int M, char *smem) {
   constexpr int EPC = FxType<E>::EPC, KW = FxType<E>::KW, KB = MT == 4 ? 4 : SPLIT ? 16 : EPI == MX_DECAY ? 4 : 8, B16 = sizeof(E) == 2;
@@ -515,6 +587,19 @@ __device__ __forceinline__ void stage_mx_head_linear_t(CStage &st, Ctx &c, int M
 #pragma unroll
         for (int q = 0; q < 4; q++) d[q] = expf(-0.6065306597126334f * mx_sigmoid(E(), r[q] + w0[q]));
         fx_stc_quad((float *)st.out2 + (size_t)t * st.ld_out2 + n0, d);
+#if MK_HAVE_HYB
+      } else if constexpr (EPI == MX_OUT32) {
+        fx_stc4((float *)st.out2 + (size_t)t * st.ld_out2, n0, N, r);
+      } else if constexpr (EPI == MX_STEP) {
+        const f32x4 b = *(const f32x4 *)(st.in_bias + n0);
+        f32x4 d;
+#pragma unroll
+        for (int q = 0; q < 4; q++) {
+          const float z = r[q] + b[q];
+          d[q] = z > 20.f ? z : log1pf(expf(z));
+        }
+        fx_stc_quad((float *)st.out2 + (size_t)t * st.ld_out2 + n0, d);
+#endif
       } else {
         fx_stc4((E *)st.out + (size_t)t * st.ld_out + (size_t)h * st.ld_out_slot, n0, N, r);
       }
@@ -525,6 +610,13 @@ __device__ __forceinline__ void stage_mx_head_linear_t(CStage &st, Ctx &c, int M
 }
 template <typename E, int MAXM>
 __device__ __forceinline__ void stage_mx_head_linear(CStage &st, Ctx &c, int M, char *smem) {
+#if MK_HAVE_HYB
+  if (st.flags & MK_F_OUT32) {
+    if (st.groups * ((st.n + 15) / 16) * 4 <= c.G && st.k / FxType<E>::KW >= 8) stage_mx_head_linear_t<E, 1, MX_OUT32, true>(st, c, M, smem);
+    else stage_mx_head_linear_t<E, 1, MX_OUT32, false>(st, c, M, smem);
+    return;
+  }
+#endif
   if (st.groups * ((st.n + 15) / 16) * 4 <= c.G && st.k / FxType<E>::KW >= 8) {
     if (st.flags & MK_F_GELU_TABLE) stage_mx_head_linear_t<E, 1, MX_GELU, true>(st, c, M, smem);
     else stage_mx_head_linear_t<E, 1, MX_PLAIN, true>(st, c, M, smem);

@@ -73,6 +73,13 @@ enum MkOp {
   MK_OP_MX_DECAY = 26,       // decays of the delta rule (low-rank product of tanh), gated activation beside it
   MK_OP_MX_DELTA = 27,       // generalised delta rule: recurrent state per request and head
   MK_OP_MX_DELTA_OUT = 28,   // norm and gate of its outputs (iterations that dealt heads in slices)
+  // selective scan, expert feed-forwards (mk_hybrid.hip); a graph that holds one, or a linear / attention / norm stage with an
+  // option of theirs, runs on the hybrid kernels
+  MK_OP_HY_CONV = 29,        // causal convolution per channel + silu
+  MK_OP_HY_STEP = 30,        // HEAD_LINEAR with a softplus behind an offset, 32-bit result (step sizes of the scan)
+  MK_OP_HY_SCAN = 31,        // selective scan: recurrent state per request, channel and state; convolution tail
+  MK_OP_HY_ROUTE = 32,       // router softmax -> top-k -> renormalise over 32-bit logits (iterations of several tokens)
+  MK_OP_HY_EXPERTS = 33,     // expert linears over the routed tokens and a shared expert over all of them
 };
 
 enum MkStageFlags {
@@ -90,6 +97,8 @@ enum MkStageFlags {
   MK_F_PRENORM = 4096,   // LINEAR (set together with MK_F_NORM): the norm in front is an MX_PRENORM; a single-token iteration forms it inside this stage
   MK_F_GELU_TABLE = 8192,  // MX_HEAD_LINEAR: out = gelu(acc) * table[id][n]
   MK_F_JOIN = 16384,     // LINEAR: a single-token iteration adds the result to the residual stream itself (the MX_PRENORM behind is multi-token only)
+  MK_F_RELU2 = 32768,    // LINEAR: out = max(acc, 0)^2
+  MK_F_OUT32 = 65536,    // MX_HEAD_LINEAR: 32-bit result in out2
   MK_F_RES_EARLY = 2048, // FX_ADDNORM / LINEAR+ADDNORM: the stage before this one does not write the residual rows, so they may be requested before its barrier
 };
 
@@ -99,6 +108,8 @@ enum MkStageFlags {
 #define MK_MX_MAX_CHUNKS 64      // split of a request's cached latents (one lane of the merging wavefront each)
 #define MK_MX_MAX_DELTA_DIM 256  // head size of the recurrence
 #define MK_MX_MAX_RANK 1024      // low-rank decay projection
+
+#define MK_HY_MAX_STATES 256     // states per channel of the selective scan
 
 #define MK_FX_MAX_HEAD_DIM 512  // largest q/k head the flex attention keeps in a wavefront's registers
 
@@ -182,7 +193,21 @@ struct MkStage {
   void *glu_out;
   int glu_n, ld_glu, glu_gate, glu_up;
   float glu_limit, glu_beta, glu_bias;
-  int pad_mx[9];
+  // hybrid stages (mk_hybrid.hip) and the options of older ones that go with them
+  int window, keep_first;  // FX_ATTN: a position sees the `window` newest ones (0: all) and the `keep_first` first ones
+  int v_col;               // FX_ATTN: column the value heads begin at
+  int slots;               // MX_PRENORM / LINEAR+PRENORM: summands per row (0: one, unweighted); HY_EXPERTS: rows per token
+  int ld_slot, ld_slot_w;  // ... columns per summand, weights per row
+  const float *slot_w;     // ... fp32 [tokens, ld_slot_w]
+  const float *in_bias;    // FX_ATTN / FX_PREP: added to the input rows; MX_PRENORM: added to the summand; HY_CONV; HY_STEP
+  const void *w_shared;    // HY_EXPERTS: weights of the expert every token visits (null: none)
+  int *ids;                // HY_ROUTE, HY_EXPERTS: int32 [tokens, topk] chosen experts
+  int n_shared, k_shared;  // HY_EXPERTS: outputs and reduction length of the shared expert
+  int states, taps;        // HY_SCAN: states per channel, taps of the convolution
+  const float *a_tab, *d_tab;  // HY_SCAN: fp32 [channels, states] log2(e) * A, [channels]
+  void *tail;              // HY_CONV / HY_SCAN: last inputs of the convolution, [state slot][taps - 1][channels]
+  const void *in3;         // HY_SCAN: step / B / C rows
+  int ld_in3, pad_hy[13];
 };
 static_assert(sizeof(MkStage) % 64 == 0, "a descriptor is whole scalar-cache lines");
 

@@ -14,7 +14,7 @@ import time
 import torch
 
 from mirage.mpk import MPK, MirageModelConfig, MPKMetadata, ServingSession
-from mirage.mpk.models import dodonex, suborax
+from mirage.mpk.models import bukatar, dodonex, suborax
 
 
 def suborax_shape(width=4096, heads=32, kv_heads=8, dim=128, vdim=128, ff=12288, layers=36, vocab=151936) -> dict:
@@ -37,14 +37,30 @@ def dodonex_shape(width=4096, heads=32, dim=128, rot_dim=64, vdim=128, q_rank=15
             "token_side": {"dim": side}, "layers": [delta if i % 2 else latent for i in range(layers)]}
 
 
+def bukatar_shape(width=4096, heads=32, kv_heads=8, dim=128, window=1024, keep_first=64, rot_dim=64, vdim=128, kv_rank=512, inner=8192, state=16, dt_rank=256, ff=12288, experts=64,
+                  top=8, expert_ff=1536, layers=36, vocab=151936) -> dict:
+    """A Bukatar config.json of the given sizes: windowed attention, latent attention and two scans by turns, dense and expert
+    feed-forwards by turns."""
+    dense = {"kind": "dense", "ff": ff}
+    moe = {"kind": "moe", "router": {"experts": experts, "top": top}, "expert": {"ff": expert_ff}, "shared": {"ff": expert_ff}}
+    att = {"type": "attention", "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "rot": {"base": 5e5, "dims": dim // 2}, "scale": dim ** -0.5,
+                                          "mask": {"size": window, "keep_first": keep_first}}}
+    lat = {"type": "latent_attention", "mixer": {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim, "kv_rank": kv_rank, "rot": {"base": 5e5, "dims": rot_dim},
+                                                 "scale": (dim + rot_dim) ** -0.5}}
+    ssm = {"type": "mamba1", "mixer": {"inner": inner, "state": state, "conv": 4, "dt_rank": dt_rank}}
+    cycle = [dict(att, mlp=dense), dict(lat, mlp=moe), dict(ssm, mlp=dense), dict(ssm, mlp=moe)]
+    return {"architecture": "Bukatar", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "layers": [cycle[i % 4] for i in range(layers)]}
+
+
 # name -> (config.json of a shape, its sizes)
 SHAPES = {"suborax-8b": (suborax_shape, {}), "suborax-2k": (suborax_shape, dict(width=2048, heads=32, kv_heads=4, ff=6144)),
-          "dodonex-8b": (dodonex_shape, {}), "dodonex-2k": (dodonex_shape, dict(width=2048, heads=16, q_rank=768, delta_heads=32, delta_dim=64, low_rank=64, ff=6144))}
+          "dodonex-8b": (dodonex_shape, {}), "dodonex-2k": (dodonex_shape, dict(width=2048, heads=16, q_rank=768, delta_heads=32, delta_dim=64, low_rank=64, ff=6144)),
+          "bukatar-8b": (bukatar_shape, {}), "bukatar-2k": (bukatar_shape, dict(width=2048, heads=16, kv_heads=4, inner=4096, dt_rank=128, ff=6144, experts=128, expert_ff=768))}
 
 
 def random_model(config: dict):
     """(MirageModelConfig with random-init weights, the reader's form of the config) of a parsed config.json."""
-    kind, module = {"Suborax": (suborax.SuboraxConfig, suborax), "Dodonex": (dodonex.DodonexConfig, dodonex)}[config["architecture"]]
+    kind, module = {"Suborax": (suborax.SuboraxConfig, suborax), "Dodonex": (dodonex.DodonexConfig, dodonex), "Bukatar": (bukatar.BukatarConfig, bukatar)}[config["architecture"]]
     sizes = kind.from_dict(config)
     return MirageModelConfig(architecture=config, state_dict=module.random_state_dict(sizes)), sizes
 

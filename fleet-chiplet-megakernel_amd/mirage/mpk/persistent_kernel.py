@@ -650,18 +650,21 @@ class PersistentKernel:
 
     def flex_attention_layer(self, input: DTensor, k_cache: DTensor, v_cache: DTensor, cos: DTensor, sin: DTensor, sink: DTensor, q_workspace: DTensor,
                              output: DTensor, num_q_heads: int, num_kv_heads: int, head_dim: int, v_dim: int, rot_dims: int, scale: float,
-                             softcap: float = 0.0, unit_norm: bool = False, eps: float = 1e-6):
+                             softcap: float = 0.0, unit_norm: bool = False, eps: float = 1e-6, window: int = 0, keep_first: int = 0, values_from_keys: bool = False,
+                             input_bias: DTensor = None):
         """Causal paged attention with rotary positions on the first `rot_dims` dims of each q/k head (rotate-half pairs;
         cos / sin are fp32 [positions, rot_dims / 2]), heads divided by their root mean square after the rotation
         (unit_norm), score = softcap * tanh(q.k * scale / softcap) (softcap 0: plain), and a per-head logit `sink` (fp32,
         None: none) that only takes part in the softmax's denominator.  input rows: all q heads, all k heads, all v heads.
-        Caches: [pages, page_size, kv_heads, flex_cache_dims(...)], in the kernel's own order inside a page."""
+        Caches: [pages, page_size, kv_heads, flex_cache_dims(...)], in the kernel's own order inside a page.  With a `window` a
+        position sees the `window` newest ones (its own among them) and the `keep_first` first ones.  values_from_keys: the rows
+        hold no value heads, the values are the key heads before rotation.  input_bias: fp32, added to the input rows."""
         assert input.num_dims == 2 and output.num_dims == 2 and q_workspace.num_dims == 2
         assert k_cache.num_dims == 4 and v_cache.num_dims == 4
-        self._task("flex_attention", (1, 1, 1), (256, 1, 1),
-                   [(input, _REPL, -1), (k_cache, _REPL, -1), (v_cache, _REPL, -1), (cos, _REPL, -1), (sin, _REPL, -1), (sink, _REPL, -1),
-                    (q_workspace, _REPL, -1), (output, _REPL, -1)],
-                   [num_q_heads, num_kv_heads, head_dim, v_dim, rot_dims, int(unit_norm), _f32_bits(eps), _f32_bits(scale), _f32_bits(softcap or 0.0)])
+        ops, p = [input, k_cache, v_cache, cos, sin, sink], [num_q_heads, num_kv_heads, head_dim, v_dim, rot_dims, int(unit_norm), _f32_bits(eps), _f32_bits(scale), _f32_bits(softcap or 0.0)]
+        if window or values_from_keys or input_bias is not None:
+            ops, p = ops + [input_bias], p + [window, keep_first, int(values_from_keys)]
+        self._task("flex_attention", (1, 1, 1), (256, 1, 1), [(t, _REPL, -1) for t in ops + [q_workspace, output]], p)
 
     # ------------------------------------------------------------------ mix layers (csrc/mk_mix.hip)
     # Like the flex layers above (and usable in one graph with them): constants are arguments, one activation type per graph.
@@ -676,22 +679,25 @@ class PersistentKernel:
         return out, [at, n, gate, up, _f32_bits(limit), _f32_bits(beta), _f32_bits(bias)]
 
     def residual_prenorm_layer(self, input: DTensor, residual: DTensor, new_residual: DTensor, output: DTensor, weight: DTensor = None, input_weight: DTensor = None,
-                               width: int = None, groups: int = 1, alpha: float = 1.0, eps: float = 1e-6, input_eps: float = 1e-6):
+                               width: int = None, groups: int = 1, alpha: float = 1.0, eps: float = 1e-6, input_eps: float = 1e-6, input_bias: DTensor = None,
+                               slot_weights: DTensor = None, slots: int = 0, slot_columns: int = 0):
         """new_residual (fp32) = v = residual + alpha * input (input None: a copy; with `input_weight`: the input is divided by
         its root mean square and multiplied by that weight first); output = v in `groups` equal parts, each divided by its
         own root mean square, times weight (weight None: v itself), rounded to the activation type.  A linear_layer over
-        `output` right behind forms it itself when an iteration has one token."""
+        `output` right behind forms it itself when an iteration has one token.  input_bias: fp32, added to the input rows.
+        slot_weights (fp32 [tokens, >= slots]): the input row is the weighted sum of `slots` rows, slot_columns apart."""
         assert residual.num_dims == 2 and new_residual.num_dims == 2 and output.num_dims == 2
-        self._task("residual_prenorm", (1, 1, 1), (256, 1, 1),
-                   [(input, _REPL, -1), (input_weight, _REPL, -1), (residual, _REPL, -1), (weight, _REPL, -1), (new_residual, _REPL, -1), (output, _REPL, -1)],
-                   [output.dim(1) if width is None else int(width), groups, _f32_bits(alpha), _f32_bits(eps), _f32_bits(input_eps)])
+        ops, p = [input, input_weight], [output.dim(1) if width is None else int(width), groups, _f32_bits(alpha), _f32_bits(eps), _f32_bits(input_eps)]
+        if input_bias is not None or slot_weights is not None:
+            ops, p = ops + [input_bias, slot_weights], p + [slots, slot_columns]
+        self._task("residual_prenorm", (1, 1, 1), (256, 1, 1), [(t, _REPL, -1) for t in ops + [residual, weight, new_residual, output]], p)
 
-    def latent_prep_layer(self, input: DTensor, q_weight: DTensor, output: DTensor, q_column: int, q_rank: int, eps: float, cache: DTensor = None,
+    def latent_prep_layer(self, input: DTensor, q_weight: DTensor = None, output: DTensor = None, q_column: int = 0, q_rank: int = 0, eps: float = 1e-6, cache: DTensor = None,
                           latent_weight: DTensor = None, cos: DTensor = None, sin: DTensor = None, latent_column: int = 0, latent_rank: int = 0, rot_column: int = 0,
                           rot_dims: int = 0, glu: tuple = None):
         """output = RMS norm of the query latent in columns [q_column, q_column + q_rank) of the input rows.  With a `cache`
         ([pages, page_size, latent_row_dim(...)]): the RMS-normalised key latent and the rotated shared key part
-        (rotate-half pairs) are appended to the request's page."""
+        (rotate-half pairs) are appended to the request's page.  Without q_weight and output there is no query latent."""
         out, p = self._glu_params(glu)
         self._task("latent_prep", (1, 1, 1), (256, 1, 1),
                    [(input, _REPL, -1), (q_weight, _REPL, -1), (latent_weight, _REPL, -1), (cos, _REPL, -1), (sin, _REPL, -1), (cache, _REPL, -1), (out, _REPL, -1),
@@ -700,7 +706,7 @@ class PersistentKernel:
     def head_linear_layer(self, input: DTensor, weight: DTensor, output: DTensor, heads: int, n: int, k: int, in_stride: int, out_stride: int, ids: DTensor = None,
                           table: DTensor = None, table_column: int = 0):
         """output[t, h * out_stride + j] = sum_i input[t, h * in_stride + i] W[h][j][i], j < n, i < k; `weight` is
-        operand_tiles(W).  With a table: gelu(tanh form) of the sum times table[ids[t], table_column + j]."""
+        operand_tiles(W).  An fp32 output of a bf16 graph (one head) receives the 32-bit sums.  With a table: gelu(tanh form) of the sum times table[ids[t], table_column + j]."""
         self._task("head_linear", (1, 1, 1), (256, 1, 1), [(input, _REPL, -1), (weight, _REPL, -1), (ids, _REPL, -1), (table, _REPL, -1), (output, _REPL, -1)],
                    [heads, n, k, in_stride, out_stride, table_column])
 
@@ -728,6 +734,46 @@ class PersistentKernel:
         self._task("general_delta", (1, 1, 1), (256, 1, 1),
                    [(input, _REPL, -1), (decay_weight, _REPL, -1), (decay_offset, _REPL, -1), (removal_offset, _REPL, -1), (norm_weight, _REPL, -1), (state, _REPL, -1),
                     (state_slots, _REPL, -1), (workspace, _REPL, -1), (out, _REPL, -1), (output, _REPL, -1)], [heads, dim, low_rank, *columns, _f32_bits(eps)] + p)
+
+    # ------------------------------------------------------------------ hybrid layers (csrc/mk_hybrid.hip)
+    # Usable in one graph with the flex and mix layers; constants are arguments.
+    def relu_squared_layer(self, input: DTensor, output: DTensor):
+        """output = max(input, 0)^2 behind the linear_layer that writes `input` (library-owned; it is the linear's epilogue and
+        `input` itself is not written)."""
+        self._task("relu_squared", (1, 1, 1), (256, 1, 1), [(input, _REPL, -1), (output, _REPL, -1)])
+
+    def short_conv_layer(self, input: DTensor, weight: DTensor, bias: DTensor, tail: DTensor, state_slots: DTensor, output: DTensor, column: int = 0):
+        """output[t, c] = silu(bias[c] + sum_j weight[j, c] x[t - (taps - 1) + j, c]) over a request's tokens, x = input[:, column + c],
+        zeros before the first.  weight fp32 [taps, channels]; tail [slots, max(taps - 1, 1), channels]: the last inputs of every
+        request, which the selective_scan_layer behind writes; state_slots as in general_delta_layer."""
+        self._task("short_conv", (1, 1, 1), (256, 1, 1), [(t, _REPL, -1) for t in (input, weight, bias, tail, state_slots, output)], [column])
+
+    def scan_step_layer(self, input: DTensor, weight: DTensor, offset: DTensor, output: DTensor, n: int, k: int, column: int = 0):
+        """output (fp32) = softplus(W input[:, column : column + k] + offset), W [n, k] given as operand_tiles."""
+        self._task("scan_step", (1, 1, 1), (256, 1, 1), [(t, _REPL, -1) for t in (input, weight, offset, output)], [n, k, column])
+
+    def selective_scan_layer(self, input: DTensor, conv: DTensor, step: DTensor, bc: DTensor, A: DTensor, D: DTensor, state: DTensor, tail: DTensor, state_slots: DTensor,
+                             output: DTensor, states: int, taps: int, x_column: int, z_column: int, b_column: int, c_column: int):
+        """Per request, channel c and state n, in fp32: S <- 2^(step_c A[c, n]) S + step_c x_c B_n, output_c = (sum_n S C_n + D_c x_c) silu(z_c)
+        with x = conv rows, z = input[:, z_column ...], B / C = bc[:, b_column / c_column ...]; A holds log2(e) times the negative rates,
+        [channels, states rounded up to 4].  state fp32 [slots, channels, states rounded up to 4] is carried from iteration to
+        iteration (zero where a request begins); the inputs input[:, x_column ...] of the last taps - 1 tokens go to `tail`."""
+        self._task("selective_scan", (1, 1, 1), (256, 1, 1), [(t, _REPL, -1) for t in (input, conv, step, bc, A, D, state, tail, state_slots, output)],
+                   [states, taps, x_column, z_column, b_column, c_column])
+
+    def expert_route_layer(self, logits: DTensor, ids: DTensor, shares: DTensor, experts: int, top: int, shared: bool = False):
+        """Softmax over the first `experts` fp32 logits, the `top` largest (ids, int32 [tokens, top]) and their scores divided by their
+        sum (shares, fp32).  shared: one more logit, whose sigmoid becomes shares[:, top].  Followed by the expert_linear_layer that
+        reads the ids (a single token is routed inside that one)."""
+        self._task("expert_route", (1, 1, 1), (256, 1, 1), [(logits, _REPL, -1), (ids, _REPL, -1), (shares, _REPL, -1)], [experts, top, int(shared)])
+
+    def expert_linear_layer(self, input: DTensor, weight: DTensor, ids: DTensor, output: DTensor, experts: int, top: int, n: int, k: int, out_stride: int, in_stride: int = 0,
+                            gated: bool = False, shared_weight: DTensor = None, shared_n: int = 0, shared_k: int = 0):
+        """output[t, s * out_stride + j] = sum_i W[ids[t, s]][j][i] input[t, s * in_stride + i] for every place s < top of a token, and with a
+        shared_weight place `top` for all tokens.  Weights are operand_tiles, rows padded to 32 per expert; gated: 16 gate rows
+        and 16 up rows by turns, output = silu(gate) up (n counts both).  in_stride 0: all places read the token's one row."""
+        self._task("expert_linear", (1, 1, 1), (256, 1, 1), [(t, _REPL, -1) for t in (input, weight, shared_weight, ids, output)],
+                   [experts, top, n, k, shared_n, shared_k, int(gated), in_stride, out_stride])
 
     # layers of the reference that are outside the one-GPU decode path
     def tensor_init_layer(self, *args, **kwargs):
@@ -1074,6 +1120,23 @@ def operand_tiles(w: torch.Tensor) -> torch.Tensor:
     w = torch.nn.functional.pad(w, (0, -k % kw, 0, -n % 16))
     n, k = w.shape[1:]
     return w.view(H, n // 16, 16, k // kw, 4, kw // 4).permute(0, 1, 3, 4, 2, 5).reshape(H * (n // 16), 16 * k).contiguous()
+
+
+def expert_tiles(w: torch.Tensor) -> torch.Tensor:
+    """[experts, n, k] matrices for expert_linear_layer: operand_tiles with n padded to 32."""
+    return operand_tiles(torch.nn.functional.pad(w, (0, 0, 0, -w.shape[1] % 32)))
+
+
+def gated_rows(gate: torch.Tensor, up: torch.Tensor) -> torch.Tensor:
+    """[experts, n, k] gate and up matrices (n a multiple of 16) as one, 16 rows of each by turns (expert_linear_layer, gated)."""
+    E, n, k = gate.shape
+    return torch.stack([gate.view(E, n // 16, 16, k), up.view(E, n // 16, 16, k)], dim=2).reshape(E, 2 * n, k)
+
+
+def pairs_to_halves(dim: int, rot_dims: int) -> torch.Tensor:
+    """Order of a head's rows that turns a rotation of neighbours (2i, 2i + 1) into the kernels' rotation of halves (i, i + rot / 2):
+    applied to the query and key rows of a projection (and to whatever reads them as values) it changes no score."""
+    return torch.tensor([*range(0, rot_dims, 2), *range(1, rot_dims, 2), *range(rot_dims, dim)])
 
 
 def latent_row_dim(rank: int, rot_dims: int, dtype: torch.dtype) -> int:
