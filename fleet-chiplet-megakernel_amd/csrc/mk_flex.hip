@@ -200,16 +200,8 @@ template <typename E> struct FxRows {
   int S;
   const float *part;
   size_t slice, ldp;
-  const float *bias;  // (hybrid kernels) added to every row, null: none
+  const float *bias;  // (hybrid kernels) added to every row where it is used, null: none
   template <int NS> __device__ __forceinline__ float get(int tok, int col) const {
-#if MK_HAVE_HYB
-    const float b = bias ? bias[col] : 0.f;
-    return sum<NS>(tok, col) + b;
-#else
-    return sum<NS>(tok, col);
-#endif
-  }
-  template <int NS> __device__ __forceinline__ float sum(int tok, int col) const {
     if constexpr (NS == 0) {
       return fx_ldc(in + (size_t)tok * ld + col);
     } else {
@@ -241,7 +233,28 @@ template <typename E> __device__ __forceinline__ FxRows<E> fx_rows(CStage &st, C
 // that computes, so that a wavefront can have the requests of two rows in flight; put(d, value) for every d < D.
 struct FxHead {
   float x[MK_FX_HEAD_REGS], xp[MK_FX_HEAD_REGS], cs[MK_FX_HEAD_REGS], sn[MK_FX_HEAD_REGS];
+#if MK_HAVE_HYB
+  float b[MK_FX_HEAD_REGS], bp[MK_FX_HEAD_REGS];  // bias of x and xp
+#endif
 };
+// Bias of a row's columns (hybrid kernels): requested beside the row, added when it is used.
+template <typename E>
+__device__ __forceinline__ void fx_bias_load(const FxRows<E> &rows, int col, int n, int rot, int lane, float (&b)[MK_FX_HEAD_REGS], float (&bp)[MK_FX_HEAD_REGS]) {
+#if MK_HAVE_HYB
+  const int half = rot >> 1;
+  const float *p = rows.bias;
+#pragma unroll
+  for (int j = 0; j < MK_FX_HEAD_REGS; j++) b[j] = bp[j] = 0.f;
+  if (!p) return;
+#pragma unroll
+  for (int j = 0; j < MK_FX_HEAD_REGS; j++)
+    if (j * 64 < n) {
+      const int d = min(j * 64 + lane, n - 1);
+      b[j] = p[col + d];
+      if (j * 64 < rot) bp[j] = p[col + (d < rot ? (d < half ? d + half : d - half) : d)];
+    }
+#endif
+}
 template <typename E>
 __device__ __forceinline__ void fx_head_load(CStage &st, const FxRows<E> &rows, int tok, int col, int pos, int lane, FxHead &h) {
   const int D = st.head_dim, rot = (st.flags & MK_F_ROPE) ? st.rot_dims : 0, half = rot >> 1;
@@ -262,6 +275,9 @@ __device__ __forceinline__ void fx_head_load(CStage &st, const FxRows<E> &rows, 
         }
       }
   });
+#if MK_HAVE_HYB
+  fx_bias_load(rows, col, D, rot, lane, h.b, h.bp);
+#endif
 }
 // ... and a value row, which is copied as it is: columns [0, n) of it, lane l holds every 64th
 template <typename E>
@@ -280,6 +296,10 @@ __device__ __forceinline__ void fx_head_finish(CStage &st, int lane, FxHead &h, 
   for (int j = 0; j < MK_FX_HEAD_REGS; j++)
     if (j * 64 < D) {
       const int d = j * 64 + lane;
+#if MK_HAVE_HYB
+      h.x[j] += h.b[j];
+      if (j * 64 < rot) h.xp[j] += h.bp[j];
+#endif
       if (j * 64 < rot && d < rot) h.x[j] = d < half ? h.x[j] * h.cs[j] - h.xp[j] * h.sn[j] : h.x[j] * h.cs[j] + h.xp[j] * h.sn[j];
       ss += d < D ? h.x[j] * h.x[j] : 0.f;
     }
@@ -341,6 +361,9 @@ __device__ __forceinline__ void stage_fx_prep(CStage &st, Ctx &c, const MkRuntim
       fx_head_load<E>(st, rows, t, s * D, pos, lane, h);
     } else {
       fx_value_load<E>(rows, t, fx_value_col(st) + (s - H - nkv) * DV, DV, lane, h.x);
+#if MK_HAVE_HYB
+      fx_bias_load(rows, fx_value_col(st) + (s - H - nkv) * DV, DV, 0, lane, h.b, h.bp);
+#endif
     }
   };
   auto finish = [&](int i, FxHead &h, int page) {
@@ -354,6 +377,10 @@ __device__ __forceinline__ void stage_fx_prep(CStage &st, Ctx &c, const MkRuntim
       fx_head_finish(st, lane, h, [&](int d, float v) { fx_stc(kc + fx_k_at<E>(page, pp, ps, nkv, s - H, nkc, d), fx_round<E>(v)); });
     } else {
       const int g = s - H - nkv;
+#if MK_HAVE_HYB
+#pragma unroll
+      for (int j = 0; j < MK_FX_HEAD_REGS; j++) h.x[j] += h.b[j];
+#endif
 #pragma unroll
       for (int j = 0; j < MK_FX_HEAD_REGS; j++)
         if (j * 64 + lane < DV) fx_stc(vc + fx_v_at<E>(page, pp, ps, nkv, g, nvb, j * 64 + lane), fx_round<E>(h.x[j]));
@@ -539,6 +566,10 @@ __device__ __forceinline__ void stage_fx_attn_t(CStage &st, Ctx &c, const MkRunt
       const int v_col = fx_value_col(st) + a.g * DV;
       float vv[MK_FX_HEAD_REGS];
       if (v_row) fx_value_load<E>(rows, a.t0, v_col, DV, lane, vv);
+#if MK_HAVE_HYB
+      float vb[MK_FX_HEAD_REGS], vbp[MK_FX_HEAD_REGS];
+      if (v_row) fx_bias_load(rows, v_col, DV, 0, lane, vb, vbp);
+#endif
       auto load_row = [&](int r, FxHead &h) {
         fx_head_load<E>(st, rows, a.t0, (r < a.nrows ? a.g * qpk + a.r0 + r : st.num_q_heads + a.g) * D, a.p, lane, h);
       };
@@ -556,7 +587,11 @@ __device__ __forceinline__ void stage_fx_attn_t(CStage &st, Ctx &c, const MkRunt
       if (v_row) {
 #pragma unroll
         for (int j = 0; j < MK_FX_HEAD_REGS; j++)
+#if MK_HAVE_HYB
+          if (j * 64 + lane < DV) vn[j * 64 + lane] = fx_round<E>(vv[j] + vb[j]);
+#else
           if (j * 64 + lane < DV) vn[j * 64 + lane] = fx_round<E>(vv[j]);
+#endif
       }
     } else {
       for (int i = tid; i < nkg * KC * 64; i += MK_THREADS) {

@@ -52,10 +52,10 @@ __device__ __forceinline__ void stage_hy_conv(CStage &st, Ctx &c, const MkRuntim
 
 // ----------------------------------------------------------------------------- selective scan
 // L lanes hold the states of a channel, Q quads each: lane j of them states 4 (i L + j) .. + 3, i < Q, so the sum over states stays
-// among L neighbours.  A workgroup takes 256 / L channels of one request and walks its tokens, TB at a time; the rows of the next
-// TB are in flight meanwhile.  A lane finishes (D x, gate, store) every L-th token's output.  State: fp32 [slot][channel][states
-// rounded up to 4], zero where a request begins.  dt: fp32 rows (in2), x: conv output rows (q_ws), B and C: columns cols[1], cols[2] of
-// in3, z: column cols[3] of in.
+// among L neighbours.  A lane works on CH channels at a time.  A workgroup takes 256 CH / L channels of one request and walks its
+// tokens, TB at a time; the rows of the next TB (or of the next unit, with its state) are in flight meanwhile.  A lane finishes (gate,
+// store) every L-th output.  State: fp32 [slot][channel][states rounded up to 4], zero where a request begins.  dt: fp32
+// rows (in2), x: conv output rows (q_ws), B and C: columns cols[1], cols[2] of in3, z: column cols[3] of in.
 template <int L>
 __device__ __forceinline__ float hy_lanes_sum(float v) {
   v += dpp_f32<0xB1>(v);  // quad_perm [1,0,3,2]
@@ -64,9 +64,9 @@ __device__ __forceinline__ float hy_lanes_sum(float v) {
   if (L >= 16) v += dpp_f32<0x140>(v);  // row_mirror
   return v;
 }
-template <typename E, int L, int Q, int TB>
+template <typename E, int L, int Q, int TB, int CH>
 __device__ __forceinline__ void stage_hy_scan_t(CStage &st, Ctx &c, const MkRuntime &rt, int M) {
-  constexpr int CW = MK_THREADS / L, KK = (TB + L - 1) / L;
+  constexpr int GW = 64 / L, CW = MK_WAVES * GW * CH, KK = (TB * CH + L - 1) / L;
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), j = lane % L;
   const int n = st.n, Np = (st.states + 3) / 4 * 4, nblk = (n + CW - 1) / CW;
   const MxDeltaUnits us = mx_delta_units(c, M);
@@ -74,21 +74,20 @@ __device__ __forceinline__ void stage_hy_scan_t(CStage &st, Ctx &c, const MkRunt
   const E *in = (const E *)st.in, *xc = (const E *)st.q_ws, *bc = (const E *)st.in3;
   const float *dtr = (const float *)st.in2;
   struct Unit {
-    int ch, t0, n, p0, slot;
-    bool real;
+    int ch0, t0, n, p0, slot;
   };
   auto unit = [&](int u) {
     Unit a;
     const int ri = u / nblk;
-    a.ch = (u - ri * nblk) * CW + wave * (64 / L) + lane / L;
-    a.real = a.ch < n;
-    a.ch = min(a.ch, n - 1);
+    a.ch0 = (u - ri * nblk) * CW + wave * GW * CH + lane / L;
     a.t0 = (int)__ffsll(__ballot(us.first && us.rank_of == ri)) - 1;
     a.n = wave_bcast(us.my_n, a.t0);
     a.p0 = __builtin_amdgcn_readfirstlane(c.sh_tok[a.t0]);
     a.slot = __builtin_amdgcn_readfirstlane(rt.state_ids[__builtin_amdgcn_readfirstlane(c.sh_tok[MK_MAX_TOKENS + a.t0])]);
     return a;
   };
+  auto channel = [&](const Unit &a, int h) { return min(a.ch0 + h * GW, n - 1); };  // (behind the last: computed, not stored)
+  auto real = [&](const Unit &a, int h) { return a.ch0 + h * GW < n; };
   int at[Q];
   bool on[Q];
 #pragma unroll
@@ -96,14 +95,16 @@ __device__ __forceinline__ void stage_hy_scan_t(CStage &st, Ctx &c, const MkRunt
     on[i] = 4 * (i * L + j) < Np;
     at[i] = min(4 * (i * L + j), Np - 4);
   }
-  auto state_of = [&](const Unit &a) { return (float *)st.k_cache + ((size_t)a.slot * n + a.ch) * Np; };
-  auto load_state = [&](const Unit &a, f32x4 (&S)[Q]) {
+  auto state_of = [&](const Unit &a, int h) { return (float *)st.k_cache + ((size_t)a.slot * n + channel(a, h)) * Np; };
+  auto load_state = [&](const Unit &a, f32x4 (&S)[CH][Q]) {
 #pragma unroll
-    for (int i = 0; i < Q; i++) S[i] = __builtin_nontemporal_load((const f32x4 *)(state_of(a) + at[i]));
+    for (int h = 0; h < CH; h++)
+#pragma unroll
+      for (int i = 0; i < Q; i++) S[h][i] = __builtin_nontemporal_load((const f32x4 *)(state_of(a, h) + at[i]));
   };
   struct Rows {
     f32x4 B[TB][Q], C[TB][Q];
-    float dt[TB], x[TB], z[KK];
+    float dt[TB][CH], x[TB][CH], z[KK];
   };
   auto load_rows = [&](const Unit &a, int tb, Rows &r) {
 #pragma unroll
@@ -114,98 +115,149 @@ __device__ __forceinline__ void stage_hy_scan_t(CStage &st, Ctx &c, const MkRunt
         r.B[t][i] = fx_ldc_quad(bc + tok * st.ld_in3 + st.cols[1] + at[i]);
         r.C[t][i] = fx_ldc_quad(bc + tok * st.ld_in3 + st.cols[2] + at[i]);
       }
-      r.dt[t] = ldc_f32(dtr + tok * st.ld_in2 + a.ch);
-      r.x[t] = fx_ldc(xc + tok * st.ld_qws + a.ch);
+#pragma unroll
+      for (int h = 0; h < CH; h++) {
+        r.dt[t][h] = ldc_f32(dtr + tok * st.ld_in2 + channel(a, h));
+        r.x[t][h] = fx_ldc(xc + tok * st.ld_qws + channel(a, h));
+      }
     }
 #pragma unroll
-    for (int k = 0; k < KK; k++) r.z[k] = fx_ldc(in + (size_t)(a.t0 + min(tb + k * L + j, a.n - 1)) * st.ld_in + st.cols[3] + a.ch);
+    for (int k = 0; k < KK; k++) r.z[k] = fx_ldc(in + (size_t)(a.t0 + min(tb + (k * L + j) / CH, a.n - 1)) * st.ld_in + st.cols[3] + channel(a, (k * L + j) % CH));
+  };
+  // The convolution's last inputs: the portion's, and before them what is left of the old ones.  Few taps: a lane per row, read with
+  // the unit's rows and written at its end; more: in ascending order by one thread (a row is read before it is written).
+  const int keep = st.taps - 1;
+  auto load_tail = [&](const Unit &a, E (&v)[CH]) {
+    const int i = a.n - keep + j;
+#pragma unroll
+    for (int h = 0; h < CH; h++) {
+      const E *old = (const E *)st.tail + ((size_t)a.slot * max(keep, 1) + min(j + a.n, max(keep, 1) - 1)) * n + channel(a, h);
+      v[h] = fx_round<E>(fx_ldc(i >= 0 ? in + (size_t)(a.t0 + min(i, a.n - 1)) * st.ld_in + st.cols[0] + channel(a, h) : old));
+    }
+  };
+  f32x4 A[CH][Q];
+  float D[CH];
+  auto load_rates = [&](const Unit &a) {
+#pragma unroll
+    for (int h = 0; h < CH; h++) {
+#pragma unroll
+      for (int i = 0; i < Q; i++) A[h][i] = *(const f32x4 *)(st.a_tab + (size_t)channel(a, h) * Np + at[i]);
+      D[h] = st.d_tab[channel(a, h)];
+    }
   };
   const int u0 = mx_spread(c);
-  f32x4 S[Q];
+  f32x4 S[CH][Q];
   Unit a{};
   // earlier iterations wrote the state: the first unit's is requested before the barrier is awaited
   const bool early = u0 < n_units && wave != 0;
   if (u0 < n_units) a = unit(u0);
-  if (early) load_state(a, S);
+  if (early) {
+    load_state(a, S);
+    load_rates(a);
+  }
   barrier_wait(c);
-  if (u0 < n_units && !early) load_state(a, S);
+  if (u0 < n_units && !early) {
+    load_state(a, S);
+    load_rates(a);
+  }
   Rows r;
-  if (u0 < n_units) load_rows(a, 0, r);
+  E tail[CH];
+  if (u0 < n_units) {
+    load_rows(a, 0, r);
+    load_tail(a, tail);
+  }
   for (int u = u0; u < n_units; u += c.G) {
     const Unit nx = u + c.G < n_units ? unit(u + c.G) : a;
-    f32x4 Sn[Q], A[Q];
+    f32x4 Sn[CH][Q];
+    E tail_n[CH];
     load_state(nx, Sn);
+    load_tail(nx, tail_n);
 #pragma unroll
-    for (int i = 0; i < Q; i++) {
-      A[i] = *(const f32x4 *)(st.a_tab + (size_t)a.ch * Np + at[i]);
-      if (!on[i] || a.p0 == 0) S[i] = (f32x4){0.f, 0.f, 0.f, 0.f};
-    }
-    const float D = st.d_tab[a.ch];
+    for (int h = 0; h < CH; h++)
+#pragma unroll
+      for (int i = 0; i < Q; i++)
+        if (!on[i] || a.p0 == 0) S[h][i] = (f32x4){0.f, 0.f, 0.f, 0.f};
     for (int tb = 0; tb < a.n; tb += TB) {
       Rows rn;
       const bool more = tb + TB < a.n;
       load_rows(more ? a : nx, more ? tb + TB : 0, rn);
-      float y[KK], x[KK];
+      float y[KK];
 #pragma unroll
       for (int t = 0; t < TB; t++) {
         if (TB > 1 && tb + t >= a.n) break;
-        const float dx = r.dt[t] * r.x[t];
-        float s = 0.f;
 #pragma unroll
-        for (int i = 0; i < Q; i++)
+        for (int h = 0; h < CH; h++) {
+          const float dx = r.dt[t][h] * r.x[t][h];
+          float s = 0.f;
 #pragma unroll
-          for (int e = 0; e < 4; e++) {
-            S[i][e] = fmaf(fx_exp2(E(), r.dt[t] * A[i][e]), S[i][e], on[i] ? dx * r.B[t][i][e] : 0.f);
-            s = fmaf(S[i][e], on[i] ? r.C[t][i][e] : 0.f, s);
-          }
-        s = hy_lanes_sum<L>(s);
-        if (t % L == j) {
-          y[t / L] = s;
-          x[t / L] = r.x[t];
+          for (int i = 0; i < Q; i++)
+#pragma unroll
+            for (int e = 0; e < 4; e++) {
+              S[h][i][e] = fmaf(fx_exp2(E(), r.dt[t][h] * A[h][i][e]), S[h][i][e], on[i] ? dx * r.B[t][i][e] : 0.f);
+              s = fmaf(S[h][i][e], on[i] ? r.C[t][i][e] : 0.f, s);
+            }
+          s = hy_lanes_sum<L>(s);
+          if ((t * CH + h) % L == j) y[(t * CH + h) / L] = s + D[h] * r.x[t][h];
         }
       }
 #pragma unroll
       for (int k = 0; k < KK; k++) {
-        const int t = k * L + j;
-        if (t < TB && tb + t < a.n && a.real) fx_stc((E *)st.out + (size_t)(a.t0 + tb + t) * st.ld_out + a.ch, fx_round<E>((y[k] + D * x[k]) * hy_silu(E(), r.z[k])));
+        const int t = (k * L + j) / CH, h = (k * L + j) % CH;
+        if (t < TB && tb + t < a.n && real(a, h)) fx_stc((E *)st.out + (size_t)(a.t0 + tb + t) * st.ld_out + channel(a, h), fx_round<E>(y[k] * hy_silu(E(), r.z[k])));
       }
       r = rn;
     }
-    if (a.real) {
+#pragma unroll
+    for (int h = 0; h < CH; h++) {
+      if (!real(a, h)) continue;
 #pragma unroll
       for (int i = 0; i < Q; i++)
-        if (on[i]) mx_stc_quad(state_of(a) + at[i], S[i]);
-      // the convolution's last inputs: the portion's, and before them what is left of the old ones (read further on than
-      // written, in ascending order, by this thread alone)
-      if (j == 0) {
-        const int keep = st.taps - 1;
-        E *tail = (E *)st.tail + (size_t)a.slot * keep * n + a.ch;
+        if (on[i]) mx_stc_quad(state_of(a, h) + at[i], S[h][i]);
+    }
+    if (keep <= L) {
+#pragma unroll
+      for (int h = 0; h < CH; h++)
+        if (j < keep && real(a, h)) fx_stc((E *)st.tail + ((size_t)a.slot * keep + j) * n + channel(a, h), tail[h]);
+    } else if (j == 0) {
+      for (int h = 0; h < CH; h++) {
+        if (!real(a, h)) continue;
+        E *rows = (E *)st.tail + (size_t)a.slot * keep * n + channel(a, h);
         for (int k = 0; k < keep; k++) {
           const int i = a.n - keep + k;
-          fx_stc(tail + (size_t)k * n, fx_round<E>(i >= 0 ? fx_ldc(in + (size_t)(a.t0 + i) * st.ld_in + st.cols[0] + a.ch) : fx_ldc(tail + (size_t)(k + a.n) * n)));
+          fx_stc(rows + (size_t)k * n, fx_round<E>(i >= 0 ? fx_ldc(in + (size_t)(a.t0 + i) * st.ld_in + st.cols[0] + channel(a, h)) : fx_ldc(rows + (size_t)(k + a.n) * n)));
         }
       }
     }
+    if (nx.ch0 != a.ch0) load_rates(nx);
     a = nx;
 #pragma unroll
-    for (int i = 0; i < Q; i++) S[i] = Sn[i];
+    for (int h = 0; h < CH; h++) {
+#pragma unroll
+      for (int i = 0; i < Q; i++) S[h][i] = Sn[h][i];
+      tail[h] = tail_n[h];
+    }
   }
   c.wrote_through = true;
 }
 template <typename E>
 __device__ __forceinline__ void stage_hy_scan(CStage &st, Ctx &c, const MkRuntime &rt, int M, bool single) {
+  // single tokens of many requests: eight channels per lane, so that a workgroup has enough in flight
+  const bool many = single && (long long)M * st.n * (st.states <= 16 ? 4 : st.states <= 32 ? 8 : 16) >= 4ll * c.G * MK_THREADS;
   if (st.states <= 16) {
-    if (single) stage_hy_scan_t<E, 4, 1, 1>(st, c, rt, M);
-    else stage_hy_scan_t<E, 4, 1, 8>(st, c, rt, M);
+    if (many) stage_hy_scan_t<E, 4, 1, 1, 8>(st, c, rt, M);
+    else if (single) stage_hy_scan_t<E, 4, 1, 1, 1>(st, c, rt, M);
+    else stage_hy_scan_t<E, 4, 1, 8, 1>(st, c, rt, M);
   } else if (st.states <= 32) {
-    if (single) stage_hy_scan_t<E, 8, 1, 1>(st, c, rt, M);
-    else stage_hy_scan_t<E, 8, 1, 8>(st, c, rt, M);
+    if (many) stage_hy_scan_t<E, 8, 1, 1, 8>(st, c, rt, M);
+    else if (single) stage_hy_scan_t<E, 8, 1, 1, 1>(st, c, rt, M);
+    else stage_hy_scan_t<E, 8, 1, 8, 1>(st, c, rt, M);
   } else if (st.states <= 64) {
-    if (single) stage_hy_scan_t<E, 16, 1, 1>(st, c, rt, M);
-    else stage_hy_scan_t<E, 16, 1, 8>(st, c, rt, M);
+    if (many) stage_hy_scan_t<E, 16, 1, 1, 8>(st, c, rt, M);
+    else if (single) stage_hy_scan_t<E, 16, 1, 1, 1>(st, c, rt, M);
+    else stage_hy_scan_t<E, 16, 1, 8, 1>(st, c, rt, M);
   } else {
-    if (single) stage_hy_scan_t<E, 16, 4, 1>(st, c, rt, M);
-    else stage_hy_scan_t<E, 16, 4, 2>(st, c, rt, M);
+    if (single) stage_hy_scan_t<E, 16, 4, 1, 1>(st, c, rt, M);
+    else stage_hy_scan_t<E, 16, 4, 2, 1>(st, c, rt, M);
   }
 }
 
@@ -275,7 +327,7 @@ __device__ __forceinline__ void stage_hy_route(CStage &st, Ctx &c, int M) {
 
 // ----------------------------------------------------------------------------- experts
 // Weights of an expert are operand tiles (see stage_mx_head_linear); a unit is a pair of 16-row tiles of one expert over all
-// tokens that visit it, its wavefronts split the reduction.  MK_F_SILU: the pair is gate and up of the same 16 outputs, out =
+// tokens that visit it.  Few units: a workgroup per unit, its wavefronts split the reduction; many: a wavefront per unit.  MK_F_SILU: the pair is gate and up of the same 16 outputs, out =
 // silu(gate) up.  Expert e < num_experts takes row (token, s) of `in` where s is its place among the token's choices (ld_in_slot 0:
 // the token's one row) and writes row (token, s) of `out`; the shared expert has its own sizes and place topk.
 // st.n / n_shared: rows of a matrix (gate and up together), st.k / k_shared: reduction length (whole operand rows).
@@ -288,11 +340,11 @@ struct HyLists {
   unsigned char place[MK_MOE_MAX_EXPERTS][MK_MAX_TOKENS];
 };
 static_assert(sizeof(HyLists) <= MK_MOE_OFFSET, "the lists lie below the scratch of the reduction");
-template <typename E, int MT, bool GLU>
+template <typename E, int MT, bool GLU, bool SPLIT>
 __device__ __forceinline__ void hy_expert_unit(CStage &st, const HyLists *ls, bool shared, int e, int pair, unsigned long long toks, int n, int K, int wave, int lane,
                                                const u32x4 *W, const u32x4 (&first)[2][4], f32x4 *red) {
   constexpr int EPC = FxType<E>::EPC, KW = FxType<E>::KW, KB = 4;
-  const int lr = lane & 15, lg = lane >> 4, nks = K / KW, kq = (nks + MK_WAVES - 1) / MK_WAVES, kb = min(nks, wave * kq), ke = min(nks, kb + kq);
+  const int lr = lane & 15, lg = lane >> 4, nks = K / KW, kq = SPLIT ? (nks + MK_WAVES - 1) / MK_WAVES : nks, kb = SPLIT ? min(nks, wave * kq) : 0, ke = min(nks, kb + kq);
   const int cnt = __popcll(toks);
   // lane r gets the r-th token of the list
   const int mine = (toks >> lane) & 1 ? __popcll(toks & ((1ull << lane) - 1ull)) : 63;
@@ -342,18 +394,23 @@ __device__ __forceinline__ void hy_expert_unit(CStage &st, const HyLists *ls, bo
 #pragma unroll
       for (int q = 0; q < KB; q++) a[h][q] = an[h][q];
   }
-  __syncthreads();
+  if constexpr (SPLIT) {
+    __syncthreads();
 #pragma unroll
-  for (int h = 0; h < 2; h++)
+    for (int h = 0; h < 2; h++)
 #pragma unroll
-    for (int m = 0; m < MT; m++) red[((wave * 2 + h) * MT + m) * 64 + lane] = acc[h][m];
-  __syncthreads();
-  auto total = [&](int h, int m) { return red[(h * MT + m) * 64 + lane] + red[((2 + h) * MT + m) * 64 + lane] + red[((4 + h) * MT + m) * 64 + lane] + red[((6 + h) * MT + m) * 64 + lane]; };
+      for (int m = 0; m < MT; m++) red[((wave * 2 + h) * MT + m) * 64 + lane] = acc[h][m];
+    __syncthreads();
+  }
+  auto total = [&](int h, int m) {
+    if constexpr (!SPLIT) return acc[h][m];
+    else return red[(h * MT + m) * 64 + lane] + red[((2 + h) * MT + m) * 64 + lane] + red[((4 + h) * MT + m) * 64 + lane] + red[((6 + h) * MT + m) * 64 + lane];
+  };
 #pragma unroll
   for (int m = 0; m < MT; m++) {
 #pragma unroll
     for (int h = 0; h < (GLU ? 1 : 2); h++) {
-      if (((GLU ? m : 2 * m + h) & (MK_WAVES - 1)) != wave || m * 16 + lr >= cnt) continue;
+      if ((SPLIT && ((GLU ? m : 2 * m + h) & (MK_WAVES - 1)) != wave) || m * 16 + lr >= cnt) continue;
       const f32x4 v = total(h, m);
       float r[4] = {v[0], v[1], v[2], v[3]};
       if (GLU) {
@@ -392,8 +449,8 @@ __device__ __forceinline__ void stage_hy_experts_t(CStage &st, Ctx &c, int M, ch
     return a;
   };
   u32x4 first[2][4];
-  auto load_first = [&](const Unit &a) {
-    const int nks = a.K / KW, kq = (nks + MK_WAVES - 1) / MK_WAVES, kb = min(nks, wave * kq);
+  auto load_first = [&](const Unit &a, bool split) {
+    const int nks = a.K / KW, kq = (nks + MK_WAVES - 1) / MK_WAVES, kb = split ? min(nks, wave * kq) : 0;
     const u32x4 *w0 = a.W + (size_t)(2 * a.pair) * nks * 64 + lane, *w1 = w0 + (size_t)nks * 64;
 #pragma unroll
     for (int q = 0; q < 4; q++) {
@@ -403,7 +460,7 @@ __device__ __forceinline__ void stage_hy_experts_t(CStage &st, Ctx &c, int M, ch
   };
   const int u0 = mx_spread(c);
   const bool early = u0 < pairs_s && wave != 0;
-  if (early) load_first(unit(u0));
+  if (early) load_first(unit(u0), true);
   if (tid == 0) __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "agent");
   barrier_wait(c);
   // ---- which experts have which tokens
@@ -441,24 +498,29 @@ __device__ __forceinline__ void stage_hy_experts_t(CStage &st, Ctx &c, int M, ch
   __syncthreads();
   const int n_units = pairs_s + __builtin_amdgcn_readfirstlane(ls->n_active) * pairs;
   const unsigned long long all = M >= 64 ? ~0ull : (1ull << M) - 1ull;
-  if (u0 < n_units && !early) load_first(unit(u0));
-  for (int u = u0; u < n_units; u += c.G) {
-    const Unit a = unit(u);
-    u32x4 f[2][4];
+  auto walk = [&](auto split, int u, int stride, bool have) {
+    constexpr bool SPLIT = decltype(split)::value;
+    if (u < n_units && !have) load_first(unit(u), SPLIT);
+    for (; u < n_units; u += stride) {
+      const Unit a = unit(u);
+      u32x4 f[2][4];
 #pragma unroll
-    for (int h = 0; h < 2; h++)
+      for (int h = 0; h < 2; h++)
 #pragma unroll
-      for (int q = 0; q < 4; q++) f[h][q] = first[h][q];
-    if (u + c.G < n_units) load_first(unit(u + c.G));
-    const bool shared = a.e < 0;
-    unsigned long long toks = all;
-    if (!shared) {
-      const unsigned long long t = ls->tok[a.e];
-      toks = (unsigned long long)(unsigned)__builtin_amdgcn_readfirstlane((int)t) | ((unsigned long long)(unsigned)__builtin_amdgcn_readfirstlane((int)(t >> 32)) << 32);
+        for (int q = 0; q < 4; q++) f[h][q] = first[h][q];
+      if (u + stride < n_units) load_first(unit(u + stride), SPLIT);
+      const bool shared = a.e < 0;
+      unsigned long long toks = all;
+      if (!shared) {
+        const unsigned long long t = ls->tok[a.e];
+        toks = (unsigned long long)(unsigned)__builtin_amdgcn_readfirstlane((int)t) | ((unsigned long long)(unsigned)__builtin_amdgcn_readfirstlane((int)(t >> 32)) << 32);
+      }
+      if (MAXM == 1 || __popcll(toks) <= 16) hy_expert_unit<E, 1, GLU, SPLIT>(st, ls, shared, a.e, a.pair, toks, a.n, a.K, wave, lane, a.W, f, red);
+      else hy_expert_unit<E, 4, GLU, SPLIT>(st, ls, shared, a.e, a.pair, toks, a.n, a.K, wave, lane, a.W, f, red);
     }
-    if (MAXM == 1 || __popcll(toks) <= 16) hy_expert_unit<E, 1, GLU>(st, ls, shared, a.e, a.pair, toks, a.n, a.K, wave, lane, a.W, f, red);
-    else hy_expert_unit<E, 4, GLU>(st, ls, shared, a.e, a.pair, toks, a.n, a.K, wave, lane, a.W, f, red);
-  }
+  };
+  if (MAXM == 1 || n_units < 3 * MK_WAVES * c.G) walk(std::true_type{}, u0, c.G, early);
+  else if constexpr (MAXM > 1) walk(std::false_type{}, mx_wave_item(c, wave), c.G * MK_WAVES, false);
   c.wrote_through = true;
 }
 template <typename E, int MAXM>

@@ -26,8 +26,8 @@ __device__ __forceinline__ void mx_stc_quad(float *p, f32x4 v) {
   asm volatile("global_store_dwordx4 %0, %1, off sc1" ::"v"((const MK_GLOBAL void *)(unsigned long long)p), "v"(v) : "memory");
 }
 
-// Four values of a norm stage's summand: row `y` from value 4 s on.  Hybrid kernels: plus a bias, and st.slots rows of the token,
-// st.ld_slot apart, weighted by `w` (four of them requested at once).
+// Four values of a norm stage's summand: row `y` from value 4 s on.  Hybrid kernels: the sum of st.slots rows of the
+// token, st.ld_slot apart, weighted by `w` (four of them requested at once).  (A bias is added by the caller, who has it in advance.)
 template <typename E>
 __device__ __forceinline__ f32x4 mx_summand(CStage &st, const E *y, const float *w, int s) {
 #if MK_HAVE_HYB
@@ -47,9 +47,7 @@ __device__ __forceinline__ f32x4 mx_summand(CStage &st, const E *y, const float 
     }
     return v;
   }
-  f32x4 v = fx_ldc_quad(y + 4 * s);
-  if (st.in_bias) v += *(const f32x4 *)(st.in_bias + 4 * s);
-  return v;
+  return fx_ldc_quad(y + 4 * s);
 #else
   return fx_ldc_quad(y + 4 * s);
 #endif
@@ -77,8 +75,25 @@ __device__ __forceinline__ void stage_mx_prenorm_t(CStage &st, Ctx &c, int M, ch
 #pragma unroll
     for (int j = 0; j < NS; j++) g[j] = w4[at(j)];
   }
+#if MK_HAVE_HYB  // (weights are requested before the barrier is awaited)
+  f32x4 yw[NS], yb[NS];
+  const f32x4 *yb4 = (const f32x4 *)st.in_bias;
+  if (yw4) {
+#pragma unroll
+    for (int j = 0; j < NS; j++) yw[j] = yw4[at(j)];
+  }
+  if (yb4) {
+#pragma unroll
+    for (int j = 0; j < NS; j++) yb[j] = yb4[at(j)];
+  }
+#endif
   // the residual row was written at least one barrier earlier than y: requested before the barrier is awaited (not by the
   // wavefront that polls it)
+#if MK_HAVE_HYB
+  auto yw_at = [&](int j) { return yw[j]; };
+#else
+  auto yw_at = [&](int j) { return yw4[at(j)]; };
+#endif
   const bool pre = (st.flags & MK_F_RES_EARLY) && t0 < M && tid >= 64;
   if (pre) load_x(t0);
   barrier_wait(c);
@@ -89,6 +104,12 @@ __device__ __forceinline__ void stage_mx_prenorm_t(CStage &st, Ctx &c, int M, ch
 #pragma unroll
       for (int j = 0; j < NS; j++) y[j] = mx_summand<E>(st, (const E *)st.in + (size_t)t * st.ld_in, MK_HAVE_HYB ? st.slot_w + (size_t)t * st.ld_slot_w : nullptr, at(j));
       float f = st.alpha;
+#if MK_HAVE_HYB
+      if (yb4) {
+#pragma unroll
+        for (int j = 0; j < NS; j++) y[j] += yb[j];
+      }
+#endif
       if (yw4) {
         float ss = 0.f;
 #pragma unroll
@@ -97,7 +118,7 @@ __device__ __forceinline__ void stage_mx_prenorm_t(CStage &st, Ctx &c, int M, ch
         ss = block_sum(ss, red);
         const float r = 1.f / sqrtf(ss / (float)st.k + st.norm_eps);
 #pragma unroll
-        for (int j = 0; j < NS; j++) y[j] = (y[j] * r) * yw4[at(j)];
+        for (int j = 0; j < NS; j++) y[j] = (y[j] * r) * yw_at(j);
       }
 #pragma unroll
       for (int j = 0; j < NS; j++)
@@ -157,7 +178,8 @@ __device__ __forceinline__ void mx_x_m1_prenorm(CStage &st, const Ctx &c, uint32
   if (st.y_in && st.y_norm_w) {
     float ss = 0.f;
     for (int i = tid; i < k4; i += MK_THREADS) {
-      const f32x4 y = mx_summand<uint16_t>(st, (const uint16_t *)st.y_in, MK_HAVE_HYB ? st.slot_w : nullptr, i);
+      f32x4 y = mx_summand<uint16_t>(st, (const uint16_t *)st.y_in, MK_HAVE_HYB ? st.slot_w : nullptr, i);
+      if (MK_HAVE_HYB && st.in_bias) y += ((const f32x4 *)st.in_bias)[i];
       ss += y[0] * y[0] + y[1] * y[1] + y[2] * y[2] + y[3] * y[3];
     }
     f = 1.f / sqrtf(block_sum(ss, red) / (float)st.k_real + st.norm_eps);
@@ -166,6 +188,7 @@ __device__ __forceinline__ void mx_x_m1_prenorm(CStage &st, const Ctx &c, uint32
     f32x4 v = fx_ldc_quad((const float *)st.res + 4 * i);
     if (st.y_in) {
       f32x4 y = mx_summand<uint16_t>(st, (const uint16_t *)st.y_in, MK_HAVE_HYB ? st.slot_w : nullptr, i);
+      if (MK_HAVE_HYB && st.in_bias) y += ((const f32x4 *)st.in_bias)[i];
       if (st.y_norm_w) y = (y * f) * ((const f32x4 *)st.y_norm_w)[i];
 #pragma unroll
       for (int e = 0; e < 4; e++) v[e] = fmaf(st.alpha, y[e], v[e]);
@@ -212,6 +235,13 @@ __device__ __forceinline__ void mx_x_m1_prenorm_wave(CStage &st, Ctx &c, uint32_
       g[kc][h] = w4[(kc * 64 + lane) * 2 + h];
       yw[kc][h] = yw4 ? yw4[(kc * 64 + lane) * 2 + h] : (f32x4){1.f, 1.f, 1.f, 1.f};
     }
+#if MK_HAVE_HYB
+  f32x4 yb[KL][2];
+#pragma unroll
+  for (int kc = 0; kc < KL; kc++)
+#pragma unroll
+    for (int h = 0; h < 2; h++) yb[kc][h] = st.in_bias ? ((const f32x4 *)st.in_bias)[(kc * 64 + lane) * 2 + h] : (f32x4){0.f, 0.f, 0.f, 0.f};
+#endif
   const bool early = st.flags & MK_F_RES_EARLY;
   if (early) load_x();
   if (c.pending && lane == 0) barrier_poll(c);
@@ -228,7 +258,7 @@ __device__ __forceinline__ void mx_x_m1_prenorm_wave(CStage &st, Ctx &c, uint32_
 #pragma unroll
         for (int h = 0; h < 2; h++) {
           y[kc][h] = (f32x4){bf_lo(raw[kc][2 * h]), bf_hi(raw[kc][2 * h]), bf_lo(raw[kc][2 * h + 1]), bf_hi(raw[kc][2 * h + 1])};
-          if (st.in_bias) y[kc][h] += *(const f32x4 *)(st.in_bias + ((kc * 64 + lane) * 2 + h) * 4);
+          y[kc][h] += yb[kc][h];
         }
     } else {
 #pragma unroll
