@@ -51,23 +51,23 @@ __device__ __forceinline__ void stage_hy_conv(CStage &st, Ctx &c, const MkRuntim
 }
 
 // ----------------------------------------------------------------------------- selective scan
-// L lanes hold the states of a channel, Q quads each: lane j of them states 4 (i L + j) .. + 3, i < Q, so the sum over states stays
+// L = 4, 8 or 16 lanes hold the states of a channel, Q quads each: lane j of them states 4 (i L + j) .. + 3, i < Q, so the sum over states stays
 // among L neighbours.  A lane works on CH channels at a time.  A workgroup takes 256 CH / L channels of one request and walks its
 // tokens, TB at a time; the rows of the next TB (or of the next unit, with its state) are in flight meanwhile.  A lane finishes (gate,
 // store) every L-th output.  State: fp32 [slot][channel][states rounded up to 4], zero where a request begins.  dt: fp32
 // rows (in2), x: conv output rows (q_ws), B and C: columns cols[1], cols[2] of in3, z: column cols[3] of in.
-template <int L>
-__device__ __forceinline__ float hy_lanes_sum(float v) {
+__device__ __forceinline__ float hy_lanes_sum(float v, int L) {
   v += dpp_f32<0xB1>(v);  // quad_perm [1,0,3,2]
   v += dpp_f32<0x4E>(v);  // quad_perm [2,3,0,1]
-  if (L >= 8) v += dpp_f32<0x141>(v);   // row_half_mirror
-  if (L >= 16) v += dpp_f32<0x140>(v);  // row_mirror
+  v += L >= 8 ? dpp_f32<0x141>(v) : 0.f;   // row_half_mirror
+  v += L >= 16 ? dpp_f32<0x140>(v) : 0.f;  // row_mirror
   return v;
 }
-template <typename E, int L, int Q, int TB, int CH>
-__device__ __forceinline__ void stage_hy_scan_t(CStage &st, Ctx &c, const MkRuntime &rt, int M) {
-  constexpr int GW = 64 / L, CW = MK_WAVES * GW * CH, KK = (TB * CH + L - 1) / L;
-  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), j = lane % L;
+template <typename E, int Q, int TB, int CH>
+__device__ __forceinline__ void stage_hy_scan_t(CStage &st, Ctx &c, const MkRuntime &rt, int M, int lg2) {
+  constexpr int KK = (TB * CH + 3) / 4;  // (outputs a lane finishes, with the fewest lanes per channel)
+  const int L = 1 << lg2, GW = 64 >> lg2, CW = MK_WAVES * GW * CH;
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), j = lane & (L - 1);
   const int n = st.n, Np = (st.states + 3) / 4 * 4, nblk = (n + CW - 1) / CW;
   const MxDeltaUnits us = mx_delta_units(c, M);
   const int n_units = us.nreq * nblk;
@@ -79,7 +79,7 @@ __device__ __forceinline__ void stage_hy_scan_t(CStage &st, Ctx &c, const MkRunt
   auto unit = [&](int u) {
     Unit a;
     const int ri = u / nblk;
-    a.ch0 = (u - ri * nblk) * CW + wave * GW * CH + lane / L;
+    a.ch0 = (u - ri * nblk) * CW + wave * GW * CH + (lane >> lg2);
     a.t0 = (int)__ffsll(__ballot(us.first && us.rank_of == ri)) - 1;
     a.n = wave_bcast(us.my_n, a.t0);
     a.p0 = __builtin_amdgcn_readfirstlane(c.sh_tok[a.t0]);
@@ -122,7 +122,8 @@ __device__ __forceinline__ void stage_hy_scan_t(CStage &st, Ctx &c, const MkRunt
       }
     }
 #pragma unroll
-    for (int k = 0; k < KK; k++) r.z[k] = fx_ldc(in + (size_t)(a.t0 + min(tb + (k * L + j) / CH, a.n - 1)) * st.ld_in + st.cols[3] + channel(a, (k * L + j) % CH));
+    for (int k = 0; k < KK; k++)
+      if (k == 0 || L == 4) r.z[k] = fx_ldc(in + (size_t)(a.t0 + min(tb + (k * L + j) / CH, a.n - 1)) * st.ld_in + st.cols[3] + channel(a, (k * L + j) % CH));
   };
   // The convolution's last inputs: the portion's, and before them what is left of the old ones.  Few taps: a lane per row, read with
   // the unit's rows and written at its end; more: in ascending order by one thread (a row is read before it is written).
@@ -182,6 +183,7 @@ __device__ __forceinline__ void stage_hy_scan_t(CStage &st, Ctx &c, const MkRunt
       const bool more = tb + TB < a.n;
       load_rows(more ? a : nx, more ? tb + TB : 0, rn);
       float y[KK];
+      static_assert(TB * CH <= 8, "with more than four lanes per channel a lane finishes one output");
 #pragma unroll
       for (int t = 0; t < TB; t++) {
         if (TB > 1 && tb + t >= a.n) break;
@@ -196,14 +198,18 @@ __device__ __forceinline__ void stage_hy_scan_t(CStage &st, Ctx &c, const MkRunt
               S[h][i][e] = fmaf(fx_exp2(E(), r.dt[t][h] * A[h][i][e]), S[h][i][e], on[i] ? dx * r.B[t][i][e] : 0.f);
               s = fmaf(S[h][i][e], on[i] ? r.C[t][i][e] : 0.f, s);
             }
-          s = hy_lanes_sum<L>(s);
-          if ((t * CH + h) % L == j) y[(t * CH + h) / L] = s + D[h] * r.x[t][h];
+          s = hy_lanes_sum(s, L) + D[h] * r.x[t][h];
+          const int e = t * CH + h;
+          if ((e & (L - 1)) == j) {
+            if (e >= 4 && L == 4) y[e / 4] = s;
+            else y[0] = s;
+          }
         }
       }
 #pragma unroll
       for (int k = 0; k < KK; k++) {
         const int t = (k * L + j) / CH, h = (k * L + j) % CH;
-        if (t < TB && tb + t < a.n && real(a, h)) fx_stc((E *)st.out + (size_t)(a.t0 + tb + t) * st.ld_out + channel(a, h), fx_round<E>(y[k] * hy_silu(E(), r.z[k])));
+        if ((k == 0 || L == 4) && t < TB && tb + t < a.n && real(a, h)) fx_stc((E *)st.out + (size_t)(a.t0 + tb + t) * st.ld_out + channel(a, h), fx_round<E>(y[k] * hy_silu(E(), r.z[k])));
       }
       r = rn;
     }
@@ -241,23 +247,16 @@ __device__ __forceinline__ void stage_hy_scan_t(CStage &st, Ctx &c, const MkRunt
 }
 template <typename E>
 __device__ __forceinline__ void stage_hy_scan(CStage &st, Ctx &c, const MkRuntime &rt, int M, bool single) {
+  const int lg2 = st.states <= 16 ? 2 : st.states <= 32 ? 3 : 4;
   // single tokens of many requests: eight channels per lane, so that a workgroup has enough in flight
-  const bool many = single && (long long)M * st.n * (st.states <= 16 ? 4 : st.states <= 32 ? 8 : 16) >= 4ll * c.G * MK_THREADS;
-  if (st.states <= 16) {
-    if (many) stage_hy_scan_t<E, 4, 1, 1, 8>(st, c, rt, M);
-    else if (single) stage_hy_scan_t<E, 4, 1, 1, 1>(st, c, rt, M);
-    else stage_hy_scan_t<E, 4, 1, 8, 1>(st, c, rt, M);
-  } else if (st.states <= 32) {
-    if (many) stage_hy_scan_t<E, 8, 1, 1, 8>(st, c, rt, M);
-    else if (single) stage_hy_scan_t<E, 8, 1, 1, 1>(st, c, rt, M);
-    else stage_hy_scan_t<E, 8, 1, 8, 1>(st, c, rt, M);
-  } else if (st.states <= 64) {
-    if (many) stage_hy_scan_t<E, 16, 1, 1, 8>(st, c, rt, M);
-    else if (single) stage_hy_scan_t<E, 16, 1, 1, 1>(st, c, rt, M);
-    else stage_hy_scan_t<E, 16, 1, 8, 1>(st, c, rt, M);
+  const bool many = single && (((long long)M * st.n) << lg2) >= 4ll * c.G * MK_THREADS;
+  if (st.states <= 64) {
+    if (many) stage_hy_scan_t<E, 1, 1, 8>(st, c, rt, M, lg2);
+    else if (single) stage_hy_scan_t<E, 1, 1, 1>(st, c, rt, M, lg2);
+    else stage_hy_scan_t<E, 1, 8, 1>(st, c, rt, M, lg2);
   } else {
-    if (single) stage_hy_scan_t<E, 16, 4, 1, 1>(st, c, rt, M);
-    else stage_hy_scan_t<E, 16, 4, 2, 1>(st, c, rt, M);
+    if (single) stage_hy_scan_t<E, 4, 1, 1>(st, c, rt, M, lg2);
+    else stage_hy_scan_t<E, 4, 2, 1>(st, c, rt, M, lg2);
   }
 }
 
@@ -340,10 +339,11 @@ struct HyLists {
   unsigned char place[MK_MOE_MAX_EXPERTS][MK_MAX_TOKENS];
 };
 static_assert(sizeof(HyLists) <= MK_MOE_OFFSET, "the lists lie below the scratch of the reduction");
-template <typename E, int MT, bool GLU, bool SPLIT>
+template <typename E, int MT, bool SPLIT>
 __device__ __forceinline__ void hy_expert_unit(CStage &st, const HyLists *ls, bool shared, int e, int pair, unsigned long long toks, int n, int K, int wave, int lane,
                                                const u32x4 *W, const u32x4 (&first)[2][4], f32x4 *red) {
   constexpr int EPC = FxType<E>::EPC, KW = FxType<E>::KW, KB = 4;
+  const bool glu = st.flags & MK_F_SILU;
   const int lr = lane & 15, lg = lane >> 4, nks = K / KW, kq = SPLIT ? (nks + MK_WAVES - 1) / MK_WAVES : nks, kb = SPLIT ? min(nks, wave * kq) : 0, ke = min(nks, kb + kq);
   const int cnt = __popcll(toks);
   // lane r gets the r-th token of the list
@@ -409,21 +409,21 @@ __device__ __forceinline__ void hy_expert_unit(CStage &st, const HyLists *ls, bo
 #pragma unroll
   for (int m = 0; m < MT; m++) {
 #pragma unroll
-    for (int h = 0; h < (GLU ? 1 : 2); h++) {
-      if ((SPLIT && ((GLU ? m : 2 * m + h) & (MK_WAVES - 1)) != wave) || m * 16 + lr >= cnt) continue;
+    for (int h = 0; h < 2; h++) {
+      if ((SPLIT && ((2 * m + h) & (MK_WAVES - 1)) != wave) || m * 16 + lr >= cnt || (glu && h)) continue;
       const f32x4 v = total(h, m);
       float r[4] = {v[0], v[1], v[2], v[3]};
-      if (GLU) {
+      if (glu) {
         const f32x4 u = total(1, m);
 #pragma unroll
         for (int q = 0; q < 4; q++) r[q] = hy_silu(E(), r[q]) * u[q];
       }
-      fx_stc4((E *)st.out + (size_t)tok[m] * st.ld_out + (size_t)place[m] * st.ld_out_slot, (GLU ? pair : 2 * pair + h) * 16 + lg * 4, GLU ? n / 2 : n, r);
+      fx_stc4((E *)st.out + (size_t)tok[m] * st.ld_out + (size_t)place[m] * st.ld_out_slot, (glu ? pair : 2 * pair + h) * 16 + lg * 4, glu ? n / 2 : n, r);
     }
   }
 }
-template <typename E, int MAXM, bool GLU>
-__device__ __forceinline__ void stage_hy_experts_t(CStage &st, Ctx &c, int M, char *smem) {
+template <typename E, int MAXM>
+__device__ __forceinline__ void stage_hy_experts(CStage &st, Ctx &c, int M, char *smem) {
   constexpr int KW = FxType<E>::KW;
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int Ex = st.num_experts, topk = st.topk;
@@ -515,16 +515,18 @@ __device__ __forceinline__ void stage_hy_experts_t(CStage &st, Ctx &c, int M, ch
         const unsigned long long t = ls->tok[a.e];
         toks = (unsigned long long)(unsigned)__builtin_amdgcn_readfirstlane((int)t) | ((unsigned long long)(unsigned)__builtin_amdgcn_readfirstlane((int)(t >> 32)) << 32);
       }
-      if (MAXM == 1 || __popcll(toks) <= 16) hy_expert_unit<E, 1, GLU, SPLIT>(st, ls, shared, a.e, a.pair, toks, a.n, a.K, wave, lane, a.W, f, red);
-      else hy_expert_unit<E, 4, GLU, SPLIT>(st, ls, shared, a.e, a.pair, toks, a.n, a.K, wave, lane, a.W, f, red);
+      const int cnt = __popcll(toks);
+      if constexpr (SPLIT) {  // 16 tokens at a time
+        const int rank = (toks >> lane) & 1 ? __popcll(toks & ((1ull << lane) - 1ull)) : -1;
+        for (int g = 0; g < cnt; g += 16) hy_expert_unit<E, 1, true>(st, ls, shared, a.e, a.pair, __ballot(rank >= g && rank < g + 16), a.n, a.K, wave, lane, a.W, f, red);
+      } else if (cnt <= 16) {
+        hy_expert_unit<E, 1, false>(st, ls, shared, a.e, a.pair, toks, a.n, a.K, wave, lane, a.W, f, red);
+      } else {
+        hy_expert_unit<E, 4, false>(st, ls, shared, a.e, a.pair, toks, a.n, a.K, wave, lane, a.W, f, red);
+      }
     }
   };
   if (MAXM == 1 || n_units < 3 * MK_WAVES * c.G) walk(std::true_type{}, u0, c.G, early);
   else if constexpr (MAXM > 1) walk(std::false_type{}, mx_wave_item(c, wave), c.G * MK_WAVES, false);
   c.wrote_through = true;
-}
-template <typename E, int MAXM>
-__device__ __forceinline__ void stage_hy_experts(CStage &st, Ctx &c, int M, char *smem) {
-  if (st.flags & MK_F_SILU) stage_hy_experts_t<E, MAXM, true>(st, c, M, smem);
-  else stage_hy_experts_t<E, MAXM, false>(st, c, M, smem);
 }
