@@ -212,10 +212,10 @@ def run_leg(torch, dec, shape, model, B, K, W, P, max_seq, mode, stage_profile=F
     }
 
 
-# ---- a model beside the closest one at equal size (bench.py --compare suborax | dodonex | bukatar) ------------------------------
+# ---- a model beside the closest one at equal size (bench.py --compare suborax | dodonex | bukatar | vizonex) ------------------------------
 # Both models with the same width, heads, head size, feed-forward, depth and vocabulary; random weights.  (Dodonex: what the
 # closest model has no counterpart for -- latent sizes, recurrence, per-token vectors -- comes from generate.py's shapes.)
-CLOSEST = {"suborax": "qwen3", "dodonex": "suborax", "bukatar": "dodonex"}
+CLOSEST = {"suborax": "qwen3", "dodonex": "suborax", "bukatar": "dodonex", "vizonex": "bukatar"}
 COMPARE_SHAPES = {"8b": dict(width=4096, heads=32, kv_heads=8, ff=12288), "2k": dict(width=2048, heads=32, kv_heads=4, ff=6144)}
 
 

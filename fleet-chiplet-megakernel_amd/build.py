@@ -19,8 +19,8 @@ CSRC = os.path.join(HERE, "csrc")
 LIB = os.path.join(HERE, "libfleet_mk.so")
 
 # kernels of mk_kernel.hip (-DMK_KERNEL_<name>): the fixed-shape pair, the flex ones, those with the mix stages beside them,
-# and those with the hybrid stages beside both
-KERNELS = ("DENSE", "FLEX", "FLEX_M1", "FLEX_F32", "MIX", "MIX_M1", "MIX_F32", "HYB", "HYB_M1", "HYB_F32")
+# those with the hybrid stages beside both, and those with the dual stages beside flex, norms, routing and experts
+KERNELS = ("DENSE", "FLEX", "FLEX_M1", "FLEX_F32", "MIX", "MIX_M1", "MIX_F32", "HYB", "HYB_M1", "HYB_F32", "DUAL", "DUAL_M1", "DUAL_F32")
 
 HIPCC_FLAGS = [
     "--offload-arch=gfx950",

@@ -45,6 +45,13 @@ __device__ __forceinline__ f32x4 fx_ldc_quad(const uint16_t *p) {
   return (f32x4){bf_lo(a), bf_hi(a), bf_lo(b), bf_hi(b)};
 }
 __device__ __forceinline__ f32x4 fx_ldc_quad(const float *p) { return __builtin_bit_cast(f32x4, ldc_16B((const u32x4 *)p)); }
+// ... of a table nobody writes during a launch
+__device__ __forceinline__ f32x4 fx_ld_quad(const uint16_t *p) {
+  const unsigned long long u = *(const unsigned long long *)p;
+  const uint32_t a = (uint32_t)u, b = (uint32_t)(u >> 32);
+  return (f32x4){bf_lo(a), bf_hi(a), bf_lo(b), bf_hi(b)};
+}
+__device__ __forceinline__ f32x4 fx_ld_quad(const float *p) { return *(const f32x4 *)p; }
 __device__ __forceinline__ void fx_stc_quad(uint16_t *p, f32x4 v) {
   stc_u64(p, (unsigned long long)pack2(v[0], v[1]) | ((unsigned long long)pack2(v[2], v[3]) << 32));
 }
@@ -86,6 +93,17 @@ __device__ __forceinline__ void stage_fx_embed(CStage &st, Ctx &c, const MkRunti
     const E *src = (const E *)st.w.seg[0] + (size_t)(id < 0 ? 0 : id) * k;
     E *out = (E *)st.out + (size_t)t * st.ld_out;
     float *out32 = st.out2 ? (float *)st.out2 + (size_t)t * st.ld_out2 : nullptr;
+#if MK_HAVE_DUAL
+    if (st.pos_tab) {  // (the caller keeps positions inside the table)
+      const E *pos = (const E *)st.pos_tab + (size_t)min(c.sh_tok[t], st.pos_rows - 1) * k;
+      for (int i = threadIdx.x; i < k; i += MK_THREADS) {
+        const float v = fmaf(fx_val(src[i]), scale, fx_val(pos[i]));
+        if (out32) stc_f32(out32 + i, v);
+        fx_stc(out + i, fx_round<E>(v));
+      }
+      continue;
+    }
+#endif
     if ((k & 3) == 0) {
       for (int i = threadIdx.x * 4; i < k; i += MK_THREADS * 4) {
         f32x4 v;
@@ -231,12 +249,47 @@ template <typename E> __device__ __forceinline__ FxRows<E> fx_rows(CStage &st, C
 // One query or key head row by one wavefront: dims [0, rot) are rotated (dim i < rot / 2 pairs with i + rot / 2), then the
 // row is divided by sqrt(mean(x^2) + eps) when the stage asks for it.  Split in a half that requests everything and a half
 // that computes, so that a wavefront can have the requests of two rows in flight; put(d, value) for every d < D.
+//
+// Dual kernels, MK_F_ROW_NORM: the row's query heads (its key heads) are together divided by their root mean square and multiplied
+// by a weight per column instead; `r` is that factor, `w` the weights.
 struct FxHead {
   float x[MK_FX_HEAD_REGS], xp[MK_FX_HEAD_REGS], cs[MK_FX_HEAD_REGS], sn[MK_FX_HEAD_REGS];
 #if MK_HAVE_HYB
   float b[MK_FX_HEAD_REGS], bp[MK_FX_HEAD_REGS];  // bias of x and xp
 #endif
+#if MK_HAVE_DUAL
+  float r, w[MK_FX_HEAD_REGS];
+#endif
 };
+#if MK_HAVE_DUAL
+// Weights of the row norm for the head whose columns begin at `col`.
+__device__ __forceinline__ void fx_row_weights(CStage &st, int col, int lane, FxHead &h) {
+  if (!(st.flags & MK_F_ROW_NORM)) return;
+  const int nq = st.num_q_heads * st.head_dim;
+  const float *w = col < nq ? (const float *)st.q_norm_w + col : (const float *)st.k_norm_w + (col - nq);
+#pragma unroll
+  for (int j = 0; j < MK_FX_HEAD_REGS; j++)
+    if (j * 64 < st.head_dim) h.w[j] = w[min(j * 64 + lane, st.head_dim - 1)];
+}
+// This lane's part of the sum of squares over columns [c0, c1) of a row, lane `id` of `n`.
+template <typename E>
+__device__ __forceinline__ float fx_row_squares(const E *row, int c0, int c1, int id, int n) {
+  float ss = 0.f;
+  for (int q0 = c0 / 4 + id; q0 * 4 < c1; q0 += 4 * n) {
+    f32x4 v[4];
+#pragma unroll
+    for (int j = 0; j < 4; j++) v[j] = fx_ldc_quad(row + 4 * min(q0 + j * n, (c1 - 1) / 4));
+#pragma unroll
+    for (int j = 0; j < 4; j++)
+#pragma unroll
+      for (int e = 0; e < 4; e++) {
+        const int at = 4 * (q0 + j * n) + e;
+        ss += at >= c0 && at < c1 ? v[j][e] * v[j][e] : 0.f;
+      }
+  }
+  return ss;
+}
+#endif
 // Bias of a row's columns (hybrid kernels): requested beside the row, added when it is used.
 template <typename E>
 __device__ __forceinline__ void fx_bias_load(const FxRows<E> &rows, int col, int n, int rot, int lane, float (&b)[MK_FX_HEAD_REGS], float (&bp)[MK_FX_HEAD_REGS]) {
@@ -309,6 +362,13 @@ __device__ __forceinline__ void fx_head_finish(CStage &st, int lane, FxHead &h, 
     for (int j = 0; j < MK_FX_HEAD_REGS; j++)
       if (j * 64 < D) h.x[j] *= r;
   }
+#if MK_HAVE_DUAL
+  if (st.flags & MK_F_ROW_NORM) {
+#pragma unroll
+    for (int j = 0; j < MK_FX_HEAD_REGS; j++)
+      if (j * 64 < D) h.x[j] = (h.x[j] * h.r) * h.w[j];
+  }
+#endif
 #pragma unroll
   for (int j = 0; j < MK_FX_HEAD_REGS; j++)
     if (j * 64 + lane < D) put(j * 64 + lane, h.x[j]);
@@ -359,6 +419,13 @@ __device__ __forceinline__ void stage_fx_prep(CStage &st, Ctx &c, const MkRuntim
     page = s < H ? 0 : rt.kv_indices[__builtin_amdgcn_readfirstlane(c.sh_tok[3 * MK_MAX_TOKENS + t]) + pos / ps];
     if (s < H + nkv) {
       fx_head_load<E>(st, rows, t, s * D, pos, lane, h);
+#if MK_HAVE_DUAL
+      if (st.flags & MK_F_ROW_NORM) {
+        const int c0 = s < H ? 0 : H * D, c1 = s < H ? H * D : (H + nkv) * D;
+        fx_row_weights(st, s * D, lane, h);
+        h.r = 1.f / sqrtf(wave_sum(fx_row_squares<E>((const E *)st.in + (size_t)t * st.ld_in, c0, c1, lane, 64)) / (float)(c1 - c0) + st.eps);
+      }
+#endif
     } else {
       fx_value_load<E>(rows, t, fx_value_col(st) + (s - H - nkv) * DV, DV, lane, h.x);
 #if MK_HAVE_HYB
@@ -482,8 +549,14 @@ __device__ __forceinline__ void stage_fx_attn_t(CStage &st, Ctx &c, const MkRunt
     a.p = a.p0 + (a.r0 + a.nrows - 1) / qpk;  // newest position any of the rows sees
     int NT = a.p / TP + 1;
     if (MK_HAVE_HYB) {
-      const int oldest = win ? max(0, a.p0 + a.r0 / qpk - win + 1) : 0;  // oldest position inside the window of the unit's first row
+      const int first = a.p0 + a.r0 / qpk;  // position of the unit's first row
+      int oldest = win ? max(0, first - win + 1) : 0;  // oldest position inside its window
+#if MK_HAVE_DUAL
+      if (st.chunk) oldest = max(oldest, first - first % st.chunk);  // ... and inside its chunk
+      a.kept = win || st.chunk ? min((keep + TP - 1) / TP, NT) : NT;
+#else
       a.kept = win ? min((keep + TP - 1) / TP, NT) : NT;
+#endif
       a.gap = max(0, oldest / TP - a.kept);
       NT -= a.gap;
     }
@@ -548,6 +621,24 @@ __device__ __forceinline__ void stage_fx_attn_t(CStage &st, Ctx &c, const MkRunt
     const bool newest = single && a.cidx == a.C - 1;
     // ---- query rows into operand order (and the new key and value)
     if (single) {
+#if MK_HAVE_DUAL
+      float rq = 0.f, rk = 0.f;
+      if (st.flags & MK_F_ROW_NORM) {
+        const int nq = st.num_q_heads * D, nk = nkv * D;
+        const E *row = (const E *)st.in + (size_t)a.t0 * st.ld_in;
+        rq = fx_row_squares<E>(row, 0, nq, tid, MK_THREADS);
+        if (newest) rk = fx_row_squares<E>(row, nq, nq + nk, tid, MK_THREADS);
+        rq = wave_sum(rq);
+        rk = wave_sum(rk);
+        if (lane == 0) {
+          part[wave] = rq;
+          part[4 + wave] = rk;
+        }
+        __syncthreads();
+        rq = 1.f / sqrtf(((part[0] + part[1]) + (part[2] + part[3])) / (float)nq + st.eps);
+        rk = 1.f / sqrtf(((part[4] + part[5]) + (part[6] + part[7])) / (float)nk + st.eps);
+      }
+#endif
       // (everything the row writers below leave out is zeroed: unused query columns, padding dims)
       const u32x4 z = {0u, 0u, 0u, 0u};
       for (int i = tid; i < nkg * KC * 64; i += MK_THREADS)
@@ -572,6 +663,10 @@ __device__ __forceinline__ void stage_fx_attn_t(CStage &st, Ctx &c, const MkRunt
 #endif
       auto load_row = [&](int r, FxHead &h) {
         fx_head_load<E>(st, rows, a.t0, (r < a.nrows ? a.g * qpk + a.r0 + r : st.num_q_heads + a.g) * D, a.p, lane, h);
+#if MK_HAVE_DUAL
+        fx_row_weights(st, (r < a.nrows ? a.g * qpk + a.r0 + r : st.num_q_heads + a.g) * D, lane, h);
+        h.r = r < a.nrows ? rq : rk;
+#endif
       };
       auto put_row = [&](int r, FxHead &h) {
         if (r < a.nrows) fx_head_finish(st, lane, h, [&](int d, float v) { q[((d / KW) * 64 + ((d % KW) / EPC) * 16 + r) * EPC + d % EPC] = fx_round<E>(v); });
@@ -612,6 +707,12 @@ __device__ __forceinline__ void stage_fx_attn_t(CStage &st, Ctx &c, const MkRunt
     }
     // ---- tiles
     const int plim = a.p0 + (a.r0 + min(lr, a.nrows - 1)) / qpk;  // newest position this lane's query row sees
+#if MK_HAVE_DUAL
+    const int olim = st.chunk ? plim - plim % st.chunk : 0;  // oldest one
+    const float sc_row = sc1 * (st.temp ? st.temp[a.g * qpk + (a.r0 + min(lr, a.nrows - 1)) % qpk] : 1.f);
+#else
+    const float sc_row = sc1;
+#endif
     float m = MK_FX_NEG, l = 0.f;
     f32x4 acc[VB], S[SUB];
 #pragma unroll
@@ -648,7 +749,7 @@ __device__ __forceinline__ void stage_fx_attn_t(CStage &st, Ctx &c, const MkRunt
       for (int u_ = 0; u_ < SUB; u_++)
 #pragma unroll
         for (int i = 0; i < 4; i++) {
-          float s = S[u_][i] * sc1;
+          float s = S[u_][i] * sc_row;
           if (cap > 0.f) {
             if constexpr (sizeof(E) == 2) {
               const float e = __builtin_amdgcn_exp2f(s * (2.f * LOG2E));
@@ -662,6 +763,9 @@ __device__ __forceinline__ void stage_fx_attn_t(CStage &st, Ctx &c, const MkRunt
           const int at = tile * TP + u_ * 16 + lg * 4 + i;
           bool seen = at <= plim;
           if (MK_HAVE_HYB) seen = seen && (win == 0 || plim - at < win || at < keep);
+#if MK_HAVE_DUAL
+          seen = seen && at >= olim;
+#endif
           s = seen ? s : MK_FX_NEG;
           sc[u_][i] = s;
           tm = fmaxf(tm, s);
@@ -869,6 +973,12 @@ __device__ __forceinline__ void stage_fx_attn(CStage &st, Ctx &c, const MkRuntim
 // ----------------------------------------------------------------------------- 32-bit linear
 // out[m, n] = sum_k x[m, k] W[n, k] in true 32-bit (v_mfma_f32_16x16x4_f32), optional SwiGLU epilogue.  A workgroup owns a
 // range of 16-column output tiles and all rows; its wavefronts split K and are reduced through LDS in a fixed order.
+__device__ __forceinline__ float fx_glu_f32(CStage &st, float g, float u) {
+#if MK_HAVE_DUAL
+  if (st.flags & MK_F_GELU) return 0.5f * g * (1.f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g))) * u;
+#endif
+  return g / (1.f + expf(-g)) * u;
+}
 template <int MT>
 __device__ __forceinline__ void stage_fx_linear_f32(CStage &st, Ctx &c, int M, char *smem) {
   if (threadIdx.x == 0) __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "agent");
@@ -926,7 +1036,7 @@ __device__ __forceinline__ void stage_fx_linear_f32(CStage &st, Ctx &c, int M, c
       if (m < M) {
         float r[4];
 #pragma unroll
-        for (int i = 0; i < 4; i++) r[i] = silu ? v[i] / (1.f + expf(-v[i])) * g[i] : linear_act(st, v[i]);
+        for (int i = 0; i < 4; i++) r[i] = silu ? fx_glu_f32(st, v[i], g[i]) : linear_act(st, v[i]);
         fx_stc4((float *)st.out + (size_t)m * st.ld_out, ot * 16 + (l >> 4) * 4, n_out, r);
       }
     }

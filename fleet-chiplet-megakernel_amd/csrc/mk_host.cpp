@@ -58,6 +58,15 @@ MK_DECLARE_KERNEL(mk_persistent_kernel_hyb_m1);
 #ifdef MK_HAVE_KERNEL_HYB_F32
 MK_DECLARE_KERNEL(mk_persistent_kernel_hyb_f32);
 #endif
+#ifdef MK_HAVE_KERNEL_DUAL
+MK_DECLARE_KERNEL(mk_persistent_kernel_dual);
+#endif
+#ifdef MK_HAVE_KERNEL_DUAL_M1
+MK_DECLARE_KERNEL(mk_persistent_kernel_dual_m1);
+#endif
+#ifdef MK_HAVE_KERNEL_DUAL_F32
+MK_DECLARE_KERNEL(mk_persistent_kernel_dual_f32);
+#endif
 
 namespace {
 
@@ -168,6 +177,7 @@ struct mk_graph {
   size_t flex_part = 0;      // floats of split-KV partials the flex and latent attention stages need
   bool mix = false;          // some stage is one of mk_mix.hip's
   bool hyb = false;          // ... of mk_hybrid.hip's, or an older stage has an option only the hybrid kernels know
+  bool dual = false;         // ... of mk_dual.hip's, or an older stage has an option only the dual kernels know
   int *state_ids = nullptr;  // batch slot -> recurrent-state slot (the caller's tensor); null: no recurrence
 };
 
@@ -273,7 +283,7 @@ int num_outputs(const Task &t) {
   if (t.name == "gang_attn_split_kv_mi300") return 3;
   if (t.name == "paged_attention_ck_fmha_split_kv_mi300" || t.name == "paged_attention_split_kv_mi300") return 2;
   if (t.name == "moe_topk_softmax_mi300") return 3;
-  if (t.name == "embedding_scaled" || t.name == "residual_rmsnorm" || t.name == "residual_prenorm" || t.name == "latent_prep" || t.name == "general_delta" || t.name == "expert_route") return 2;
+  if (t.name == "embedding_scaled" || t.name == "residual_rmsnorm" || t.name == "residual_prenorm" || t.name == "latent_prep" || t.name == "general_delta" || t.name == "expert_route" || t.name == "ring_conv") return 2;
   return 1;
 }
 
@@ -347,7 +357,8 @@ int lower_linear(mk_graph *g, size_t &i) {
   st.eps = g->cfg.rms_eps;
   // a following silu_mul over this linear's (library-owned) output is folded into the epilogue
   const Task *act = nullptr;
-  if (!silu && !res && i + 1 < g->ltasks.size() && g->ltasks[i + 1].name == "silu_mul" && g->ltasks[i + 1].ops.size() == 2 &&
+  const bool gelu = i + 1 < g->ltasks.size() && g->ltasks[i + 1].name == "gelu_mul";
+  if (!silu && !res && i + 1 < g->ltasks.size() && (gelu || g->ltasks[i + 1].name == "silu_mul") && g->ltasks[i + 1].ops.size() == 2 &&
       g->ltasks[i + 1].ops[0] == out_id && tout.kind == T_OWNED) {
     act = &g->ltasks[i + 1];
   }
@@ -363,6 +374,12 @@ int lower_linear(mk_graph *g, size_t &i) {
   }
   if (silu || act) {
     st.flags |= MK_F_SILU;
+    if (act && gelu) {
+      st.flags |= MK_F_GELU;
+      g->mix = g->hyb = g->dual = true;
+      int rc2 = set_flex(g, tin.dtype, "gelu_mul");
+      if (rc2) return rc2;
+    }
     if (act) {
       final_out = act->ops[1];
       const int groups = act->grid[0] * act->grid[1] * act->grid[2];
@@ -427,7 +444,7 @@ int lower_linear(mk_graph *g, size_t &i) {
   }
   g->stages.push_back(st);
   g->stage_desc.push_back(fmt("LINEAR%s%s%s%s %s x %s -> %s n=%d k=%d segs=%d", f32 ? "_F32" : "", (st.flags & MK_F_NORM) ? "+norm" : "", (st.flags & MK_F_RES) ? "+res" : "",
-                              (st.flags & MK_F_SILU) ? "+silu" : sq ? "+relu2" : "", tin.name.c_str(), g->tensors[w_id].name.c_str(), tfo.name.c_str(), st.n, st.k,
+                              (st.flags & MK_F_GELU) ? "+gelu" : (st.flags & MK_F_SILU) ? "+silu" : sq ? "+relu2" : "", tin.name.c_str(), g->tensors[w_id].name.c_str(), tfo.name.c_str(), st.n, st.k,
                               st.w.nseg));
   g->weight_bytes += (int64_t)st.n * st.k * (int64_t)dtype_size(tin.dtype);
   g->stage_weight.resize(g->stages.size(), -1);
@@ -661,11 +678,13 @@ int lower_attention(mk_graph *g, size_t &i) {
 
 
 // ---- flex tasks (mk_flex.hip): sizes and constants are data --------------------------------------------------------
-// embedding_scaled [ids, table, residual rows (fp32), rows] params [source, scale bits]
+// embedding_scaled [ids, table, residual rows (fp32), rows] params [source, scale bits]; with one more operand behind the table, [positions,
+// table columns]: its row at the token's position is added (behind the last row: the last one).
 int lower_embedding_scaled(mk_graph *g, size_t &i) {
   const Task &t = g->ltasks[i];
-  if (t.ops.size() != 4 || t.params.size() != 2) return fail(MK_EINVAL, "embedding_scaled expects 4 operands / 2 params");
-  const Tensor &ids = g->tensors[t.ops[0]], &w = g->tensors[t.ops[1]], &r = g->tensors[t.ops[2]], &o = g->tensors[t.ops[3]];
+  const bool ext = t.ops.size() == 5;
+  if ((!ext && t.ops.size() != 4) || t.params.size() != 2) return fail(MK_EINVAL, "embedding_scaled expects 4 or 5 operands / 2 params");
+  const Tensor &ids = g->tensors[t.ops[0]], &w = g->tensors[t.ops[1]], &r = g->tensors[t.ops[2 + ext]], &o = g->tensors[t.ops[3 + ext]];
   const int B = g->cfg.max_num_batched_tokens;
   if (ids.dtype != MK_DT_I64 || (int64_t)ids.elems() < B) return fail(MK_EINVAL, "embedding_scaled: ids must be int64, one per token row");
   if (w.ndims != 2 || o.ndims != 2 || r.ndims != 2 || o.dims[1] < w.dims[1] || r.dims[1] < w.dims[1] || o.dims[0] < B || r.dims[0] < B || w.dtype != o.dtype || r.dtype != MK_DT_F32 ||
@@ -686,8 +705,15 @@ int lower_embedding_scaled(mk_graph *g, size_t &i) {
   st.w.nseg = 1;
   st.w.seg[0] = w.ptr;
   if (t.params[0] == 0) st.flags |= MK_F_EMBED_FROM_TOKENS;
+  if (ext) {
+    const Tensor &pos = g->tensors[t.ops[2]];
+    if (pos.ndims != 2 || pos.dims[0] < 1 || pos.dims[1] != w.dims[1] || pos.strides[0] != w.dims[1] || pos.dtype != w.dtype) return fail(MK_EINVAL, "embedding_scaled: position vectors are [positions, %d] of the table's type", st.k);
+    st.pos_tab = pos.ptr;
+    st.pos_rows = (int)pos.dims[0];
+    g->mix = g->hyb = g->dual = true;
+  }
   g->stages.push_back(st);
-  g->stage_desc.push_back(fmt("FX_EMBED %s[%s] * %g -> %s, %s k=%d", w.name.c_str(), ids.name.c_str(), st.alpha, r.name.c_str(), o.name.c_str(), st.k));
+  g->stage_desc.push_back(fmt("FX_EMBED %s[%s] * %g%s -> %s, %s k=%d", w.name.c_str(), ids.name.c_str(), st.alpha, ext ? " + position" : "", r.name.c_str(), o.name.c_str(), st.k));
   i++;
   return MK_OK;
 }
@@ -767,12 +793,15 @@ int lower_residual_rmsnorm(mk_graph *g, size_t &i) {
 // qkv rows are all query heads, then all key heads, then all value heads; caches are [pages, page_size, kv heads, padded
 // dim] with a layout of the library's own inside a page.  With three more params [window, kept first positions, values from
 // keys 0/1] and one more operand behind the sink, fp32 [input columns] added to the rows: a position sees the `window` newest
-// ones and the kept first ones; the value heads are the key heads before rotation (the rows hold no others).
+// ones and the kept first ones; the value heads are the key heads before rotation (the rows hold no others).  With one more param and
+// three more operands behind those [q row weights, k row weights, score factors; all optional]: a position sees only its own chunk
+// (param, 0: none) of positions; all query heads of a row are divided by their common root mean square and multiplied by a
+// weight per column, all key heads likewise; scores are multiplied by a factor per head.
 int lower_flex_attention(mk_graph *g, size_t &i) {
   const Task &t = g->ltasks[i];
-  const bool ext = t.ops.size() == 9 && t.params.size() == 12;
-  if (!ext && (t.ops.size() != 8 || t.params.size() != 9)) return fail(MK_EINVAL, "flex_attention expects 8 operands / 9 params, or 9 / 12");
-  const Tensor &in = g->tensors[t.ops[0]], &kc = g->tensors[t.ops[1]], &vc = g->tensors[t.ops[2]], &qw = g->tensors[t.ops[6 + ext]], &o = g->tensors[t.ops[7 + ext]];
+  const bool ext2 = t.ops.size() == 12 && t.params.size() == 13, ext = ext2 || (t.ops.size() == 9 && t.params.size() == 12);
+  if (!ext && (t.ops.size() != 8 || t.params.size() != 9)) return fail(MK_EINVAL, "flex_attention expects 8 operands / 9 params, or 9 / 12, or 12 / 13");
+  const Tensor &in = g->tensors[t.ops[0]], &kc = g->tensors[t.ops[1]], &vc = g->tensors[t.ops[2]], &qw = g->tensors[t.ops[t.ops.size() - 2]], &o = g->tensors[t.ops.back()];
   const int window = ext ? t.params[9] : 0, keep = ext ? t.params[10] : 0, own_v = !(ext && t.params[11]);
   const int B = g->cfg.max_num_batched_tokens, ps = g->cfg.page_size;
   const int H = t.params[0], G = t.params[1], D = t.params[2], DV = t.params[3], rot = t.params[4];
@@ -814,6 +843,20 @@ int lower_flex_attention(mk_graph *g, size_t &i) {
   st.keep_first = window ? keep : 0;
   st.in_bias = ext && t.ops[6] >= 0 ? (const float *)g->tensors[t.ops[6]].ptr : nullptr;
   if (ext) g->mix = g->hyb = true;
+  if (ext2) {
+    const int qn = t.ops[7], kn = t.ops[8], tp = t.ops[9];
+    if (t.params[12] < 0 || (qn >= 0) != (kn >= 0) || (qn >= 0 && (t.params[5] || rot || st.in_bias || !vector_ok(g->tensors[qn], (int64_t)H * D) || !vector_ok(g->tensors[kn], (int64_t)G * D))) ||
+        (tp >= 0 && !vector_ok(g->tensors[tp], H)))
+      return fail(MK_EINVAL, "flex_attention: chunks of %d; row norms need fp32 weights for all query and all key columns, and no rotation, bias or unit norm beside them; a score factor per head", t.params[12]);
+    g->dual = true;
+    st.chunk = t.params[12];
+    if (qn >= 0) {
+      st.flags |= MK_F_ROW_NORM;
+      st.q_norm_w = g->tensors[qn].ptr;
+      st.k_norm_w = g->tensors[kn].ptr;
+    }
+    st.temp = tp >= 0 ? (const float *)g->tensors[tp].ptr : nullptr;
+  }
   st.rot_dims = rot;
   st.eps = bits_f32(t.params[6]);
   st.sm_scale = bits_f32(t.params[7]);
@@ -847,7 +890,7 @@ int lower_flex_attention(mk_graph *g, size_t &i) {
   g->flex_part = std::max(g->flex_part, (size_t)g->G * 16 * (st.v_tiles * 16 + 32));
   if (!g->stages.empty()) {
     MkStage &pl = g->stages.back();  // the q/k/v linear may leave its K-slice sum to this stage's row fetch
-    if (pl.op == MK_OP_LINEAR && !(pl.flags & (MK_F_SILU | MK_F_RES)) && pl.out == st.in && pl.ld_out == st.ld_in && pl.n >= cols) pl.flags |= MK_F_DEFER_SUM;
+    if (pl.op == MK_OP_LINEAR && !(pl.flags & (MK_F_SILU | MK_F_RES)) && pl.out == st.in && pl.ld_out == st.ld_in && pl.n >= cols && !(st.flags & MK_F_ROW_NORM)) pl.flags |= MK_F_DEFER_SUM;
   }
   if (B > 1) {
     MkStage sp = st;
@@ -856,7 +899,7 @@ int lower_flex_attention(mk_graph *g, size_t &i) {
     g->stage_desc.push_back(fmt("FX_PREP[portions] %s", in.name.c_str()));
   }
   g->stages.push_back(st);
-  g->stage_desc.push_back(fmt("FX_ATTN %s -> %s q=%d kv=%d d=%d dv=%d rot=%d norm=%d softcap=%g sink=%d window=%d+%d bias=%d", in.name.c_str(), o.name.c_str(), H, G, D, DV, rot, t.params[5], st.softcap, t.ops[5] >= 0, st.window, st.keep_first, st.in_bias != nullptr));
+  g->stage_desc.push_back(fmt("FX_ATTN %s -> %s q=%d kv=%d d=%d dv=%d rot=%d norm=%d softcap=%g sink=%d window=%d+%d bias=%d chunk=%d rownorm=%d", in.name.c_str(), o.name.c_str(), H, G, D, DV, rot, t.params[5], st.softcap, t.ops[5] >= 0, st.window, st.keep_first, st.in_bias != nullptr, st.chunk, !!(st.flags & MK_F_ROW_NORM)));
   i++;
   return MK_OK;
 }
@@ -873,28 +916,36 @@ int set_mix(mk_graph *g, int dtype, const char *task) {
 // y); new residual = v, rows = the RMS norm of v in `groups` equal parts times weight (no weight: v).  A bf16 linear that
 // reads the rows next forms them itself when an iteration has one token.
 // With two more operands behind the y weight (fp32 [columns] added to y, optional; fp32 [tokens, >= slots] weights, optional) and
-// two more params [slots, columns per slot]: y is the weighted sum of `slots` rows that lie side by side.
+// two more params [slots, columns per slot]: y is the weighted sum of `slots` rows that lie side by side.  With three more operands
+// behind those (y factor, y2, y2 factor; factors are fp32 [columns], all optional): v = residual + alpha * y factor * y + y2 factor * y2,
+// and the slots belong to y2.  The new residual rows are optional then.  A ring_conv that adds the rows' convolution to them right behind is
+// done by this stage when every request brings one token, and the linear may follow that.
+int lower_ring_conv(mk_graph *g, size_t &i, MkStage *out, std::string *desc);
 int lower_residual_prenorm(mk_graph *g, size_t &i) {
   const Task t = g->ltasks[i];
-  const bool ext = t.ops.size() == 8 && t.params.size() == 7;
-  const int e2 = ext ? 2 : 0;
-  if (!ext && (t.ops.size() != 6 || t.params.size() != 5)) return fail(MK_EINVAL, "residual_prenorm expects 6 operands / 5 params, or 8 / 7");
+  const bool ext2 = t.ops.size() == 11 && t.params.size() == 7, ext = ext2 || (t.ops.size() == 8 && t.params.size() == 7);
+  const int e2 = ext2 ? 5 : ext ? 2 : 0;
+  if (!ext && (t.ops.size() != 6 || t.params.size() != 5)) return fail(MK_EINVAL, "residual_prenorm expects 6 operands / 5 params, or 8 / 7, or 11 / 7");
   auto opt = [&](int k) { return t.ops[k] >= 0 ? &g->tensors[t.ops[k]] : nullptr; };
   const Tensor *y = opt(0), *yw = opt(1), *yb = ext ? opt(2) : nullptr, *sw = ext ? opt(3) : nullptr, *w = opt(3 + e2);
-  const Tensor x = g->tensors[t.ops[2 + e2]], xo = g->tensors[t.ops[4 + e2]], o = g->tensors[t.ops[5 + e2]];
+  const Tensor *ys = ext2 ? opt(4) : nullptr, *y2 = ext2 ? opt(5) : nullptr, *y2s = ext2 ? opt(6) : nullptr, *ys_of = sw && y2 ? y2 : y;
+  const bool no_xo = t.ops[4 + e2] < 0;
+  if (no_xo && (!ext2 || !w)) return fail(MK_EINVAL, "residual_prenorm: the new residual rows are missing");
+  const Tensor x = g->tensors[t.ops[2 + e2]], o = g->tensors[t.ops[5 + e2]], xo = no_xo ? x : g->tensors[t.ops[4 + e2]];
   const int slots = sw ? t.params[5] : 0, ld_slot = sw ? t.params[6] : 0;
   const int B = g->cfg.max_num_batched_tokens, width = t.params[0], groups = t.params[1];
   const int64_t n = o.ndims == 2 ? o.dims[1] : 0;
   int rc = set_mix(g, o.dtype, "residual_prenorm");
   if (rc) return rc;
   if (n < 4 || n % 4 || width < 1 || width > n || !rows_ok(o, B, n, o.dtype) || !rows_ok(x, B, n, MK_DT_F32) || !rows_ok(xo, B, n, MK_DT_F32) || x.dims[1] != n || xo.dims[1] != n ||
-      (y && (!rows_ok(*y, B, n, o.dtype) || (!sw && y->dims[1] != n))) || (w && !vector_ok(*w, n)) || (yw && (!y || !vector_ok(*yw, n))))
+      (y && (!rows_ok(*y, B, n, o.dtype) || (!(sw && !y2) && y->dims[1] != n))) || (y2 && (!y || !rows_ok(*y2, B, n, o.dtype) || (!sw && y2->dims[1] != n))) || (ys && (!y || !vector_ok(*ys, n))) ||
+      (y2s && (!y2 || !vector_ok(*y2s, n))) || (w && !vector_ok(*w, n)) || (yw && (!y || !vector_ok(*yw, n))))
     return fail(MK_EINVAL, "residual_prenorm: every row tensor is [tokens, %lld] (a multiple of 4; residual fp32), weights are fp32 of that size, width=%d of it real", (long long)n, width);
   if (w && (groups < 1 || groups > MK_MX_MAX_GROUPS || width % groups)) return fail(MK_EINVAL, "residual_prenorm: %d parts of a row of %d (at most %d)", groups, width, MK_MX_MAX_GROUPS);
-  if ((yb && (!y || !vector_ok(*yb, n))) || (sw && (!y || yb || slots < 1 || slots > MK_MOE_MAX_TOPK + 1 || ld_slot < n || ld_slot % 8 || y->dims[1] < (int64_t)(slots - 1) * ld_slot + n || !rows_ok(*sw, B, slots, MK_DT_F32))))
+  if ((yb && (!y || !vector_ok(*yb, n))) || (sw && (!y || (yb && !y2) || slots < 1 || slots > MK_MOE_MAX_TOPK + 1 || ld_slot < n || ld_slot % 8 || ys_of->dims[1] < (int64_t)(slots - 1) * ld_slot + n || !rows_ok(*sw, B, slots, MK_DT_F32))))
     return fail(MK_EINVAL, "residual_prenorm: a bias has %lld entries; %d slots of %d columns with fp32 weights of that many columns (and no bias)", (long long)n, slots, ld_slot);
   if (n > 12 * 4 * MK_THREADS) return fail(MK_EUNSUPPORTED, "residual_prenorm: rows of %lld values (most %d)", (long long)n, 12 * 4 * MK_THREADS);
-  if (x.ptr == xo.ptr || (xo.ptr == o.ptr && w)) return fail(MK_EINVAL, "residual_prenorm: the new residual rows must not overwrite the old ones (other workgroups may still read them), nor the rows them");
+  if (!no_xo && (x.ptr == xo.ptr || (xo.ptr == o.ptr && w))) return fail(MK_EINVAL, "residual_prenorm: the new residual rows must not overwrite the old ones (other workgroups may still read them), nor the rows them");
   MkStage st;
   memset(&st, 0, sizeof(st));
   st.op = MK_OP_MX_PRENORM;
@@ -913,16 +964,21 @@ int lower_residual_prenorm(mk_graph *g, size_t &i) {
   st.slot_w = sw ? (const float *)sw->ptr : nullptr;
   st.ld_slot_w = sw ? (int)sw->strides[0] : 0;
   if (yb || sw) g->hyb = true;
+  if (ext2) g->hyb = g->dual = true;
+  st.y_scale = ys ? (const float *)ys->ptr : nullptr;
+  st.y2 = y2 ? y2->ptr : nullptr;
+  st.ld_y2 = y2 ? (int)y2->strides[0] : 0;
+  st.y2_scale = y2s ? (const float *)y2s->ptr : nullptr;
   st.res = x.ptr;
   st.ld_res = (int)x.strides[0];
   st.norm_w = w ? w->ptr : nullptr;
   st.out = xo.ptr == o.ptr ? nullptr : o.ptr;
   st.ld_out = (int)o.strides[0];
-  st.out2 = xo.ptr;
+  st.out2 = no_xo ? nullptr : xo.ptr;
   st.ld_out2 = (int)xo.strides[0];
   if (!g->stages.empty()) {
     MkStage &pl = g->stages.back();
-    if (!w && !yw && !yb && !sw && y && st.out && pl.op == MK_OP_LINEAR && !(pl.flags & (MK_F_SILU | MK_F_RES)) && pl.out == st.in && (pl.k & 63) == 0) {
+    if (!w && !yw && !yb && !sw && !ys && !y2 && y && st.out && pl.op == MK_OP_LINEAR && !(pl.flags & (MK_F_SILU | MK_F_RES)) && pl.out == st.in && (pl.k & 63) == 0) {
       // a plain linear in front adds its single-token result to the stream itself
       pl.flags |= MK_F_JOIN;
       pl.res = st.res;
@@ -938,16 +994,46 @@ int lower_residual_prenorm(mk_graph *g, size_t &i) {
   }
   bool res, silu;
   int extra;
-  const bool fuse = g->flex == FLEX_BF16 && w && i + 1 < g->ltasks.size() && linear_kind(g->ltasks[i + 1].name, &res, &silu, &extra) && !res && g->ltasks[i + 1].ops[0] == t.ops[5 + e2];
+  i++;
+  int rows_id = t.ops[5 + e2];
+  MkStage conv;
+  std::string conv_desc;
+  if (w && st.out && i < g->ltasks.size() && g->ltasks[i].name == "ring_conv" && g->ltasks[i].ops.size() == 9 && g->ltasks[i].ops[0] == rows_id && g->ltasks[i].params.size() == 6 &&
+      g->ltasks[i].params[0] == 0 && g->ltasks[i].params[2] && !g->ltasks[i].params[1] && g->ltasks[i].ops[2] < 0 && g->ltasks[i].ops[5] < 0) {
+    rows_id = g->ltasks[i].ops[7];
+    if ((rc = lower_ring_conv(g, i, &conv, &conv_desc))) return rc;
+    if (conv.n != n) return fail(MK_EINVAL, "ring_conv: %d channels over rows of %lld", conv.n, (long long)n);
+    conv.flags |= MK_F_PORTIONS;
+    st.conv_w = conv.conv_w;
+    st.taps = conv.taps;
+    st.tail = conv.tail;
+    st.out3 = conv.out;
+    st.ld_out3 = conv.ld_out;
+  }
+  bool fuse = g->flex == FLEX_BF16 && w && i < g->ltasks.size() && linear_kind(g->ltasks[i].name, &res, &silu, &extra) && !res && g->ltasks[i].ops[0] == rows_id;
+  if (fuse && (ys || y2 || st.conv_w)) {  // these forms: a plain linear, one part of the norm, nothing else in front
+    const std::string behind = i + 1 < g->ltasks.size() ? g->ltasks[i + 1].name : "";
+    fuse = !silu && !yw && !yb && groups == 1 && n % 64 == 0 && behind != "silu_mul" && behind != "gelu_mul" && behind != "silu_mul_linear_with_residual";
+  }
   if (fuse) st.flags |= MK_F_ONLY_MULTI;
   g->stages.push_back(st);
-  g->stage_desc.push_back(fmt("MX_PRENORM%s %s + %g * %s%s -> %s, %s k=%d parts=%d", (st.flags & MK_F_ONLY_MULTI) ? "[multi-token only]" : "", x.name.c_str(), st.alpha, yw ? "norm of " : "", y ? y->name.c_str() : "0", xo.name.c_str(),
-                              o.name.c_str(), width, st.norm_groups));
-  i++;
+  g->stage_desc.push_back(fmt("MX_PRENORM%s %s + %g * %s%s%s%s%s -> %s, %s k=%d parts=%d", (st.flags & MK_F_ONLY_MULTI) ? "[multi-token only]" : "", x.name.c_str(), st.alpha, yw ? "norm of " : "", y ? y->name.c_str() : "0", y2 ? " + " : "",
+                              y2 ? y2->name.c_str() : "", st.conv_w ? " (+conv)" : "", no_xo ? "-" : xo.name.c_str(), o.name.c_str(), width, st.norm_groups));
+  if (st.conv_w && B > 1) {
+    g->stages.push_back(conv);
+    g->stage_desc.push_back(conv_desc);
+  }
   if (!fuse) return MK_OK;
   rc = lower_linear(g, i);
   if (rc) return rc;
   MkStage &l = g->stages.back();
+  l.y_scale = st.y_scale;
+  l.y2 = st.y2;
+  l.ld_y2 = st.ld_y2;
+  l.y2_scale = st.y2_scale;
+  l.conv_w = st.conv_w;
+  l.taps = st.taps;
+  l.tail = st.tail;
   l.flags |= MK_F_NORM | MK_F_PRENORM | (st.flags & MK_F_RES_EARLY);
   l.y_in = st.in;
   l.ld_y = st.ld_in;
@@ -960,8 +1046,9 @@ int lower_residual_prenorm(mk_graph *g, size_t &i) {
   l.res = st.res;
   l.ld_res = st.ld_res;
   l.norm_w = st.norm_w;
-  l.norm_out = st.out;
-  l.ld_norm = st.ld_out;
+  l.norm_out = st.conv_w ? st.out3 : st.out;  // the rows its multi-token forms read
+  l.ld_norm = st.conv_w ? st.ld_out3 : st.ld_out;
+  l.out3 = st.conv_w ? st.out : nullptr;      // (the normed rows, which the single-token form writes)
   l.out2 = st.out2;
   l.ld_out2 = st.ld_out2;
   l.alpha = st.alpha;
@@ -1291,6 +1378,107 @@ int lower_short_conv(mk_graph *g, size_t &i) {
   return MK_OK;
 }
 
+// ring_conv [rows, weights [taps, channels], bias (fp32, optional), ring [slots, taps, channels], state slots (int32), step bias (fp32 [heads],
+// optional), log2(e) x rates (fp32 [heads]), output, steps and decays (fp32, optional)] params [column, silu 0/1, identity 0/1, heads, step
+// column, column of the decays]: see stage_du_conv.
+int lower_ring_conv(mk_graph *g, size_t &i, MkStage *to, std::string *desc) {
+  const Task &t = g->ltasks[i];
+  if (t.ops.size() != 9 || t.params.size() != 6) return fail(MK_EINVAL, "ring_conv expects 9 operands / 6 params");
+  const Tensor &in = g->tensors[t.ops[0]], &w = g->tensors[t.ops[1]], &ring = g->tensors[t.ops[3]], &o = g->tensors[t.ops[7]];
+  const Tensor *b = t.ops[2] >= 0 ? &g->tensors[t.ops[2]] : nullptr, *sb = t.ops[5] >= 0 ? &g->tensors[t.ops[5]] : nullptr;
+  const int B = g->cfg.max_num_batched_tokens, col = t.params[0], taps = w.ndims == 2 ? (int)w.dims[0] : 0, n = w.ndims == 2 ? (int)w.dims[1] : 0, H = t.params[3], scol = t.params[4], dcol = t.params[5];
+  int rc = set_hyb(g, in.dtype, "ring_conv");
+  if (rc) return rc;
+  g->dual = true;
+  if (taps > MK_DU_MAX_TAPS) return fail(MK_EUNSUPPORTED, "ring_conv: %d taps (at most %d)", taps, MK_DU_MAX_TAPS);
+  if (taps < 1 || n < 4 || n % 4 || col < 0 || col % 4 || w.dtype != in.dtype || w.strides[0] != n || (b && !vector_ok(*b, n)) || !rows_ok(in, B, (int64_t)col + n, in.dtype) || !rows_ok(o, B, n, in.dtype) ||
+      o.ptr == in.ptr || ring.ndims != 3 || ring.dtype != in.dtype || ring.dims[0] < g->cfg.max_num_batched_requests || ring.dims[1] != taps || ring.dims[2] != n || ring.strides[0] != (int64_t)taps * n || ring.strides[1] != n)
+    return fail(MK_EINVAL, "ring_conv: %d taps over %d channels (a multiple of 4) at column %d do not fit the operands", taps, n, col);
+  if (sb && (t.ops[6] < 0 || t.ops[8] < 0 || H < 1 || scol < 0 || scol + H > in.dims[1] || dcol < H || !vector_ok(*sb, H) || !vector_ok(g->tensors[t.ops[6]], H) || !rows_ok(g->tensors[t.ops[8]], B, (int64_t)dcol + H, MK_DT_F32)))
+    return fail(MK_EINVAL, "ring_conv: %d steps at column %d, decays from column %d on, do not fit the operands", H, scol, dcol);
+  if ((rc = set_state_slots(g, g->tensors[t.ops[4]], "ring_conv"))) return rc;
+  MkStage st;
+  memset(&st, 0, sizeof(st));
+  st.op = MK_OP_DU_CONV;
+  if (t.params[1]) st.flags |= MK_F_SILU;
+  if (t.params[2]) st.flags |= MK_F_IDENTITY;
+  st.n = n;
+  st.taps = taps;
+  st.in = in.ptr;
+  st.ld_in = (int)in.strides[0];
+  st.cols[0] = col;
+  st.conv_w = w.ptr;
+  st.in_bias = b ? (const float *)b->ptr : nullptr;
+  st.tail = ring.ptr;
+  st.out = o.ptr;
+  st.ld_out = (int)o.strides[0];
+  if (sb) {
+    st.num_q_heads = H;
+    st.step_bias = (const float *)sb->ptr;
+    st.a_tab = (const float *)g->tensors[t.ops[6]].ptr;
+    st.cols[1] = scol;
+    st.cols[2] = dcol;
+    st.out2 = g->tensors[t.ops[8]].ptr;
+    st.ld_out2 = (int)g->tensors[t.ops[8]].strides[0];
+  }
+  const std::string d = fmt("DU_CONV%s %s -> %s n=%d taps=%d steps=%d", to ? "[portions]" : "", in.name.c_str(), o.name.c_str(), n, taps, sb ? H : 0);
+  if (to) {
+    *to = st;
+    *desc = d;
+  } else {
+    g->stages.push_back(st);
+    g->stage_desc.push_back(d);
+  }
+  i++;
+  return MK_OK;
+}
+
+// dual_scan [rows, convolved rows, steps and decays (fp32), D (fp32 [heads]), state (fp32), state slots (int32), output (fp32)] params [heads,
+// values per head, states, groups, z column of the rows, x, B and C column of the convolved rows, column of the decays]
+int lower_dual_scan(mk_graph *g, size_t &i) {
+  const Task &t = g->ltasks[i];
+  if (t.ops.size() != 7 || t.params.size() != 9) return fail(MK_EINVAL, "dual_scan expects 7 operands / 9 params");
+  const Tensor &in = g->tensors[t.ops[0]], &xc = g->tensors[t.ops[1]], &dt = g->tensors[t.ops[2]], &D = g->tensors[t.ops[3]], &state = g->tensors[t.ops[4]], &o = g->tensors[t.ops[6]];
+  const int B = g->cfg.max_num_batched_tokens, H = t.params[0], V = t.params[1], N = t.params[2], G = t.params[3], zc = t.params[4], x0 = t.params[5], b0 = t.params[6], c0 = t.params[7], dc = t.params[8], np = (N + 3) / 4 * 4;
+  int rc = set_hyb(g, in.dtype, "dual_scan");
+  if (rc) return rc;
+  g->dual = true;
+  if (N < 1 || N > MK_HY_MAX_STATES || H < 1 || V < 1 || G < 1 || H % G) return fail(MK_EUNSUPPORTED, "dual_scan: %d heads of %d values in %d groups, %d states (at most %d)", H, V, G, N, MK_HY_MAX_STATES);
+  if (zc < 0 || x0 < 0 || b0 < 0 || b0 % 4 || c0 < 0 || c0 % 4 || dc < H || !vector_ok(D, H) || !rows_ok(in, B, (int64_t)zc + (int64_t)H * V, in.dtype) ||
+      !rows_ok(xc, B, std::max((int64_t)x0 + (int64_t)H * V, (int64_t)std::max(b0, c0) + (int64_t)G * np), in.dtype) || !rows_ok(dt, B, (int64_t)dc + H, MK_DT_F32) || !rows_ok(o, B, (int64_t)H * V, MK_DT_F32))
+    return fail(MK_EINVAL, "dual_scan: %d heads of %d values, %d groups of %d states do not fit the operands", H, V, G, N);
+  if (state.dtype != MK_DT_F32 || state.ndims != 4 || state.dims[0] < g->cfg.max_num_batched_requests || state.dims[1] != H || state.dims[2] != V || state.dims[3] != np || state.strides[2] != np ||
+      state.strides[1] != (int64_t)V * np || state.strides[0] != (int64_t)H * V * np)
+    return fail(MK_EINVAL, "dual_scan: the state is fp32 [>= %d slots, %d, %d, %d]", g->cfg.max_num_batched_requests, H, V, np);
+  if ((rc = set_state_slots(g, g->tensors[t.ops[5]], "dual_scan"))) return rc;
+  MkStage st;
+  memset(&st, 0, sizeof(st));
+  st.op = MK_OP_DU_SCAN;
+  st.num_q_heads = H;
+  st.v_dim = V;
+  st.states = N;
+  st.groups = G;
+  st.in = in.ptr;
+  st.ld_in = (int)in.strides[0];
+  st.cols[0] = x0;
+  st.cols[1] = b0;
+  st.cols[2] = c0;
+  st.cols[3] = zc;
+  st.cols[4] = dc;
+  st.q_ws = xc.ptr;
+  st.ld_qws = (int)xc.strides[0];
+  st.in2 = dt.ptr;
+  st.ld_in2 = (int)dt.strides[0];
+  st.d_tab = (const float *)D.ptr;
+  st.k_cache = state.ptr;
+  st.out = o.ptr;
+  st.ld_out = (int)o.strides[0];
+  g->stages.push_back(st);
+  g->stage_desc.push_back(fmt("DU_SCAN %s -> %s heads=%d n=%d states=%d groups=%d", xc.name.c_str(), o.name.c_str(), H, V, N, G));
+  i++;
+  return MK_OK;
+}
+
 // scan_step [rows, weights (operand order), offset (fp32), output (fp32)] params [n, k, column]: softplus(W x + offset)
 int lower_scan_step(mk_graph *g, size_t &i) {
   const Task &t = g->ltasks[i];
@@ -1373,20 +1561,31 @@ int lower_selective_scan(mk_graph *g, size_t &i) {
 }
 
 // expert_route [logits (fp32), ids (int32 [tokens, top]), shares (fp32)] params [experts, top, shared 0/1]: the stage runs for
-// iterations of several tokens; the expert_linear behind it routes a single one itself.
+// iterations of several tokens; the expert_linear behind it routes a single one itself.  With one more operand behind the logits (correction,
+// fp32 [experts]) and three more params [groups, groups kept, scale bits]: sigmoid scores, choices among the best groups (MK_F_GROUPS); the
+// shared expert's share is 1 and has no logit.
 // expert_linear [rows, weights, shared weights (optional), ids, output] params [experts, top, n, k, shared n, shared k, gated 0/1, input
-// columns per place (0: one row for all), output columns per place]
+// columns per place (0: one row for all), output columns per place]; four more params [limit, beta, bias, shared expert's limit; bits]: the
+// clamped activation (MK_F_CLAMP_GLU).
 bool route_ok(int experts, int top) { return experts >= 1 && experts <= MK_MOE_MAX_EXPERTS && top >= 1 && top <= experts && top <= MK_MOE_MAX_TOPK; }
 int lower_expert_route(mk_graph *g, size_t &i) {
   const Task &t = g->ltasks[i];
-  if (t.ops.size() != 3 || t.params.size() != 3) return fail(MK_EINVAL, "expert_route expects 3 operands / 3 params");
-  const Tensor &z = g->tensors[t.ops[0]], &ids = g->tensors[t.ops[1]], &w = g->tensors[t.ops[2]];
+  const bool ext = t.ops.size() == 4 && t.params.size() == 6;
+  if (!ext && (t.ops.size() != 3 || t.params.size() != 3)) return fail(MK_EINVAL, "expert_route expects 3 operands / 3 params, or 4 / 6");
+  const Tensor &z = g->tensors[t.ops[0]], &ids = g->tensors[t.ops[1 + ext]], &w = g->tensors[t.ops[2 + ext]];
+  const int ids_id = t.ops[1 + ext];
   const int B = g->cfg.max_num_batched_tokens, E = t.params[0], top = t.params[1], sh = t.params[2] ? 1 : 0;
+  if (ext) {
+    const int groups = t.params[3], keep = t.params[4];
+    if (groups < 1 || E % groups || keep < 1 || keep > groups || top > keep * (E / groups) || !vector_ok(g->tensors[t.ops[1]], E))
+      return fail(MK_EINVAL, "expert_route: %d of %d experts in %d groups of which %d stay open, a correction per expert", top, E, groups, keep);
+    g->dual = true;
+  }
   g->mix = g->hyb = true;
   if (!route_ok(E, top)) return fail(MK_EUNSUPPORTED, "expert_route: %d of %d experts (at most %d of %d)", top, E, MK_MOE_MAX_TOPK, MK_MOE_MAX_EXPERTS);
-  if (!rows_ok(z, B, E + sh, MK_DT_F32) || ids.ndims != 2 || ids.dtype != MK_DT_I32 || ids.dims[0] < B || ids.dims[1] != top || ids.strides[0] != top || !rows_ok(w, B, top + sh, MK_DT_F32))
+  if (!rows_ok(z, B, E + (ext ? 0 : sh), MK_DT_F32) || ids.ndims != 2 || ids.dtype != MK_DT_I32 || ids.dims[0] < B || ids.dims[1] != top || ids.strides[0] != top || !rows_ok(w, B, top + sh, MK_DT_F32))
     return fail(MK_EINVAL, "expert_route: logits fp32 [tokens, %d], ids int32 [tokens, %d], shares fp32 [tokens, >= %d]", E + sh, top, top + sh);
-  if (i + 1 >= g->ltasks.size() || g->ltasks[i + 1].name != "expert_linear" || g->ltasks[i + 1].ops.size() != 5 || g->ltasks[i + 1].ops[3] != t.ops[1] ||
+  if (i + 1 >= g->ltasks.size() || g->ltasks[i + 1].name != "expert_linear" || g->ltasks[i + 1].ops.size() != 5 || g->ltasks[i + 1].ops[3] != ids_id ||
       (g->ltasks[i + 1].ops[2] >= 0) != (sh != 0))
     return fail(MK_EUNSUPPORTED, "expert_route is followed by the expert_linear that reads its ids");
   MkStage st;
@@ -1401,6 +1600,13 @@ int lower_expert_route(mk_graph *g, size_t &i) {
   st.slot_w = (const float *)w.ptr;
   st.ld_slot_w = (int)w.strides[0];
   st.w_shared = sh ? z.ptr : nullptr;  // (only its presence counts here)
+  if (ext) {
+    st.flags |= MK_F_GROUPS;
+    st.choice_bias = (const float *)g->tensors[t.ops[1]].ptr;
+    st.groups = t.params[3];
+    st.groups_keep = t.params[4];
+    st.choice_scale = bits_f32(t.params[5]);
+  }
   g->stages.push_back(st);
   g->stage_desc.push_back(fmt("HY_ROUTE[multi-token only] %s -> %s experts=%d top=%d shared=%d", z.name.c_str(), w.name.c_str(), E, top, sh));
   i++;
@@ -1408,7 +1614,8 @@ int lower_expert_route(mk_graph *g, size_t &i) {
 }
 int lower_expert_linear(mk_graph *g, size_t &i) {
   const Task &t = g->ltasks[i];
-  if (t.ops.size() != 5 || t.params.size() != 9) return fail(MK_EINVAL, "expert_linear expects 5 operands / 9 params");
+  const bool clamp = t.params.size() == 13;
+  if (t.ops.size() != 5 || (!clamp && t.params.size() != 9)) return fail(MK_EINVAL, "expert_linear expects 5 operands / 9 or 13 params");
   const Tensor &in = g->tensors[t.ops[0]], &w = g->tensors[t.ops[1]], &ids = g->tensors[t.ops[3]], &o = g->tensors[t.ops[4]];
   const Tensor *ws = t.ops[2] >= 0 ? &g->tensors[t.ops[2]] : nullptr;
   const int B = g->cfg.max_num_batched_tokens, E = t.params[0], top = t.params[1], n = t.params[2], k = t.params[3], ns = ws ? t.params[4] : 0, ks = ws ? t.params[5] : 0, glu = t.params[6] ? 2 : 1,
@@ -1428,6 +1635,15 @@ int lower_expert_linear(mk_graph *g, size_t &i) {
   memset(&st, 0, sizeof(st));
   st.op = MK_OP_HY_EXPERTS;
   if (glu == 2) st.flags |= MK_F_SILU;
+  if (clamp) {
+    if (glu != 2) return fail(MK_EINVAL, "expert_linear: the clamped activation belongs to a gated linear");
+    g->dual = true;
+    st.flags |= MK_F_CLAMP_GLU;
+    st.glu_limit = bits_f32(t.params[9]);
+    st.glu_beta = bits_f32(t.params[10]);
+    st.glu_bias = bits_f32(t.params[11]);
+    st.glu_limit_shared = bits_f32(t.params[12]);
+  }
   st.num_experts = E;
   st.topk = top;
   st.n = n;
@@ -1452,9 +1668,14 @@ int lower_expert_linear(mk_graph *g, size_t &i) {
     st.ld_logits = r.ld_logits;
     st.slot_w = r.slot_w;
     st.ld_slot_w = r.ld_slot_w;
+    st.flags |= r.flags & MK_F_GROUPS;
+    st.choice_bias = r.choice_bias;
+    st.groups = r.groups;
+    st.groups_keep = r.groups_keep;
+    st.choice_scale = r.choice_scale;
   }
   g->stages.push_back(st);
-  g->stage_desc.push_back(fmt("HY_EXPERTS%s%s %s -> %s experts=%d top=%d n=%d k=%d shared=%dx%d", (st.flags & MK_F_MOE_INLINE_TOPK) ? "+route" : "", glu == 2 ? "+silu" : "", in.name.c_str(), o.name.c_str(), E,
+  g->stage_desc.push_back(fmt("HY_EXPERTS%s%s %s -> %s experts=%d top=%d n=%d k=%d shared=%dx%d", (st.flags & MK_F_MOE_INLINE_TOPK) ? "+route" : "", clamp ? "+clamped" : glu == 2 ? "+silu" : "", in.name.c_str(), o.name.c_str(), E,
                               top, n, k, ns, ks));
   g->weight_bytes += ((int64_t)top * n * k + (int64_t)ns * ks) * es;
   i++;
@@ -1640,7 +1861,7 @@ int lower(mk_graph *g) {
   g->last_linear_task = g->last_linear_stage = -1;
   g->flex = FLEX_NONE;
   g->flex_items = g->flex_part = 0;
-  g->mix = g->hyb = false;
+  g->mix = g->hyb = g->dual = false;
   g->state_ids = nullptr;
   const int B = g->cfg.max_num_batched_tokens;
   // The list that is lowered: the recorded tasks, with the composite ones spelt out as the tasks they stand for (the
@@ -1792,6 +2013,14 @@ int lower(mk_graph *g) {
     } else if (t.name == "short_conv") {
       int rc = lower_short_conv(g, i);
       if (rc) return rc;
+    } else if (t.name == "ring_conv") {
+      int rc = lower_ring_conv(g, i, nullptr, nullptr);
+      if (rc) return rc;
+    } else if (t.name == "dual_scan") {
+      int rc = lower_dual_scan(g, i);
+      if (rc) return rc;
+    } else if (t.name == "gelu_mul") {
+      return fail(MK_EUNSUPPORTED, "gelu_mul follows the linear that writes its input");
     } else if (t.name == "scan_step") {
       int rc = lower_scan_step(g, i);
       if (rc) return rc;
@@ -1996,7 +2225,8 @@ int lower(mk_graph *g) {
     const bool f32_op = op == MK_OP_LINEAR_F32 || op == MK_OP_FX_ARGMAX_F32;
     const bool fixed_op = op == MK_OP_EMBED || op == MK_OP_NORM || op == MK_OP_ATTN || op == MK_OP_SILU_MUL || op == MK_OP_MOE_TOPK || op == MK_OP_MOE_LINEAR || op == MK_OP_MOE_COMBINE;
     const bool ok = g->flex == FLEX_NONE ? !f32_op : g->flex == FLEX_BF16 ? !f32_op && !fixed_op : !fixed_op && op != MK_OP_LINEAR && op != MK_OP_ARGMAX_PARTIAL;
-    if (!ok) return fail(MK_EUNSUPPORTED, "stage %zu (%s) cannot run in one graph with the others", s, g->stage_desc[s].c_str());
+    const bool not_dual = (op >= MK_OP_MX_LATENT_PREP && op <= MK_OP_MX_DELTA_OUT && op != MK_OP_MX_HEAD_LINEAR) || (op >= MK_OP_HY_CONV && op <= MK_OP_HY_SCAN);
+    if (!ok || (g->dual && not_dual)) return fail(MK_EUNSUPPORTED, "stage %zu (%s) cannot run in one graph with the others", s, g->stage_desc[s].c_str());
   }
   for (auto &st : g->stages) {  // the task type a stage is shown as in a profiler trace (runtime_header.h:91-188)
     switch (st.op) {
@@ -2024,7 +2254,9 @@ int lower(mk_graph *g) {
       case MK_OP_MX_DELTA:
       case MK_OP_MX_DELTA_OUT:
       case MK_OP_HY_CONV:
-      case MK_OP_HY_SCAN: st.prof_event = 116; break;
+      case MK_OP_HY_SCAN:
+      case MK_OP_DU_CONV:
+      case MK_OP_DU_SCAN: st.prof_event = 116; break;
       case MK_OP_HY_STEP: st.prof_event = 120; break;
       case MK_OP_HY_ROUTE: st.prof_event = 172; break;
       case MK_OP_HY_EXPERTS: st.prof_event = (st.flags & MK_F_SILU) ? 170 : 171; break;
@@ -2085,7 +2317,8 @@ int task_type_id(const std::string &n) {
       {"find_ngram_partial", 112}, {"find_ngram_global", 113}, {"target_verify_greedy", 114}, {"single_batch_extend_attention", 115},
       {"embedding_scaled", 101}, {"residual_rmsnorm", 119}, {"flex_attention", 116},
       {"residual_prenorm", 119}, {"latent_prep", 116}, {"head_linear", 120}, {"latent_attention", 116}, {"general_delta", 116},
-      {"relu_squared", 118}, {"short_conv", 116}, {"scan_step", 120}, {"selective_scan", 116}, {"expert_route", 172}, {"expert_linear", 170}};
+      {"relu_squared", 118}, {"short_conv", 116}, {"scan_step", 120}, {"selective_scan", 116}, {"expert_route", 172}, {"expert_linear", 170}, {"ring_conv", 116},
+      {"dual_scan", 116}, {"gelu_mul", 118}};
   auto it = ids.find(n);
   return it == ids.end() ? 0 : it->second;
 }
@@ -2385,6 +2618,16 @@ static const void *kernel_of(const mk_graph *g) {
   if (g->flex == FLEX_NONE) {
 #ifdef MK_HAVE_KERNEL_DENSE
     k = m1 ? (const void *)mk_persistent_kernel_m1 : (const void *)mk_persistent_kernel;
+#endif
+  } else if (g->dual) {
+#ifdef MK_HAVE_KERNEL_DUAL
+    if (g->flex == FLEX_BF16 && !m1) k = (const void *)mk_persistent_kernel_dual;
+#endif
+#ifdef MK_HAVE_KERNEL_DUAL_M1
+    if (g->flex == FLEX_BF16 && m1) k = (const void *)mk_persistent_kernel_dual_m1;
+#endif
+#ifdef MK_HAVE_KERNEL_DUAL_F32
+    if (g->flex == FLEX_F32) k = (const void *)mk_persistent_kernel_dual_f32;
 #endif
   } else if (g->hyb) {
 #ifdef MK_HAVE_KERNEL_HYB
@@ -2711,9 +2954,10 @@ int mk_add_task(mk_graph *g, const char *task_name, const int grid_dim[3], const
     // (and the sink of flex_attention, the summand of residual_rmsnorm, what the mix tasks may leave out)
     const bool optional = ((t.name == "gang_attn_split_kv_mi300" || t.name == "kv_cache_update_mi300" || t.name == "paged_attention" ||
                            t.name == "paged_attention_split_kv_mi300" || t.name == "attention" || t.name == "single_batch_extend_attention") && i >= 3 && i <= 6) ||
-                          (t.name == "flex_attention" && i >= 3 && i <= (n_operands == 9 ? 6 : 5)) || (t.name == "expert_linear" && i == 2) || (t.name == "residual_rmsnorm" && i == 0) ||
-                          (t.name == "residual_prenorm" && (i == 0 || i == 1 || i == 3 || (n_operands == 8 && (i == 2 || i == 5)))) || (t.name == "latent_prep" && i >= 1 && i <= 7) ||
-                          (t.name == "head_linear" && (i == 2 || i == 3)) || (t.name == "latent_attention" && (i == 3 || i == 4)) || (t.name == "general_delta" && i == 8);
+                          (t.name == "flex_attention" && i >= 3 && i <= (n_operands == 12 ? 9 : n_operands == 9 ? 6 : 5)) || (t.name == "expert_linear" && i == 2) || (t.name == "residual_rmsnorm" && i == 0) ||
+                          (t.name == "residual_prenorm" && (i == 0 || i == 1 || i == 3 || (n_operands == 8 && (i == 2 || i == 5)) || (n_operands == 11 && i != 7 && i != 10))) || (t.name == "latent_prep" && i >= 1 && i <= 7) ||
+                          (t.name == "head_linear" && (i == 2 || i == 3)) || (t.name == "latent_attention" && (i == 3 || i == 4)) || (t.name == "general_delta" && i == 8) ||
+                          (t.name == "ring_conv" && (i == 2 || i == 5 || i == 6 || i == 8));
     if (tensor_ids[i] >= (int)g->tensors.size() || tensor_ids[i] < (optional ? -1 : 0))
       return fail(MK_EINVAL, "task '%s': bad tensor id %d for operand %d", task_name, tensor_ids[i], i);
     t.ops.push_back(tensor_ids[i]);
@@ -2733,7 +2977,7 @@ int mk_add_task(mk_graph *g, const char *task_name, const int grid_dim[3], const
                                 "paged_attention_ck_fmha_merge_mi300", "gang_attn_merge_mi300", "splitk_reduce_mi300", "silu_mul_linear_with_residual", "rmsnorm_linear", "identity", "argmax", "attention",
                                 "find_ngram_partial", "find_ngram_global", "target_verify_greedy", "single_batch_extend_attention",
                                 "embedding_scaled", "residual_rmsnorm", "flex_attention", "residual_prenorm", "latent_prep", "head_linear", "latent_attention", "general_delta",
-                                "relu_squared", "short_conv", "scan_step", "selective_scan", "expert_route", "expert_linear"};
+                                "relu_squared", "short_conv", "scan_step", "selective_scan", "expert_route", "expert_linear", "ring_conv", "dual_scan", "gelu_mul"};
   bool ok = linear_kind(t.name, &a, &b, &c);
   for (auto k : known) ok = ok || t.name == k;
   if (!ok) return fail(MK_EUNSUPPORTED, "Unsupported task name: %s", task_name);

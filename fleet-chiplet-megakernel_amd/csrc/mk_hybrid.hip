@@ -263,7 +263,78 @@ __device__ __forceinline__ void stage_hy_scan(CStage &st, Ctx &c, const MkRuntim
 // ----------------------------------------------------------------------------- routing
 // One wavefront, one token: z fp32 [experts (+ 1: the shared expert's gate)].  Lane s < topk ends up with the s-th choice (ties: the
 // lower index) and its share, lane topk with sigmoid of the gate.
-__device__ __forceinline__ void hy_route_wave(CStage &st, const float *z, int lane, float &w, int &id) {
+// With MK_F_GROUPS (dual kernels): scores are sigmoids, choices are made on score + correction among the experts of the best groups, a
+// group's worth being the sum of its two largest; the shares are choice_scale times the scores, the shared expert's is 1.  `scr`: 2 KB
+// of LDS of the wavefront.
+#if MK_HAVE_DUAL
+__device__ __forceinline__ void hy_route_groups(CStage &st, const float *z, int lane, float &w, int &id, float *scr) {
+  const int E = st.num_experts, count = st.groups, size = E / count;
+  float s[4], p[4];
+#pragma unroll
+  for (int q = 0; q < 4; q++) {
+    const int e = q * 64 + lane, ec = min(e, E - 1);
+    const float zv = ldc_f32(z + ec), b = st.choice_bias[ec];
+    s[q] = 1.f / (1.f + expf(-zv));
+    p[q] = e < E ? s[q] + b : -3.0e38f;
+    scr[e] = p[q];
+  }
+  __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+  if (count > 1) {
+    for (int g = lane; g < count; g += 64) {
+      float a = -3.0e38f, b = -3.0e38f;
+      for (int i = 0; i < size; i++) {
+        const float v = scr[g * size + i];
+        b = fmaxf(b, fminf(a, v));
+        a = fmaxf(a, v);
+      }
+      scr[256 + g] = size > 1 ? a + b : a;
+    }
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+#pragma unroll
+    for (int q = 0; q < 4; q++) {
+      if (q * 64 >= E) continue;
+      const int g = min(q * 64 + lane, E - 1) / size;
+      const float mine = scr[256 + g];
+      int better = 0;
+      for (int i = 0; i < count; i++) {
+        const float v = scr[256 + i];
+        better += v > mine || (v == mine && i < g);
+      }
+      if (better >= st.groups_keep) p[q] = -3.0e38f;
+    }
+  }
+  w = 0.f;
+  id = 0;
+  for (int k = 0; k < st.topk; k++) {
+    float bv = p[0];
+    int be = lane;
+#pragma unroll
+    for (int q = 1; q < 4; q++)
+      if (p[q] > bv) {
+        bv = p[q];
+        be = q * 64 + lane;
+      }
+    wave_argmax(bv, be);
+    be = __builtin_amdgcn_readfirstlane(be);
+    const float sv = lane_f32(be < 64 ? s[0] : be < 128 ? s[1] : be < 192 ? s[2] : s[3], be & 63);
+    if (lane == k) {
+      w = sv * st.choice_scale;
+      id = be;
+    }
+#pragma unroll
+    for (int q = 0; q < 4; q++)
+      if (q * 64 + lane == be) p[q] = -3.4e38f;
+  }
+  if (lane == st.topk) w = 1.f;
+}
+#endif
+__device__ __forceinline__ void hy_route_wave(CStage &st, const float *z, int lane, float &w, int &id, float *scr) {
+#if MK_HAVE_DUAL
+  if (st.flags & MK_F_GROUPS) {
+    hy_route_groups(st, z, lane, w, id, scr);
+    return;
+  }
+#endif
   const int E = st.num_experts;
   float p[4], mx = -3.0e38f;
 #pragma unroll
@@ -312,13 +383,13 @@ __device__ __forceinline__ void hy_route_store(CStage &st, int t, int lane, floa
   if (lane < st.topk + (st.w_shared ? 1 : 0)) stc_f32((float *)st.slot_w + (size_t)t * st.ld_slot_w + lane, w);
 }
 // (iterations of several tokens; a single token is routed by the expert stage itself)
-__device__ __forceinline__ void stage_hy_route(CStage &st, Ctx &c, int M) {
+__device__ __forceinline__ void stage_hy_route(CStage &st, Ctx &c, int M, char *smem) {
   barrier_wait(c);
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   for (int t = mx_wave_item(c, wave); t < M; t += c.G * MK_WAVES) {
     float w;
     int id;
-    hy_route_wave(st, (const float *)st.moe_logits + (size_t)t * st.ld_logits, lane, w, id);
+    hy_route_wave(st, (const float *)st.moe_logits + (size_t)t * st.ld_logits, lane, w, id, (float *)smem + wave * 512);
     hy_route_store(st, t, lane, w, id);
   }
   c.wrote_through = true;
@@ -338,7 +409,17 @@ struct HyLists {
   int pad[3];
   unsigned char place[MK_MOE_MAX_EXPERTS][MK_MAX_TOKENS];
 };
-static_assert(sizeof(HyLists) <= MK_MOE_OFFSET, "the lists lie below the scratch of the reduction");
+static_assert(sizeof(HyLists) <= MK_OUT_OFFSET, "the lists lie below the scratch of the routing and of the reduction");
+template <typename E>
+__device__ __forceinline__ float hy_glu(E, CStage &st, bool shared, float a, float b) {
+#if MK_HAVE_DUAL
+  if (st.flags & MK_F_CLAMP_GLU) {
+    const float lim = shared ? st.glu_limit_shared : st.glu_limit, g = fminf(a, lim), u = fminf(fmaxf(b, -lim), lim);
+    return g * mx_sigmoid(E(), st.glu_beta * g) * (u + st.glu_bias);
+  }
+#endif
+  return hy_silu(E(), a) * b;
+}
 template <typename E, int MT, bool SPLIT>
 __device__ __forceinline__ void hy_expert_unit(CStage &st, const HyLists *ls, bool shared, int e, int pair, unsigned long long toks, int n, int K, int wave, int lane,
                                                const u32x4 *W, const u32x4 (&first)[2][4], f32x4 *red) {
@@ -416,7 +497,7 @@ __device__ __forceinline__ void hy_expert_unit(CStage &st, const HyLists *ls, bo
       if (glu) {
         const f32x4 u = total(1, m);
 #pragma unroll
-        for (int q = 0; q < 4; q++) r[q] = hy_silu(E(), r[q]) * u[q];
+        for (int q = 0; q < 4; q++) r[q] = hy_glu(E(), st, shared, r[q], u[q]);
       }
       fx_stc4((E *)st.out + (size_t)tok[m] * st.ld_out + (size_t)place[m] * st.ld_out_slot, (glu ? pair : 2 * pair + h) * 16 + lg * 4, glu ? n / 2 : n, r);
     }
@@ -470,7 +551,7 @@ __device__ __forceinline__ void stage_hy_experts(CStage &st, Ctx &c, int M, char
     if (wave == MK_WAVES - 1) {
       float w;
       int id;
-      hy_route_wave(st, (const float *)st.moe_logits, lane, w, id);
+      hy_route_wave(st, (const float *)st.moe_logits, lane, w, id, (float *)(smem + MK_OUT_OFFSET));
       if (lane < topk) {
         ls->tok[id] = 1ull;
         ls->place[id][0] = (unsigned char)lane;

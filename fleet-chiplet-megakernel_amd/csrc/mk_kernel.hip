@@ -74,7 +74,12 @@ typedef const __attribute__((address_space(4))) MkWeight CWeight;
 #define MK_TUNE_R24 2
 #endif
 
-#if defined(MK_KERNEL_HYB) || defined(MK_KERNEL_HYB_M1) || defined(MK_KERNEL_HYB_F32)
+#if defined(MK_KERNEL_DUAL) || defined(MK_KERNEL_DUAL_M1) || defined(MK_KERNEL_DUAL_F32)
+#define MK_HAVE_DUAL 1  // ... the dual stages (mk_dual.hip) beside flex, mix and hybrid ones, without latent attention, delta rule and selective scan
+#else
+#define MK_HAVE_DUAL 0
+#endif
+#if defined(MK_KERNEL_HYB) || defined(MK_KERNEL_HYB_M1) || defined(MK_KERNEL_HYB_F32) || MK_HAVE_DUAL
 #define MK_HAVE_HYB 1
 #else
 #define MK_HAVE_HYB 0
@@ -119,6 +124,9 @@ struct Ctx {
   int defer_ld_res;
 #if MK_HAVE_MIX
   bool mx_split;  // the latent attention (delta rule) that just ran left some request in chunks (its heads in slices)
+#endif
+#if MK_HAVE_DUAL
+  const int *state_ids;  // MkRuntime::state_ids
 #endif
 #ifdef MK_TRACE
   long long mark[4];  // (tracing builds) wall-clock marks the running stage sets, stored next to its stage timing
@@ -910,6 +918,16 @@ __device__ __forceinline__ void stage_norm(CStage &st, Ctx &c, int M, char *smem
 }
 
 __device__ __forceinline__ float silu_mul(float g, float u) { return g / (1.f + __expf(-g)) * u; }
+// gated activation of a [gate ; up] linear (dual kernels: gelu where the stage asks for it, 32-bit: library functions)
+__device__ __forceinline__ float gelu_tanh(float z) {  // z / (1 + e^-2y) = z (1 + tanh y) / 2
+  return z / (1.f + __expf(-1.5957691216057308f * (z + 0.044715f * z * z * z)));
+}
+__device__ __forceinline__ float linear_glu(CStage &st, float g, float u) {
+#if MK_HAVE_DUAL
+  if (st.flags & MK_F_GELU) return gelu_tanh(g) * u;
+#endif
+  return silu_mul(g, u);
+}
 // activation of a plain linear's outputs (hybrid kernels: the square of relu where the stage asks for it)
 __device__ __forceinline__ float linear_act(CStage &st, float v) {
 #if MK_HAVE_HYB
@@ -1249,7 +1267,7 @@ __device__ __forceinline__ void stage_linear_m1_t(CStage &st, Ctx &c, char *smem
         }
 #pragma unroll
         for (int h = 0; h < NROW; h++) a[h] = wave_sum(a[h]);
-        const float v = SILU ? silu_mul(a[0], a[NROW - 1]) : linear_act(st, a[0] + lres[i]);
+        const float v = SILU ? linear_glu(st, a[0], a[NROW - 1]) : linear_act(st, a[0] + lres[i]);
         if (lane == 0) so[lo_[i] - o_begin] = (uint16_t)f2bf(v);
       }
     }
@@ -1276,7 +1294,7 @@ __device__ __forceinline__ void stage_linear_m1_t(CStage &st, Ctx &c, char *smem
         }
 #pragma unroll
         for (int h = 0; h < NROW; h++) a[h] = wave_sum(a[h]);
-        const float v = SILU ? silu_mul(a[0], a[NROW - 1]) : linear_act(st, a[0] + r);
+        const float v = SILU ? linear_glu(st, a[0], a[NROW - 1]) : linear_act(st, a[0] + r);
         if (lane == 0) so[o - o_begin] = (uint16_t)f2bf(v);
       }
     }
@@ -1318,7 +1336,7 @@ __device__ __forceinline__ void stage_linear_m1_generic(CStage &st, Ctx &c, char
         ag = dot8(ldg_stream(wg + kc), x, ag);
         au = dot8(ldg_stream(wu + kc), x, au);
       }
-      v = silu_mul(wave_sum(ag), wave_sum(au));
+      v = linear_glu(st, wave_sum(ag), wave_sum(au));
     } else {
       const u32x4 *w0 = weight_row(st.w, r, k8);
       float a0 = 0.f;
@@ -1536,7 +1554,7 @@ __device__ __forceinline__ void stage_linear_small(CStage &st, Ctx &c, int M, ch
     const float tot = transpose_sum<NV>(vv, lane);
     const int m = lane & (MB - 1), q = SILU ? 0 : lane / MB;
     float v;
-    if (SILU) v = silu_mul(tot, dpp_f32<0x100 + MB>(tot));  // row_shl:MB: the up sum sits MB lanes above the gate sum
+    if (SILU) v = linear_glu(st, tot, dpp_f32<0x100 + MB>(tot));  // row_shl:MB: the up sum sits MB lanes above the gate sum
     else v = linear_act(st, tot + rf);
     if (lane < Q * MB && m < M && o + q < o_end) so[m * n_loc + (o + q - o_begin)] = (uint16_t)f2bf(v);
   };
@@ -1838,7 +1856,7 @@ __device__ __forceinline__ void stage_linear_mfma_tiles(CStage &st, Ctx &c, cons
           for (int i = 0; i < 4; i++) {
             const int n = otile * 16 + lg * 4 + i;
             float r;
-            if (silu) r = TW >= 2 ? silu_mul(acc[(2 * u) % TW][mt][i], acc[(2 * u + 1) % TW][mt][i]) : 0.f;
+            if (silu) r = TW >= 2 ? linear_glu(st, acc[(2 * u) % TW][mt][i], acc[(2 * u + 1) % TW][mt][i]) : 0.f;
             else r = acc[u][mt][i];
             if ((st.flags & MK_F_RES) && n < n_out) r += bf2f(rrow[n]);
             rr[i] = linear_act(st, r);
@@ -2179,13 +2197,13 @@ __device__ __forceinline__ void stage_linear_mfma_xres(CStage &st, Ctx &c, const
 #pragma unroll
           for (int mt = 0; mt < MT; mt++)
 #pragma unroll
-            for (int i = 0; i < 4; i++) v[mt][i] = silu_mul(acc[t][mt][i], acc[(t + 1) % TW][mt][i]);
+            for (int i = 0; i < 4; i++) v[mt][i] = linear_glu(st, acc[t][mt][i], acc[(t + 1) % TW][mt][i]);
         } else {
 #pragma unroll
           for (int mt = 0; mt < MT; mt++) {
             const f32x4 up = __builtin_bit_cast(f32x4, xl[mt * 64 + lane]);
 #pragma unroll
-            for (int i = 0; i < 4; i++) v[mt][i] = silu_mul(acc[t][mt][i], up[i]);
+            for (int i = 0; i < 4; i++) v[mt][i] = linear_glu(st, acc[t][mt][i], up[i]);
           }
         }
         store_tile(ti >> 1, v);
@@ -2354,7 +2372,7 @@ __device__ __forceinline__ void stage_linear_mfma(CStage &st, Ctx &c, int M, cha
 #pragma unroll
         for (int i = 0; i < 4; i++) {
           const int n = n0 + i;
-          float r = silu ? silu_mul(v[i], v2[i]) : v[i];
+          float r = silu ? linear_glu(st, v[i], v2[i]) : v[i];
           if ((st.flags & MK_F_RES) && n < n_out) r += bf2f(rrow[n]);
           rr[i] = linear_act(st, r);
         }
@@ -4154,6 +4172,9 @@ __device__ __attribute__((noinline)) void mk_verify_greedy(int stage, const MkRu
 #if MK_HAVE_HYB
 #include "mk_hybrid.hip"
 #endif
+#if MK_HAVE_DUAL
+#include "mk_dual.hip"
+#endif
 #define MK_HAVE_FLEX 1
 #else
 #define MK_HAVE_FLEX 0
@@ -4177,6 +4198,9 @@ __device__ __forceinline__ void run_stage_program(const MkRuntime &rt, const MkR
       const bool packed_only = MAXM > 1 && rt.packed_only;
       if ((flags & MK_F_ONLY_MULTI) && M == 1 && !(packed_only && (op == MK_OP_NORM || (FX && (op == MK_OP_FX_ADDNORM || op == MK_OP_MX_PRENORM))))) continue;
       if (FX && op == MK_OP_FX_PREP && single) continue;
+#if MK_HAVE_DUAL
+      if (op == MK_OP_DU_CONV && (flags & MK_F_PORTIONS) && (MAXM == 1 || single)) continue;
+#endif
 #if MK_HAVE_MIX
       if ((op == MK_OP_MX_LATENT_MERGE || op == MK_OP_MX_DELTA_OUT) && !c.mx_split) continue;
 #endif
@@ -4202,20 +4226,27 @@ __device__ __forceinline__ void run_stage_program(const MkRuntime &rt, const MkR
         case MK_OP_FX_ARGMAX_F32: if constexpr (F32) stage_fx_argmax_f32(st, c, rt, M); break;
 #endif
 #if MK_HAVE_MIX
-        case MK_OP_MX_PRENORM: stage_mx_prenorm<E>(st, c, M, smem); break;
+        case MK_OP_MX_PRENORM: stage_mx_prenorm<E>(st, c, M, MAXM == 1 || single, smem); break;
+#if !MK_HAVE_DUAL
         case MK_OP_MX_LATENT_PREP: stage_mx_latent_prep<E>(st, c, rt, M); break;
-        case MK_OP_MX_HEAD_LINEAR: stage_mx_head_linear<E, MAXM>(st, c, M, smem); break;
         case MK_OP_MX_LATENT_ATTN: stage_mx_latent_attn<E>(st, c, rt, M, smem); break;
         case MK_OP_MX_LATENT_MERGE: stage_mx_latent_merge<E>(st, c, rt, M); break;
         case MK_OP_MX_DECAY: stage_mx_head_linear_t<E, 1, MX_DECAY, false>(st, c, M, smem); break;
         case MK_OP_MX_DELTA: stage_mx_delta<E>(st, c, rt, M, MAXM == 1 || single, smem); break;
         case MK_OP_MX_DELTA_OUT: stage_mx_delta_out<E>(st, c, M); break;
 #endif
+        case MK_OP_MX_HEAD_LINEAR: stage_mx_head_linear<E, MAXM>(st, c, M, smem); break;
+#endif
 #if MK_HAVE_HYB
+#if MK_HAVE_DUAL
+        case MK_OP_DU_CONV: stage_du_conv<E>(st, c, M); break;
+        case MK_OP_DU_SCAN: stage_du_scan<E>(st, c, rt, M, MAXM == 1 || single); break;
+#else
         case MK_OP_HY_CONV: stage_hy_conv<E>(st, c, rt, M); break;
         case MK_OP_HY_STEP: stage_mx_head_linear_t<E, 1, MX_STEP, false>(st, c, M, smem); break;
         case MK_OP_HY_SCAN: stage_hy_scan<E>(st, c, rt, M, MAXM == 1 || single); break;
-        case MK_OP_HY_ROUTE: stage_hy_route(st, c, M); break;
+#endif
+        case MK_OP_HY_ROUTE: stage_hy_route(st, c, M, smem); break;
         case MK_OP_HY_EXPERTS: stage_hy_experts<E, MAXM>(st, c, M, smem); break;
 #endif
         case MK_OP_EMBED: if constexpr (!FX) stage_embed(st, c, rt, M); break;
@@ -4352,6 +4383,9 @@ __device__ __forceinline__ void mk_kernel_body(const MkRuntime &rt, const MkRunt
   c.sh_tok = &sh_tok[0][0];
   c.sh_ticket = sh_ticket;
   c.seq = 0;
+#if MK_HAVE_DUAL
+  c.state_ids = rt.state_ids;
+#endif
   c.prof_n = 0;
   c.defer_S = 0;
   c.wrote_through = false;
@@ -4509,6 +4543,21 @@ extern "C" __global__ __launch_bounds__(MK_THREADS, 1) void mk_persistent_kernel
 #endif
 #ifdef MK_KERNEL_HYB_F32
 extern "C" __global__ __launch_bounds__(MK_THREADS, 1) void mk_persistent_kernel_hyb_f32(MK_KERNEL_ARGS) {
+  mk_kernel_body<MK_MAX_TOKENS, float>(rt, rtp, max_iters, run_scheduler);
+}
+#endif
+#ifdef MK_KERNEL_DUAL  // graphs with dual stages (mk_dual.hip): those, the flex stages, norms and head linears, routing and experts
+extern "C" __global__ __launch_bounds__(MK_THREADS, 1) void mk_persistent_kernel_dual(MK_KERNEL_ARGS) {
+  mk_kernel_body<MK_MAX_TOKENS, uint16_t>(rt, rtp, max_iters, run_scheduler);
+}
+#endif
+#ifdef MK_KERNEL_DUAL_M1
+extern "C" __global__ __launch_bounds__(MK_THREADS, 1) void mk_persistent_kernel_dual_m1(MK_KERNEL_ARGS) {
+  mk_kernel_body<1, uint16_t>(rt, rtp, max_iters, run_scheduler);
+}
+#endif
+#ifdef MK_KERNEL_DUAL_F32
+extern "C" __global__ __launch_bounds__(MK_THREADS, 1) void mk_persistent_kernel_dual_f32(MK_KERNEL_ARGS) {
   mk_kernel_body<MK_MAX_TOKENS, float>(rt, rtp, max_iters, run_scheduler);
 }
 #endif

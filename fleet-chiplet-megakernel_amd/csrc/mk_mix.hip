@@ -53,12 +53,37 @@ __device__ __forceinline__ f32x4 mx_summand(CStage &st, const E *y, const float 
 #endif
 }
 
+#if MK_HAVE_DUAL
+// Convolution over time of normed rows, added to them (see mk_dual.hip): one quad of a row whose request brings this one token.  h:
+// the row's values as they are stored, ring: the request's ring of st.taps rows.  Taps b0 .. (counted back from the token's own).
+template <typename E>
+__device__ __forceinline__ f32x4 mx_ring_conv(CStage &st, const E *ring, int n, int pos, int q, int b0, f32x4 acc) {
+  const int taps = st.taps;
+  for (int b = b0; b < taps; b += 4) {
+    f32x4 v[4], g[4];
+#pragma unroll
+    for (int y = 0; y < 4; y++) {
+      const int back = min(b + y, taps - 1);
+      v[y] = fx_ldc_quad(ring + (size_t)(max(pos - back, 0) % taps) * n + 4 * q);
+      g[y] = fx_ld_quad((const E *)st.conv_w + (size_t)(taps - 1 - back) * n + 4 * q);
+    }
+#pragma unroll
+    for (int y = 0; y < 4; y++)
+#pragma unroll
+      for (int e = 0; e < 4; e++) acc[e] = b + y < taps && b + y <= pos ? fmaf(v[y][e], g[y][e], acc[e]) : acc[e];
+  }
+  return acc;
+}
+#endif
+
 // ----------------------------------------------------------------------------- residual sum + norm in parts
 // v = x + alpha * f(y),  f(y) = y or y / sqrt(mean(y^2) + norm_eps) * y_norm_w;  out2 = v (32-bit);  out = the RMS norm of v in
 // st.norm_groups equal parts times norm_w (norm_groups 0: v itself), rounded to E.  Rows are st.n long, st.k of them real (the
 // rest is zero in every operand).  A workgroup per row.
+// Dual kernels: v = x + alpha * y_scale f(y) + y2_scale y2 (both factors element by element; `slots` then belongs to y2), and when every
+// request brings one token also out3 = the normed row plus its convolution over time, which keeps the row in the request's ring.
 template <typename E, int NS>
-__device__ __forceinline__ void stage_mx_prenorm_t(CStage &st, Ctx &c, int M, char *smem) {
+__device__ __forceinline__ void stage_mx_prenorm_t(CStage &st, Ctx &c, int M, bool single, char *smem) {
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), n4 = st.n / 4;
   float *red = (float *)smem, *gs = red + 64, *row = gs + MK_MX_MAX_GROUPS;
   const int ng = st.norm_groups, gl = ng ? st.k / ng : st.k;
@@ -87,6 +112,17 @@ __device__ __forceinline__ void stage_mx_prenorm_t(CStage &st, Ctx &c, int M, ch
     for (int j = 0; j < NS; j++) yb[j] = yb4[at(j)];
   }
 #endif
+#if MK_HAVE_DUAL
+  f32x4 ys[NS], y2s[NS];
+  if (st.y_scale) {
+#pragma unroll
+    for (int j = 0; j < NS; j++) ys[j] = ((const f32x4 *)st.y_scale)[at(j)];
+  }
+  if (st.y2) {
+#pragma unroll
+    for (int j = 0; j < NS; j++) y2s[j] = st.y2_scale ? ((const f32x4 *)st.y2_scale)[at(j)] : (f32x4){1.f, 1.f, 1.f, 1.f};
+  }
+#endif
   // the residual row was written at least one barrier earlier than y: requested before the barrier is awaited (not by the
   // wavefront that polls it)
 #if MK_HAVE_HYB
@@ -102,7 +138,26 @@ __device__ __forceinline__ void stage_mx_prenorm_t(CStage &st, Ctx &c, int M, ch
     if (st.in) {
       f32x4 y[NS];
 #pragma unroll
-      for (int j = 0; j < NS; j++) y[j] = mx_summand<E>(st, (const E *)st.in + (size_t)t * st.ld_in, MK_HAVE_HYB ? st.slot_w + (size_t)t * st.ld_slot_w : nullptr, at(j));
+      for (int j = 0; j < NS; j++) {
+#if MK_HAVE_DUAL
+        if (st.y2) {
+          y[j] = fx_ldc_quad((const E *)st.in + (size_t)t * st.ld_in + 4 * at(j));
+          continue;
+        }
+#endif
+        y[j] = mx_summand<E>(st, (const E *)st.in + (size_t)t * st.ld_in, MK_HAVE_HYB ? st.slot_w + (size_t)t * st.ld_slot_w : nullptr, at(j));
+      }
+#if MK_HAVE_DUAL
+      if (st.y2) {
+        f32x4 y2[NS];
+#pragma unroll
+        for (int j = 0; j < NS; j++) y2[j] = mx_summand<E>(st, (const E *)st.y2 + (size_t)t * st.ld_y2, st.slot_w + (size_t)t * st.ld_slot_w, at(j));
+#pragma unroll
+        for (int j = 0; j < NS; j++)
+#pragma unroll
+          for (int e = 0; e < 4; e++) x[j][e] = fmaf(y2s[j][e], y2[j][e], x[j][e]);
+      }
+#endif
       float f = st.alpha;
 #if MK_HAVE_HYB
       if (yb4) {
@@ -120,6 +175,12 @@ __device__ __forceinline__ void stage_mx_prenorm_t(CStage &st, Ctx &c, int M, ch
 #pragma unroll
         for (int j = 0; j < NS; j++) y[j] = (y[j] * r) * yw_at(j);
       }
+#if MK_HAVE_DUAL
+      if (st.y_scale) {
+#pragma unroll
+        for (int j = 0; j < NS; j++) y[j] *= ys[j];
+      }
+#endif
 #pragma unroll
       for (int j = 0; j < NS; j++)
 #pragma unroll
@@ -158,15 +219,31 @@ __device__ __forceinline__ void stage_mx_prenorm_t(CStage &st, Ctx &c, int M, ch
           for (int e = 0; e < 4; e++) o[e] = (o[e] * gs[q0 == q3 ? q0 : min((4 * s + e) / gl, ng - 1)]) * g[j][e];
         }
         if (st.out) fx_stc_quad((E *)st.out + (size_t)t * st.ld_out + 4 * s, o);
+#if MK_HAVE_DUAL
+        if (st.conv_w && single) {
+          const int pos = __builtin_amdgcn_readfirstlane(c.sh_tok[t]), taps = st.taps;
+          E *ring = (E *)st.tail + (size_t)__builtin_amdgcn_readfirstlane(c.state_ids[__builtin_amdgcn_readfirstlane(c.sh_tok[MK_MAX_TOKENS + t])]) * taps * st.n;
+          const f32x4 w0 = fx_ld_quad((const E *)st.conv_w + (size_t)(taps - 1) * st.n + 4 * s);
+          f32x4 h, acc;
+#pragma unroll
+          for (int e = 0; e < 4; e++) {
+            h[e] = fx_val(fx_round<E>(o[e]));
+            acc[e] = fmaf(w0[e], h[e], h[e]);
+          }
+          acc = mx_ring_conv<E>(st, ring, st.n, pos, s, 1, acc);
+          fx_stc_quad((E *)st.out3 + (size_t)t * st.ld_out3 + 4 * s, acc);
+          fx_stc_quad(ring + (size_t)(pos % taps) * st.n + 4 * s, h);
+        }
+#endif
       }
     __syncthreads();
   }
   c.wrote_through = true;
 }
 template <typename E>
-__device__ __forceinline__ void stage_mx_prenorm(CStage &st, Ctx &c, int M, char *smem) {
-  if (st.n <= 4 * 4 * MK_THREADS) stage_mx_prenorm_t<E, 4>(st, c, M, smem);
-  else stage_mx_prenorm_t<E, 12>(st, c, M, smem);
+__device__ __forceinline__ void stage_mx_prenorm(CStage &st, Ctx &c, int M, bool single, char *smem) {
+  if (st.n <= 4 * 4 * MK_THREADS) stage_mx_prenorm_t<E, 4>(st, c, M, single, smem);
+  else stage_mx_prenorm_t<E, 12>(st, c, M, single, smem);
 }
 
 // The same in front of a single-token bf16 linear, whose input row it leaves in LDS (virtual workgroup 0 also stores the rows).
@@ -343,12 +420,115 @@ __device__ __forceinline__ void mx_x_m1_prenorm_wave(CStage &st, Ctx &c, uint32_
   }
 }
 
+#if MK_HAVE_DUAL
+// What a residual_prenorm with dual options does in front of a single-token linear, by the workgroup: v = res + alpha y_scale y + y2_scale y2,
+// the normed row (norm_out, with a convolution: out3) and the linear's input row in LDS, which is the normed row or the sum of it and its convolution.  In two
+// halves: whatever the previous stage does not write is requested before its barrier is awaited.  NS: quads per thread (0: none of this).
+// One part of the norm; the norm weight, both factors and the convolution are optional as in the stage.
+#define MX_EARLY_TAPS 4
+template <int NS>
+struct MxPrologue {
+  f32x4 g[NS], ys[NS], y2s[NS], x[NS];
+  unsigned long long cw[NS][MX_EARLY_TAPS], ring[NS][MX_EARLY_TAPS];
+  int pos, k4;
+  uint16_t *rows;
+  __device__ __forceinline__ int at(int j) const { return min((int)threadIdx.x + j * MK_THREADS, k4 - 1); }
+  __device__ __forceinline__ void load_x(CStage &st) {
+#pragma unroll
+    for (int j = 0; j < NS; j++) x[j] = fx_ldc_quad((const float *)st.res + 4 * at(j));
+  }
+  __device__ __forceinline__ void load(CStage &st, const Ctx &c) {
+    k4 = st.k / 4;
+    pos = __builtin_amdgcn_readfirstlane(c.sh_tok[0]);
+    const f32x4 one = {1.f, 1.f, 1.f, 1.f};
+#pragma unroll
+    for (int j = 0; j < NS; j++) {
+      g[j] = ((const f32x4 *)st.norm_w)[at(j)];
+      ys[j] = st.y_scale ? ((const f32x4 *)st.y_scale)[at(j)] : one;
+      y2s[j] = st.y2_scale ? ((const f32x4 *)st.y2_scale)[at(j)] : one;
+    }
+    if (st.conv_w) {
+      const int taps = st.taps;
+      rows = (uint16_t *)st.tail + (size_t)__builtin_amdgcn_readfirstlane(c.state_ids[__builtin_amdgcn_readfirstlane(c.sh_tok[MK_MAX_TOKENS])]) * taps * st.k;
+#pragma unroll
+      for (int b = 0; b < MX_EARLY_TAPS; b++) {
+        const int back = min(b, taps - 1), row = max(pos - back, 0) % taps;
+#pragma unroll
+        for (int j = 0; j < NS; j++) {
+          cw[j][b] = ((const unsigned long long *)((const uint16_t *)st.conv_w + (size_t)(taps - 1 - back) * st.k))[at(j)];
+          if (b) ring[j][b] = ldc_u64(rows + (size_t)row * st.k + 4 * at(j));
+        }
+      }
+    }
+    if (st.flags & MK_F_RES_EARLY) load_x(st);
+  }
+  __device__ __forceinline__ void finish(CStage &st, const Ctx &c, uint32_t *xs, float *red) {
+    auto quad = [](unsigned long long u) { return (f32x4){bf_lo((uint32_t)u), bf_hi((uint32_t)u), bf_lo((uint32_t)(u >> 32)), bf_hi((uint32_t)(u >> 32))}; };
+    const int tid = threadIdx.x;
+    if (!(st.flags & MK_F_RES_EARLY)) load_x(st);
+    f32x4 y[NS], y2[NS];
+    if (st.y_in) {
+#pragma unroll
+      for (int j = 0; j < NS; j++) y[j] = st.y2 ? fx_ldc_quad((const uint16_t *)st.y_in + 4 * at(j)) : mx_summand<uint16_t>(st, (const uint16_t *)st.y_in, st.slot_w, at(j));
+      if (st.y2) {
+#pragma unroll
+        for (int j = 0; j < NS; j++) y2[j] = mx_summand<uint16_t>(st, (const uint16_t *)st.y2, st.slot_w, at(j));
+      }
+#pragma unroll
+      for (int j = 0; j < NS; j++)
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+          if (st.y2) x[j][e] = fmaf(y2s[j][e], y2[j][e], x[j][e]);
+          x[j][e] = fmaf(st.alpha, y[j][e] * ys[j][e], x[j][e]);
+        }
+    }
+    float ss = 0.f;
+#pragma unroll
+    for (int j = 0; j < NS; j++)
+      if (tid + j * MK_THREADS < k4) ss += x[j][0] * x[j][0] + x[j][1] * x[j][1] + x[j][2] * x[j][2] + x[j][3] * x[j][3];
+    const float r = 1.f / sqrtf(block_sum(ss, red) / (float)st.k_real + st.eps);
+#pragma unroll
+    for (int j = 0; j < NS; j++) {
+      const int i = tid + j * MK_THREADS;
+      if (i >= k4) continue;
+      const f32x4 o = (x[j] * r) * g[j];
+      unsigned long long hp = (unsigned long long)pack2(o[0], o[1]) | ((unsigned long long)pack2(o[2], o[3]) << 32);
+      if (c.vid == 0) {
+        if (st.out2) stc_16B((u32x4 *)st.out2 + i, __builtin_bit_cast(u32x4, x[j]));
+        stc_u64((unsigned long long *)(st.conv_w ? st.out3 : st.norm_out) + i, hp);
+        if (st.conv_w) stc_u64(rows + (size_t)(pos % st.taps) * st.k + 4 * i, hp);  // (a row nobody reads in this iteration)
+      }
+      if (st.conv_w) {
+        const f32x4 h = quad(hp);
+        f32x4 acc = h;
+#pragma unroll
+        for (int b = 0; b < MX_EARLY_TAPS; b++) {
+          const f32x4 w = quad(cw[j][b]), v = b ? quad(ring[j][b]) : h;
+#pragma unroll
+          for (int e = 0; e < 4; e++) acc[e] = b < st.taps && b <= pos ? fmaf(v[e], w[e], acc[e]) : acc[e];
+        }
+        if (st.taps > MX_EARLY_TAPS) acc = mx_ring_conv<uint16_t>(st, rows, st.k, pos, i, MX_EARLY_TAPS, acc);
+        hp = (unsigned long long)pack2(acc[0], acc[1]) | ((unsigned long long)pack2(acc[2], acc[3]) << 32);
+      }
+      ((unsigned long long *)xs)[i] = hp;
+    }
+    __syncthreads();
+  }
+};
+template <> struct MxPrologue<0> {};
+__device__ __forceinline__ bool mx_dual_prenorm(CStage &st) { return (st.flags & MK_F_PRENORM) && (st.y_scale || st.y2 || st.conv_w); }
+#else
+template <int NS> struct MxPrologue {};
+__device__ __forceinline__ bool mx_dual_prenorm(CStage &) { return false; }
+#endif
+
 // ----------------------------------------------------------------------------- single-token linear, any reduction length
 // out[n] = sum_k W[n, k] x[k], k a multiple of 64.  A wavefront owns a run of rows and takes R of them at a time, 512 U values of
 // k per step, two steps' loads in flight; the first step's are requested before the previous stage's barrier is awaited (not by
 // the wavefront that polls it).  MK_F_JOIN: the sum joins the residual stream, out2 = res + alpha * sum (32-bit), norm_out = the
 // same rounded, and st.out is not written.
-template <int R, int U>
+// PRO: the row comes from an MxPrologue of that many quads per thread (dual kernels; 0: it does not).
+template <int R, int U, int PRO = 0>
 __device__ __forceinline__ void stage_mx_linear_m1_t(CStage &st, Ctx &c, char *smem) {
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int K = st.k, k8 = K / 8, nkb = (k8 + 64 * U - 1) / (64 * U), n = st.n;
@@ -366,10 +546,19 @@ __device__ __forceinline__ void stage_mx_linear_m1_t(CStage &st, Ctx &c, char *s
       for (int u = 0; u < U; u++) b[r][u] = ldg_stream(w + min((kb * U + u) * 64 + lane, k8 - 1));
     }
   };
+  MxPrologue<PRO> pro;
+  if constexpr (PRO > 0) {
+    if (wave != 0) pro.load(st, c);
+  }
   if (wave != 0) load(0, A);
   barrier_wait(c);
   for (int i = k8 + tid; i < nkb * U * 64; i += MK_THREADS) xs4[i] = (u32x4){0u, 0u, 0u, 0u};  // (nothing multiplies the repeated loads)
-  stage_x_m1<true>(st, c, (uint32_t *)smem, (float *)(smem + MK_RED_OFFSET));
+  if constexpr (PRO > 0) {
+    if (wave == 0) pro.load(st, c);
+    pro.finish(st, c, (uint32_t *)smem, (float *)(smem + MK_RED_OFFSET));
+  } else {
+    stage_x_m1<true>(st, c, (uint32_t *)smem, (float *)(smem + MK_RED_OFFSET));
+  }
   if (wave == 0) load(0, A);
   const bool join = st.flags & MK_F_JOIN;
   float acc[R];
@@ -415,9 +604,17 @@ __device__ __forceinline__ void stage_mx_linear_m1_t(CStage &st, Ctx &c, char *s
 }
 // (which single-token linears: those that join the stream, and those no tuned instantiation exists for)
 __device__ __forceinline__ bool mx_linear_m1_form(CStage &st) {
-  return !(st.flags & (MK_F_SILU | MK_F_RES)) && (st.k & 63) == 0 && ((st.flags & MK_F_JOIN) || (st.k != 4096 && st.k != 2048 && st.k != 1024 && st.k != 12288));
+  return !(st.flags & (MK_F_SILU | MK_F_RES)) && (st.k & 63) == 0 && ((st.flags & MK_F_JOIN) || mx_dual_prenorm(st) || (st.k != 4096 && st.k != 2048 && st.k != 1024 && st.k != 12288));
 }
 __device__ __forceinline__ void stage_mx_linear_m1(CStage &st, Ctx &c, char *smem) {
+#if MK_HAVE_DUAL
+  if (mx_dual_prenorm(st)) {
+    if (st.k <= 1024) stage_mx_linear_m1_t<4, 2, 1>(st, c, smem);
+    else if (st.k <= 4 * 4 * MK_THREADS) stage_mx_linear_m1_t<4, 4, 4>(st, c, smem);
+    else stage_mx_linear_m1_t<4, 4, 12>(st, c, smem);
+    return;
+  }
+#endif
   if (st.k <= 512) stage_mx_linear_m1_t<4, 1>(st, c, smem);
   else if (st.k <= 1536) stage_mx_linear_m1_t<4, 3>(st, c, smem);
   else stage_mx_linear_m1_t<4, 4>(st, c, smem);

@@ -80,6 +80,10 @@ enum MkOp {
   MK_OP_HY_SCAN = 31,        // selective scan: recurrent state per request, channel and state; convolution tail
   MK_OP_HY_ROUTE = 32,       // router softmax -> top-k -> renormalise over 32-bit logits (iterations of several tokens)
   MK_OP_HY_EXPERTS = 33,     // expert linears over the routed tokens and a shared expert over all of them
+  // parallel sub-layers, state-space recurrence with one decay per head (mk_dual.hip); a graph that holds one, or an older stage
+  // with an option of theirs, runs on the dual kernels
+  MK_OP_DU_CONV = 34,        // causal convolution per channel whose inputs stay in a ring of rows per request; step sizes and decays beside it
+  MK_OP_DU_SCAN = 35,        // recurrence per head, [states x values] of state, gated 32-bit result
 };
 
 enum MkStageFlags {
@@ -99,6 +103,12 @@ enum MkStageFlags {
   MK_F_JOIN = 16384,     // LINEAR: a single-token iteration adds the result to the residual stream itself (the MX_PRENORM behind is multi-token only)
   MK_F_RELU2 = 32768,    // LINEAR: out = max(acc, 0)^2
   MK_F_OUT32 = 65536,    // MX_HEAD_LINEAR: 32-bit result in out2
+  MK_F_GELU = 131072,    // with MK_F_SILU: the gate is gelu (tanh form) instead of silu
+  MK_F_CLAMP_GLU = 262144,  // with MK_F_SILU, HY_EXPERTS: out = a / (1 + exp(-beta a)) * (b + bias), a = min(gate, limit), b = clamp(up, -limit, limit)
+  MK_F_GROUPS = 524288,  // HY_ROUTE / HY_EXPERTS: sigmoid scores, choice with a correction among the best groups of experts
+  MK_F_ROW_NORM = 1048576,  // FX_ATTN / FX_PREP: all query heads of a row are RMS-normalised together, all key heads likewise
+  MK_F_PORTIONS = 2097152,  // DU_CONV: iterations in which some request brings several tokens (the norm in front does it otherwise)
+  MK_F_IDENTITY = 4194304,  // DU_CONV: the input itself is added
   MK_F_RES_EARLY = 2048, // FX_ADDNORM / LINEAR+ADDNORM: the stage before this one does not write the residual rows, so they may be requested before its barrier
 };
 
@@ -110,6 +120,7 @@ enum MkStageFlags {
 #define MK_MX_MAX_RANK 1024      // low-rank decay projection
 
 #define MK_HY_MAX_STATES 256     // states per channel of the selective scan
+#define MK_DU_MAX_TAPS 16        // taps of the convolutions that keep a ring of rows
 
 #define MK_FX_MAX_HEAD_DIM 512  // largest q/k head the flex attention keeps in a wavefront's registers
 
@@ -207,7 +218,21 @@ struct MkStage {
   const float *a_tab, *d_tab;  // HY_SCAN: fp32 [channels, states] log2(e) * A, [channels]
   void *tail;              // HY_CONV / HY_SCAN: last inputs of the convolution, [state slot][taps - 1][channels]
   const void *in3;         // HY_SCAN: step / B / C rows
-  int ld_in3, pad_hy[13];
+  int ld_in3;
+  // dual stages (mk_dual.hip) and the options of older ones that go with them
+  int chunk;               // FX_ATTN: a position sees only its own chunk of this many (0: no chunks)
+  const float *temp;       // FX_ATTN: fp32 [num_q_heads] factor of the scores
+  const float *y_scale;    // MX_PRENORM / LINEAR+PRENORM: fp32 factor of the summand, element by element (null: none)
+  const void *y2;          // ... a second summand (null: none; `slots` then belongs to it) and its factor
+  const float *y2_scale;
+  const void *conv_w;      // ... and LINEAR: [taps][n] convolution over time of the normed rows, added to them: MX_PRENORM's out3, LINEAR's norm_out (ring: tail; LINEAR's out3: the normed rows); DU_CONV: its weights
+  void *out3;
+  const void *pos_tab;     // FX_EMBED: [pos_rows, k] added by position (null: none)
+  int ld_y2, ld_out3, pos_rows, groups_keep;  // groups_keep: MK_F_GROUPS: groups (field `groups`) that stay open
+  const float *choice_bias;  // MK_F_GROUPS: fp32 [num_experts] correction of the choice
+  float choice_scale, glu_limit_shared;  // ... factor of the chosen scores; MK_F_CLAMP_GLU: limit of the shared expert
+  const float *step_bias;  // DU_CONV: fp32 [num_q_heads] added to the step inputs (column cols[1]); rates in a_tab; steps and decays (column cols[2]) in out2
+  int pad_du[4];
 };
 static_assert(sizeof(MkStage) % 64 == 0, "a descriptor is whole scalar-cache lines");
 

@@ -14,7 +14,7 @@ import time
 import torch
 
 from mirage.mpk import MPK, MirageModelConfig, MPKMetadata, ServingSession
-from mirage.mpk.models import bukatar, dodonex, suborax
+from mirage.mpk.models import bukatar, dodonex, suborax, vizonex
 
 
 def suborax_shape(width=4096, heads=32, kv_heads=8, dim=128, vdim=128, ff=12288, layers=36, vocab=151936) -> dict:
@@ -52,15 +52,29 @@ def bukatar_shape(width=4096, heads=32, kv_heads=8, dim=128, window=1024, keep_f
     return {"architecture": "Bukatar", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "layers": [cycle[i % 4] for i in range(layers)]}
 
 
+def vizonex_shape(width=4096, heads=32, kv_heads=8, dim=128, chunk=1024, dual_heads=64, dual_dim=128, state=128, groups=8, ff=12288, experts=64, top=8, expert_groups=8, expert_groups_kept=4,
+                  expert_ff=1536, layers=36, vocab=151936, positions=32768) -> dict:
+    """A Vizonex config.json of the given sizes: chunked attention and recurrence by turns, dense and expert feed-forwards by turns."""
+    dense = {"kind": "dense", "ff": ff}
+    moe = {"kind": "moe", "router": {"experts": experts, "top": top, "groups": {"count": expert_groups, "keep": expert_groups_kept}, "scale": 2.5},
+           "expert": {"ff": expert_ff, "limit": 7.0}, "shared": {"ff": expert_ff, "limit": 7.0}}
+    att = {"type": "attention", "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "mask": {"size": chunk}}}
+    ssm = {"type": "mamba2", "mixer": {"heads": dual_heads, "vdim": dual_dim, "state": state, "groups": groups, "norm_groups": groups, "conv": 4}}
+    cycle = [dict(att, mlp=dense), dict(ssm, mlp=moe), dict(ssm, mlp=dense), dict(att, mlp=moe)]
+    return {"architecture": "Vizonex", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "canon": {"taps": 4}, "max_positions": positions, "layers": [cycle[i % 4] for i in range(layers)]}
+
+
 # name -> (config.json of a shape, its sizes)
 SHAPES = {"suborax-8b": (suborax_shape, {}), "suborax-2k": (suborax_shape, dict(width=2048, heads=32, kv_heads=4, ff=6144)),
           "dodonex-8b": (dodonex_shape, {}), "dodonex-2k": (dodonex_shape, dict(width=2048, heads=16, q_rank=768, delta_heads=32, delta_dim=64, low_rank=64, ff=6144)),
-          "bukatar-8b": (bukatar_shape, {}), "bukatar-2k": (bukatar_shape, dict(width=2048, heads=16, kv_heads=4, inner=4096, dt_rank=128, ff=6144, experts=128, expert_ff=768))}
+          "bukatar-8b": (bukatar_shape, {}), "bukatar-2k": (bukatar_shape, dict(width=2048, heads=16, kv_heads=4, inner=4096, dt_rank=128, ff=6144, experts=128, expert_ff=768)),
+          "vizonex-8b": (vizonex_shape, {}), "vizonex-2k": (vizonex_shape, dict(width=2048, heads=16, kv_heads=4, dual_heads=32, ff=6144, experts=128, expert_ff=768))}
 
 
 def random_model(config: dict):
     """(MirageModelConfig with random-init weights, the reader's form of the config) of a parsed config.json."""
-    kind, module = {"Suborax": (suborax.SuboraxConfig, suborax), "Dodonex": (dodonex.DodonexConfig, dodonex), "Bukatar": (bukatar.BukatarConfig, bukatar)}[config["architecture"]]
+    kind, module = {"Suborax": (suborax.SuboraxConfig, suborax), "Dodonex": (dodonex.DodonexConfig, dodonex), "Bukatar": (bukatar.BukatarConfig, bukatar),
+                    "Vizonex": (vizonex.VizonexConfig, vizonex)}[config["architecture"]]
     sizes = kind.from_dict(config)
     return MirageModelConfig(architecture=config, state_dict=module.random_state_dict(sizes)), sizes
 

@@ -30,13 +30,10 @@ from typing import List, Optional
 import torch
 
 from ...model_registry import register_model_builder
-from ...persistent_kernel import PersistentKernel, expert_tiles, flex_cache_dims, gated_rows, latent_row_dim, operand_row, operand_tiles, pairs_to_halves
-from ....kernel import bfloat16, float32, int32, int64
-from ..graph_builder import GraphBuilder, MirageModelConfig
-
-
-def _up(n: int, m: int) -> int:
-    return -(-n // m) * m
+from ...persistent_kernel import PersistentKernel, flex_cache_dims, latent_row_dim, operand_row, operand_tiles, pairs_to_halves
+from ....kernel import float32, int32
+from ..graph_builder import MirageModelConfig
+from ..layer_list import LayerListBuilder, up_to as _up
 
 
 def _rot(m: dict):
@@ -232,17 +229,12 @@ def random_state_dict(cfg: BukatarConfig, seed: int = 0, device="cuda", std: flo
 
 
 @register_model_builder("Bukatar")
-class BukatarBuilder(GraphBuilder):
-    owns_kv_cache = True
-    dtypes = (torch.bfloat16, torch.float32)
+class BukatarBuilder(LayerListBuilder):
 
     def __init__(self, mpk: PersistentKernel, weights: Optional[dict] = None):
         super().__init__(mpk, weights)
-        self.tokenizer = None
-        self.returned_hidden_state = None
-        self.logits = None
         self.k_cache, self.v_cache, self.latent_cache, self.state, self.tail, self.state_slots = {}, {}, {}, {}, {}, None
-        self._keep, self._tables, self._attached = {}, {}, {}
+        self._tables, self._attached = {}, {}
 
     @classmethod
     def kernels(cls, dtype, max_num_batched_tokens):
@@ -266,39 +258,6 @@ class BukatarBuilder(GraphBuilder):
         self.build_from_dict(state_dict, True)
 
     # ------------------------------------------------------------------ tensors
-    def _attach(self, t: torch.Tensor, name: str):
-        t = t.contiguous()
-        self._keep[name] = t
-        return self.mpk.attach_input(torch_tensor=t, name=name)
-
-    def release_weights(self, names):
-        return sum(self._keep.pop(n, None) is not None for n in names)
-
-    def _w(self, name: str) -> torch.Tensor:
-        w = self._state[name]
-        if tuple(w.shape) != self._shapes[name]:
-            raise ValueError(f"{name} has shape {tuple(w.shape)}, expected {self._shapes[name]}")
-        return w
-
-    def _matrix(self, name: str, rows: int = None, cols: int = None):
-        return self._pad(self._w(name).to(self.dtype), rows, cols)
-
-    @staticmethod
-    def _pad(w: torch.Tensor, rows: int = None, cols: int = None):
-        return torch.nn.functional.pad(w, (0, (cols or w.shape[-1]) - w.shape[-1], 0, (rows or w.shape[-2]) - w.shape[-2]))
-
-    def _vector(self, name: str, size: int):
-        """Attach a norm weight, a bias or an offset in fp32, zero-padded to `size`."""
-        v = self._w(name).to(torch.float32)
-        return self._attach(torch.nn.functional.pad(v, (0, size - len(v))), name)
-
-    def _rows(self, name: str, cols: int, dt):
-        """Activation rows of one iteration (library-owned, zero-filled), one tensor per name and size."""
-        key = f"{name}_{cols}"
-        if key not in self._acts:
-            self._acts[key] = self.mpk.new_tensor(dims=(self.mpk.max_num_batched_tokens, cols), dtype=dt, name=key, io_category="cuda_tensor")
-        return self._acts[key]
-
     def _rotary(self, dims: int, base: float):
         from .. import checkpoint
         if dims == 0:
@@ -331,25 +290,9 @@ class BukatarBuilder(GraphBuilder):
             elif m.kv_from is None:
                 self.latent_cache[i] = zeros(mpk.max_num_pages, mpk.page_size, latent_row_dim(m.kv_rank, m.rot_dim, self.dtype))
         if self.state:
-            self.state_slots = mpk.meta_tensors.get("state_slots_buffer")
-            if self.state_slots is None:
-                self.state_slots = torch.arange(mpk.max_num_batched_requests, dtype=torch.int32, device=mpk.device)
+            self.state_slots = self._new_state_slots()
 
     # ------------------------------------------------------------------ sub-layers: each returns what the next residual sum takes
-    def _linear(self, inp, w: torch.Tensor, name: str, out):
-        self.mpk.linear_layer(input=inp, weight=self._attach(w, name), output=out, grid_dim=(1, 1, 1), block_dim=(256, 1, 1))
-        return out
-
-    def _sections(self, parts):
-        """parts: (name, matrix, rows it takes).  Returns the stacked matrix, zero-padded, and every part's first row."""
-        col, at = {}, 0
-        for n, _, size in parts:
-            col[n], at = at, at + size
-        w_in = torch.zeros(at, self._W, dtype=self.dtype, device=parts[0][1].device)
-        for n, w, _ in parts:
-            w_in[col[n]:col[n] + w.shape[0], :w.shape[1]] = w.to(self.dtype)
-        return w_in, col, at
-
     def _window(self, i: int, p: str, m: WindowMixer, h):
         mpk, E, H, G, D = self.mpk, self._E, m.heads, m.kv_heads, m.dim
         order = pairs_to_halves(D, m.rot_dims).to(self._w(p + "q").device)
@@ -434,7 +377,7 @@ class BukatarBuilder(GraphBuilder):
         return dict(input=self._linear(act, self._matrix(p + "down", cols=F), p + "down", self._y))
 
     def _experts(self, i: int, p: str, f: ExpertFF, h):
-        mpk, E, W, KW, B = self.mpk, self._E, self._W, operand_row(self.dtype), self.mpk.max_num_batched_tokens
+        mpk, W = self.mpk, self._W
         shared, top = f.shared_ff is not None, f.top
         router = self._matrix(p + "router", cols=W)
         if shared:
@@ -445,37 +388,18 @@ class BukatarBuilder(GraphBuilder):
         ids, shares = self._rows(f"expert_ids_{i}", top, int32), self._rows(f"expert_shares_{i}", _up(top + 1, 4), float32)
         mpk.expert_route_layer(z, ids, shares, f.experts, top, shared)
 
-        def matrices(names, ff):
-            F = _up(ff, max(KW, 16))
-            pick = lambda part, rows, cols: torch.stack([self._matrix(f"{p}{x}.{part}", rows, cols) for x in names])
-            return F, expert_tiles(gated_rows(pick("gate", F, W), pick("up", F, W))), expert_tiles(pick("down", W, F))
-
-        F, w13, w2 = matrices([f"e{j}" for j in range(f.experts)], f.ff)
-        Fs, s13, s2 = matrices(["shared"], f.shared_ff) if shared else (0, None, None)
-        attach = lambda t, name: None if t is None else self._attach(t, p + name)
-        places, A = top + int(shared), max(F, Fs)
-        act = self._rows(f"expert_act_{f.ff}_{f.shared_ff}_{top}", places * A, E)
-        mpk.expert_linear_layer(h, attach(w13, "gate_up"), ids, act, f.experts, top, 2 * F, W, A, gated=True, shared_weight=attach(s13, "shared.gate_up"), shared_n=2 * Fs, shared_k=W)
-        y = self._rows("expert_out", places * W, E)
-        mpk.expert_linear_layer(act, attach(w2, "down"), ids, y, f.experts, top, W, F, W, in_stride=A, shared_weight=attach(s2, "shared.down"), shared_n=W, shared_k=Fs)
+        y, places = self._expert_linears(p, h, ids, f.experts, top, f.ff, f.shared_ff)
         return dict(input=y, slot_weights=shares, slots=places, slot_columns=W)
 
     # ------------------------------------------------------------------ graph
     def build_from_dict(self, state_dict: dict, with_lm_head: bool = True):
         mpk, c = self.mpk, self.config
-        self._shapes = c.tensor_shapes()
-        missing = sorted(set(self._shapes) - set(state_dict))
-        if missing:
-            raise KeyError(f"the state dict lacks {missing}")
+        self._begin(c, state_dict, with_lm_head)
         if mpk.spec_decode_config is not None and any(isinstance(l.mixer, ScanMixer) for l in c.layers):
             raise NotImplementedError("speculative decoding: rows of rejected guesses cannot be taken back out of a recurrent state")
-        self._state, self._acts, self.with_lm_head = state_dict, {}, with_lm_head
-        f32 = self.dtype == torch.float32
-        self._E = E = float32 if f32 else bfloat16
-        self._W = W = _up(c.width, 64)
+        f32, E, W = self.dtype == torch.float32, self._E, self._W
         self.allocate_caches()
         self._slots = self._attach(self.state_slots, "state_slots") if self.state else None
-        one = dict(grid_dim=(1, 1, 1), block_dim=(256, 1, 1))
         # the residual rows alternate between two buffers: a single-token iteration forms the new rows in every workgroup of
         # the linear that reads them, from the old ones
         streams = [self._rows("residual_a", W, float32), self._rows("residual_b", W, float32)]
@@ -489,12 +413,7 @@ class BukatarBuilder(GraphBuilder):
             mpk.residual_prenorm_layer(**{"input": None, **summand}, input_weight=norm_behind, residual=old, weight=weight, new_residual=streams[which], output=h, width=c.width,
                                        eps=c.eps, input_eps=c.eps)
 
-        ids = self._attach(mpk.meta_tensors["input_tokens"], "input_token")
-        spec, spec_tokens = mpk.spec_decode_config, None
-        if spec is not None:
-            all_tokens = self._attach(mpk.meta_tensors["tokens"], "all_tokens")
-            spec_tokens = mpk.draft_forward_layer_dispatcher(spec_decode_config=spec, tokens=all_tokens, grid_dim=(96, 1, 1), block_dim=(128, 1, 1))
-            ids = spec_tokens
+        ids, spec, spec_tokens = self._token_ids(with_lm_head)
         embed = self._attach(self._matrix("embed", cols=W), "embed")
         mpk.embed_scaled_layer(input=ids, weight=embed, residual=streams[which], output=streams[which] if f32 else x16)
         summand, behind = {}, None
@@ -510,19 +429,7 @@ class BukatarBuilder(GraphBuilder):
         join(behind, self._vector("final.norm", W), **summand)
         self.hidden = h
         if not with_lm_head:
-            if spec_tokens is not None:
-                raise ValueError("speculative decoding needs the LM head and the sampling stages in the graph (with_lm_head)")
             self._state = None
             return
-        self.logits = self._rows("logits", c.vocab, E)
-        mpk.linear_layer(input=h, weight=embed, output=self.logits, **one)
-        out = self._attach(mpk.meta_tensors["output_tokens"], "output_token")
-        part = (self._rows("argmax_value", mpk.num_workers, E), self._rows("argmax_index", mpk.num_workers, int64))
-        mpk.argmax_partial_layer(input=self.logits, output=part, grid_dim=(mpk.num_workers, 1, 1), block_dim=(128, 1, 1))
-        mpk.argmax_reduce_layer(input=part, output=out, grid_dim=(1, 1, 1), block_dim=(128, 1, 1))
-        if spec_tokens is not None:
-            self.verify_out = mpk.verify_layer_dispatcher(spec_decode_config=spec, spec_tokens=spec_tokens, target_output=out)
+        self._head_and_sampling(h, embed, c.vocab, spec, spec_tokens)
         self._state = None
-
-    def decode(self, ids: torch.Tensor):
-        return self.tokenizer.decode(ids, skip_special_tokens=True)

@@ -42,6 +42,7 @@ class MirageModelConfig:
 class GraphBuilder(abc.ABC):
     owns_kv_cache = False        # True: the builder allocates the K/V caches when the caller brings none
     default_eos_token_id = None  # used when neither the caller nor the checkpoint names one
+    max_positions = None         # most positions of a sequence where the model itself bounds them
     dtypes = (torch.bfloat16,)   # activation / weight types the model can be built in
 
     def __init__(self, mpk, weights: Optional[Dict[str, Any]] = None):

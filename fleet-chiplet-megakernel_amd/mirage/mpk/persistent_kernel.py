@@ -631,12 +631,13 @@ class PersistentKernel:
     # ------------------------------------------------------------------ layers whose sizes and constants are data (csrc/mk_flex.hip)
     # No counterpart in the reference.  A graph uses them in one activation type, bf16 or fp32 (weights and caches of the same
     # type); the residual stream, norms, angles, scores and softmax are 32-bit in both.
-    def embed_scaled_layer(self, input: DTensor, weight: DTensor, residual: DTensor, output: DTensor, scale: float = 1.0, input_source: int = 1):
+    def embed_scaled_layer(self, input: DTensor, weight: DTensor, residual: DTensor, output: DTensor, scale: float = 1.0, input_source: int = 1, positions: DTensor = None):
         """residual (fp32) = weight[id] * scale, output = the same rounded to the activation type (the two may be one
-        tensor in an fp32 graph).  input_source as in embed_layer."""
+        tensor in an fp32 graph).  input_source as in embed_layer.  positions [n, columns]: the row at the token's position is
+        added (a position behind the last row takes that one: callers keep sequences within the table)."""
         assert input.num_dims == 2 and weight.num_dims == 2 and residual.num_dims == 2 and output.num_dims == 2
-        self._task("embedding_scaled", (1, 1, 1), (256, 1, 1),
-                   [(input, _REPL, -1), (weight, _REPL, -1), (residual, _REPL, -1), (output, _REPL, -1)], [input_source, _f32_bits(scale)])
+        ops = [input, weight] + ([] if positions is None else [positions]) + [residual, output]
+        self._task("embedding_scaled", (1, 1, 1), (256, 1, 1), [(t, _REPL, -1) for t in ops], [input_source, _f32_bits(scale)])
 
     def residual_rmsnorm_layer(self, input: DTensor, residual: DTensor, weight: DTensor, new_residual: DTensor, output: DTensor, width: int = None,
                                alpha: float = 1.0, eps: float = 1e-6, weight_offset: float = 0.0):
@@ -651,19 +652,25 @@ class PersistentKernel:
     def flex_attention_layer(self, input: DTensor, k_cache: DTensor, v_cache: DTensor, cos: DTensor, sin: DTensor, sink: DTensor, q_workspace: DTensor,
                              output: DTensor, num_q_heads: int, num_kv_heads: int, head_dim: int, v_dim: int, rot_dims: int, scale: float,
                              softcap: float = 0.0, unit_norm: bool = False, eps: float = 1e-6, window: int = 0, keep_first: int = 0, values_from_keys: bool = False,
-                             input_bias: DTensor = None):
+                             input_bias: DTensor = None, chunk: int = 0, q_row_weight: DTensor = None, k_row_weight: DTensor = None, score_factors: DTensor = None):
         """Causal paged attention with rotary positions on the first `rot_dims` dims of each q/k head (rotate-half pairs;
         cos / sin are fp32 [positions, rot_dims / 2]), heads divided by their root mean square after the rotation
         (unit_norm), score = softcap * tanh(q.k * scale / softcap) (softcap 0: plain), and a per-head logit `sink` (fp32,
         None: none) that only takes part in the softmax's denominator.  input rows: all q heads, all k heads, all v heads.
         Caches: [pages, page_size, kv_heads, flex_cache_dims(...)], in the kernel's own order inside a page.  With a `window` a
         position sees the `window` newest ones (its own among them) and the `keep_first` first ones.  values_from_keys: the rows
-        hold no value heads, the values are the key heads before rotation.  input_bias: fp32, added to the input rows."""
+        hold no value heads, the values are the key heads before rotation.  input_bias: fp32, added to the input rows.  chunk: a
+        position sees only positions of its own chunk, counted from position 0.  q_row_weight / k_row_weight (fp32, one value per
+        query / key column): all query heads of a row are divided by their common root mean square and multiplied by the weight, all
+        key heads likewise.  score_factors: fp32, one factor of the scores per query head (the sink stays as it is)."""
         assert input.num_dims == 2 and output.num_dims == 2 and q_workspace.num_dims == 2
         assert k_cache.num_dims == 4 and v_cache.num_dims == 4
         ops, p = [input, k_cache, v_cache, cos, sin, sink], [num_q_heads, num_kv_heads, head_dim, v_dim, rot_dims, int(unit_norm), _f32_bits(eps), _f32_bits(scale), _f32_bits(softcap or 0.0)]
-        if window or values_from_keys or input_bias is not None:
+        dual = chunk or q_row_weight is not None or k_row_weight is not None or score_factors is not None
+        if dual or window or values_from_keys or input_bias is not None:
             ops, p = ops + [input_bias], p + [window, keep_first, int(values_from_keys)]
+        if dual:
+            ops, p = ops + [q_row_weight, k_row_weight, score_factors], p + [chunk]
         self._task("flex_attention", (1, 1, 1), (256, 1, 1), [(t, _REPL, -1) for t in ops + [q_workspace, output]], p)
 
     # ------------------------------------------------------------------ mix layers (csrc/mk_mix.hip)
@@ -680,16 +687,21 @@ class PersistentKernel:
 
     def residual_prenorm_layer(self, input: DTensor, residual: DTensor, new_residual: DTensor, output: DTensor, weight: DTensor = None, input_weight: DTensor = None,
                                width: int = None, groups: int = 1, alpha: float = 1.0, eps: float = 1e-6, input_eps: float = 1e-6, input_bias: DTensor = None,
-                               slot_weights: DTensor = None, slots: int = 0, slot_columns: int = 0):
+                               slot_weights: DTensor = None, slots: int = 0, slot_columns: int = 0, factor: DTensor = None, input2: DTensor = None, factor2: DTensor = None):
         """new_residual (fp32) = v = residual + alpha * input (input None: a copy; with `input_weight`: the input is divided by
         its root mean square and multiplied by that weight first); output = v in `groups` equal parts, each divided by its
         own root mean square, times weight (weight None: v itself), rounded to the activation type.  A linear_layer over
         `output` right behind forms it itself when an iteration has one token.  input_bias: fp32, added to the input rows.
-        slot_weights (fp32 [tokens, >= slots]): the input row is the weighted sum of `slots` rows, slot_columns apart."""
-        assert residual.num_dims == 2 and new_residual.num_dims == 2 and output.num_dims == 2
+        slot_weights (fp32 [tokens, >= slots]): the input row is the weighted sum of `slots` rows, slot_columns apart.  input2: a
+        second summand (the slots then belong to it); factor / factor2 (fp32 vectors) multiply the summands element by element.
+        new_residual None: nobody reads v.  A ring_conv_layer(identity=True) over `output` right behind is done by this stage where
+        every request brings one token, and a linear_layer may follow that instead."""
+        assert residual.num_dims == 2 and output.num_dims == 2
         ops, p = [input, input_weight], [output.dim(1) if width is None else int(width), groups, _f32_bits(alpha), _f32_bits(eps), _f32_bits(input_eps)]
         if input_bias is not None or slot_weights is not None:
             ops, p = ops + [input_bias, slot_weights], p + [slots, slot_columns]
+        if factor is not None or input2 is not None or new_residual is None:
+            ops, p = (ops + [None, None] if len(ops) == 2 else ops) + [factor, input2, factor2], p + [0, 0] if len(p) == 5 else p
         self._task("residual_prenorm", (1, 1, 1), (256, 1, 1), [(t, _REPL, -1) for t in ops + [residual, weight, new_residual, output]], p)
 
     def latent_prep_layer(self, input: DTensor, q_weight: DTensor = None, output: DTensor = None, q_column: int = 0, q_rank: int = 0, eps: float = 1e-6, cache: DTensor = None,
@@ -761,19 +773,53 @@ class PersistentKernel:
         self._task("selective_scan", (1, 1, 1), (256, 1, 1), [(t, _REPL, -1) for t in (input, conv, step, bc, A, D, state, tail, state_slots, output)],
                    [states, taps, x_column, z_column, b_column, c_column])
 
-    def expert_route_layer(self, logits: DTensor, ids: DTensor, shares: DTensor, experts: int, top: int, shared: bool = False):
+    def expert_route_layer(self, logits: DTensor, ids: DTensor, shares: DTensor, experts: int, top: int, shared: bool = False, correction: DTensor = None, groups: int = 1,
+                           groups_kept: int = 1, scale: float = 1.0):
         """Softmax over the first `experts` fp32 logits, the `top` largest (ids, int32 [tokens, top]) and their scores divided by their
         sum (shares, fp32).  shared: one more logit, whose sigmoid becomes shares[:, top].  Followed by the expert_linear_layer that
-        reads the ids (a single token is routed inside that one)."""
-        self._task("expert_route", (1, 1, 1), (256, 1, 1), [(logits, _REPL, -1), (ids, _REPL, -1), (shares, _REPL, -1)], [experts, top, int(shared)])
+        reads the ids (a single token is routed inside that one).  With a `correction` (fp32 [experts]): scores are sigmoids of the logits;
+        choices are made on score + correction among the experts of the `groups_kept` best of `groups` equal groups of neighbours, a
+        group's worth being the sum of its two largest; shares are scale times the chosen scores, the shared expert's is 1 (no logit)."""
+        ops, p = [logits, ids, shares], [experts, top, int(shared)]
+        if correction is not None:
+            ops, p = [logits, correction, ids, shares], p + [groups, groups_kept, _f32_bits(scale)]
+        self._task("expert_route", (1, 1, 1), (256, 1, 1), [(t, _REPL, -1) for t in ops], p)
 
     def expert_linear_layer(self, input: DTensor, weight: DTensor, ids: DTensor, output: DTensor, experts: int, top: int, n: int, k: int, out_stride: int, in_stride: int = 0,
-                            gated: bool = False, shared_weight: DTensor = None, shared_n: int = 0, shared_k: int = 0):
+                            gated: bool = False, shared_weight: DTensor = None, shared_n: int = 0, shared_k: int = 0, clamp: tuple = None):
         """output[t, s * out_stride + j] = sum_i W[ids[t, s]][j][i] input[t, s * in_stride + i] for every place s < top of a token, and with a
         shared_weight place `top` for all tokens.  Weights are operand_tiles, rows padded to 32 per expert; gated: 16 gate rows
-        and 16 up rows by turns, output = silu(gate) up (n counts both).  in_stride 0: all places read the token's one row."""
+        and 16 up rows by turns, output = silu(gate) up (n counts both).  in_stride 0: all places read the token's one row.
+        clamp (limit, beta, bias, limit of the shared expert): output = a / (1 + exp(-beta a)) * (b + bias), a = min(gate, limit), b = up clamped
+        to [-limit, limit]."""
         self._task("expert_linear", (1, 1, 1), (256, 1, 1), [(t, _REPL, -1) for t in (input, weight, shared_weight, ids, output)],
-                   [experts, top, n, k, shared_n, shared_k, int(gated), in_stride, out_stride])
+                   [experts, top, n, k, shared_n, shared_k, int(gated), in_stride, out_stride] + ([] if clamp is None else [_f32_bits(x) for x in clamp]))
+
+    # ------------------------------------------------------------------ dual layers (csrc/mk_dual.hip)
+    # Usable in one graph with the flex layers, norms, head linears, routing and experts, not with latent attention, the delta rule or the
+    # selective scan; constants are arguments.
+    def gelu_mul_layer(self, input: DTensor, output: DTensor, groups: int = 1):
+        """output = gelu(gate) up (tanh form) behind the linear_layer that writes `input` through a shuffled [gate ; up] weight of that many
+        groups (library-owned; it is the linear's epilogue and `input` itself is not written)."""
+        self._task("gelu_mul", (groups, 1, 1), (256, 1, 1), [(input, _REPL, -1), (output, _REPL, -1)])
+
+    def ring_conv_layer(self, input: DTensor, weight: DTensor, ring: DTensor, state_slots: DTensor, output: DTensor, bias: DTensor = None, column: int = 0, silu: bool = False,
+                        identity: bool = False, heads: int = 0, step_column: int = 0, decay_column: int = 0, step_bias: DTensor = None, rates: DTensor = None, steps: DTensor = None):
+        """output[t, c] = act(bias[c] + sum_j weight[j, c] x[t - (taps - 1) + j, c]) over a request's tokens, x = input[:, column + c], zeros before
+        the first; silu: act; identity: x[t, c] is added.  weight [taps, channels] of the rows' type; ring [slots, taps, channels] holds a
+        request's last inputs, position p in row p % taps.  With a step_bias (fp32 [heads]): steps[:, h] = softplus(input[:, step_column + h] +
+        step_bias[h]) and steps[:, decay_column + h] = 2^(rates[h] times that), fp32."""
+        self._task("ring_conv", (1, 1, 1), (256, 1, 1), [(t, _REPL, -1) for t in (input, weight, bias, ring, state_slots, step_bias, rates, output, steps)],
+                   [column, int(silu), int(identity), heads, step_column, decay_column])
+
+    def dual_scan_layer(self, input: DTensor, conv: DTensor, steps: DTensor, D: DTensor, state: DTensor, state_slots: DTensor, output: DTensor, heads: int, values: int, states: int,
+                        groups: int, z_column: int, x_column: int, b_column: int, c_column: int, decay_column: int):
+        """Per request and head, in fp32: S <- decay S + step B x^T (S is states x values), output = (S^T C + D x) silu(z), an fp32 row.  x, B and C
+        are columns of the conv rows (a group's B and C take the states rounded up to 4; head h reads group h // (heads / groups)),
+        z of the input rows, steps and decays come from ring_conv_layer.  state fp32 [slots, heads, values, states rounded up to 4] is carried
+        from iteration to iteration (zero where a request begins)."""
+        self._task("dual_scan", (1, 1, 1), (256, 1, 1), [(t, _REPL, -1) for t in (input, conv, steps, D, state, state_slots, output)],
+                   [heads, values, states, groups, z_column, x_column, b_column, c_column, decay_column])
 
     # layers of the reference that are outside the one-GPU decode path
     def tensor_init_layer(self, *args, **kwargs):

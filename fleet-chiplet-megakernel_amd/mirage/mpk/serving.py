@@ -53,7 +53,7 @@ class ServingSession:
         self.mpk = mpk
         pk = mpk.persistent_kernel
         self.page_size, self.max_rows, self.max_requests = pk.page_size, pk.max_num_batched_tokens, pk.max_num_batched_requests
-        self.rows_per_request, self.max_seq = pk.max_tokens_per_request, pk.max_seq_length
+        self.rows_per_request, self.max_seq = pk.max_tokens_per_request, min(pk.max_seq_length, mpk.model_builder.max_positions or pk.max_seq_length)
         self.pool = PagePool(pk.max_num_pages)
         # one state slot per batch slot: the kernel starts a request's state from zero where its position is zero
         self.state_slots = getattr(mpk.model_builder, "state_slots", None)
@@ -179,8 +179,8 @@ class ServingSession:
         out = [list(p) for p in prompts]
         need = [-(-(len(p) + max_new_tokens) // self.page_size) for p in prompts]
         for i, p in enumerate(prompts):
-            if not p or need[i] > self.pool.num_pages:
-                raise ValueError(f"prompt {i} is empty or its {len(p) + max_new_tokens} positions exceed the cache")
+            if not p or need[i] > self.pool.num_pages or len(p) + max_new_tokens - 1 > self.max_seq:
+                raise ValueError(f"prompt {i} is empty or its {len(p) + max_new_tokens} positions exceed the cache or max_seq_length={self.max_seq}")
         waiting, live, reserved = list(range(len(prompts))), {}, 0
         while waiting or live:
             while waiting and len(live) < self.max_requests and reserved + need[waiting[0]] <= self.pool.num_pages:
