@@ -96,10 +96,18 @@ __device__ __forceinline__ void stage_fx_embed(CStage &st, Ctx &c, const MkRunti
 #if MK_HAVE_DUAL
     if (st.pos_tab) {  // (the caller keeps positions inside the table)
       const E *pos = (const E *)st.pos_tab + (size_t)min(c.sh_tok[t], st.pos_rows - 1) * k;
-      for (int i = threadIdx.x; i < k; i += MK_THREADS) {
-        const float v = fmaf(fx_val(src[i]), scale, fx_val(pos[i]));
-        if (out32) stc_f32(out32 + i, v);
-        fx_stc(out + i, fx_round<E>(v));
+      if ((k & 3) == 0) {
+        for (int i = threadIdx.x * 4; i < k; i += MK_THREADS * 4) {
+          const f32x4 v = fx_ld_quad(src + i) * scale + fx_ld_quad(pos + i);
+          if (out32) fx_stc_quad(out32 + i, v);
+          fx_stc_quad(out + i, v);
+        }
+      } else {
+        for (int i = threadIdx.x; i < k; i += MK_THREADS) {
+          const float v = fmaf(fx_val(src[i]), scale, fx_val(pos[i]));
+          if (out32) stc_f32(out32 + i, v);
+          fx_stc(out + i, fx_round<E>(v));
+        }
       }
       continue;
     }

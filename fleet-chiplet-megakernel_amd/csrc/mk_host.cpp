@@ -1015,6 +1015,8 @@ int lower_residual_prenorm(mk_graph *g, size_t &i) {
     const std::string behind = i + 1 < g->ltasks.size() ? g->ltasks[i + 1].name : "";
     fuse = !silu && !yw && !yb && groups == 1 && n % 64 == 0 && behind != "silu_mul" && behind != "gelu_mul" && behind != "silu_mul_linear_with_residual";
   }
+  // rows that are only normalised: a stage whose wavefronts share the parts is faster than every workgroup of the linear reading all of them
+  if (!y && no_xo) fuse = false;
   if (fuse) st.flags |= MK_F_ONLY_MULTI;
   g->stages.push_back(st);
   g->stage_desc.push_back(fmt("MX_PRENORM%s %s + %g * %s%s%s%s%s -> %s, %s k=%d parts=%d", (st.flags & MK_F_ONLY_MULTI) ? "[multi-token only]" : "", x.name.c_str(), st.alpha, yw ? "norm of " : "", y ? y->name.c_str() : "0", y2 ? " + " : "",

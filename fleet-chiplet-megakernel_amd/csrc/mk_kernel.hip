@@ -4240,7 +4240,7 @@ __device__ __forceinline__ void run_stage_program(const MkRuntime &rt, const MkR
 #if MK_HAVE_HYB
 #if MK_HAVE_DUAL
         case MK_OP_DU_CONV: stage_du_conv<E>(st, c, M); break;
-        case MK_OP_DU_SCAN: stage_du_scan<E>(st, c, rt, M, MAXM == 1 || single); break;
+        case MK_OP_DU_SCAN: stage_du_scan<E>(st, c, rt, M, MAXM == 1 || single, smem); break;
 #else
         case MK_OP_HY_CONV: stage_hy_conv<E>(st, c, rt, M); break;
         case MK_OP_HY_STEP: stage_mx_head_linear_t<E, 1, MX_STEP, false>(st, c, M, smem); break;

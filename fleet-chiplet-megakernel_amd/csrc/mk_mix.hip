@@ -26,31 +26,43 @@ __device__ __forceinline__ void mx_stc_quad(float *p, f32x4 v) {
   asm volatile("global_store_dwordx4 %0, %1, off sc1" ::"v"((const MK_GLOBAL void *)(unsigned long long)p), "v"(v) : "memory");
 }
 
-// Four values of a norm stage's summand: row `y` from value 4 s on.  Hybrid kernels: the sum of st.slots rows of the
-// token, st.ld_slot apart, weighted by `w` (four of them requested at once).  (A bias is added by the caller, who has it in advance.)
-template <typename E>
-__device__ __forceinline__ f32x4 mx_summand(CStage &st, const E *y, const float *w, int s) {
+// Values of a norm stage's summand: this thread's NS quads of row `y`, at(j) the index of quad j.  Hybrid kernels: with `places` the sum of
+// st.slots rows of the token, st.ld_slot apart, weighted by `w`; the quads of SQ rows are requested at once.  (A bias is added by the caller, who has
+// it in advance.)
+template <typename E, int NS, typename At>
+__device__ __forceinline__ void mx_summands(CStage &st, const E *y, const float *w, bool places, f32x4 (&v)[NS], At at) {
 #if MK_HAVE_HYB
-  if (st.slots) {
-    f32x4 v = {0.f, 0.f, 0.f, 0.f};
-    for (int q0 = 0; q0 < st.slots; q0 += 4) {
-      f32x4 x[4];
-      float f[4];
+  if (places) {
+    constexpr int SQ = NS <= 4 ? 4 : 1;
 #pragma unroll
-      for (int q = 0; q < 4; q++) {
-        const int at = min(q0 + q, st.slots - 1);
-        x[q] = fx_ldc_quad(y + (size_t)at * st.ld_slot + 4 * s);
-        f[q] = q0 + q < st.slots ? ldc_f32(w + at) : 0.f;
+    for (int j = 0; j < NS; j++) v[j] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    for (int q0 = 0; q0 < st.slots; q0 += SQ) {
+      f32x4 x[SQ][NS];
+      float f[SQ];
+#pragma unroll
+      for (int q = 0; q < SQ; q++) {
+        const int r = min(q0 + q, st.slots - 1);
+        f[q] = q0 + q < st.slots ? ldc_f32(w + r) : 0.f;
+#pragma unroll
+        for (int j = 0; j < NS; j++) x[q][j] = fx_ldc_quad(y + (size_t)r * st.ld_slot + 4 * at(j));
       }
 #pragma unroll
-      for (int q = 0; q < 4; q++) v += x[q] * f[q];
+      for (int q = 0; q < SQ; q++)
+#pragma unroll
+        for (int j = 0; j < NS; j++) v[j] += x[q][j] * f[q];
     }
-    return v;
+    return;
   }
-  return fx_ldc_quad(y + 4 * s);
-#else
-  return fx_ldc_quad(y + 4 * s);
 #endif
+#pragma unroll
+  for (int j = 0; j < NS; j++) v[j] = fx_ldc_quad(y + 4 * at(j));
+}
+// ... one quad
+template <typename E>
+__device__ __forceinline__ f32x4 mx_summand(CStage &st, const E *y, const float *w, int s) {
+  f32x4 v[1];
+  mx_summands<E, 1>(st, y, w, MK_HAVE_HYB && st.slots, v, [&](int) { return s; });
+  return v[0];
 }
 
 #if MK_HAVE_DUAL
@@ -113,15 +125,26 @@ __device__ __forceinline__ void stage_mx_prenorm_t(CStage &st, Ctx &c, int M, bo
   }
 #endif
 #if MK_HAVE_DUAL
-  f32x4 ys[NS], y2s[NS];
-  if (st.y_scale) {
+  // factors and the convolution's weights (short rows: in advance; long ones: where they are used)
+  constexpr bool AHEAD = NS <= 4;
+  constexpr int NA = AHEAD ? NS : 1, TA = AHEAD ? 4 : 1;
+  const f32x4 one = {1.f, 1.f, 1.f, 1.f};
+  f32x4 ys[NA], y2s[NA], cw[NA][TA], rg[NA][TA];
+  if constexpr (AHEAD) {
 #pragma unroll
-    for (int j = 0; j < NS; j++) ys[j] = ((const f32x4 *)st.y_scale)[at(j)];
-  }
-  if (st.y2) {
+    for (int j = 0; j < NS; j++) {
+      ys[j] = st.y_scale ? ((const f32x4 *)st.y_scale)[at(j)] : one;
+      y2s[j] = st.y2_scale ? ((const f32x4 *)st.y2_scale)[at(j)] : one;
+    }
+    if (st.conv_w && single) {
 #pragma unroll
-    for (int j = 0; j < NS; j++) y2s[j] = st.y2_scale ? ((const f32x4 *)st.y2_scale)[at(j)] : (f32x4){1.f, 1.f, 1.f, 1.f};
+      for (int b = 0; b < TA; b++)
+#pragma unroll
+        for (int j = 0; j < NS; j++) cw[j][b] = fx_ld_quad((const E *)st.conv_w + (size_t)(st.taps - 1 - min(b, st.taps - 1)) * st.n + 4 * at(j));
+    }
   }
+  auto ys_at = [&](int j) { return AHEAD ? ys[AHEAD ? j : 0] : st.y_scale ? ((const f32x4 *)st.y_scale)[at(j)] : one; };
+  auto y2s_at = [&](int j) { return AHEAD ? y2s[AHEAD ? j : 0] : st.y2_scale ? ((const f32x4 *)st.y2_scale)[at(j)] : one; };
 #endif
   // the residual row was written at least one barrier earlier than y: requested before the barrier is awaited (not by the
   // wavefront that polls it)
@@ -135,28 +158,36 @@ __device__ __forceinline__ void stage_mx_prenorm_t(CStage &st, Ctx &c, int M, bo
   barrier_wait(c);
   for (int t = t0; t < M; t += c.G) {
     if (!(pre && t == t0)) load_x(t);
+#if MK_HAVE_DUAL
+    const bool conv = st.conv_w && single;
+    const int pos = __builtin_amdgcn_readfirstlane(c.sh_tok[t]), taps = st.taps;
+    E *ring = conv ? (E *)st.tail + (size_t)__builtin_amdgcn_readfirstlane(c.state_ids[__builtin_amdgcn_readfirstlane(c.sh_tok[MK_MAX_TOKENS + t])]) * taps * st.n : nullptr;
+    if constexpr (AHEAD) {
+      if (conv) {
+#pragma unroll
+        for (int b = 1; b < TA; b++)
+#pragma unroll
+          for (int j = 0; j < NS; j++) rg[j][b] = fx_ldc_quad(ring + (size_t)(max(pos - min(b, taps - 1), 0) % taps) * st.n + 4 * at(j));
+      }
+    }
+#endif
     if (st.in) {
       f32x4 y[NS];
-#pragma unroll
-      for (int j = 0; j < NS; j++) {
+      const float *sw = MK_HAVE_HYB ? st.slot_w + (size_t)t * st.ld_slot_w : nullptr;
 #if MK_HAVE_DUAL
-        if (st.y2) {
-          y[j] = fx_ldc_quad((const E *)st.in + (size_t)t * st.ld_in + 4 * at(j));
-          continue;
-        }
-#endif
-        y[j] = mx_summand<E>(st, (const E *)st.in + (size_t)t * st.ld_in, MK_HAVE_HYB ? st.slot_w + (size_t)t * st.ld_slot_w : nullptr, at(j));
-      }
-#if MK_HAVE_DUAL
+      mx_summands<E, NS>(st, (const E *)st.in + (size_t)t * st.ld_in, sw, st.slots && !st.y2, y, at);
       if (st.y2) {
         f32x4 y2[NS];
+        mx_summands<E, NS>(st, (const E *)st.y2 + (size_t)t * st.ld_y2, sw, st.slots, y2, at);
 #pragma unroll
-        for (int j = 0; j < NS; j++) y2[j] = mx_summand<E>(st, (const E *)st.y2 + (size_t)t * st.ld_y2, st.slot_w + (size_t)t * st.ld_slot_w, at(j));
+        for (int j = 0; j < NS; j++) {
+          const f32x4 f2 = y2s_at(j);
 #pragma unroll
-        for (int j = 0; j < NS; j++)
-#pragma unroll
-          for (int e = 0; e < 4; e++) x[j][e] = fmaf(y2s[j][e], y2[j][e], x[j][e]);
+          for (int e = 0; e < 4; e++) x[j][e] = fmaf(f2[e], y2[j][e], x[j][e]);
+        }
       }
+#else
+      mx_summands<E, NS>(st, (const E *)st.in + (size_t)t * st.ld_in, sw, MK_HAVE_HYB && st.slots, y, at);
 #endif
       float f = st.alpha;
 #if MK_HAVE_HYB
@@ -178,7 +209,7 @@ __device__ __forceinline__ void stage_mx_prenorm_t(CStage &st, Ctx &c, int M, bo
 #if MK_HAVE_DUAL
       if (st.y_scale) {
 #pragma unroll
-        for (int j = 0; j < NS; j++) y[j] *= ys[j];
+        for (int j = 0; j < NS; j++) y[j] *= ys_at(j);
       }
 #endif
 #pragma unroll
@@ -220,17 +251,23 @@ __device__ __forceinline__ void stage_mx_prenorm_t(CStage &st, Ctx &c, int M, bo
         }
         if (st.out) fx_stc_quad((E *)st.out + (size_t)t * st.ld_out + 4 * s, o);
 #if MK_HAVE_DUAL
-        if (st.conv_w && single) {
-          const int pos = __builtin_amdgcn_readfirstlane(c.sh_tok[t]), taps = st.taps;
-          E *ring = (E *)st.tail + (size_t)__builtin_amdgcn_readfirstlane(c.state_ids[__builtin_amdgcn_readfirstlane(c.sh_tok[MK_MAX_TOKENS + t])]) * taps * st.n;
-          const f32x4 w0 = fx_ld_quad((const E *)st.conv_w + (size_t)(taps - 1) * st.n + 4 * s);
+        if (conv) {
           f32x4 h, acc;
 #pragma unroll
-          for (int e = 0; e < 4; e++) {
-            h[e] = fx_val(fx_round<E>(o[e]));
-            acc[e] = fmaf(w0[e], h[e], h[e]);
+          for (int e = 0; e < 4; e++) h[e] = fx_val(fx_round<E>(o[e]));
+          acc = h;
+          if constexpr (AHEAD) {
+#pragma unroll
+            for (int b = 0; b < TA; b++)
+#pragma unroll
+              for (int e = 0; e < 4; e++) acc[e] = b < taps && b <= pos ? fmaf(b ? rg[j][b][e] : h[e], cw[j][b][e], acc[e]) : acc[e];
+            if (taps > TA) acc = mx_ring_conv<E>(st, ring, st.n, pos, s, TA, acc);
+          } else {
+            const f32x4 w0 = fx_ld_quad((const E *)st.conv_w + (size_t)(taps - 1) * st.n + 4 * s);
+#pragma unroll
+            for (int e = 0; e < 4; e++) acc[e] = fmaf(w0[e], h[e], acc[e]);
+            acc = mx_ring_conv<E>(st, ring, st.n, pos, s, 1, acc);
           }
-          acc = mx_ring_conv<E>(st, ring, st.n, pos, s, 1, acc);
           fx_stc_quad((E *)st.out3 + (size_t)t * st.ld_out3 + 4 * s, acc);
           fx_stc_quad(ring + (size_t)(pos % taps) * st.n + 4 * s, h);
         }
@@ -240,8 +277,30 @@ __device__ __forceinline__ void stage_mx_prenorm_t(CStage &st, Ctx &c, int M, bo
   }
   c.wrote_through = true;
 }
+#if MK_HAVE_DUAL
+template <typename E, typename Put>
+__device__ __forceinline__ void mx_norm_row(const E *src, const float *w, int n, float eps, int lane, Put put);
+// Rows that are only normalised, in parts of whole quads: a wavefront per (row, part).
+template <typename E>
+__device__ __forceinline__ void stage_mx_norm_parts(CStage &st, Ctx &c, int M) {
+  barrier_wait(c);
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), ng = st.norm_groups, gl = st.k / ng;
+  for (int i = mx_wave_item(c, wave); i < M * ng; i += c.G * MK_WAVES) {
+    const int t = i / ng, q = i - t * ng;
+    E *o = (E *)st.out + (size_t)t * st.ld_out + q * gl;
+    mx_norm_row<float>((const float *)st.res + (size_t)t * st.ld_res + q * gl, (const float *)st.norm_w + q * gl, gl, st.eps, lane, [&](int s, f32x4 v) { fx_stc_quad(o + 4 * s, v); });
+  }
+  c.wrote_through = true;
+}
+#endif
 template <typename E>
 __device__ __forceinline__ void stage_mx_prenorm(CStage &st, Ctx &c, int M, bool single, char *smem) {
+#if MK_HAVE_DUAL
+  if (!st.in && !st.out2 && st.out && !st.conv_w && st.norm_groups && (st.k / st.norm_groups) % 4 == 0 && st.k / st.norm_groups <= MK_MX_MAX_NORM_ROW) {
+    stage_mx_norm_parts<E>(st, c, M);
+    return;
+  }
+#endif
   if (st.n <= 4 * 4 * MK_THREADS) stage_mx_prenorm_t<E, 4>(st, c, M, single, smem);
   else stage_mx_prenorm_t<E, 12>(st, c, M, single, smem);
 }
@@ -428,7 +487,7 @@ __device__ __forceinline__ void mx_x_m1_prenorm_wave(CStage &st, Ctx &c, uint32_
 #define MX_EARLY_TAPS 4
 template <int NS>
 struct MxPrologue {
-  f32x4 g[NS], ys[NS], y2s[NS], x[NS];
+  f32x4 g[NS], x[NS], ys[NS], y2s[NS];
   unsigned long long cw[NS][MX_EARLY_TAPS], ring[NS][MX_EARLY_TAPS];
   int pos, k4;
   uint16_t *rows;
@@ -464,16 +523,14 @@ struct MxPrologue {
   }
   __device__ __forceinline__ void finish(CStage &st, const Ctx &c, uint32_t *xs, float *red) {
     auto quad = [](unsigned long long u) { return (f32x4){bf_lo((uint32_t)u), bf_hi((uint32_t)u), bf_lo((uint32_t)(u >> 32)), bf_hi((uint32_t)(u >> 32))}; };
+    auto pack = [](f32x4 o) { return (unsigned long long)pack2(o[0], o[1]) | ((unsigned long long)pack2(o[2], o[3]) << 32); };
     const int tid = threadIdx.x;
     if (!(st.flags & MK_F_RES_EARLY)) load_x(st);
-    f32x4 y[NS], y2[NS];
     if (st.y_in) {
-#pragma unroll
-      for (int j = 0; j < NS; j++) y[j] = st.y2 ? fx_ldc_quad((const uint16_t *)st.y_in + 4 * at(j)) : mx_summand<uint16_t>(st, (const uint16_t *)st.y_in, st.slot_w, at(j));
-      if (st.y2) {
-#pragma unroll
-        for (int j = 0; j < NS; j++) y2[j] = mx_summand<uint16_t>(st, (const uint16_t *)st.y2, st.slot_w, at(j));
-      }
+      f32x4 y[NS], y2[NS];
+      auto at_ = [&](int j) { return at(j); };
+      mx_summands<uint16_t, NS>(st, (const uint16_t *)st.y_in, st.slot_w, st.slots && !st.y2, y, at_);
+      if (st.y2) mx_summands<uint16_t, NS>(st, (const uint16_t *)st.y2, st.slot_w, st.slots, y2, at_);
 #pragma unroll
       for (int j = 0; j < NS; j++)
 #pragma unroll
@@ -491,8 +548,7 @@ struct MxPrologue {
     for (int j = 0; j < NS; j++) {
       const int i = tid + j * MK_THREADS;
       if (i >= k4) continue;
-      const f32x4 o = (x[j] * r) * g[j];
-      unsigned long long hp = (unsigned long long)pack2(o[0], o[1]) | ((unsigned long long)pack2(o[2], o[3]) << 32);
+      unsigned long long hp = pack((x[j] * r) * g[j]);
       if (c.vid == 0) {
         if (st.out2) stc_16B((u32x4 *)st.out2 + i, __builtin_bit_cast(u32x4, x[j]));
         stc_u64((unsigned long long *)(st.conv_w ? st.out3 : st.norm_out) + i, hp);
@@ -508,7 +564,7 @@ struct MxPrologue {
           for (int e = 0; e < 4; e++) acc[e] = b < st.taps && b <= pos ? fmaf(v[e], w[e], acc[e]) : acc[e];
         }
         if (st.taps > MX_EARLY_TAPS) acc = mx_ring_conv<uint16_t>(st, rows, st.k, pos, i, MX_EARLY_TAPS, acc);
-        hp = (unsigned long long)pack2(acc[0], acc[1]) | ((unsigned long long)pack2(acc[2], acc[3]) << 32);
+        hp = pack(acc);
       }
       ((unsigned long long *)xs)[i] = hp;
     }

@@ -212,7 +212,7 @@ def test_lowering():
     c = config([chunked(4, 2, 16, 24, 20, dense(48)), dual(4, 12, 8, 2, 2, 4, moe(6, 2, 3, 2, 24, 24)), chunked(4, 2, 16, 24, 20, None)], 64, 90)
     n, conv = "MX_PRENORM[multi-token", "DU_CONV[portions]"
     att = [n, conv, "LINEAR", "FX_PREP[portions]", "FX_ATTN", "LINEAR"]
-    want = (["FX_EMBED"] + att + ["LINEAR+gelu", "LINEAR"] + [n, conv, "LINEAR", "DU_CONV", "DU_SCAN", n, "LINEAR", "MX_HEAD_LINEAR", "HY_ROUTE[multi-token", "HY_EXPERTS+route+clamped", "HY_EXPERTS"] +
+    want = (["FX_EMBED"] + att + ["LINEAR+gelu", "LINEAR"] + [n, conv, "LINEAR", "DU_CONV", "DU_SCAN", "MX_PRENORM", "LINEAR", "MX_HEAD_LINEAR", "HY_ROUTE[multi-token", "HY_EXPERTS+route+clamped", "HY_EXPERTS"] +
             att + [n, "LINEAR", "ARGMAX_PARTIAL", "ARGMAX_REDUCE"])
     m = _host_mpk(c)
     assert _ops(m) == want

@@ -37,8 +37,10 @@ CONFIGS = {
 }
 
 
-def weights(cfg, seed=0):
-    """bf16-valued weights under their checkpoint names; norm weights, factors and offsets away from their neutral values."""
+def weights(cfg, seed=None):
+    """bf16-valued weights under their checkpoint names; norm weights, factors and offsets away from their neutral values.  (The "odd" model's seed is
+    one whose routers have next to no near ties on the tests' prompts: a choice that rounding turns changes a request for good.)"""
+    seed = (17 if cfg is CONFIGS["odd"] else 0) if seed is None else seed
     g = torch.Generator().manual_seed(seed)
     out = {}
     for name, shape in VizonexConfig.from_dict(cfg).tensor_shapes().items():
